@@ -49,6 +49,10 @@ extern "C" {
 #define MLORA_F16 0
 #define MLORA_F32 1
 
+/* gated products: silu(g) * u, and g sigmoid(alpha g) (u + 1) with g and u clipped to a limit */
+#define MLORA_GLU_SILU    0
+#define MLORA_GLU_CLIPPED 1
+
 /* y = acc, or y += acc, in the epilogue of the linear kernels */
 #define MLORA_STORE       0
 #define MLORA_ACCUMULATE  1
@@ -568,6 +572,14 @@ typedef struct mlora_decode_plan {
 } mlora_decode_plan;
 
 int mlora_decode_step(const mlora_decode_plan* plan, void* stream);
+
+/* act = clipped gated product of [gate | up] = xf . Wp^T: with g = min(scale gate, limit), u = clamp(scale up, +-limit),
+ * g sigmoid(alpha g) (u + 1).  The forms of mlora_gemv_frag_silu (interleaved tiles, T <= 64), mlora_linear_frag_silu
+ * (persistent GEMM shapes) and mlora_silu_mul. */
+int mlora_gemv_frag_clipglu(void* act, const void* xf, const void* Wil_p, int T, int K, int I, float scale, float limit, float alpha, void* stream);
+int mlora_linear_frag_clipglu(void* act, const void* xf, const void* Wp, int T, int K, int I, float scale, float limit, float alpha, void* stream);
+int mlora_clipglu_mul(void* out, int out_layout, const void* gate, const void* up, int ld, int T, int I, float scale, float limit, float alpha,
+                      void* stream);
 
 #ifdef __cplusplus
 }

@@ -1,0 +1,72 @@
+/*
+ * mlora_decoder.h - C ABI of the kernels for decoders with latent attention, experts and a one-number norm.
+ *
+ * The library is built once per element type (libmlora_hip.so fp16, libmlora_bf16.so bfloat16, libmlora_f32.so fp32) with
+ * the same entry points; "elements" below are of that type, and MLORA_F16 names it in dtype arguments.  The functions
+ * declared here are in the bfloat16 and the fp32 library.  In the latter activations are row-major, weights are plain
+ * [N, K] and fragment-ordered outputs are refused.  Conventions as in mlora.h.
+ */
+#ifndef MLORA_DECODER_H
+#define MLORA_DECODER_H
+
+#include "mlora.h"
+
+#ifdef __cplusplus
+extern "C" {
+#endif
+
+/* Residual stream x [T, Hp] fp32 (columns H..Hp-1 zero): x += the n_part blocks part[q][T][Hp], in order; with a branch
+ * x += branch / rms(branch) * branch_w; then, where an output is given, out = x / rms(x) * gain, rms over the H columns with
+ * eps inside the root; in fragment order and / or row-major [T, Hp]. */
+int mlora_stream_norm(void* out_frag, void* out_row, float* x, const float* part, int n_part, const float* branch, const void* branch_w,
+                      float eps, float gain, int T, int H, int Hp, void* stream);
+
+/* Per-layer token input: out[t, n] = gelu_tanh(W[n] . x[t]) * table[ids[t], col0 + n] for n < dim, 0 for dim <= n < N.
+ * mlora_token_gate takes the residual stream (with pending partial sums, as above), W packed [N, K], and writes fragment
+ * order; mlora_token_gate_mul takes the product z [T, N] of a separate linear. */
+int mlora_token_gate(void* out_frag, const float* x, const float* part, int n_part, const void* Wp, const void* table, int ld_table, int col0,
+                     int dim, const int32_t* ids, int V, int T, int K, int N, void* stream);
+int mlora_token_gate_mul(void* out, const void* z, const void* table, int ld_table, int col0, int dim, const int32_t* ids, int V, int T, int N,
+                         void* stream);
+
+/* Latent attention (layouts at the top of latent_attention.hip).  mlora_latent_prep takes the token's projections
+ * qkv [T, ld] times `gain`: rotates the heads' query parts (columns off_rot .. + H rot) into q [T, H, NB 32], and, with c_norm,
+ * norms the latent (off_c .. + R), rotates the shared key part (off_kr .. + rot) and stores both in the token's page slot.
+ * mlora_head_linear: y[t, h] = alpha W[h] . x[t, h].  mlora_latent_attn: causal softmax over the sequence's pages with
+ * scores (q . cached) * scale and, with `sink`, exp(sink[h]) in the denominator; out [T, H, ceil32(R)].  splits > 1 needs
+ * a workspace. */
+int mlora_latent_prep(void* q, void* cache, const void* qkv, int ld, int off_rot, int off_c, int off_kr, float gain, const void* c_norm,
+                      float eps, const int32_t* block_table, int max_blocks, const int32_t* tok_seq, const int32_t* tok_pos,
+                      const float* rope_cos, const float* rope_sin, int max_pos, int T, int H, int R, int rot, int n_pages, int n_seq,
+                      void* stream);
+int mlora_head_linear(void* y, int y_layout, long ldy, long head_y, const void* x, long ldx, long head_x, const void* W, int heads, int T,
+                      int K, int N, float alpha, void* stream);
+int mlora_latent_attn_splits(int T, int H, int max_ctx);
+size_t mlora_latent_attn_workspace_bytes(int T, int H, int R, int splits);
+int mlora_latent_attn(void* out, const void* q, const void* cache, const int32_t* block_table, int max_blocks, const int32_t* tok_seq,
+                      const int32_t* tok_pos, const float* sink, float scale, int T, int H, int R, int rot, int n_pages, int n_seq,
+                      int splits, void* workspace, size_t workspace_bytes, void* stream);
+
+/* Mixture of experts.  mlora_moe_route: z = scale logits[t] + bias, the `top` largest per token (lower index on ties), softmax
+ * over those.  mlora_moe_plan sorts the (token, choice) entries by expert into tiles {expert, first place, places, 0} of
+ * mlora_moe_tile_rows places (at most mlora_moe_max_tiles of them).  mlora_moe_linear multiplies tile by tile with the
+ * experts' weights (one [N, K] block each): stage UP reads token rows x [T, K] and writes place rows, stage DOWN reads place
+ * rows and writes entry rows; `act` is applied to alpha times the product.  mlora_moe_combine: x[t] += sum over the
+ * choices of weight * row. */
+#define MLORA_ACT_NONE  0
+#define MLORA_ACT_RELU2 1   /* max(v, 0)^2 */
+#define MLORA_MOE_UP    0
+#define MLORA_MOE_DOWN  1
+int mlora_moe_route(int32_t* pick, float* weight, const float* logits, int ld, const float* bias, float scale, int T, int E, int top,
+                    void* stream);
+int mlora_moe_tile_rows(int T, int E, int top);
+int mlora_moe_max_tiles(int T, int E, int top);
+int mlora_moe_plan(int32_t* perm, int32_t* tiles, int32_t* n_tiles, const int32_t* pick, int T, int E, int top, void* stream);
+int mlora_moe_linear(void* y, const void* x, const void* W, const int32_t* perm, const int32_t* tiles, const int32_t* n_tiles, int tile_rows,
+                     int max_tiles, int T, int K, int N, int top, int stage, int act, float alpha, void* stream);
+int mlora_moe_combine(float* x, const void* y, const float* weight, int T, int top, int N, void* stream);
+
+#ifdef __cplusplus
+}
+#endif
+#endif /* MLORA_DECODER_H */

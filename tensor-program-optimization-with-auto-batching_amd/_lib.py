@@ -1,6 +1,7 @@
-"""ctypes binding of libmlora_hip.so (the C ABI declared in include/mlora.h).
+"""ctypes binding of the kernel libraries (the C ABI declared in include/mlora.h and include/mlora_decoder.h): one library
+per element type, with the same entry points.
 
-There is no fallback: if the library has not been built, loading raises and every operator fails.
+There is no fallback: if a library has not been built, loading it raises and every operator fails.
 """
 from __future__ import annotations
 
@@ -9,13 +10,17 @@ import os
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "libmlora_hip.so")
+LIB_PATHS = {"float16": LIB_PATH, "bfloat16": os.path.join(_HERE, "libmlora_bf16.so"), "float32": os.path.join(_HERE, "libmlora_f32.so")}
 
-F16, F32 = 0, 1
+F16, F32 = 0, 1          # F16: the library's own 16-bit element type (in the fp32 library: fp32)
+GLU_SILU, GLU_CLIPPED = 0, 1
+ACT_NONE, ACT_RELU2 = 0, 1
+MOE_UP, MOE_DOWN = 0, 1
 ROWMAJOR, FRAG = 0, 1
 STORE, ACCUMULATE = 0, 1
 PAGE_SIZE = 16
 
-_p, _i, _f, _z = C.c_void_p, C.c_int, C.c_float, C.c_size_t
+_p, _i, _f, _z, _l = C.c_void_p, C.c_int, C.c_float, C.c_size_t, C.c_long
 
 # name -> (restype, argtypes); mirrors include/mlora.h one to one
 SIGNATURES = {
@@ -50,6 +55,9 @@ SIGNATURES = {
     "mlora_linear_frag_silu": (_i, [_p, _p, _p, _i, _i, _i, _p, _i, _p, _i, _p]),
     "mlora_gemv_frag_lora": (_i, [_p, _i, _i, _p, _p, _i, _i, _i, _p, _p, _i, _p, _i, _i, _p]),
     "mlora_gemv_frag_silu": (_i, [_p, _p, _p, _i, _i, _i, _p]),
+    "mlora_gemv_frag_clipglu": (_i, [_p, _p, _p, _i, _i, _i, _f, _f, _f, _p]),
+    "mlora_linear_frag_clipglu": (_i, [_p, _p, _p, _i, _i, _i, _f, _f, _f, _p]),
+    "mlora_clipglu_mul": (_i, [_p, _i, _p, _p, _i, _i, _i, _f, _f, _f, _p]),
     "mlora_gemv_frag_split": (_i, [_p, _i, _i, _p, _p, _p, _i, _i, _i, _i, _p]),
     "mlora_gemv_split_kq": (_i, [_i, _i, _i, _i]),
     "mlora_gemv_frag_split_kq": (_i, [_p, _p, _i, _p, _p, _i, _i, _i, _i, _p]),
@@ -109,7 +117,25 @@ class DecodePlan(C.Structure):
 
 SIGNATURES["mlora_decode_step"] = (_i, [C.POINTER(DecodePlan), _p])
 
-_lib = None
+# mirrors include/mlora_decoder.h (the bfloat16 and fp32 libraries)
+DECODER_SIGNATURES = {
+    "mlora_stream_norm": (_i, [_p, _p, _p, _p, _i, _p, _p, _f, _f, _i, _i, _i, _p]),
+    "mlora_token_gate": (_i, [_p, _p, _p, _i, _p, _p, _i, _i, _i, _p, _i, _i, _i, _i, _p]),
+    "mlora_token_gate_mul": (_i, [_p, _p, _p, _i, _i, _i, _p, _i, _i, _i, _p]),
+    "mlora_latent_prep": (_i, [_p, _p, _p, _i, _i, _i, _i, _f, _p, _f, _p, _i, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _p]),
+    "mlora_head_linear": (_i, [_p, _i, _l, _l, _p, _l, _l, _p, _i, _i, _i, _i, _f, _p]),
+    "mlora_latent_attn_splits": (_i, [_i, _i, _i]),
+    "mlora_latent_attn_workspace_bytes": (_z, [_i, _i, _i, _i]),
+    "mlora_latent_attn": (_i, [_p, _p, _p, _p, _i, _p, _p, _p, _f, _i, _i, _i, _i, _i, _i, _i, _p, _z, _p]),
+    "mlora_moe_route": (_i, [_p, _p, _p, _i, _p, _f, _i, _i, _i, _p]),
+    "mlora_moe_tile_rows": (_i, [_i, _i, _i]),
+    "mlora_moe_max_tiles": (_i, [_i, _i, _i]),
+    "mlora_moe_plan": (_i, [_p, _p, _p, _p, _i, _i, _i, _p]),
+    "mlora_moe_linear": (_i, [_p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _f, _p]),
+    "mlora_moe_combine": (_i, [_p, _p, _p, _i, _i, _i, _p]),
+}
+
+_libs = {}
 
 
 class MloraError(RuntimeError):
@@ -118,22 +144,31 @@ class MloraError(RuntimeError):
         self.code = code
 
 
-def lib() -> C.CDLL:
-    """The loaded library; raises if libmlora_hip.so is missing (build it with build.py)."""
-    global _lib
-    if _lib is None:
-        if not os.path.exists(LIB_PATH):
-            raise RuntimeError(
-                f"{LIB_PATH} not found: the HIP library is not built (run build.py). There is no CPU fallback.")
-        l = C.CDLL(LIB_PATH)
-        for name, (res, args) in SIGNATURES.items():
+def lib(dtype: str = "float16") -> C.CDLL:
+    """The loaded library of an element type; raises if it is missing (build it with build.py).  The bfloat16 and fp32
+    libraries hold the decoder kernels and those of mlora.h that their sources give (no adapter kernels)."""
+    l = _libs.get(dtype)
+    if l is None:
+        path = LIB_PATHS[dtype]
+        if not os.path.exists(path):
+            raise RuntimeError(f"{path} not found: the HIP library is not built (run build.py). There is no CPU fallback.")
+        l = C.CDLL(path)
+        table = SIGNATURES if dtype == "float16" else {**{n: v for n, v in SIGNATURES.items() if hasattr(l, n)}, **DECODER_SIGNATURES}
+        if dtype == "float32":
+            table.pop("mlora_token_gate")              # a matrix-core kernel
+        for name, (res, args) in table.items():
             fn = getattr(l, name)
             fn.restype = res
             fn.argtypes = args
-        _lib = l
-    return _lib
+        _libs[dtype] = l
+    return l
 
 
-def check(code: int) -> None:
+def loaded() -> C.CDLL:
+    """A library for what does not depend on the element type: one that is loaded already, else the fp16 one."""
+    return next(iter(_libs.values()), None) or lib()
+
+
+def check(code: int, dtype: str = "float16") -> None:
     if code != 0:
-        raise MloraError(code, lib().mlora_last_error().decode())
+        raise MloraError(code, lib(dtype).mlora_last_error().decode())

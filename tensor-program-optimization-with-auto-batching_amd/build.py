@@ -1,4 +1,8 @@
-"""Compile the HIP sources in csrc/ into libmlora_hip.so (gfx950), in-tree, with hipcc.
+"""Compile the HIP sources in csrc/ (gfx950) in-tree with hipcc: one library per element type.
+
+    libmlora_hip.so    fp16: the Llama / LoRA hot path
+    libmlora_bf16.so   bfloat16: the linear and row kernels and those of the latent-attention decoders
+    libmlora_f32.so    fp32: the same decoders in IEEE fp32
 
 Usage: python build.py [--force]
 """
@@ -11,8 +15,17 @@ from concurrent.futures import ThreadPoolExecutor
 
 HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
-LIB = os.path.join(HERE, "libmlora_hip.so")
 SOURCES = ["api.hip", "gather_mm.hip", "gather_mm_batch.hip", "gemv.hip", "gemm.hip", "rowops.hip", "attention.hip", "decode_step.hip"]
+DECODER_SOURCES = ["stream_ops.hip", "latent_attention.hip", "moe.hip"]
+LIBS = {   # element type -> (library, sources, suffix of the objects, extra flags)
+    "float16": (os.path.join(HERE, "libmlora_hip.so"), SOURCES, "", []),
+    "bfloat16": (os.path.join(HERE, "libmlora_bf16.so"), ["api.hip", "gemv.hip", "gemm.hip", "rowops.hip", *DECODER_SOURCES], "_bf16",
+                 ["-DMLORA_ELT_BF16"]),
+    "float32": (os.path.join(HERE, "libmlora_f32.so"), ["api.hip", "rowops.hip", "linear_f32.hip", *DECODER_SOURCES], "_f32", ["-DMLORA_ELT_F32"]),
+}
+LIB = LIBS["float16"][0]
+HEADERS = [os.path.join(CSRC, h) for h in ("common.h", "lora_device.h", "gather_mm_batch.h", "moe.h")] + \
+          [os.path.join(HERE, "..", "include", h) for h in ("mlora.h", "mlora_decoder.h")]
 FLAGS = ["--offload-arch=gfx950", "-O3", "-fPIC", "-std=c++17", "-mllvm", "-amdgpu-kernarg-preload-count=16",
          "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
@@ -34,24 +47,35 @@ def _run(cmd):
         sys.stderr.write(err + "\n")
 
 
-def build(force: bool = True, jobs: int = 6) -> str:
-    """Compile every source to an object and link the shared library; returns its path."""
-    objs = []
-    todo = []
-    hdr_m = max(os.path.getmtime(os.path.join(CSRC, "common.h")), os.path.getmtime(os.path.join(CSRC, "lora_device.h")),
-                os.path.getmtime(os.path.join(CSRC, "gather_mm_batch.h")),
-                os.path.getmtime(os.path.join(HERE, "..", "include", "mlora.h")))
-    for src in SOURCES:
-        s = os.path.join(CSRC, src)
-        o = os.path.join(CSRC, src.replace(".hip", ".o"))
-        objs.append(o)
-        if force or not os.path.exists(o) or os.path.getmtime(o) < max(os.path.getmtime(s), hdr_m):
-            todo.append([_hipcc(), *FLAGS, "-c", s, "-o", o])
+def build(force: bool = True, jobs: int = 0, dtypes=tuple(LIBS)) -> str:
+    """Compile every source of the libraries of `dtypes` to an object and link them; returns the path of the last one.
+    jobs: compiler processes at once (0: MAX_JOBS, else 6)."""
+    jobs = jobs or int(os.environ.get("MAX_JOBS") or 6)
+    hdr_m = max(os.path.getmtime(h) for h in HEADERS)
+    todo, links = [], []
+    for dt in dtypes:
+        lib, sources, suffix, extra = LIBS[dt]
+        objs, stale = [], force or not os.path.exists(lib)
+        for src in sources:
+            s = os.path.join(CSRC, src)
+            o = os.path.join(CSRC, src.replace(".hip", suffix + ".o"))
+            objs.append(o)
+            if force or not os.path.exists(o) or os.path.getmtime(o) < max(os.path.getmtime(s), hdr_m):
+                todo.append([_hipcc(), *FLAGS, *extra, "-c", s, "-o", o])
+                stale = True
+        if stale or any(os.path.getmtime(o) > os.path.getmtime(lib) for o in objs):
+            links.append([_hipcc(), "--offload-arch=gfx950", "-shared", "-fPIC", *objs, "-o", lib])
     with ThreadPoolExecutor(max_workers=jobs) as ex:
         list(ex.map(_run, todo))
-    if todo or not os.path.exists(LIB):
-        _run([_hipcc(), "--offload-arch=gfx950", "-shared", "-fPIC", *objs, "-o", LIB])
-    return LIB
+    for cmd in links:
+        _run(cmd)
+    return LIBS[dtypes[-1]][0]
+
+
+def ensure(dtype: str) -> str:
+    """Build the library of one element type if it is not there (a fresh checkout); returns its path."""
+    lib = LIBS[dtype][0]
+    return lib if os.path.exists(lib) else build(force=False, dtypes=(dtype,))
 
 
 if __name__ == "__main__":

@@ -8,6 +8,7 @@
 #include <stdarg.h>
 
 #include "../../include/mlora.h"
+#include "../../include/mlora_decoder.h"
 
 typedef _Float16 f16;
 typedef f16 f16x2 __attribute__((ext_vector_type(2)));
@@ -15,6 +16,20 @@ typedef f16 f16x4 __attribute__((ext_vector_type(4)));
 typedef f16 f16x8 __attribute__((ext_vector_type(8)));
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 typedef float f32x2 __attribute__((ext_vector_type(2)));
+
+// The element type of a build of the library: weights and stored activations.  The same sources are compiled once per
+// element type into separate libraries with the same entry points - fp16 by default, bfloat16 with MLORA_ELT_BF16,
+// float with MLORA_ELT_F32 (the sources that do not need the 16-bit matrix cores).
+#if defined(MLORA_ELT_BF16)
+typedef __bf16 elt;
+#elif defined(MLORA_ELT_F32)
+typedef float elt;
+#else
+typedef f16 elt;
+#endif
+typedef elt eltx2 __attribute__((ext_vector_type(2)));
+typedef elt eltx4 __attribute__((ext_vector_type(4)));
+typedef elt eltx8 __attribute__((ext_vector_type(8)));
 
 #define WAVE 64
 
@@ -64,6 +79,36 @@ __device__ __forceinline__ float wave_max(float v) {
 // 16-byte global load of 8 fp16 values
 __device__ __forceinline__ f16x8 ld8(const f16* p) { return *reinterpret_cast<const f16x8*>(p); }
 __device__ __forceinline__ void st8(f16* p, f16x8 v) { *reinterpret_cast<f16x8*>(p) = v; }
+#if defined(MLORA_ELT_BF16) || defined(MLORA_ELT_F32)
+__device__ __forceinline__ eltx8 ld8(const elt* p) { return *reinterpret_cast<const eltx8*>(p); }
+__device__ __forceinline__ void st8(elt* p, eltx8 v) { *reinterpret_cast<eltx8*>(p) = v; }
+#endif
+
+// D[16 x 16] += A[16 x 32] . B[32 x 16] on the matrix cores, fp32 accumulation: a lane holds 8 consecutive k of row
+// (column) lane % 16 from k-group lane / 16, and rows 4 (lane / 16) .. + 3 of column lane % 16 of the result
+#if defined(MLORA_ELT_BF16)
+__device__ __forceinline__ f32x4 mfma_16x16x32(eltx8 a, eltx8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
+#elif !defined(MLORA_ELT_F32)
+__device__ __forceinline__ f32x4 mfma_16x16x32(eltx8 a, eltx8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_f16(a, b, c, 0, 0, 0); }
+#endif
+
+// The product of a gated feed-forward, act(gate) * up:
+//   MLORA_GLU_SILU     silu(g) * u on the operands as stored (rounded to the element type)
+//   MLORA_GLU_CLIPPED  g = min(scale g, limit), u = clamp(scale u, -limit, limit): g sigmoid(alpha g) (u + 1)
+struct GluArgs {
+  float scale, limit, alpha;
+};
+template <int KIND>
+__device__ __forceinline__ float glu(float g, float u, const GluArgs& a) {
+  if constexpr (KIND == MLORA_GLU_SILU) {
+    const float gf = (float)(elt)g;
+    return gf / (1.f + expf(-gf)) * (float)(elt)u;
+  } else {
+    g = fminf(g * a.scale, a.limit);
+    u = fminf(fmaxf(u * a.scale, -a.limit), a.limit);
+    return g / (1.f + expf(-a.alpha * g)) * (u + 1.f);
+  }
+}
 
 // a.x*b.x + a.y*b.y + c with fp32 accumulation (v_dot2_f32_f16)
 __device__ __forceinline__ float dot2(f16x2 a, f16x2 b, float c) {

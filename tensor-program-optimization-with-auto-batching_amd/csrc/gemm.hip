@@ -18,7 +18,7 @@ int mlora_check_linear(const char* who, const void* y, int y_dtype, int mode, co
 
 namespace {
 
-enum { OUT_F16 = 0, OUT_F32 = 1, OUT_ACC_F32 = 2, OUT_SILU = 3 };
+enum { OUT_F16 = 0, OUT_F32 = 1, OUT_ACC_F32 = 2, OUT_SILU = 3, OUT_CLIP = 4 };   // the last two: a gated product (MLORA_GLU_*) in fragment order
 
 // compute units of the current device (0 if it cannot be asked), read once
 int gemm_n_cu() {
@@ -33,8 +33,8 @@ int gemm_n_cu() {
 constexpr int WT = 4;   // 16-wide MFMA tiles per wave along N and along T
 
 template <int OUT, bool PACKED>
-__global__ __launch_bounds__(256) void gemm_kernel(void* __restrict__ yv, const f16* __restrict__ x, int ldx,
-                                                   const f16* __restrict__ W, int T, int K, int N) {
+__global__ __launch_bounds__(256) void gemm_kernel(void* __restrict__ yv, const elt* __restrict__ x, int ldx,
+                                                   const elt* __restrict__ W, int T, int K, int N) {
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int r16 = lane & 15, kg = lane >> 4;
   const int n0 = blockIdx.x * 128 + (wave & 1) * 64;
@@ -43,8 +43,8 @@ __global__ __launch_bounds__(256) void gemm_kernel(void* __restrict__ yv, const 
 
   constexpr int WSTEP = PACKED ? 512 : 32;   // elements between consecutive k-steps of one fragment stream
   const int tiles = (N + 15) / 16;
-  const f16* wp[WT];
-  const f16* xp[WT];
+  const elt* wp[WT];
+  const elt* xp[WT];
 #pragma unroll
   for (int i = 0; i < WT; ++i) {
     if constexpr (PACKED) {
@@ -66,7 +66,7 @@ __global__ __launch_bounds__(256) void gemm_kernel(void* __restrict__ yv, const 
 #pragma unroll
     for (int j = 0; j < WT; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
 
-  f16x8 a[WT], b[WT];
+  eltx8 a[WT], b[WT];
 #pragma unroll
   for (int i = 0; i < WT; ++i) {
     a[i] = ld8(wp[i]);
@@ -74,7 +74,7 @@ __global__ __launch_bounds__(256) void gemm_kernel(void* __restrict__ yv, const 
   }
   const int KB = K / 32;
   for (int ks = 1; ks <= KB; ++ks) {
-    f16x8 an[WT], bn[WT];
+    eltx8 an[WT], bn[WT];
     const int kc = ks < KB ? ks : 0;   // the last prefetch wraps to a valid address and is discarded
 #pragma unroll
     for (int i = 0; i < WT; ++i) {
@@ -84,7 +84,7 @@ __global__ __launch_bounds__(256) void gemm_kernel(void* __restrict__ yv, const 
 #pragma unroll
     for (int i = 0; i < WT; ++i)
 #pragma unroll
-      for (int j = 0; j < WT; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_f16(a[i], b[j], acc[i][j], 0, 0, 0);
+      for (int j = 0; j < WT; ++j) acc[i][j] = mfma_16x16x32(a[i], b[j], acc[i][j]);
 #pragma unroll
     for (int i = 0; i < WT; ++i) {
       a[i] = an[i];
@@ -104,7 +104,7 @@ __global__ __launch_bounds__(256) void gemm_kernel(void* __restrict__ yv, const 
       const size_t o = (size_t)t * N + n;
       const f32x4 s = acc[i][j];
       if constexpr (OUT == OUT_F16) {
-        *reinterpret_cast<f16x4*>((f16*)yv + o) = f16x4{(f16)s[0], (f16)s[1], (f16)s[2], (f16)s[3]};
+        *reinterpret_cast<eltx4*>((elt*)yv + o) = eltx4{(elt)s[0], (elt)s[1], (elt)s[2], (elt)s[3]};
       } else if constexpr (OUT == OUT_F32) {
         *reinterpret_cast<f32x4*>((float*)yv + o) = s;
       } else {
@@ -130,15 +130,15 @@ constexpr int LBK = 64;              // k per stage
 
 // FT x FN: 16-row fragments of tokens / of weight rows per block; WT x WN: MFMA tiles of a wave (FT/WT * FN/WN == 4 waves)
 template <int OUT, int FT, int FN, int WT_, int WN_>
-__global__ __launch_bounds__(256) void gemm_lds_kernel(void* __restrict__ yv, const f16* __restrict__ x, int ldx,
-                                                       const f16* __restrict__ Wp, int T, int K, int N) {
+__global__ __launch_bounds__(256) void gemm_lds_kernel(void* __restrict__ yv, const elt* __restrict__ x, int ldx,
+                                                       const elt* __restrict__ Wp, int T, int K, int N) {
   static_assert((FT / WT_) * (FN / WN_) == 4, "four waves cover the block");
   constexpr int KS = LBK / 32;                      // 32-k steps per stage
   constexpr int WELEMS = KS * FN * 512, XELEMS = KS * FT * 512;   // fp16 elements of a stage: W, then x
   constexpr int STAGE = WELEMS + XELEMS;
   constexpr int WCH = KS * FN * WAVE / 256, XCH = KS * FT * WAVE / 256;   // 16-byte chunks per thread and stage
   static_assert(WCH >= 1 && XCH >= 1, "a stage gives every thread at least one chunk of each operand");
-  extern __shared__ __align__(16) f16 smem[];       // [2][STAGE]
+  extern __shared__ __align__(16) elt smem[];       // [2][STAGE]
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int n0 = blockIdx.x * FN * 16, t0 = blockIdx.y * FT * 16;
   constexpr int WAVES_N = FN / WN_;
@@ -147,8 +147,8 @@ __global__ __launch_bounds__(256) void gemm_lds_kernel(void* __restrict__ yv, co
   const int tiles = (N + 15) / 16;
 
   // chunk c = threadIdx.x + 256 j of an operand's stage: fragment f = c / 64 = ks * F + tile, lane slot l = c % 64
-  const f16* wsrc[WCH];
-  const f16* xsrc[XCH];
+  const elt* wsrc[WCH];
+  const elt* xsrc[XCH];
 #pragma unroll
   for (int j = 0; j < WCH; ++j) {
     const int c = threadIdx.x + 256 * j;
@@ -173,7 +173,7 @@ __global__ __launch_bounds__(256) void gemm_lds_kernel(void* __restrict__ yv, co
     xsrc[j] = x + (size_t)t * ldx + ks * 32 + gq * 8;
     xdst[j] = ((ks * FT + (row >> 4)) * 64 + gq * 16 + ((row & 15) ^ (gq << 2))) * 8;
   }
-  f16x8 wst[WCH], xst[XCH];
+  eltx8 wst[WCH], xst[XCH];
   auto load_stage = [&](int s) {                    // s: stage index; k-steps KS*s .. (the last may be past K)
 #pragma unroll
     for (int j = 0; j < WCH; ++j) {
@@ -191,7 +191,7 @@ __global__ __launch_bounds__(256) void gemm_lds_kernel(void* __restrict__ yv, co
     }
   };
   auto store_stage = [&](int buf) {
-    f16* dst = smem + buf * STAGE;
+    elt* dst = smem + buf * STAGE;
 #pragma unroll
     for (int j = 0; j < WCH; ++j) st8(dst + (threadIdx.x + 256 * j) * 8, wst[j]);
 #pragma unroll
@@ -211,12 +211,12 @@ __global__ __launch_bounds__(256) void gemm_lds_kernel(void* __restrict__ yv, co
   __syncthreads();
   for (int s = 0; s < S; ++s) {
     if (s + 1 < S) load_stage(s + 1);
-    const f16* ws = smem + (s & 1) * STAGE;
-    const f16* xs = ws + WELEMS;
+    const elt* ws = smem + (s & 1) * STAGE;
+    const elt* xs = ws + WELEMS;
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) {
       if (s * KS + ks < KB) {                        // workgroup-uniform
-        f16x8 a[WN_], b[WT_];
+        eltx8 a[WN_], b[WT_];
 #pragma unroll
         for (int i = 0; i < WN_; ++i) a[i] = ld8(ws + (ks * FN + wn * WN_ + i) * 512 + lane * 8);
 #pragma unroll
@@ -224,7 +224,7 @@ __global__ __launch_bounds__(256) void gemm_lds_kernel(void* __restrict__ yv, co
 #pragma unroll
         for (int i = 0; i < WN_; ++i)
 #pragma unroll
-          for (int j = 0; j < WT_; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_f16(a[i], b[j], acc[i][j], 0, 0, 0);
+          for (int j = 0; j < WT_; ++j) acc[i][j] = mfma_16x16x32(a[i], b[j], acc[i][j]);
       }
     }
     if (s + 1 < S) store_stage((s + 1) & 1);
@@ -243,7 +243,7 @@ __global__ __launch_bounds__(256) void gemm_lds_kernel(void* __restrict__ yv, co
       const size_t o = (size_t)t * N + n;
       const f32x4 sacc = acc[i][j];
       if constexpr (OUT == OUT_F16) {
-        *reinterpret_cast<f16x4*>((f16*)yv + o) = f16x4{(f16)sacc[0], (f16)sacc[1], (f16)sacc[2], (f16)sacc[3]};
+        *reinterpret_cast<eltx4*>((elt*)yv + o) = eltx4{(elt)sacc[0], (elt)sacc[1], (elt)sacc[2], (elt)sacc[3]};
       } else if constexpr (OUT == OUT_F32) {
         *reinterpret_cast<f32x4*>((float*)yv + o) = sacc;
       } else {
@@ -284,9 +284,9 @@ constexpr int PP_OUT_ELEMS = 16 * PP_OUT_LD;   // per wave: 16 tokens x 64 colum
 // Projections are row ranges of the fused weight, each with its own B table [n_ad][rows][r] (row-major, r in {32, 64})
 // and its own v; a 256-row block lies inside one range (checked by the launcher).  n_proj == 0: a plain GEMM.
 struct PPLora {
-  const f16* B[3];
-  const f16* vh[3];
-  const f16* vl[3];
+  const elt* B[3];
+  const elt* vh[3];
+  const elt* vl[3];
   int n_begin[3], n_rows[3];
   int n_proj, r;
   const int32_t* blk_adapter;
@@ -297,22 +297,22 @@ __device__ __forceinline__ unsigned long long uniform64(unsigned long long v) {
   return ((unsigned long long)hi << 32) | lo;
 }
 
-// OUT_SILU: Wp is the fused [2 I, K] gate / up matrix (N = 2 I, gate rows first) and the output is
-// act = silu(f16(gate)) * f16(up) [T, I] in fragment order (tiles per 32-k step: x_tt).  A block is 256 tokens x 128
+// OUT_SILU (and likewise OUT_CLIP with its own product): Wp is the fused [2 I, K] gate / up matrix (N = 2 I, gate rows first) and the output is
+// act = silu(elt(gate)) * elt(up) [T, I] in fragment order (tiles per 32-k step: x_tt).  A block is 256 tokens x 128
 // channels: the ring slots of a stage hold, for each of the two row groups of waves, four gate tiles and then the four
 // up tiles of the same channels, so that a lane ends up with both halves of its channels and the product never leaves
 // the registers.  LoRA deltas: slot 0 of `lo` is the gate projection, slot 1 the up projection (B == nullptr: not
 // adapted); each rides as its own extra k-steps, in which only that half of a wave's tiles is multiplied.
 // LORA = false is the plain GEMM (lo is ignored)
 template <int OUT, bool LORA>
-__global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __restrict__ yv, const f16* __restrict__ x, int ldx, int x_tt,
-                                                                   const f16* __restrict__ Wp, int T, int K, int N, int gx, int gy,
-                                                                   PPLora lo) {
-  extern __shared__ __align__(16) f16 smem[];  // [PP_STAGES][PP_STAGE_ELEMS], then [PP_WAVES][PP_OUT_ELEMS]
+__global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __restrict__ yv, const elt* __restrict__ x, int ldx, int x_tt,
+                                                                   const elt* __restrict__ Wp, int T, int K, int N, int gx, int gy,
+                                                                   PPLora lo, GluArgs ga) {
+  extern __shared__ __align__(16) elt smem[];  // [PP_STAGES][PP_STAGE_ELEMS], then [PP_WAVES][PP_OUT_ELEMS]
   constexpr int NW = PP_WAVES;
   constexpr int LQ = 2 * PP_F / NW;            // fragments a wave fetches per stage (4)
   constexpr int WTF = 4;                       // token fragments of a wave's tile (64 tokens)
-  constexpr bool SILU = OUT == OUT_SILU;
+  constexpr bool SILU = OUT == OUT_SILU || OUT == OUT_CLIP;   // a gated product
   constexpr int BN = SILU ? PP_F * 8 : PP_F * 16;   // output columns of a block (SILU: channels, each a gate and an up row)
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
   const int nb = gx * gy;
@@ -346,11 +346,11 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
   const int E = SILU ? EP * ((lo.B[0] != nullptr) + (lo.B[1] != nullptr)) : EP;
 
   // ---- loader role: wave w fetches fragments 4 w .. 4 w + 3 of every stage (waves 0-3: weights, waves 4-7: tokens)
-  const f16* src[LQ];
+  const elt* src[LQ];
   int step = 0;                                // elements between consecutive k-steps of this wave's sources
   int load_L = blockIdx.x, load_kb = 0;        // the stage the loader issues next
   int load_nst = KB;                           // stages of the block being loaded (KB, or KB + E with a delta)
-  const f16* l_src = nullptr;                  // LoRA stages of that block (all uniform): row 0 of the block in B[a] (weight waves) or in v_hi (token waves) ...
+  const elt* l_src = nullptr;                  // LoRA stages of that block (all uniform): row 0 of the block in B[a] (weight waves) or in v_hi (token waves) ...
   long l_lo = 0;                               // ... the distance from v_hi to v_lo (token waves; 0 for weight waves) ...
   int l_rows = 1;                              // ... and the rows that exist from there on (rows past them repeat the last one; their results are dropped)
   int l_a = -1, l_n0 = 0, l_t0 = 0;            // SILU: adapter, first channel and first token of that block (the stages' addresses are formed per stage)
@@ -367,9 +367,9 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
         l_n0 = n0;
         l_t0 = t0;
       } else if (a >= 0) {
-        const f16* Bt = lo.B[0];
-        const f16* vh = lo.vh[0];
-        const f16* vl = lo.vl[0];
+        const elt* Bt = lo.B[0];
+        const elt* vh = lo.vh[0];
+        const elt* vl = lo.vl[0];
         int nbeg = lo.n_begin[0], nrows = lo.n_rows[0];
 #pragma unroll
         for (int i = 1; i < 3; ++i)
@@ -386,7 +386,7 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
           l_rows = T - t0;
         }
         // all of this is the same in every lane: say so, it lives in scalar registers across the K loop
-        l_src = (const f16*)uniform64((unsigned long long)l_src);
+        l_src = (const elt*)uniform64((unsigned long long)l_src);
         l_lo = (long)uniform64((unsigned long long)l_lo);
         l_rows = __builtin_amdgcn_readfirstlane(l_rows);
       }
@@ -428,7 +428,7 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
   // PLAIN: the caller knows that this stage is an ordinary k-step and not the last of its block (no tests at all)
   auto issue = [&](auto PLAIN) {
     constexpr bool plain = decltype(PLAIN)::value;
-    f16* dst = smem + ring * PP_STAGE_ELEMS + wave * LQ * 512;
+    elt* dst = smem + ring * PP_STAGE_ELEMS + wave * LQ * 512;
     if (plain || !LORA || load_kb < KB) {
 #pragma unroll
       for (int q = 0; q < LQ; ++q)
@@ -440,7 +440,7 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
       const int jj = has_gate && up ? j - EP : j;
       const bool lo_half = jj >= RB;
       const int ks = (lo_half ? jj - RB : jj) * 32;
-      const f16* base;
+      const elt* base;
       int row0, rows;
       if (wave < NW / 2) {                     // rows of the projection's table for this wave's channels (used by the waves of that half only)
         base = (up ? lo.B[1] : lo.B[0]) + (size_t)l_a * I * lo.r;
@@ -455,7 +455,7 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
       for (int q = 0; q < LQ; ++q) {
         int row = row0 + q * 16 + (lane & 15);
         row = row < rows ? row : rows - 1;
-        const f16* p = base + ((size_t)row * lo.r + ks + (lane >> 4) * 8);
+        const elt* p = base + ((size_t)row * lo.r + ks + (lane >> 4) * 8);
         __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)p,
                                          (__attribute__((address_space(3))) void*)(dst + q * 512), 16, 0, 0);
       }
@@ -466,7 +466,7 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
       for (int q = 0; q < LQ; ++q) {
         int row = ((wave & 3) * LQ + q) * 16 + (lane & 15);
         row = row < l_rows ? row : l_rows - 1;
-        const f16* p = l_src + (j < RB ? 0 : l_lo) + ((size_t)row * lo.r + ks + (lane >> 4) * 8);
+        const elt* p = l_src + (j < RB ? 0 : l_lo) + ((size_t)row * lo.r + ks + (lane >> 4) * 8);
         __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)p,
                                          (__attribute__((address_space(3))) void*)(dst + q * 512), 16, 0, 0);
       }
@@ -485,11 +485,11 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
   // ---- compute role: rows wn * 128 .., tokens wt * 64 ..
   const int wn = wave & 1, wt = wave >> 1;
   f32x4 acc[8][WTF];
-  f16x8 a[2][8], b[2][WTF];
+  eltx8 a[2][8], b[2][WTF];
   int rd = 0;                                  // ring slot of the stage whose fragments are read next
   auto read_frags = [&](auto U) {
     constexpr int u = decltype(U)::value;
-    const f16* st = smem + rd * PP_STAGE_ELEMS + lane * 8;
+    const elt* st = smem + rd * PP_STAGE_ELEMS + lane * 8;
 #pragma unroll
     for (int j = 0; j < WTF; ++j) b[u][j] = ld8(st + (PP_F + wt * WTF + j) * 512);
 #pragma unroll
@@ -503,13 +503,13 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
 #pragma unroll
       for (int i = 0; i < 4; ++i)
 #pragma unroll
-        for (int j = 0; j < WTF; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_f16(a[u][i], b[u][j], acc[i][j], 0, 0, 0);
+        for (int j = 0; j < WTF; ++j) acc[i][j] = mfma_16x16x32(a[u][i], b[u][j], acc[i][j]);
     }
     if (half != 0) {
 #pragma unroll
       for (int i = 4; i < 8; ++i)
 #pragma unroll
-        for (int j = 0; j < WTF; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_f16(a[u][i], b[u][j], acc[i][j], 0, 0, 0);
+        for (int j = 0; j < WTF; ++j) acc[i][j] = mfma_16x16x32(a[u][i], b[u][j], acc[i][j]);
     }
   };
   // One stage: its successor must be in LDS (this wave's share: at most the two stages issued after it still in flight;
@@ -535,7 +535,7 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
   __syncthreads();
   issue(std::false_type());
   read_frags(std::integral_constant<int, 0>());
-  f16* ostage = smem + PP_STAGES * PP_STAGE_ELEMS + wave * PP_OUT_ELEMS;
+  elt* ostage = smem + PP_STAGES * PP_STAGE_ELEMS + wave * PP_OUT_ELEMS;
   const int r16 = lane & 15, g = lane >> 4;
   for (int L = blockIdx.x; L < nb; L += G) {
 #pragma unroll
@@ -577,15 +577,12 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
         for (int i = 0; i < 4; ++i) {
           const int c = n0 + (wn * 4 + i) * 16 + g * 4;
           if (c >= I) continue;
-          f16x4 o = f16x4{0, 0, 0, 0};                   // rows past T inside the last tile: zeros, as the separate kernel writes them
+          eltx4 o = eltx4{0, 0, 0, 0};                   // rows past T inside the last tile: zeros, as the separate kernel writes them
           if (t < T) {
 #pragma unroll
-            for (int r = 0; r < 4; ++r) {
-              const float gf = (float)(f16)acc[i][j][r];
-              o[r] = (f16)(gf / (1.f + expf(-gf)) * (float)(f16)acc[4 + i][j][r]);
-            }
+            for (int r = 0; r < 4; ++r) o[r] = (elt)glu<OUT == OUT_CLIP ? MLORA_GLU_CLIPPED : MLORA_GLU_SILU>(acc[i][j][r], acc[4 + i][j][r], ga);
           }
-          *reinterpret_cast<f16x4*>((f16*)yv + ((size_t)(c >> 5) * x_tt + (t >> 4)) * 512 + ((c & 31) >> 3) * 128 + (t & 15) * 8 + (c & 7)) = o;
+          *reinterpret_cast<eltx4*>((elt*)yv + ((size_t)(c >> 5) * x_tt + (t >> 4)) * 512 + ((c & 31) >> 3) * 128 + (t & 15) * 8 + (c & 7)) = o;
         }
       }
     } else if constexpr (OUT == OUT_F16) {
@@ -597,7 +594,7 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
             const f32x4 sacc = acc[h * 4 + i][j];
-            *reinterpret_cast<f16x4*>(ostage + r16 * PP_OUT_LD + i * 16 + g * 4) = f16x4{(f16)sacc[0], (f16)sacc[1], (f16)sacc[2], (f16)sacc[3]};
+            *reinterpret_cast<eltx4*>(ostage + r16 * PP_OUT_LD + i * 16 + g * 4) = eltx4{(elt)sacc[0], (elt)sacc[1], (elt)sacc[2], (elt)sacc[3]};
           }
           __builtin_amdgcn_wave_barrier();
 #pragma unroll
@@ -606,15 +603,15 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
             const int tr = c >> 3, cc = (c & 7) * 8;
             const int t = t0 + (wt * WTF + j) * 16 + tr;
             const int n = n0 + (wn * 8 + h * 4) * 16 + cc;
-            const f16x4 lo = *reinterpret_cast<const f16x4*>(ostage + tr * PP_OUT_LD + cc);
-            const f16x4 hi = *reinterpret_cast<const f16x4*>(ostage + tr * PP_OUT_LD + cc + 4);
+            const eltx4 lo = *reinterpret_cast<const eltx4*>(ostage + tr * PP_OUT_LD + cc);
+            const eltx4 hi = *reinterpret_cast<const eltx4*>(ostage + tr * PP_OUT_LD + cc + 4);
             if (t < T && n + 8 <= N) {
-              st8((f16*)yv + (size_t)t * N + n, f16x8{lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]});
+              st8((elt*)yv + (size_t)t * N + n, eltx8{lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]});
             } else if (t < T) {
 #pragma unroll
               for (int e = 0; e < 4; ++e) {
-                if (n + e < N) ((f16*)yv)[(size_t)t * N + n + e] = lo[e];
-                if (n + 4 + e < N) ((f16*)yv)[(size_t)t * N + n + 4 + e] = hi[e];
+                if (n + e < N) ((elt*)yv)[(size_t)t * N + n + e] = lo[e];
+                if (n + 4 + e < N) ((elt*)yv)[(size_t)t * N + n + 4 + e] = hi[e];
               }
             }
           }
@@ -645,24 +642,24 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
 }
 
 template <int OUT>
-int launch_gemm_pp(void* y, const f16* x, int ldx, int x_tt, const f16* Wp, int T, int K, int N, hipStream_t s,
-                   const PPLora& lo = PPLora()) {
-  constexpr size_t lds = ((size_t)PP_STAGES * PP_STAGE_ELEMS + (size_t)PP_WAVES * PP_OUT_ELEMS) * sizeof(f16);
+int launch_gemm_pp(void* y, const elt* x, int ldx, int x_tt, const elt* Wp, int T, int K, int N, hipStream_t s,
+                   const PPLora& lo = PPLora(), const GluArgs& ga = GluArgs()) {
+  constexpr size_t lds = ((size_t)PP_STAGES * PP_STAGE_ELEMS + (size_t)PP_WAVES * PP_OUT_ELEMS) * sizeof(elt);
   // the attribute is per kernel, set once per process (the initialiser of a local static runs once, also when several
   // host threads make their first call together)
   static const hipError_t configured = [] {
     hipError_t e = hipFuncSetAttribute((const void*)gemm_pp_kernel<OUT, false>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-    if (e == hipSuccess) e = hipFuncSetAttribute((const void*)gemm_pp_kernel<OUT, true>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    if (e == hipSuccess) e = hipFuncSetAttribute((const void*)gemm_pp_kernel<OUT, OUT != OUT_CLIP>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     return e;
   }();
   if (configured != hipSuccess)
     return mlora_set_error(MLORA_ERR_LAUNCH, "gemm_packed: cannot reserve %zu bytes of LDS: %s", lds, hipGetErrorString(configured));
-  const int gx = OUT == OUT_SILU ? ceil_div(N / 2, PP_F * 8) : ceil_div(N, PP_F * 16), gy = ceil_div(T, PP_F * 16);
+  const int gx = OUT == OUT_SILU || OUT == OUT_CLIP ? ceil_div(N / 2, PP_F * 8) : ceil_div(N, PP_F * 16), gy = ceil_div(T, PP_F * 16);
   int n_cu = gemm_n_cu();
   if (n_cu <= 0) n_cu = 256;
   const int grid = gx * gy < n_cu ? gx * gy : n_cu;
-  if (lo.n_proj > 0) hipLaunchKernelGGL((gemm_pp_kernel<OUT, true>), dim3(grid), dim3(PP_WAVES * WAVE), lds, s, y, x, ldx, x_tt, Wp, T, K, N, gx, gy, lo);
-  else hipLaunchKernelGGL((gemm_pp_kernel<OUT, false>), dim3(grid), dim3(PP_WAVES * WAVE), lds, s, y, x, ldx, x_tt, Wp, T, K, N, gx, gy, lo);
+  if (lo.n_proj > 0 && OUT != OUT_CLIP) hipLaunchKernelGGL((gemm_pp_kernel<OUT, OUT != OUT_CLIP>), dim3(grid), dim3(PP_WAVES * WAVE), lds, s, y, x, ldx, x_tt, Wp, T, K, N, gx, gy, lo, ga);
+  else hipLaunchKernelGGL((gemm_pp_kernel<OUT, false>), dim3(grid), dim3(PP_WAVES * WAVE), lds, s, y, x, ldx, x_tt, Wp, T, K, N, gx, gy, lo, ga);
   return MLORA_OK;
 }
 
@@ -689,7 +686,7 @@ constexpr int MID_KS = 2;                      // 32-k steps per stage
 
 template <int OUT, int FT, int FN>
 __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_mid_kernel(void* __restrict__ yv, float* __restrict__ part, int ld_part,
-                                                                    const f16* __restrict__ xf, int x_tt, const f16* __restrict__ Wp,
+                                                                    const elt* __restrict__ xf, int x_tt, const elt* __restrict__ Wp,
                                                                     int T, int K, int N) {
   constexpr int MID_STAGES = FT == 16 ? 3 : 4;
   constexpr int SF = FN + FT;                  // fragments of one 32-k step: weights, then tokens
@@ -704,7 +701,7 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_mid_kernel(void* __res
   static_assert(FT % 4 == 0 && FN % 2 == 0 && WNF <= 4, "the tile divides over the waves");
   static_assert(VM == 5 || VM == 6 || VM == 8, "wait_next has an instruction for each of these");
   static_assert(LREM == 0 || VM1 == 5 || VM1 == 6, "wait_next has an instruction for each of these");
-  extern __shared__ __align__(16) f16 smem[];  // [MID_STAGES][STAGE_ELEMS]; the output staging reuses it after the K loop
+  extern __shared__ __align__(16) elt smem[];  // [MID_STAGES][STAGE_ELEMS]; the output staging reuses it after the K loop
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
   const int KB = K / 32;
   const int tiles = (N + 15) / 16;
@@ -715,7 +712,7 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_mid_kernel(void* __res
   const int nks = kb1 - kb0;                   // 32-k steps of this slice (>= 1: checked by the launcher)
   const int nst = (nks + MID_KS - 1) / MID_KS; // stages
 
-  const f16* src[LQ];
+  const elt* src[LQ];
   int step[LQ], kso[LQ];
 #pragma unroll
   for (int q = 0; q < LQ; ++q) {
@@ -735,7 +732,7 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_mid_kernel(void* __res
   }
   int ring = 0, load_kb = kb0;
   auto issue = [&]() {
-    f16* dst = smem + ring * STAGE_ELEMS + wave * 512;
+    elt* dst = smem + ring * STAGE_ELEMS + wave * 512;
 #pragma unroll
     for (int q = 0; q < LQ; ++q) {
       if (LREM != 0 && q == LQ - 1 && wave >= LREM) break;      // uniform
@@ -750,7 +747,7 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_mid_kernel(void* __res
 
   const int wn = wave & 1, wt = wave >> 1;     // weight rows wn * WNF * 16 .., tokens wt * WTF * 16 ..
   f32x4 acc[WNF][WTF];
-  f16x8 a[2][MID_KS][WNF], b[2][MID_KS][WTF];  // two register sets: the stage being multiplied and its successor
+  eltx8 a[2][MID_KS][WNF], b[2][MID_KS][WTF];  // two register sets: the stage being multiplied and its successor
 #pragma unroll
   for (int i = 0; i < WNF; ++i)
 #pragma unroll
@@ -758,7 +755,7 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_mid_kernel(void* __res
   int rd = 0;
   auto read_frags = [&](auto U) {
     constexpr int u = decltype(U)::value;
-    const f16* st = smem + rd * STAGE_ELEMS + lane * 8;
+    const elt* st = smem + rd * STAGE_ELEMS + lane * 8;
 #pragma unroll
     for (int ks = 0; ks < MID_KS; ++ks) {
 #pragma unroll
@@ -777,7 +774,7 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_mid_kernel(void* __res
 #pragma unroll
         for (int i = 0; i < WNF; ++i)
 #pragma unroll
-          for (int j = 0; j < WTF; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_f16(a[u][ks][i], b[u][ks][j], acc[i][j], 0, 0, 0);
+          for (int j = 0; j < WTF; ++j) acc[i][j] = mfma_16x16x32(a[u][ks][i], b[u][ks][j], acc[i][j]);
       }
     }
     done_ks += MID_KS;
@@ -837,14 +834,14 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_mid_kernel(void* __res
   }
   if constexpr (OUT == OUT_F16) {
     // 16 tokens x (16 WNF) columns at a time through the wave's staging buffer: D[n][t] fragments in, token rows out
-    f16* ostage = smem + wave * PP_OUT_ELEMS;
+    elt* ostage = smem + wave * PP_OUT_ELEMS;
     constexpr int CPR = WNF * 2;               // 16-byte chunks per token row
 #pragma unroll
     for (int j = 0; j < WTF; ++j) {
 #pragma unroll
       for (int i = 0; i < WNF; ++i) {
         const f32x4 sacc = acc[i][j];
-        *reinterpret_cast<f16x4*>(ostage + r16 * PP_OUT_LD + i * 16 + gq * 4) = f16x4{(f16)sacc[0], (f16)sacc[1], (f16)sacc[2], (f16)sacc[3]};
+        *reinterpret_cast<eltx4*>(ostage + r16 * PP_OUT_LD + i * 16 + gq * 4) = eltx4{(elt)sacc[0], (elt)sacc[1], (elt)sacc[2], (elt)sacc[3]};
       }
       __builtin_amdgcn_wave_barrier();
 #pragma unroll
@@ -854,15 +851,15 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_mid_kernel(void* __res
         const int tr = c / CPR, cc = (c % CPR) * 8;
         const int t = t0 + (wt * WTF + j) * 16 + tr;
         const int n = n0 + wn * WNF * 16 + cc;
-        const f16x4 lo = *reinterpret_cast<const f16x4*>(ostage + tr * PP_OUT_LD + cc);
-        const f16x4 hi = *reinterpret_cast<const f16x4*>(ostage + tr * PP_OUT_LD + cc + 4);
+        const eltx4 lo = *reinterpret_cast<const eltx4*>(ostage + tr * PP_OUT_LD + cc);
+        const eltx4 hi = *reinterpret_cast<const eltx4*>(ostage + tr * PP_OUT_LD + cc + 4);
         if (t < T && n + 8 <= N) {
-          st8((f16*)yv + (size_t)t * N + n, f16x8{lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]});
+          st8((elt*)yv + (size_t)t * N + n, eltx8{lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]});
         } else if (t < T) {
 #pragma unroll
           for (int e = 0; e < 4; ++e) {
-            if (n + e < N) ((f16*)yv)[(size_t)t * N + n + e] = lo[e];
-            if (n + 4 + e < N) ((f16*)yv)[(size_t)t * N + n + 4 + e] = hi[e];
+            if (n + e < N) ((elt*)yv)[(size_t)t * N + n + e] = lo[e];
+            if (n + 4 + e < N) ((elt*)yv)[(size_t)t * N + n + 4 + e] = hi[e];
           }
         }
       }
@@ -922,10 +919,10 @@ MidShape gemm_mid_shape(int T, int K, int N, int ksplit_max) {
 }
 
 template <int OUT, int FT, int FN>
-int launch_gemm_mid_shape(void* y, float* part, int ld_part, int ksplit, const f16* xf, int x_tt, const f16* Wp, int T, int K, int N,
+int launch_gemm_mid_shape(void* y, float* part, int ld_part, int ksplit, const elt* xf, int x_tt, const elt* Wp, int T, int K, int N,
                           hipStream_t s) {
-  constexpr size_t lds = (size_t)(FT == 16 ? 3 : 4) * MID_KS * (FN + FT) * 512 * sizeof(f16);
-  static_assert(lds >= (size_t)PP_WAVES * PP_OUT_ELEMS * sizeof(f16), "the output staging fits the ring");
+  constexpr size_t lds = (size_t)(FT == 16 ? 3 : 4) * MID_KS * (FN + FT) * 512 * sizeof(elt);
+  static_assert(lds >= (size_t)PP_WAVES * PP_OUT_ELEMS * sizeof(elt), "the output staging fits the ring");
   static const hipError_t configured =               // the attribute is per kernel, set once per process, by one thread
       hipFuncSetAttribute((const void*)gemm_mid_kernel<OUT, FT, FN>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
   if (configured != hipSuccess)
@@ -936,7 +933,7 @@ int launch_gemm_mid_shape(void* y, float* part, int ld_part, int ksplit, const f
 }
 
 template <int OUT>
-int launch_gemm_mid(void* y, float* part, int ld_part, const MidShape& m, const f16* xf, int x_tt, const f16* Wp, int T, int K, int N,
+int launch_gemm_mid(void* y, float* part, int ld_part, const MidShape& m, const elt* xf, int x_tt, const elt* Wp, int T, int K, int N,
                     hipStream_t s) {
   if (m.ft == 8) {
     if (m.fn == 4) return launch_gemm_mid_shape<OUT, 8, 4>(y, part, ld_part, m.ksplit, xf, x_tt, Wp, T, K, N, s);
@@ -949,8 +946,8 @@ int launch_gemm_mid(void* y, float* part, int ld_part, const MidShape& m, const 
 }
 
 template <int OUT, int FT, int FN, int WT_, int WN_>
-int launch_gemm_lds(void* y, const f16* x, int ldx, const f16* Wp, int T, int K, int N, hipStream_t s) {
-  constexpr size_t lds = 2 * (LBK / 32) * (FT + FN) * 512 * sizeof(f16);
+int launch_gemm_lds(void* y, const elt* x, int ldx, const elt* Wp, int T, int K, int N, hipStream_t s) {
+  constexpr size_t lds = 2 * (LBK / 32) * (FT + FN) * 512 * sizeof(elt);
   static const hipError_t configured =               // the attribute is per kernel, set once per process, by one thread
       lds > 64 * 1024 ? hipFuncSetAttribute((const void*)gemm_lds_kernel<OUT, FT, FN, WT_, WN_>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)
                       : hipSuccess;
@@ -965,7 +962,7 @@ int launch_gemm_lds(void* y, const f16* x, int ldx, const f16* Wp, int T, int K,
 // 256 tokens x 64 columns (wave 64 x 64, several workgroups per CU) so that a few hundred tokens still spread
 // over all CUs.
 template <int OUT>
-int launch_gemm_lds_auto(void* y, const f16* x, int ldx, const f16* Wp, int T, int K, int N, hipStream_t s) {
+int launch_gemm_lds_auto(void* y, const elt* x, int ldx, const elt* Wp, int T, int K, int N, hipStream_t s) {
   if ((long)ceil_div(T, 256) * ceil_div(N, 256) >= 256) {
     // x rows must be 16-byte aligned for the direct-to-LDS loads (ldx % 8 == 0 is checked; the base may be a slice)
     if (((uintptr_t)x & 15) == 0 && K % 64 == 0) return launch_gemm_pp<OUT>(y, x, ldx, 0, Wp, T, K, N, s);
@@ -982,8 +979,8 @@ int gemm_dispatch(const char* who, void* y, int y_dtype, int mode, const void* x
   MLORA_CHECK(ceil_div(T, 128) <= 65535, MLORA_ERR_UNSUPPORTED, "%s: T=%d too large", who, T);
   const dim3 grid(ceil_div(N, 128), ceil_div(T, 128)), block(256);
   hipStream_t s = (hipStream_t)stream;
-  const f16* xp = (const f16*)x;
-  const f16* Wp = (const f16*)W;
+  const elt* xp = (const elt*)x;
+  const elt* Wp = (const elt*)W;
   if constexpr (PACKED) {
     if (T > 128) {
       int e;
@@ -1037,8 +1034,8 @@ extern "C" int mlora_linear_frag(void* y, int y_dtype, int mode, const void* xf,
   MLORA_CHECK(K % 32 == 0, MLORA_ERR_UNSUPPORTED, "linear_frag: K %% 32 != 0 (K=%d)", K);
   MLORA_CHECK(((uintptr_t)xf & 15) == 0, MLORA_ERR_INVALID, "linear_frag: xf must be 16-byte aligned");
   hipStream_t s = (hipStream_t)stream;
-  const f16* x = (const f16*)xf;
-  const f16* W = (const f16*)Wp;
+  const elt* x = (const elt*)xf;
+  const elt* W = (const elt*)Wp;
   const int tt = mlora_frag_tiles(T);
   int e;
   if (mlora_gemm_frag_preferred(T, K, N)) {
@@ -1054,6 +1051,19 @@ extern "C" int mlora_linear_frag(void* y, int y_dtype, int mode, const void* xf,
   return e ? e : mlora_launch_status("linear_frag");
 }
 
+extern "C" int mlora_linear_frag_clipglu(void* act, const void* xf, const void* Wp, int T, int K, int I, float scale, float limit,
+                                         float alpha, void* stream) {
+  MLORA_CHECK(act && xf && Wp, MLORA_ERR_INVALID, "linear_frag_clipglu: null pointer");
+  MLORA_CHECK(T > 0 && K > 0 && I > 0 && I % 32 == 0 && I <= (1 << 29), MLORA_ERR_UNSUPPORTED,
+              "linear_frag_clipglu: need I %% 32 == 0 (T=%d K=%d I=%d)", T, K, I);
+  MLORA_CHECK(mlora_gemm_frag_preferred(T, K, 2 * I) && (((uintptr_t)xf | (uintptr_t)act) & 15) == 0, MLORA_ERR_UNSUPPORTED,
+              "linear_frag_clipglu: only shapes of the persistent GEMM (mlora_gemm_frag_preferred; T=%d K=%d N=%d)", T, K, 2 * I);
+  const int e = launch_gemm_pp<OUT_CLIP>(act, (const elt*)xf, 0, mlora_frag_tiles(T), (const elt*)Wp, T, K, 2 * I, (hipStream_t)stream,
+                                         PPLora(), GluArgs{scale, limit, alpha});
+  return e ? e : mlora_launch_status("linear_frag_clipglu");
+}
+
+#ifndef MLORA_ELT_BF16      // the adapter kernels are fp16
 extern "C" int mlora_linear_frag_lora(void* y, int y_dtype, int mode, const void* xf, const void* Wp, int T, int K, int N,
                                       const mlora_fused_lora* projs, int n_proj, const int32_t* blk_adapter, int r, void* stream) {
   if (int e = mlora_check_linear("linear_frag_lora", y, y_dtype, mode, xf, K, Wp, T, K, N)) return e;
@@ -1071,16 +1081,16 @@ extern "C" int mlora_linear_frag_lora(void* y, int y_dtype, int mode, const void
                     (p.n_rows % (PP_F * 16) == 0 || p.n_begin + p.n_rows == N),
                 MLORA_ERR_UNSUPPORTED, "linear_frag_lora: rows %d..%d of projection %d do not fall on 256-row blocks", p.n_begin,
                 p.n_begin + p.n_rows, i);
-    lo.B[i] = (const f16*)p.B; lo.vh[i] = (const f16*)p.v_hi; lo.vl[i] = (const f16*)p.v_lo;
+    lo.B[i] = (const elt*)p.B; lo.vh[i] = (const elt*)p.v_hi; lo.vl[i] = (const elt*)p.v_lo;
     lo.n_begin[i] = p.n_begin; lo.n_rows[i] = p.n_rows;
   }
   lo.n_proj = n_proj; lo.r = r; lo.blk_adapter = blk_adapter;
   hipStream_t s = (hipStream_t)stream;
   const int tt = mlora_frag_tiles(T);
   int e;
-  if (mode == MLORA_ACCUMULATE) e = launch_gemm_pp<OUT_ACC_F32>(y, (const f16*)xf, 0, tt, (const f16*)Wp, T, K, N, s, lo);
-  else if (y_dtype == MLORA_F32) e = launch_gemm_pp<OUT_F32>(y, (const f16*)xf, 0, tt, (const f16*)Wp, T, K, N, s, lo);
-  else e = launch_gemm_pp<OUT_F16>(y, (const f16*)xf, 0, tt, (const f16*)Wp, T, K, N, s, lo);
+  if (mode == MLORA_ACCUMULATE) e = launch_gemm_pp<OUT_ACC_F32>(y, (const elt*)xf, 0, tt, (const elt*)Wp, T, K, N, s, lo);
+  else if (y_dtype == MLORA_F32) e = launch_gemm_pp<OUT_F32>(y, (const elt*)xf, 0, tt, (const elt*)Wp, T, K, N, s, lo);
+  else e = launch_gemm_pp<OUT_F16>(y, (const elt*)xf, 0, tt, (const elt*)Wp, T, K, N, s, lo);
   return e ? e : mlora_launch_status("linear_frag_lora");
 }
 
@@ -1105,14 +1115,15 @@ extern "C" int mlora_linear_frag_silu(void* act, const void* xf, const void* Wp,
                   p.n_begin, p.n_rows, I);
       const int slot = p.n_begin == 0 ? 0 : 1;
       MLORA_CHECK(lo.B[slot] == nullptr, MLORA_ERR_INVALID, "linear_frag_silu: two projections over the same rows");
-      lo.B[slot] = (const f16*)p.B; lo.vh[slot] = (const f16*)p.v_hi; lo.vl[slot] = (const f16*)p.v_lo;
+      lo.B[slot] = (const elt*)p.B; lo.vh[slot] = (const elt*)p.v_hi; lo.vl[slot] = (const elt*)p.v_lo;
       lo.n_begin[slot] = p.n_begin; lo.n_rows[slot] = p.n_rows;
     }
     lo.n_proj = n_proj; lo.r = r; lo.blk_adapter = blk_adapter;
   }
-  const int e = launch_gemm_pp<OUT_SILU>(act, (const f16*)xf, 0, mlora_frag_tiles(T), (const f16*)Wp, T, K, 2 * I, (hipStream_t)stream, lo);
+  const int e = launch_gemm_pp<OUT_SILU>(act, (const elt*)xf, 0, mlora_frag_tiles(T), (const elt*)Wp, T, K, 2 * I, (hipStream_t)stream, lo);
   return e ? e : mlora_launch_status("linear_frag_silu");
 }
+#endif
 
 // K slices the mid-size kernel would use for resid [T, N] += xf . Wp^T with at most ks_max slices (T > 64)
 int mlora_gemm_mid_ksplit(int T, int K, int N, int ks_max) { return gemm_mid_shape(T, K, N, ks_max).ksplit; }
@@ -1124,7 +1135,7 @@ int mlora_gemm_mid_acc(float* resid, float* part, int ld_part, int ks, const voi
               "linear_frag (K slices): need K %% 32 == 0 and at least one 32-k step per slice (K=%d ks=%d)", K, ks);
   MidShape m = gemm_mid_shape(T, K, N, ks);
   m.ksplit = ks;                               // the caller's partial buffers were sized for ks slices
-  const int e = launch_gemm_mid<OUT_ACC_F32>(resid, part, ld_part, m, (const f16*)xf, mlora_frag_tiles(T), (const f16*)Wp, T, K, N,
+  const int e = launch_gemm_mid<OUT_ACC_F32>(resid, part, ld_part, m, (const elt*)xf, mlora_frag_tiles(T), (const elt*)Wp, T, K, N,
                                              (hipStream_t)stream);
   return e ? e : mlora_launch_status("linear_frag (K slices)");
 }

@@ -20,7 +20,7 @@ namespace {
 constexpr int GEMV_WAVES = 8;
 constexpr int KSTEP = 32;   // k per MFMA
 
-enum { OUT_F16 = 0, OUT_F32 = 1, OUT_ACC_F32 = 2, OUT_SILU_FRAG = 3 };
+enum { OUT_F16 = 0, OUT_F32 = 1, OUT_ACC_F32 = 2, OUT_SILU_FRAG = 3, OUT_CLIP_FRAG = 4 };   // the last two: a gated product (MLORA_GLU_*) in fragment order
 
 // v / d for a uniform divisor 1..4 (the slice counts of a launch): shifts and one multiply instead of the division
 // sequences - a hundred scalar instructions each, three times over - that stood before a workgroup's first load
@@ -38,7 +38,7 @@ __device__ __forceinline__ int udiv_le4(int v, int d) {
 // KiB per rider, under the shadow of the weight stream.
 struct LoraDeltaRide {
   const float* vpart;   // [n_vpart, T, r]
-  const f16* B;         // [n_ad, N, r]
+  const elt* B;         // [n_ad, N, r]
   const int32_t* ids;   // [T]
   float* out;           // [T, N]
   float scaling;
@@ -65,8 +65,8 @@ __device__ __forceinline__ void lora_delta_ride(const LoraDeltaRide& d, int unit
   const int r = d.r, lpr = r >> 3;                           // 16-byte chunks per row of B
   const int nq = ncol * lpr;                                 // chunks of this rider's rows of B: at most BQ per thread
   // one round of requests: the rider's rows of B (uniform base + 32-bit lane offset) and the shares of v
-  f16x8 bv[BQ];
-  const f16* __restrict__ Bp = d.B + ((size_t)id * d.N + c0) * r;
+  eltx8 bv[BQ];
+  const elt* __restrict__ Bp = d.B + ((size_t)id * d.N + c0) * r;
 #pragma unroll
   for (int u = 0; u < BQ; ++u) {
     const int q = u * NTH + tid;
@@ -123,11 +123,11 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE) void lora_expand_shares_kernel(Lo
 // x instead of a GEMV tile: the adapter work rides in the GEMV launch and finishes long before it does.
 // An accumulating launch without shrink units may instead carry `ride_blocks` delta riders (lora_delta_ride).
 template <int NT, int TT, int OUT, bool PACKED, bool XFRAG, bool SHRINK, int PIPE = 4>   // PIPE: k-steps in flight per wave
-__global__ __launch_bounds__(GEMV_WAVES* WAVE, (NT * TT > 8 ? 2 : 4)) void gemv_kernel(void* __restrict__ yv, const f16* __restrict__ x, int ldx,
-                                                                const f16* __restrict__ W, int T, int K, int N,
+__global__ __launch_bounds__(GEMV_WAVES* WAVE, (NT * TT > 8 ? 2 : 4)) void gemv_kernel(void* __restrict__ yv, const elt* __restrict__ x, int ldx,
+                                                                const elt* __restrict__ W, int T, int K, int N,
                                                                 LoraShrinkBatch sb, int shrink_blocks, int n_main,
                                                                 float* __restrict__ y2, int ksplit, float* __restrict__ part,
-                                                                LoraDeltaRide dr, int ride_blocks) {
+                                                                LoraDeltaRide dr, int ride_blocks, GluArgs ga) {
   constexpr int TILES = NT * TT;
   constexpr int HT = TILES > 8 ? TILES / 2 : TILES;   // accumulator tiles summed per pass through LDS (64 KiB holds 8)
   constexpr bool RIDE = OUT == OUT_ACC_F32 && PACKED && XFRAG && !SHRINK;   // the launches that may carry delta riders
@@ -167,9 +167,9 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE, (NT * TT > 8 ? 2 : 4)) void gemv_
   const int KB = K / KSTEP;
   constexpr int WSTEP = PACKED ? 512 : KSTEP;   // elements between consecutive k-steps of one fragment stream
 
-  const f16* wp[PACKED ? 1 : NT];
+  const elt* wp[PACKED ? 1 : NT];
   int woff[NT];                                    // packed: element offset of tile i from the block's first tile (uniform)
-  const f16* xp[TT];
+  const elt* xp[TT];
   if constexpr (PACKED) wp[0] = W + ((size_t)bid * NT * KB) * 512 + lane * 8;
 #pragma unroll
   for (int i = 0; i < NT; ++i) {
@@ -206,14 +206,14 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE, (NT * TT > 8 ? 2 : 4)) void gemv_
   const int kb0 = ksplit > 1 ? udiv_le4(slice * KB, ksplit) : 0;
   const int kb1 = ksplit > 1 ? udiv_le4((slice + 1) * KB, ksplit) : KB;
   const int S = (kb1 - kb0 - wave + GEMV_WAVES - 1) / GEMV_WAVES;
-  f16x8 a[PIPE][NT], b[PIPE][TT];
+  eltx8 a[PIPE][NT], b[PIPE][TT];
   auto load_stage = [&](int u, int s) {
     const bool in = s < S;
     const int ks = in ? kb0 + wave + GEMV_WAVES * s : 0;
 #pragma unroll
     for (int i = 0; i < NT; ++i) {
-      a[u][i] = __builtin_nontemporal_load(reinterpret_cast<const f16x8*>(wp[PACKED ? 0 : i] + (woff[i] + ks * WSTEP)));
-      if (!in) a[u][i] = f16x8{0, 0, 0, 0, 0, 0, 0, 0};
+      a[u][i] = __builtin_nontemporal_load(reinterpret_cast<const eltx8*>(wp[PACKED ? 0 : i] + (woff[i] + ks * WSTEP)));
+      if (!in) a[u][i] = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
     }
 #pragma unroll
     for (int j = 0; j < TT; ++j) b[u][j] = ld8(xp[j] + (size_t)ks * XSTEP);
@@ -226,14 +226,15 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE, (NT * TT > 8 ? 2 : 4)) void gemv_
 #pragma unroll
       for (int i = 0; i < NT; ++i)
 #pragma unroll
-        for (int j = 0; j < TT; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_f16(a[u][i], b[u][j], acc[i][j], 0, 0, 0);
+        for (int j = 0; j < TT; ++j) acc[i][j] = mfma_16x16x32(a[u][i], b[u][j], acc[i][j]);
       load_stage(u, s0 + u + PIPE);
     }
   }
 
-  if constexpr (OUT == OUT_SILU_FRAG) {
+  if constexpr (OUT == OUT_SILU_FRAG || OUT == OUT_CLIP_FRAG) {
+    constexpr int KIND = OUT == OUT_SILU_FRAG ? MLORA_GLU_SILU : MLORA_GLU_CLIPPED;
     // The weight interleaves 16-row tiles of gate and up, so this block's two tiles are gate rows c..c+15 and up
-    // rows c..c+15 of the same channels: out[t, c + ..] = silu(f16(gate)) * f16(up), written in fragment order.
+    // rows c..c+15 of the same channels: out[t, c + ..] = silu(elt(gate)) * elt(up), written in fragment order.
     static_assert(NT % 2 == 0 && TILES <= 8, "the SiLU epilogue pairs a gate tile with an up tile and sums all tiles in one pass");
 #pragma unroll
     for (int i = 0; i < NT; ++i)
@@ -252,13 +253,10 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE, (NT * TT > 8 ? 2 : 4)) void gemv_
       const int c = (bid * (NT / 2) + p) * 16 + (sl >> 4) * 4;   // output channel of the first of this lane's 4 rows
       const int t = j * 16 + (sl & 15);
       if (t < T && c < N / 2) {
-        f16x4 o;
+        eltx4 o;
 #pragma unroll
-        for (int q = 0; q < 4; ++q) {
-          const float gf = (float)(f16)sg[q];
-          o[q] = (f16)(gf / (1.f + expf(-gf)) * (float)(f16)su[q]);
-        }
-        *reinterpret_cast<f16x4*>((f16*)yv + frag_offset(t, c, TT)) = o;
+        for (int q = 0; q < 4; ++q) o[q] = (elt)glu<KIND>(sg[q], su[q], ga);
+        *reinterpret_cast<eltx4*>((elt*)yv + frag_offset(t, c, TT)) = o;
       }
     }
     return;
@@ -292,7 +290,7 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE, (NT * TT > 8 ? 2 : 4)) void gemv_
       } else if (t < T && n < N) {                 // N % 4 == 0: the 4 rows are inside together
         const size_t o = (size_t)t * n_main + n;
         if constexpr (OUT == OUT_F16) {
-          *reinterpret_cast<f16x4*>((f16*)yv + o) = f16x4{(f16)s[0], (f16)s[1], (f16)s[2], (f16)s[3]};
+          *reinterpret_cast<eltx4*>((elt*)yv + o) = eltx4{(elt)s[0], (elt)s[1], (elt)s[2], (elt)s[3]};
         } else if constexpr (OUT == OUT_F32) {
           *reinterpret_cast<f32x4*>((float*)yv + o) = s;
         } else if constexpr (OUT == OUT_ACC_F32) {
@@ -304,15 +302,15 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE, (NT * TT > 8 ? 2 : 4)) void gemv_
   }
 }
 
-// Gate/up GEMV with the SiLU epilogue as ONE workgroup per compute unit.  A unit takes in first-level-cache fills at a
+// Gate/up GEMV with the gated product as its epilogue, as ONE workgroup per compute unit.  A unit takes in first-level-cache fills at a
 // bounded rate, weights and token block together, so a launch is as fast as its most loaded unit: here every unit gets
 // an equal share of the (gate tile, up tile) pairs - NP or NP - 1 of them - and reads the token block once for all of
 // them, instead of once per pair.  Same k-split over the 8 waves and the same fixed-order reduction as gemv_kernel, so
 // the result bits are the same.  The reduction goes through LDS one pair at a time.
-template <int NP, int TT, int PIPE>
-__global__ __launch_bounds__(GEMV_WAVES* WAVE, 2) void gemv_silu_cu_kernel(f16* __restrict__ act, const f16* __restrict__ x,
-                                                                        const f16* __restrict__ W, int T, int K, int I,
-                                                                        int base, int rem) {
+template <int NP, int TT, int PIPE, int KIND>
+__global__ __launch_bounds__(GEMV_WAVES* WAVE, 2) void gemv_glu_cu_kernel(elt* __restrict__ act, const elt* __restrict__ x,
+                                                                        const elt* __restrict__ W, int T, int K, int I,
+                                                                        int base, int rem, GluArgs ga) {
   constexpr int NT = 2 * NP;
   __shared__ f32x4 red[GEMV_WAVES][2 * TT][WAVE];
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
@@ -321,11 +319,11 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE, 2) void gemv_silu_cu_kernel(f16* 
   const int p0 = wg * base + (wg < rem ? wg : rem);    // first pair of this workgroup
   const int np = base + (wg < rem ? 1 : 0);            // and how many it has
   const int KB = K / KSTEP;
-  const f16* wp = W + ((size_t)(2 * p0) * KB) * 512 + lane * 8;
+  const elt* wp = W + ((size_t)(2 * p0) * KB) * 512 + lane * 8;
   int woff[NT];                                        // a missing last pair repeats the first tile (cache hits) and is not stored
 #pragma unroll
   for (int i = 0; i < NT; ++i) woff[i] = (i < 2 * np ? i : 0) * KB * 512;
-  const f16* xp = x + lane * 8;
+  const elt* xp = x + lane * 8;
   constexpr int XSTEP = TT * 512;
 
   f32x4 acc[NT][TT];
@@ -334,14 +332,14 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE, 2) void gemv_silu_cu_kernel(f16* 
 #pragma unroll
     for (int j = 0; j < TT; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
   const int S = (KB - wave + GEMV_WAVES - 1) / GEMV_WAVES;
-  f16x8 a[PIPE][NT], b[PIPE][TT];
+  eltx8 a[PIPE][NT], b[PIPE][TT];
   auto load_stage = [&](int u, int s) {
     const bool in = s < S;
     const int ks = in ? wave + GEMV_WAVES * s : 0;
 #pragma unroll
     for (int i = 0; i < NT; ++i) {
-      a[u][i] = __builtin_nontemporal_load(reinterpret_cast<const f16x8*>(wp + (woff[i] + ks * 512)));
-      if (!in) a[u][i] = f16x8{0, 0, 0, 0, 0, 0, 0, 0};
+      a[u][i] = __builtin_nontemporal_load(reinterpret_cast<const eltx8*>(wp + (woff[i] + ks * 512)));
+      if (!in) a[u][i] = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
     }
 #pragma unroll
     for (int j = 0; j < TT; ++j) b[u][j] = ld8(xp + j * 512 + (size_t)ks * XSTEP);
@@ -354,7 +352,7 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE, 2) void gemv_silu_cu_kernel(f16* 
 #pragma unroll
       for (int i = 0; i < NT; ++i)
 #pragma unroll
-        for (int j = 0; j < TT; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_f16(a[u][i], b[u][j], acc[i][j], 0, 0, 0);
+        for (int j = 0; j < TT; ++j) acc[i][j] = mfma_16x16x32(a[u][i], b[u][j], acc[i][j]);
       load_stage(u, s0 + u + PIPE);
     }
   }
@@ -377,13 +375,10 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE, 2) void gemv_silu_cu_kernel(f16* 
         const int c = (p0 + p) * 16 + (sl >> 4) * 4;   // output channel of the first of this lane's 4 rows
         const int t = j * 16 + (sl & 15);
         if (t < T && c < I) {
-          f16x4 o;
+          eltx4 o;
 #pragma unroll
-          for (int q = 0; q < 4; ++q) {
-            const float gf = (float)(f16)sg[q];
-            o[q] = (f16)(gf / (1.f + expf(-gf)) * (float)(f16)su[q]);
-          }
-          *reinterpret_cast<f16x4*>(act + frag_offset(t, c, TT)) = o;
+          for (int q = 0; q < 4; ++q) o[q] = (elt)glu<KIND>(sg[q], su[q], ga);
+          *reinterpret_cast<eltx4*>(act + frag_offset(t, c, TT)) = o;
         }
       }
       __syncthreads();
@@ -396,11 +391,11 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE, 2) void gemv_silu_cu_kernel(f16* 
 // and every (tile, range) piece goes to a unit of its own, starting with the units that got one main tile fewer, so
 // that no unit takes in more than NM tiles plus a 1/kq piece - with whole appended tiles in the deal, the units that
 // drew one would set the time of the launch.  A piece's fp32 partial goes to block `range` of y2 [kq][T][n_ext];
-// whoever reads the shrink results adds the blocks in range order.  Main rows: f16 store, the k order and the wave
+// whoever reads the shrink results adds the blocks in range order.  Main rows: elt store, the k order and the wave
 // reduction of gemv_kernel, hence its bits.
 template <int NM, int TT, int PIPE>
-__global__ __launch_bounds__(GEMV_WAVES* WAVE, 2) void gemv_split_cu_kernel(f16* __restrict__ y, float* __restrict__ y2,
-                                                                         const f16* __restrict__ x, const f16* __restrict__ W,
+__global__ __launch_bounds__(GEMV_WAVES* WAVE, 2) void gemv_split_cu_kernel(elt* __restrict__ y, float* __restrict__ y2,
+                                                                         const elt* __restrict__ x, const elt* __restrict__ W,
                                                                          int T, int K, int n_main, int n_ext, int base, int rem,
                                                                          int kq, int n_wg) {   // n_wg: the grid size, as an argument (gridDim comes from a later scalar load)
   constexpr int NT = NM + 1;                           // register tile NM is the piece of an appended tile
@@ -416,12 +411,12 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE, 2) void gemv_split_cu_kernel(f16*
   const bool has_ext = piece < (n_ext / 16) * kq;
   const int et = has_ext ? udiv_le4(piece, kq) : 0, eq = has_ext ? piece - et * kq : 0;
   const int ekb0 = has_ext ? udiv_le4(eq * KB, kq) : 0, ekb1 = has_ext ? udiv_le4((eq + 1) * KB, kq) : 0;
-  const f16* wp = W + lane * 8;
+  const elt* wp = W + lane * 8;
   size_t woff[NT];                                     // a missing main tile repeats the first one (cache hits) and is not stored
 #pragma unroll
   for (int i = 0; i < NM; ++i) woff[i] = (size_t)(m0 + (i < nm ? i : 0)) * KB * 512;
   woff[NM] = (size_t)(n_main / 16 + et) * KB * 512;
-  const f16* xp = x + lane * 8;
+  const elt* xp = x + lane * 8;
   constexpr int XSTEP = TT * 512;
 
   f32x4 acc[NT][TT];
@@ -430,18 +425,18 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE, 2) void gemv_split_cu_kernel(f16*
 #pragma unroll
     for (int j = 0; j < TT; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
   const int S = (KB - wave + GEMV_WAVES - 1) / GEMV_WAVES;
-  f16x8 a[PIPE][NT], b[PIPE][TT];
+  eltx8 a[PIPE][NT], b[PIPE][TT];
   auto load_stage = [&](int u, int s) {
     const bool in = s < S;
     const int ks = in ? wave + GEMV_WAVES * s : 0;
 #pragma unroll
     for (int i = 0; i < NM; ++i) {
-      a[u][i] = __builtin_nontemporal_load(reinterpret_cast<const f16x8*>(wp + (woff[i] + (size_t)ks * 512)));
-      if (!in) a[u][i] = f16x8{0, 0, 0, 0, 0, 0, 0, 0};
+      a[u][i] = __builtin_nontemporal_load(reinterpret_cast<const eltx8*>(wp + (woff[i] + (size_t)ks * 512)));
+      if (!in) a[u][i] = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
     }
-    a[u][NM] = f16x8{0, 0, 0, 0, 0, 0, 0, 0};
+    a[u][NM] = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
     if (in && ks >= ekb0 && ks < ekb1)                 // wave-uniform: the piece covers only its range of K
-      a[u][NM] = __builtin_nontemporal_load(reinterpret_cast<const f16x8*>(wp + (woff[NM] + (size_t)ks * 512)));
+      a[u][NM] = __builtin_nontemporal_load(reinterpret_cast<const eltx8*>(wp + (woff[NM] + (size_t)ks * 512)));
 #pragma unroll
     for (int j = 0; j < TT; ++j) b[u][j] = ld8(xp + j * 512 + (size_t)ks * XSTEP);
   };
@@ -453,7 +448,7 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE, 2) void gemv_split_cu_kernel(f16*
 #pragma unroll
       for (int i = 0; i < NT; ++i)
 #pragma unroll
-        for (int j = 0; j < TT; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_f16(a[u][i], b[u][j], acc[i][j], 0, 0, 0);
+        for (int j = 0; j < TT; ++j) acc[i][j] = mfma_16x16x32(a[u][i], b[u][j], acc[i][j]);
       load_stage(u, s0 + u + PIPE);
     }
   }
@@ -474,7 +469,7 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE, 2) void gemv_split_cu_kernel(f16*
         if (t < T) {
           if (i < NM) {
             const int n = (m0 + i) * 16 + (sl >> 4) * 4;
-            *reinterpret_cast<f16x4*>(y + (size_t)t * n_main + n) = f16x4{(f16)s[0], (f16)s[1], (f16)s[2], (f16)s[3]};
+            *reinterpret_cast<eltx4*>(y + (size_t)t * n_main + n) = eltx4{(elt)s[0], (elt)s[1], (elt)s[2], (elt)s[3]};
           } else {
             const int n = et * 16 + (sl >> 4) * 4;
             *reinterpret_cast<f32x4*>(y2 + ((size_t)eq * T + t) * n_ext + n) = s;
@@ -487,7 +482,7 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE, 2) void gemv_split_cu_kernel(f16*
 }
 
 // one thread per 16-byte chunk of the packed array
-__global__ __launch_bounds__(256) void pack_weight_kernel(f16* __restrict__ dst, const f16* __restrict__ src, int N, int K,
+__global__ __launch_bounds__(256) void pack_weight_kernel(elt* __restrict__ dst, const elt* __restrict__ src, int N, int K,
                                                           size_t chunks) {
   const size_t c = (size_t)blockIdx.x * 256 + threadIdx.x;
   if (c >= chunks) return;
@@ -498,33 +493,33 @@ __global__ __launch_bounds__(256) void pack_weight_kernel(f16* __restrict__ dst,
   const int ks = blk % KB;
   const size_t nt = blk / KB;
   const size_t n = nt * 16 + row;
-  f16x8 v = f16x8{0, 0, 0, 0, 0, 0, 0, 0};
+  eltx8 v = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
   if (n < (size_t)N) v = ld8(src + n * K + ks * KSTEP + g * 8);
   st8(dst + c * 8, v);
 }
 
 // one thread per 16-byte chunk of the fragment-ordered activation block
-__global__ __launch_bounds__(256) void pack_activation_kernel(f16* __restrict__ dst, const f16* __restrict__ src, int ldsrc,
+__global__ __launch_bounds__(256) void pack_activation_kernel(elt* __restrict__ dst, const elt* __restrict__ src, int ldsrc,
                                                               int T, int K, int TT, int chunks) {
   const int c = blockIdx.x * 256 + threadIdx.x;
   if (c >= chunks) return;
   const int t16 = c & 15, kg = (c >> 4) & 3, blk = c >> 6;
   const int tt = blk % TT, ks = blk / TT;
   const int t = tt * 16 + t16;
-  f16x8 v = f16x8{0, 0, 0, 0, 0, 0, 0, 0};
+  eltx8 v = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
   if (t < T) v = ld8(src + (size_t)t * ldsrc + ks * KSTEP + kg * 8);
   st8(dst + (size_t)c * 8, v);
 }
 
 template <int NT, int TT, bool PACKED, bool XFRAG, bool SHRINK, int PIPE = 4>
-void launch_gemv(void* y, int out, const f16* x, int ldx, const f16* W, int T, int K, int N, hipStream_t s,
+void launch_gemv(void* y, int out, const elt* x, int ldx, const elt* W, int T, int K, int N, hipStream_t s,
                  const LoraShrinkBatch& sb, int n_main, float* y2, int ksplit = 1, float* part = nullptr,
                  const LoraDeltaRide& dr = LoraDeltaRide(), int rblocks = 0) {
   const int sblocks = SHRINK ? ceil_div(lora_shrink_units(sb), GEMV_WAVES) : 0;
   const dim3 grid(ceil_div(N, 16 * NT) * ksplit + sblocks + rblocks), block(GEMV_WAVES * WAVE);
-  if (out == OUT_F16) hipLaunchKernelGGL((gemv_kernel<NT, TT, OUT_F16, PACKED, XFRAG, SHRINK, PIPE>), grid, block, 0, s, y, x, ldx, W, T, K, N, sb, sblocks, n_main, y2, ksplit, part, dr, 0);
-  else if (out == OUT_F32) hipLaunchKernelGGL((gemv_kernel<NT, TT, OUT_F32, PACKED, XFRAG, SHRINK, PIPE>), grid, block, 0, s, y, x, ldx, W, T, K, N, sb, sblocks, n_main, y2, ksplit, part, dr, 0);
-  else hipLaunchKernelGGL((gemv_kernel<NT, TT, OUT_ACC_F32, PACKED, XFRAG, SHRINK, PIPE>), grid, block, 0, s, y, x, ldx, W, T, K, N, sb, sblocks, n_main, y2, ksplit, part, dr, rblocks);
+  if (out == OUT_F16) hipLaunchKernelGGL((gemv_kernel<NT, TT, OUT_F16, PACKED, XFRAG, SHRINK, PIPE>), grid, block, 0, s, y, x, ldx, W, T, K, N, sb, sblocks, n_main, y2, ksplit, part, dr, 0, GluArgs());
+  else if (out == OUT_F32) hipLaunchKernelGGL((gemv_kernel<NT, TT, OUT_F32, PACKED, XFRAG, SHRINK, PIPE>), grid, block, 0, s, y, x, ldx, W, T, K, N, sb, sblocks, n_main, y2, ksplit, part, dr, 0, GluArgs());
+  else hipLaunchKernelGGL((gemv_kernel<NT, TT, OUT_ACC_F32, PACKED, XFRAG, SHRINK, PIPE>), grid, block, 0, s, y, x, ldx, W, T, K, N, sb, sblocks, n_main, y2, ksplit, part, dr, rblocks, GluArgs());
 }
 
 // Rows per workgroup.  Every workgroup reads the whole token block, so its L2 traffic is T / (16 NT) of the weight
@@ -548,8 +543,8 @@ int gemv_dispatch(void* y, int y_dtype, int mode, const void* x, int ldx, const 
   if (n_main < 0) n_main = N;
   const int out = mode == MLORA_ACCUMULATE ? OUT_ACC_F32 : (y_dtype == MLORA_F32 ? OUT_F32 : OUT_F16);
   hipStream_t s = (hipStream_t)stream;
-  const f16* xp = (const f16*)x;
-  const f16* Wp = (const f16*)W;
+  const elt* xp = (const elt*)x;
+  const elt* Wp = (const elt*)W;
   const int tiles = ceil_div(N, 16);
   if constexpr (PACKED && XFRAG) {
     if (T <= 32 && (ksplit > 1 || tiles >= 768)) {
@@ -656,6 +651,7 @@ static LoraShrinkBatch shrink_batch(const void* xf, void* v_part, const void* co
   return b;
 }
 
+#ifndef MLORA_ELT_BF16      // the adapter kernels are fp16
 extern "C" int mlora_gemv_frag_lora(void* y, int y_dtype, int mode, const void* xf, const void* Wp, int T, int K, int N,
                                     void* v_part, const void* const* A, int n_proj, const int32_t* tok_adapter, int r,
                                     int n_ad, void* stream) {
@@ -666,6 +662,7 @@ extern "C" int mlora_gemv_frag_lora(void* y, int y_dtype, int mode, const void* 
   return gemv_dispatch<true, true, true>(y, y_dtype, mode, xf, K, Wp, T, K, N, stream,
                                          shrink_batch(xf, v_part, A, n_proj, tok_adapter, T, K, r, n_ad));
 }
+#endif
 
 // A narrow weight (fewer than 512 row tiles) gives too few workgroups for four tiles each; splitting K over up to four
 // workgroups restores one equal workgroup per compute unit.  At least 24 k-steps per slice keep every wave's pipeline full.
@@ -724,6 +721,7 @@ extern "C" int mlora_gemv_frag_acc_ksplit(float* y, float* y2, float* part, int 
                                           ks, part);
 }
 
+#ifndef MLORA_ELT_BF16      // the adapter kernels are fp16
 // Riders per token of the delta-carrying launch below (0: the shape is not served): a rider thread keeps at most
 // RIDE_BQ 16-byte chunks of B, the launch must be K-split (it is the split form of the kernel that carries riders),
 // and with riders the slices are chosen as if the matrix had 256 more rows (sixteen workgroups' worth, as for the
@@ -757,7 +755,7 @@ extern "C" int mlora_gemv_frag_acc_ksplit_delta(float* y, float* part, int ks, c
   MLORA_CHECK(n_vpart >= 1, MLORA_ERR_INVALID, "gemv_frag_acc_ksplit_delta: no shares");
   LoraDeltaRide dr;
   dr.vpart = vpart;
-  dr.B = (const f16*)B;
+  dr.B = (const elt*)B;
   dr.ids = tok_adapter;
   dr.out = part + (size_t)(ks - 1) * T * N;       // the slot behind the K-slice partials
   dr.scaling = scaling;
@@ -785,7 +783,7 @@ extern "C" int mlora_lora_expand_shares(float* y, const float* vpart, int n_vpar
   if (T == 0) return MLORA_OK;
   LoraDeltaRide dr;
   dr.vpart = vpart;
-  dr.B = (const f16*)B;
+  dr.B = (const elt*)B;
   dr.ids = tok_adapter;
   dr.out = y;
   dr.scaling = scaling;
@@ -795,13 +793,16 @@ extern "C" int mlora_lora_expand_shares(float* y, const float* vpart, int n_vpar
   hipLaunchKernelGGL(lora_expand_shares_kernel, dim3(T * per_token), dim3(GEMV_WAVES * WAVE), 0, (hipStream_t)stream, dr);
   return mlora_launch_status("lora_expand_shares");
 }
+#endif
 
-extern "C" int mlora_gemv_frag_silu(void* act, const void* xf, const void* Wil_p, int T, int K, int I, void* stream) {
-  MLORA_CHECK(act && xf && Wil_p, MLORA_ERR_INVALID, "gemv_frag_silu: null pointer");
+template <int KIND>
+static int gemv_frag_glu(const char* who, void* act, const void* xf, const void* Wil_p, int T, int K, int I, const GluArgs& ga, void* stream) {
+  constexpr int OUT = KIND == MLORA_GLU_SILU ? OUT_SILU_FRAG : OUT_CLIP_FRAG;
+  MLORA_CHECK(act && xf && Wil_p, MLORA_ERR_INVALID, "%s: null pointer", who);
   MLORA_CHECK(T > 0 && T <= 64 && K > 0 && K % 32 == 0 && I > 0 && I % 32 == 0, MLORA_ERR_UNSUPPORTED,
-              "gemv_frag_silu: need 0 < T <= 64, K %% 32 == 0, I %% 32 == 0 (T=%d K=%d I=%d)", T, K, I);
-  const f16* xp = (const f16*)xf;
-  const f16* Wp = (const f16*)Wil_p;
+              "%s: need 0 < T <= 64, K %% 32 == 0, I %% 32 == 0 (T=%d K=%d I=%d)", who, T, K, I);
+  const elt* xp = (const elt*)xf;
+  const elt* Wp = (const elt*)Wil_p;
   hipStream_t s = (hipStream_t)stream;
   const LoraShrinkBatch sb = LoraShrinkBatch();
   const dim3 grid(I / 16), block(GEMV_WAVES * WAVE);
@@ -812,27 +813,36 @@ extern "C" int mlora_gemv_frag_silu(void* act, const void* xf, const void* Wil_p
   if ((T <= 32 || per <= 3) && n_cu > 0 && pairs >= 2 * n_cu && per <= 4) {
     const int base = pairs / n_cu, rem = pairs % n_cu;
     const dim3 g(n_cu);
-#define MLORA_SILU_CU(NP, TT, PIPE) \
-  hipLaunchKernelGGL((gemv_silu_cu_kernel<NP, TT, PIPE>), g, block, 0, s, (f16*)act, xp, Wp, T, K, I, base, rem)
+#define MLORA_GLU_CU(NP, TT, PIPE) \
+  hipLaunchKernelGGL((gemv_glu_cu_kernel<NP, TT, PIPE, KIND>), g, block, 0, s, (elt*)act, xp, Wp, T, K, I, base, rem, ga)
     if (T <= 16) {
-      if (per <= 2) MLORA_SILU_CU(2, 1, 4);
-      else if (per == 3) MLORA_SILU_CU(3, 1, 4);
-      else MLORA_SILU_CU(4, 1, 3);
+      if (per <= 2) MLORA_GLU_CU(2, 1, 4);
+      else if (per == 3) MLORA_GLU_CU(3, 1, 4);
+      else MLORA_GLU_CU(4, 1, 3);
     } else if (T <= 32) {
-      if (per <= 2) MLORA_SILU_CU(2, 2, 4);
-      else if (per == 3) MLORA_SILU_CU(3, 2, 3);
-      else MLORA_SILU_CU(4, 2, 2);
+      if (per <= 2) MLORA_GLU_CU(2, 2, 4);
+      else if (per == 3) MLORA_GLU_CU(3, 2, 3);
+      else MLORA_GLU_CU(4, 2, 2);
     } else {                                   // 33..64 tokens: four token tiles, at most three pairs fit the registers
-      if (per <= 2) MLORA_SILU_CU(2, 4, 2);
-      else MLORA_SILU_CU(3, 4, 2);
+      if (per <= 2) MLORA_GLU_CU(2, 4, 2);
+      else MLORA_GLU_CU(3, 4, 2);
     }
-#undef MLORA_SILU_CU
-    return mlora_launch_status("gemv_frag_silu");
+#undef MLORA_GLU_CU
+    return mlora_launch_status(who);
   }
-  if (T <= 16) hipLaunchKernelGGL((gemv_kernel<2, 1, OUT_SILU_FRAG, true, true, false>), grid, block, 0, s, act, xp, K, Wp, T, K, 2 * I, sb, 0, 2 * I, nullptr, 1, nullptr, LoraDeltaRide(), 0);
-  else if (T <= 32) hipLaunchKernelGGL((gemv_kernel<2, 2, OUT_SILU_FRAG, true, true, false>), grid, block, 0, s, act, xp, K, Wp, T, K, 2 * I, sb, 0, 2 * I, nullptr, 1, nullptr, LoraDeltaRide(), 0);
-  else hipLaunchKernelGGL((gemv_kernel<2, 4, OUT_SILU_FRAG, true, true, false, 2>), grid, block, 0, s, act, xp, K, Wp, T, K, 2 * I, sb, 0, 2 * I, nullptr, 1, nullptr, LoraDeltaRide(), 0);
-  return mlora_launch_status("gemv_frag_silu");
+  if (T <= 16) hipLaunchKernelGGL((gemv_kernel<2, 1, OUT, true, true, false>), grid, block, 0, s, act, xp, K, Wp, T, K, 2 * I, sb, 0, 2 * I, nullptr, 1, nullptr, LoraDeltaRide(), 0, ga);
+  else if (T <= 32) hipLaunchKernelGGL((gemv_kernel<2, 2, OUT, true, true, false>), grid, block, 0, s, act, xp, K, Wp, T, K, 2 * I, sb, 0, 2 * I, nullptr, 1, nullptr, LoraDeltaRide(), 0, ga);
+  else hipLaunchKernelGGL((gemv_kernel<2, 4, OUT, true, true, false, 2>), grid, block, 0, s, act, xp, K, Wp, T, K, 2 * I, sb, 0, 2 * I, nullptr, 1, nullptr, LoraDeltaRide(), 0, ga);
+  return mlora_launch_status(who);
+}
+
+extern "C" int mlora_gemv_frag_silu(void* act, const void* xf, const void* Wil_p, int T, int K, int I, void* stream) {
+  return gemv_frag_glu<MLORA_GLU_SILU>("gemv_frag_silu", act, xf, Wil_p, T, K, I, GluArgs(), stream);
+}
+
+extern "C" int mlora_gemv_frag_clipglu(void* act, const void* xf, const void* Wil_p, int T, int K, int I, float scale, float limit,
+                                       float alpha, void* stream) {
+  return gemv_frag_glu<MLORA_GLU_CLIPPED>("gemv_frag_clipglu", act, xf, Wil_p, T, K, I, GluArgs{scale, limit, alpha}, stream);
 }
 
 extern "C" int mlora_gemv_frag_split(void* y, int y_dtype, int mode, float* y2, const void* xf, const void* Wp, int T, int K,
@@ -874,7 +884,7 @@ extern "C" int mlora_gemv_frag_split_kq(void* y, float* y2, int kq, const void* 
   const dim3 g(n_cu), block(GEMV_WAVES * WAVE);
   hipStream_t s = (hipStream_t)stream;
 #define MLORA_SPLIT_CU(NM, TT, PIPE)                                                                                       \
-  hipLaunchKernelGGL((gemv_split_cu_kernel<NM, TT, PIPE>), g, block, 0, s, (f16*)y, y2, (const f16*)xf, (const f16*)Wp, T, K, \
+  hipLaunchKernelGGL((gemv_split_cu_kernel<NM, TT, PIPE>), g, block, 0, s, (elt*)y, y2, (const elt*)xf, (const elt*)Wp, T, K, \
                      N_main, N_ext, base, rem, kq, n_cu)
   if (T <= 16) {
     if (per <= 2) MLORA_SPLIT_CU(2, 1, 4);
@@ -897,8 +907,8 @@ extern "C" int mlora_pack_activation(void* dst, const void* src, int ldsrc, int 
   MLORA_CHECK(T > 0 && K > 0 && K % 32 == 0 && ldsrc >= K && ldsrc % 8 == 0 && (size_t)mlora_frag_tiles(T) * 2 * K < 0x7fffffffULL,
               MLORA_ERR_UNSUPPORTED, "pack_activation: need T > 0, K %% 32 == 0, ldsrc >= K (T=%d K=%d ldsrc=%d)", T, K, ldsrc);
   const int chunks = mlora_frag_tiles(T) * 16 * (K / 8);
-  hipLaunchKernelGGL(pack_activation_kernel, dim3(ceil_div(chunks, 256)), dim3(256), 0, (hipStream_t)stream, (f16*)dst,
-                     (const f16*)src, ldsrc, T, K, mlora_frag_tiles(T), chunks);
+  hipLaunchKernelGGL(pack_activation_kernel, dim3(ceil_div(chunks, 256)), dim3(256), 0, (hipStream_t)stream, (elt*)dst,
+                     (const elt*)src, ldsrc, T, K, mlora_frag_tiles(T), chunks);
   return mlora_launch_status("pack_activation");
 }
 
@@ -912,7 +922,7 @@ extern "C" int mlora_pack_weight(void* dst, const void* src, int N, int K, void*
   MLORA_CHECK(N > 0 && K > 0 && K % 32 == 0, MLORA_ERR_UNSUPPORTED, "pack_weight: need K %% 32 == 0 (N=%d K=%d)", N, K);
   const size_t chunks = mlora_packed_weight_elems(N, K) / 8;
   MLORA_CHECK(chunks / 256 + 1 < 0x7fffffffULL, MLORA_ERR_UNSUPPORTED, "pack_weight: matrix too large");
-  hipLaunchKernelGGL(pack_weight_kernel, dim3((unsigned)((chunks + 255) / 256)), dim3(256), 0, (hipStream_t)stream, (f16*)dst,
-                     (const f16*)src, N, K, chunks);
+  hipLaunchKernelGGL(pack_weight_kernel, dim3((unsigned)((chunks + 255) / 256)), dim3(256), 0, (hipStream_t)stream, (elt*)dst,
+                     (const elt*)src, N, K, chunks);
   return mlora_launch_status("pack_weight");
 }

@@ -1,0 +1,327 @@
+// Mixture of experts: routing, the plan that sorts (token, choice) entries by expert, the expert linears over that plan,
+// and the weighted sum.  Compiled for every element type (the fp32 build has its linears in linear_f32.hip).
+#include "moe.h"
+
+namespace {
+
+constexpr int RT_WAVES = 4;
+constexpr int RT_MAX_E = 1024;
+
+// One wave per token: z = scale * logit + bias, the `top` largest (the lower index on ties), softmax over those.
+__global__ __launch_bounds__(RT_WAVES* WAVE) void moe_route_kernel(int32_t* __restrict__ pick, float* __restrict__ weight,
+                                                                  const float* __restrict__ logits, int ld, const float* __restrict__ bias,
+                                                                  float scale, int T, int E, int top) {
+  __shared__ float zs[RT_WAVES][RT_MAX_E];
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int t = blockIdx.x * RT_WAVES + wave;
+  if (t >= T) return;                       // no barrier below: the waves are independent
+  float* z = zs[wave];
+  for (int e = lane; e < E; e += WAVE) z[e] = fmaf(logits[(size_t)t * ld + e], scale, bias[e]);
+  float z0 = 0.f, sum = 0.f;
+  for (int k = 0; k < top; ++k) {
+    float bv = -INFINITY;
+    int bi = 0x7fffffff;
+    for (int e = lane; e < E; e += WAVE) {  // a lane reads and marks only its own entries
+      const float v = z[e];
+      if (v > bv) {
+        bv = v;
+        bi = e;
+      }
+    }
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const float ov = __shfl_xor(bv, o, WAVE);
+      const int oi = __shfl_xor(bi, o, WAVE);
+      if (ov > bv || (ov == bv && oi < bi)) {
+        bv = ov;
+        bi = oi;
+      }
+    }
+    if (bi >= E) bi = k;                    // only if the logits are not numbers
+    if (k == 0) z0 = bv;
+    const float ex = expf(bv - z0);
+    sum += ex;
+    if (lane == (bi & 63)) z[bi] = -INFINITY;
+    if (lane == 0) {
+      pick[(size_t)t * top + k] = bi;
+      weight[(size_t)t * top + k] = ex;
+    }
+  }
+  // lane 0 wrote the exponentials and scales them itself
+  if (lane == 0)
+    for (int k = 0; k < top; ++k) weight[(size_t)t * top + k] /= sum;
+}
+
+constexpr int PL_THREADS = 1024;
+constexpr int PL_MAX_E = RT_MAX_E;
+
+// Counting sort of the entries by expert, one workgroup.  The order of an expert's entries among themselves may differ
+// from run to run; nothing depends on it (every row of a tile is computed by itself).
+__global__ __launch_bounds__(PL_THREADS) void moe_plan_kernel(int32_t* __restrict__ perm, int4* __restrict__ tiles, int32_t* __restrict__ n_tiles,
+                                                              const int32_t* __restrict__ pick, int n, int E, int tile_rows) {
+  __shared__ int count[PL_MAX_E], first[PL_MAX_E], tile0[PL_MAX_E];
+  for (int e = threadIdx.x; e < E; e += PL_THREADS) count[e] = 0;
+  __syncthreads();
+  for (int i = threadIdx.x; i < n; i += PL_THREADS) atomicAdd(&count[pick[i]], 1);
+  __syncthreads();
+  if (threadIdx.x < WAVE) {                 // one wave scans, 64 experts at a time
+    const int lane = threadIdx.x;
+    int base = 0, tbase = 0;
+    for (int e0 = 0; e0 < E; e0 += WAVE) {
+      const int c = e0 + lane < E ? count[e0 + lane] : 0;
+      const int nt = (c + tile_rows - 1) / tile_rows;
+      int s = c, ts = nt;
+#pragma unroll
+      for (int o = 1; o < WAVE; o <<= 1) {
+        const int a = __shfl_up(s, o, WAVE), b = __shfl_up(ts, o, WAVE);
+        if (lane >= o) {
+          s += a;
+          ts += b;
+        }
+      }
+      if (e0 + lane < E) {
+        first[e0 + lane] = base + s - c;
+        tile0[e0 + lane] = tbase + ts - nt;
+      }
+      base += __shfl(s, WAVE - 1, WAVE);
+      tbase += __shfl(ts, WAVE - 1, WAVE);
+    }
+    if (lane == 0) *n_tiles = tbase;
+  }
+  __syncthreads();
+  for (int e = threadIdx.x; e < E; e += PL_THREADS) {
+    const int c = count[e];
+    for (int i = 0, k = 0; i < c; i += tile_rows, ++k) tiles[tile0[e] + k] = make_int4(e, first[e] + i, c - i < tile_rows ? c - i : tile_rows, 0);
+    count[e] = 0;
+  }
+  __syncthreads();
+  for (int i = threadIdx.x; i < n; i += PL_THREADS) {
+    const int e = pick[i];
+    perm[first[e] + atomicAdd(&count[e], 1)] = i;
+  }
+}
+
+// x[t, :] += sum_k weight[t, k] * y[t * top + k, :], choices in order
+__global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ x, const elt* __restrict__ y, const float* __restrict__ weight,
+                                                          int top, int N) {
+  const int t = blockIdx.y, c = (blockIdx.x * 256 + threadIdx.x) * 4;
+  if (c >= N) return;
+  f32x4 s = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int k = 0; k < top; ++k) {
+    const float w = weight[(size_t)t * top + k];
+    const eltx4 v = *reinterpret_cast<const eltx4*>(y + ((size_t)t * top + k) * N + c);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) s[e] = fmaf(w, (float)v[e], s[e]);
+  }
+  f32x4* p = reinterpret_cast<f32x4*>(x + (size_t)t * N + c);
+  *p = *p + s;
+}
+
+#ifndef MLORA_ELT_F32
+struct MoeLinear {
+  elt* y;
+  const elt* x;
+  const elt* W;             // packed, one [N, K] block per expert
+  size_t w_elems;
+  int K, N, top, up, act;
+  float alpha;
+};
+
+__device__ __forceinline__ eltx4 moe_out(f32x4 s, const MoeLinear& a) {
+  eltx4 o;
+#pragma unroll
+  for (int q = 0; q < 4; ++q) {
+    float v = s[q] * a.alpha;
+    if (a.act == MLORA_ACT_RELU2) {
+      v = fmaxf(v, 0.f);
+      v = v * v;
+    }
+    o[q] = (elt)v;
+  }
+  return o;
+}
+
+// Tiles of 16 entries (a decode step: a few tokens per expert): the weights are what is read.  A workgroup takes 16 NT rows
+// of one expert, its waves split K, the partial tiles meet in LDS in wave order.
+constexpr int MG_WAVES = 8;
+template <int NT, int PIPE>
+__global__ __launch_bounds__(MG_WAVES* WAVE) void moe_gemv_kernel(MoeLinear a, MoePlan plan) {
+  if ((int)blockIdx.y >= *plan.n_tiles) return;
+  __shared__ f32x4 red[MG_WAVES][NT][WAVE];
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
+  const int4 tile = plan.tiles[blockIdx.y];
+  const int KB = a.K / 32, ntiles = a.N / 16, nt0 = blockIdx.x * NT;
+  const int i16 = lane & 15;
+  const int place = tile.y + (i16 < tile.z ? i16 : tile.z - 1);
+  const int entry = plan.perm[place];
+  const elt* xp = a.x + (size_t)(a.up ? entry / a.top : place) * a.K + (lane >> 4) * 8;
+  const elt* wp = a.W + tile.x * a.w_elems + lane * 8;
+  int woff[NT];
+#pragma unroll
+  for (int i = 0; i < NT; ++i) woff[i] = (nt0 + i < ntiles ? nt0 + i : ntiles - 1) * KB * 512;
+  f32x4 acc[NT];
+#pragma unroll
+  for (int i = 0; i < NT; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  const int S = (KB - wave + MG_WAVES - 1) / MG_WAVES;
+  eltx8 w[PIPE][NT], b[PIPE];
+  auto load = [&](int u, int s) {
+    const int ks = s < S ? wave + MG_WAVES * s : 0;
+#pragma unroll
+    for (int i = 0; i < NT; ++i) w[u][i] = ld8(wp + woff[i] + ks * 512);
+    b[u] = ld8(xp + ks * 32);
+    if (s >= S) b[u] = eltx8{0, 0, 0, 0, 0, 0, 0, 0};     // past this wave's share: valid addresses, no contribution
+  };
+#pragma unroll
+  for (int u = 0; u < PIPE; ++u) load(u, u);
+  for (int s0 = 0; s0 < S; s0 += PIPE)
+#pragma unroll
+    for (int u = 0; u < PIPE; ++u) {
+#pragma unroll
+      for (int i = 0; i < NT; ++i) acc[i] = mfma_16x16x32(w[u][i], b[u], acc[i]);
+      load(u, s0 + u + PIPE);
+    }
+#pragma unroll
+  for (int i = 0; i < NT; ++i) red[wave][i][lane] = acc[i];
+  __syncthreads();
+  for (int e = threadIdx.x; e < NT * WAVE; e += MG_WAVES * WAVE) {
+    const int i = e >> 6, sl = e & 63, row = sl & 15;
+    const int n = (nt0 + i) * 16 + (sl >> 4) * 4;
+    if (row >= tile.z || n >= a.N) continue;
+    f32x4 s = red[0][i][sl];
+#pragma unroll
+    for (int q = 1; q < MG_WAVES; ++q) s += red[q][i][sl];
+    const int p = tile.y + row;
+    *reinterpret_cast<eltx4*>(a.y + (size_t)(a.up ? p : plan.perm[p]) * a.N + n) = moe_out(s, a);
+  }
+}
+
+// Tiles of 128 entries: a wave owns 64 entries x 64 rows, four waves 128 x 128, operands straight into registers, one k-step
+// ahead.  Blocks of one expert's rows are neighbours in the grid.
+constexpr int MM_ROWS = 128;
+__global__ __launch_bounds__(256) void moe_gemm_kernel(MoeLinear a, MoePlan plan) {
+  if ((int)blockIdx.y >= *plan.n_tiles) return;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
+  const int4 tile = plan.tiles[blockIdx.y];
+  const int KB = a.K / 32, ntiles = a.N / 16;
+  const int nt0 = blockIdx.x * 8 + (wave & 1) * 4, r0 = (wave >> 1) * 64;
+  if (nt0 >= ntiles || r0 >= tile.z) return;
+  const int r16 = lane & 15, g = lane >> 4;
+  const elt* xp[4];
+  const elt* wp[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int r = r0 + j * 16 + r16;
+    const int place = tile.y + (r < tile.z ? r : tile.z - 1);
+    xp[j] = a.x + (size_t)(a.up ? plan.perm[place] / a.top : place) * a.K + g * 8;
+    const int nt = nt0 + j < ntiles ? nt0 + j : ntiles - 1;
+    wp[j] = a.W + tile.x * a.w_elems + (size_t)nt * KB * 512 + lane * 8;
+  }
+  f32x4 acc[4][4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+  eltx8 w[4], b[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    w[i] = ld8(wp[i]);
+    b[i] = ld8(xp[i]);
+  }
+  for (int ks = 1; ks <= KB; ++ks) {
+    const int kc = ks < KB ? ks : 0;         // the last prefetch wraps to a valid address and is discarded
+    eltx8 wn[4], bn[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      wn[i] = ld8(wp[i] + (size_t)kc * 512);
+      bn[i] = ld8(xp[i] + kc * 32);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) acc[i][j] = mfma_16x16x32(w[i], b[j], acc[i][j]);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      w[i] = wn[i];
+      b[i] = bn[i];
+    }
+  }
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int r = r0 + j * 16 + r16;
+    if (r >= tile.z) continue;
+    const int p = tile.y + r;
+    elt* yr = a.y + (size_t)(a.up ? p : plan.perm[p]) * a.N;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int n = (nt0 + i) * 16 + g * 4;
+      if (n < a.N) *reinterpret_cast<eltx4*>(yr + n) = moe_out(acc[i][j], a);
+    }
+  }
+}
+#endif
+
+}  // namespace
+
+extern "C" int mlora_moe_route(int32_t* pick, float* weight, const float* logits, int ld, const float* bias, float scale, int T, int E, int top,
+                               void* stream) {
+  MLORA_CHECK(pick && weight && logits && bias, MLORA_ERR_INVALID, "moe_route: null pointer");
+  MLORA_CHECK(T >= 0 && E > 0 && E <= RT_MAX_E && top > 0 && top <= E && ld >= E, MLORA_ERR_UNSUPPORTED,
+              "moe_route: need 0 < top <= experts <= %d (T=%d E=%d top=%d)", RT_MAX_E, T, E, top);
+  if (T == 0) return MLORA_OK;
+  hipLaunchKernelGGL(moe_route_kernel, dim3(ceil_div(T, RT_WAVES)), dim3(RT_WAVES * WAVE), 0, (hipStream_t)stream, pick, weight, logits, ld, bias,
+                     scale, T, E, top);
+  return mlora_launch_status("moe_route");
+}
+
+// rows per expert tile for this many entries (the fp32 build has one size)
+extern "C" int mlora_moe_tile_rows(int T, int E, int top) {
+#ifdef MLORA_ELT_F32
+  return 64;
+#else
+  return E > 0 && (long)T * top > 16L * E ? MM_ROWS : 16;
+#endif
+}
+
+// an upper bound of the tiles of a plan, whatever the routing
+extern "C" int mlora_moe_max_tiles(int T, int E, int top) {
+  if (T <= 0 || E <= 0 || top <= 0) return 0;
+  const long n = (long)T * top;
+  return (int)(n / mlora_moe_tile_rows(T, E, top) + (n < E ? n : E));
+}
+
+extern "C" int mlora_moe_plan(int32_t* perm, int32_t* tiles, int32_t* n_tiles, const int32_t* pick, int T, int E, int top, void* stream) {
+  MLORA_CHECK(perm && tiles && n_tiles && pick && ((uintptr_t)tiles & 15) == 0, MLORA_ERR_INVALID, "moe_plan: null or unaligned pointer");
+  MLORA_CHECK(T > 0 && E > 0 && E <= PL_MAX_E && top > 0 && (long)T * top < 0x7fffffffL, MLORA_ERR_UNSUPPORTED,
+              "moe_plan: need experts <= %d (T=%d E=%d top=%d)", PL_MAX_E, T, E, top);
+  hipLaunchKernelGGL(moe_plan_kernel, dim3(1), dim3(PL_THREADS), 0, (hipStream_t)stream, perm, (int4*)tiles, n_tiles, pick, T * top, E,
+                     mlora_moe_tile_rows(T, E, top));
+  return mlora_launch_status("moe_plan");
+}
+
+extern "C" int mlora_moe_combine(float* x, const void* y, const float* weight, int T, int top, int N, void* stream) {
+  MLORA_CHECK(x && y && weight, MLORA_ERR_INVALID, "moe_combine: null pointer");
+  MLORA_CHECK(T >= 0 && T <= 65535 && top > 0 && N > 0 && N % 4 == 0, MLORA_ERR_UNSUPPORTED, "moe_combine: T=%d top=%d N=%d", T, top, N);
+  if (T == 0) return MLORA_OK;
+  hipLaunchKernelGGL(moe_combine_kernel, dim3(ceil_div(N, 1024), T), dim3(256), 0, (hipStream_t)stream, x, (const elt*)y, weight, top, N);
+  return mlora_launch_status("moe_combine");
+}
+
+#ifndef MLORA_ELT_F32
+extern "C" int mlora_moe_linear(void* y, const void* x, const void* W, const int32_t* perm, const int32_t* tiles, const int32_t* n_tiles,
+                                int tile_rows, int max_tiles, int T, int K, int N, int top, int stage, int act, float alpha, void* stream) {
+  MLORA_CHECK(y && x && W && perm && tiles && n_tiles, MLORA_ERR_INVALID, "moe_linear: null pointer");
+  MLORA_CHECK(T >= 0 && K > 0 && K % 32 == 0 && N > 0 && N % 16 == 0 && top > 0 && max_tiles >= 0 && max_tiles <= 65535 &&
+                  (long)N * K < (1L << 31) && (tile_rows == 16 || tile_rows == MM_ROWS),
+              MLORA_ERR_UNSUPPORTED, "moe_linear: need K %% 32 == 0, N %% 16 == 0 (T=%d K=%d N=%d tiles=%d)", T, K, N, max_tiles);
+  if (T == 0 || max_tiles == 0) return MLORA_OK;
+  MoeLinear a;
+  a.y = (elt*)y; a.x = (const elt*)x; a.W = (const elt*)W; a.w_elems = (size_t)N * K;
+  a.K = K; a.N = N; a.top = top; a.up = stage == MLORA_MOE_UP; a.act = act; a.alpha = alpha;
+  MoePlan p;
+  p.perm = perm; p.tiles = (const int4*)tiles; p.n_tiles = n_tiles;
+  hipStream_t s = (hipStream_t)stream;
+  if (tile_rows == 16) hipLaunchKernelGGL((moe_gemv_kernel<2, 4>), dim3(ceil_div(N, 32), max_tiles), dim3(MG_WAVES * WAVE), 0, s, a, p);
+  else hipLaunchKernelGGL(moe_gemm_kernel, dim3(ceil_div(N, 128), max_tiles), dim3(256), 0, s, a, p);
+  return mlora_launch_status("moe_linear");
+}
+#endif

@@ -10,7 +10,7 @@ constexpr int ROW_THREADS = 256;
 // LoRA expand carried by the RMSNorm launch: resid[t, :] += scaling * B[id_t] . v[t] before the row is normed.
 struct LoraExpandRow {
   LoraVSource src;      // shrink results, one slot (src.v == nullptr: plain RMSNorm)
-  const f16* B;         // [n_ad, H, r]
+  const elt* B;         // [n_ad, H, r]
   const int32_t* ids;
   float scaling;
   int r, n_ad;
@@ -45,8 +45,8 @@ constexpr int NORM_THREADS = 512;
 // residual row in place, and then norms the updated row.
 // With PARTS the K-split partials of the row are added after the expand, in slice order, and the row is stored back.
 template <typename XT, int VPT, bool PARTS = false>
-__global__ __launch_bounds__(NORM_THREADS) void rmsnorm_kernel(f16* __restrict__ y, XT* __restrict__ x,
-                                                               const f16* __restrict__ w, float eps, int H, int frag_tt,
+__global__ __launch_bounds__(NORM_THREADS) void rmsnorm_kernel(elt* __restrict__ y, XT* __restrict__ x,
+                                                               const elt* __restrict__ w, float eps, int H, int frag_tt,
                                                                LoraExpandRow lx, KSplitParts kp) {
   __shared__ float lds[NORM_THREADS / WAVE];
   __shared__ float lv[64];
@@ -60,14 +60,14 @@ __global__ __launch_bounds__(NORM_THREADS) void rmsnorm_kernel(f16* __restrict__
   // The row and the norm weight are requested first: neither depends on the adapter id, so their latency
   // overlaps the id -> (shrink results, B table) chain below.
   float v[VPT][8];
-  f16x8 wv[VPT];
+  eltx8 wv[VPT];
 #pragma unroll
   for (int i = 0; i < VPT; ++i) {
     const int c = (i * NORM_THREADS + threadIdx.x) * 8;
     if (c < H) {
       wv[i] = ld8(w + c);
       if constexpr (sizeof(XT) == 2) {
-        const f16x8 t = ld8((const f16*)xr + c);
+        const eltx8 t = ld8((const elt*)xr + c);
 #pragma unroll
         for (int e = 0; e < 8; ++e) v[i][e] = (float)t[e];
       } else {
@@ -107,18 +107,18 @@ __global__ __launch_bounds__(NORM_THREADS) void rmsnorm_kernel(f16* __restrict__
       const int id = lx.ids[row];
       if (id >= 0 && id < lx.n_ad) {
         has_delta = true;
-        const f16* __restrict__ B = lx.B + (size_t)id * H * lx.r;
+        const elt* __restrict__ B = lx.B + (size_t)id * H * lx.r;
         const int lpr = lx.r >> 3;                  // lanes (16-byte chunks) per output column
         const int chunks = H * lpr;
         // one batch is 16 chunks per thread: all of B[id] for rank 16 and H = 4096, so that the table is requested once,
         // as a whole, right behind the adapter id
         constexpr int NB = VPT == 1 ? 16 : 8;
-        f16x8 bv[NB];
+        eltx8 bv[NB];
         auto load_batch = [&](int q0) {
 #pragma unroll
           for (int u = 0; u < NB; ++u) {
             const int q = q0 + u * NORM_THREADS + threadIdx.x;
-            bv[u] = f16x8{0, 0, 0, 0, 0, 0, 0, 0};
+            bv[u] = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
             if (q < chunks) bv[u] = ld8(B + (size_t)q * 8);
           }
         };
@@ -202,41 +202,39 @@ __global__ __launch_bounds__(NORM_THREADS) void rmsnorm_kernel(f16* __restrict__
   for (int i = 0; i < VPT; ++i) {
     const int c = (i * NORM_THREADS + threadIdx.x) * 8;
     if (c < H) {
-      f16x8 o;
+      eltx8 o;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) o[e] = (f16)(v[i][e] * inv * (float)wv[i][e]);
+      for (int e = 0; e < 8; ++e) o[e] = (elt)(v[i][e] * inv * (float)wv[i][e]);
       st8(y + (frag_tt ? frag_offset(row, c, frag_tt) : (size_t)row * H + c), o);
     }
   }
 }
 
-__global__ __launch_bounds__(ROW_THREADS) void silu_mul_kernel(f16* __restrict__ out, const f16* __restrict__ gate,
-                                                               const f16* __restrict__ up, int ld, int I, int frag_tt) {
+template <int KIND>
+__global__ __launch_bounds__(ROW_THREADS) void glu_mul_kernel(elt* __restrict__ out, const elt* __restrict__ gate,
+                                                              const elt* __restrict__ up, int ld, int I, int frag_tt, GluArgs ga) {
   const int row = blockIdx.y;
   const int c = (blockIdx.x * ROW_THREADS + threadIdx.x) * 8;
   if (c >= I) return;
-  const f16x8 g = ld8(gate + (size_t)row * ld + c);
-  const f16x8 u = ld8(up + (size_t)row * ld + c);
-  f16x8 o;
+  const eltx8 g = ld8(gate + (size_t)row * ld + c);
+  const eltx8 u = ld8(up + (size_t)row * ld + c);
+  eltx8 o;
 #pragma unroll
-  for (int e = 0; e < 8; ++e) {
-    const float gf = (float)g[e];
-    o[e] = (f16)(gf / (1.f + expf(-gf)) * (float)u[e]);
-  }
+  for (int e = 0; e < 8; ++e) o[e] = (elt)glu<KIND>((float)g[e], (float)u[e], ga);
   st8(out + (frag_tt ? frag_offset(row, c, frag_tt) : (size_t)row * I + c), o);
 }
 
 template <typename OT>
-__global__ __launch_bounds__(ROW_THREADS) void embed_kernel(OT* __restrict__ out, const f16* __restrict__ table,
+__global__ __launch_bounds__(ROW_THREADS) void embed_kernel(OT* __restrict__ out, const elt* __restrict__ table,
                                                             const int32_t* __restrict__ ids, int H, int V) {
   const int row = blockIdx.x;
   const int id = ids[row];
   const bool ok = id >= 0 && id < V;
   for (int c = threadIdx.x * 8; c < H; c += ROW_THREADS * 8) {
-    f16x8 t = f16x8{0, 0, 0, 0, 0, 0, 0, 0};
+    eltx8 t = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
     if (ok) t = ld8(table + (size_t)id * H + c);
     if constexpr (sizeof(OT) == 2) {
-      st8((f16*)out + (size_t)row * H + c, t);
+      st8((elt*)out + (size_t)row * H + c, t);
     } else {
       float* o = (float*)out + (size_t)row * H + c;
       *reinterpret_cast<f32x4*>(o) = f32x4{(float)t[0], (float)t[1], (float)t[2], (float)t[3]};
@@ -307,9 +305,9 @@ __global__ __launch_bounds__(AMAX_THREADS) void argmax_kernel(int32_t* __restric
 constexpr int TILE_PITCH = 128 + 8;    // fp16 elements per (k-step, k-group) slot of the staging buffer: 16 rows x 8, padded
 
 template <typename XT, int MC>
-__global__ __launch_bounds__(1024) void rmsnorm_tile_kernel(f16* __restrict__ y, const XT* __restrict__ x, const f16* __restrict__ w,
+__global__ __launch_bounds__(1024) void rmsnorm_tile_kernel(elt* __restrict__ y, const XT* __restrict__ x, const elt* __restrict__ w,
                                                             float eps, int T, int H, int frag_tt) {
-  __shared__ __align__(16) f16 buf[2][64 * TILE_PITCH];
+  __shared__ __align__(16) elt buf[2][64 * TILE_PITCH];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int tt = blockIdx.x, row = tt * 16 + wave;
   const bool live = row < T;
@@ -326,7 +324,7 @@ __global__ __launch_bounds__(1024) void rmsnorm_tile_kernel(f16* __restrict__ y,
     for (int e = 0; e < 8; ++e) v[m][e] = 0.f;
     if (live && c < H) {
       if constexpr (sizeof(XT) == 2) {
-        const f16x8 t = ld8((const f16*)xr + c);
+        const eltx8 t = ld8((const elt*)xr + c);
 #pragma unroll
         for (int e = 0; e < 8; ++e) v[m][e] = (float)t[e];
       } else {
@@ -350,13 +348,13 @@ __global__ __launch_bounds__(1024) void rmsnorm_tile_kernel(f16* __restrict__ y,
   for (int m = 0; m < MC; ++m) {
     if (m < M) {                                       // uniform
       const int c = m * 512 + lane * 8;
-      f16x8 o = f16x8{0, 0, 0, 0, 0, 0, 0, 0};
+      eltx8 o = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
       if (c < H) {
-        const f16x8 wv = ld8(w + c);
+        const eltx8 wv = ld8(w + c);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) o[e] = (f16)(v[m][e] * inv * (float)wv[e]);
+        for (int e = 0; e < 8; ++e) o[e] = (elt)(v[m][e] * inv * (float)wv[e]);
       }
-      f16* b = buf[m & 1];
+      elt* b = buf[m & 1];
       st8(b + lane * TILE_PITCH + wave * 8, o);        // slot = (k-step within the block) * 4 + k-group = lane
       __syncthreads();
       const int ks = m * 16 + wave;                    // this wave's fragment of the block
@@ -365,25 +363,23 @@ __global__ __launch_bounds__(1024) void rmsnorm_tile_kernel(f16* __restrict__ y,
   }
 }
 
-// SiLU(gate) * up of a token block of prefill size into fragment order: a wave produces one whole fragment (16 tokens x
+// act(gate) * up of a token block of prefill size into fragment order: a wave produces one whole fragment (16 tokens x
 // 32 columns, 1 KiB contiguous), the four waves of a workgroup four neighbouring k-steps, so that the rows are read in
 // runs of 256 bytes.
-__global__ __launch_bounds__(ROW_THREADS) void silu_mul_tile_kernel(f16* __restrict__ out, const f16* __restrict__ gate,
-                                                                    const f16* __restrict__ up, int ld, int T, int I, int frag_tt) {
+template <int KIND>
+__global__ __launch_bounds__(ROW_THREADS) void glu_mul_tile_kernel(elt* __restrict__ out, const elt* __restrict__ gate,
+                                                                   const elt* __restrict__ up, int ld, int T, int I, int frag_tt, GluArgs ga) {
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int tt = blockIdx.y, ks = blockIdx.x * (ROW_THREADS / WAVE) + wave;
   const int c = ks * 32 + (lane >> 4) * 8;
   if (c >= I) return;
   const int t = tt * 16 + (lane & 15);
-  f16x8 o = f16x8{0, 0, 0, 0, 0, 0, 0, 0};
+  eltx8 o = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
   if (t < T) {
-    const f16x8 g = ld8(gate + (size_t)t * ld + c);
-    const f16x8 u = ld8(up + (size_t)t * ld + c);
+    const eltx8 g = ld8(gate + (size_t)t * ld + c);
+    const eltx8 u = ld8(up + (size_t)t * ld + c);
 #pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      const float gf = (float)g[e];
-      o[e] = (f16)(gf / (1.f + expf(-gf)) * (float)u[e]);
-    }
+    for (int e = 0; e < 8; ++e) o[e] = (elt)glu<KIND>((float)g[e], (float)u[e], ga);
   }
   st8(out + ((size_t)ks * frag_tt + tt) * 512 + lane * 8, o);
 }
@@ -402,11 +398,11 @@ static int rmsnorm_impl(const char* who, void* y, int y_layout, void* x, int x_d
   hipStream_t s = (hipStream_t)stream;
   if (frag_tt && T > 64 && H <= 4096 && lx.src.v == nullptr && kp.n == 0) {      // a prefill-sized block: whole fragments per store
 #define MLORA_RMS_TILE(XT, MC) \
-  hipLaunchKernelGGL((rmsnorm_tile_kernel<XT, MC>), dim3(frag_tt), dim3(1024), 0, s, (f16*)y, (const XT*)x, (const f16*)w, eps, T, H, frag_tt)
+  hipLaunchKernelGGL((rmsnorm_tile_kernel<XT, MC>), dim3(frag_tt), dim3(1024), 0, s, (elt*)y, (const XT*)x, (const elt*)w, eps, T, H, frag_tt)
     if (x_dtype == MLORA_F16) {
-      if (H <= 1024) MLORA_RMS_TILE(f16, 2);
-      else if (H <= 2048) MLORA_RMS_TILE(f16, 4);
-      else MLORA_RMS_TILE(f16, 8);
+      if (H <= 1024) MLORA_RMS_TILE(elt, 2);
+      else if (H <= 2048) MLORA_RMS_TILE(elt, 4);
+      else MLORA_RMS_TILE(elt, 8);
     } else {
       if (H <= 1024) MLORA_RMS_TILE(float, 2);
       else if (H <= 2048) MLORA_RMS_TILE(float, 4);
@@ -418,16 +414,16 @@ static int rmsnorm_impl(const char* who, void* y, int y_layout, void* x, int x_d
   const int vpt = ceil_div(H, NORM_THREADS * 8);
   const size_t dyn = lx.src.v ? (size_t)H * sizeof(float) : 0;   // LDS staging of the expand deltas
 #define MLORA_RMS(XT, VPT) \
-  hipLaunchKernelGGL((rmsnorm_kernel<XT, VPT>), dim3(T), dim3(NORM_THREADS), dyn, s, (f16*)y, (XT*)x, (const f16*)w, eps, H, frag_tt, lx, kp)
+  hipLaunchKernelGGL((rmsnorm_kernel<XT, VPT>), dim3(T), dim3(NORM_THREADS), dyn, s, (elt*)y, (XT*)x, (const elt*)w, eps, H, frag_tt, lx, kp)
   if (kp.n > 0) {
     MLORA_CHECK(x_dtype == MLORA_F32 && vpt <= 2 && kp.n <= MAX_PARTS && kp.p, MLORA_ERR_UNSUPPORTED,
                 "%s: K-split partials need an fp32 row, H <= 8192 and at most %d partial blocks (H=%d n=%d)", who, H, MAX_PARTS, kp.n);
-    if (vpt <= 1) hipLaunchKernelGGL((rmsnorm_kernel<float, 1, true>), dim3(T), dim3(NORM_THREADS), dyn, s, (f16*)y, (float*)x, (const f16*)w, eps, H, frag_tt, lx, kp);
-    else hipLaunchKernelGGL((rmsnorm_kernel<float, 2, true>), dim3(T), dim3(NORM_THREADS), dyn, s, (f16*)y, (float*)x, (const f16*)w, eps, H, frag_tt, lx, kp);
+    if (vpt <= 1) hipLaunchKernelGGL((rmsnorm_kernel<float, 1, true>), dim3(T), dim3(NORM_THREADS), dyn, s, (elt*)y, (float*)x, (const elt*)w, eps, H, frag_tt, lx, kp);
+    else hipLaunchKernelGGL((rmsnorm_kernel<float, 2, true>), dim3(T), dim3(NORM_THREADS), dyn, s, (elt*)y, (float*)x, (const elt*)w, eps, H, frag_tt, lx, kp);
   } else if (x_dtype == MLORA_F16) {
-    if (vpt <= 1) MLORA_RMS(f16, 1);
-    else if (vpt <= 2) MLORA_RMS(f16, 2);
-    else MLORA_RMS(f16, 4);
+    if (vpt <= 1) MLORA_RMS(elt, 1);
+    else if (vpt <= 2) MLORA_RMS(elt, 2);
+    else MLORA_RMS(elt, 4);
   } else {
     if (vpt <= 1) MLORA_RMS(float, 1);
     else if (vpt <= 2) MLORA_RMS(float, 2);
@@ -453,7 +449,7 @@ extern "C" int mlora_lora_expand_rmsnorm(void* y, int y_layout, float* resid, co
   lx.src.kc = v_dense ? 0 : lora_k_split(K).kc;
   lx.src.kq = 1;
   lx.src.T = T; lx.src.n_ad = n_ad; lx.src.ld = n_ad * r;
-  lx.B = (const f16*)B;
+  lx.B = (const elt*)B;
   lx.ids = tok_adapter;
   lx.scaling = scaling;
   lx.r = r; lx.n_ad = n_ad;
@@ -476,7 +472,7 @@ extern "C" int mlora_rmsnorm_ksplit(void* y, int y_layout, float* resid, const f
     lx.src.kc = v_dense ? 0 : lora_k_split(K).kc;
     lx.src.kq = 1;
     lx.src.T = T; lx.src.n_ad = n_ad; lx.src.ld = n_ad * r;
-    lx.B = (const f16*)B;
+    lx.B = (const elt*)B;
     lx.ids = tok_adapter;
     lx.scaling = scaling;
     lx.r = r; lx.n_ad = n_ad;
@@ -488,23 +484,33 @@ extern "C" int mlora_rmsnorm_ksplit(void* y, int y_layout, float* resid, const f
   return rmsnorm_impl("rmsnorm_ksplit", y, y_layout, resid, MLORA_F32, w, eps, T, H, lx, stream, kp);
 }
 
-extern "C" int mlora_silu_mul(void* out, int out_layout, const void* gate, const void* up, int ld, int T, int I,
-                              void* stream) {
+template <int KIND>
+static int glu_mul(const char* who, void* out, int out_layout, const void* gate, const void* up, int ld, int T, int I, const GluArgs& ga,
+                   void* stream) {
   MLORA_CHECK(out_layout == MLORA_ROWMAJOR || (out_layout == MLORA_FRAG && I % 32 == 0), MLORA_ERR_UNSUPPORTED,
-              "silu_mul: fragment-ordered output needs I %% 32 == 0 (layout=%d I=%d)", out_layout, I);
+              "%s: fragment-ordered output needs I %% 32 == 0 (layout=%d I=%d)", who, out_layout, I);
   const int frag_tt = out_layout == MLORA_FRAG ? mlora_frag_tiles(T) : 0;
-  MLORA_CHECK(out && gate && up, MLORA_ERR_INVALID, "silu_mul: null pointer");
-  MLORA_CHECK(T >= 0 && I > 0 && I % 8 == 0 && ld >= I && ld % 8 == 0, MLORA_ERR_UNSUPPORTED, "silu_mul: need I %% 8 == 0, ld >= I, ld %% 8 == 0 (T=%d I=%d ld=%d)", T, I, ld);
-  MLORA_CHECK(T <= 65535, MLORA_ERR_UNSUPPORTED, "silu_mul: T=%d exceeds 65535", T);
+  MLORA_CHECK(out && gate && up, MLORA_ERR_INVALID, "%s: null pointer", who);
+  MLORA_CHECK(T >= 0 && I > 0 && I % 8 == 0 && ld >= I && ld % 8 == 0, MLORA_ERR_UNSUPPORTED, "%s: need I %% 8 == 0, ld >= I, ld %% 8 == 0 (T=%d I=%d ld=%d)", who, T, I, ld);
+  MLORA_CHECK(T <= 65535, MLORA_ERR_UNSUPPORTED, "%s: T=%d exceeds 65535", who, T);
   if (T == 0) return MLORA_OK;
   if (frag_tt && T > 64) {
-    hipLaunchKernelGGL(silu_mul_tile_kernel, dim3(ceil_div(I, 32 * (ROW_THREADS / WAVE)), frag_tt), dim3(ROW_THREADS), 0,
-                       (hipStream_t)stream, (f16*)out, (const f16*)gate, (const f16*)up, ld, T, I, frag_tt);
-    return mlora_launch_status("silu_mul");
+    hipLaunchKernelGGL(glu_mul_tile_kernel<KIND>, dim3(ceil_div(I, 32 * (ROW_THREADS / WAVE)), frag_tt), dim3(ROW_THREADS), 0,
+                       (hipStream_t)stream, (elt*)out, (const elt*)gate, (const elt*)up, ld, T, I, frag_tt, ga);
+    return mlora_launch_status(who);
   }
-  hipLaunchKernelGGL(silu_mul_kernel, dim3(ceil_div(I, ROW_THREADS * 8), T), dim3(ROW_THREADS), 0, (hipStream_t)stream,
-                     (f16*)out, (const f16*)gate, (const f16*)up, ld, I, frag_tt);
-  return mlora_launch_status("silu_mul");
+  hipLaunchKernelGGL(glu_mul_kernel<KIND>, dim3(ceil_div(I, ROW_THREADS * 8), T), dim3(ROW_THREADS), 0, (hipStream_t)stream,
+                     (elt*)out, (const elt*)gate, (const elt*)up, ld, I, frag_tt, ga);
+  return mlora_launch_status(who);
+}
+
+extern "C" int mlora_silu_mul(void* out, int out_layout, const void* gate, const void* up, int ld, int T, int I, void* stream) {
+  return glu_mul<MLORA_GLU_SILU>("silu_mul", out, out_layout, gate, up, ld, T, I, GluArgs(), stream);
+}
+
+extern "C" int mlora_clipglu_mul(void* out, int out_layout, const void* gate, const void* up, int ld, int T, int I, float scale, float limit,
+                                 float alpha, void* stream) {
+  return glu_mul<MLORA_GLU_CLIPPED>("clipglu_mul", out, out_layout, gate, up, ld, T, I, GluArgs{scale, limit, alpha}, stream);
 }
 
 extern "C" int mlora_embed(void* out, int out_dtype, const void* table, const int32_t* ids, int T, int H, int V, void* stream) {
@@ -513,8 +519,8 @@ extern "C" int mlora_embed(void* out, int out_dtype, const void* table, const in
   MLORA_CHECK(out_dtype == MLORA_F16 || out_dtype == MLORA_F32, MLORA_ERR_INVALID, "embed: bad out_dtype %d", out_dtype);
   if (T == 0) return MLORA_OK;
   hipStream_t s = (hipStream_t)stream;
-  if (out_dtype == MLORA_F16) hipLaunchKernelGGL(embed_kernel<f16>, dim3(T), dim3(ROW_THREADS), 0, s, (f16*)out, (const f16*)table, ids, H, V);
-  else hipLaunchKernelGGL(embed_kernel<float>, dim3(T), dim3(ROW_THREADS), 0, s, (float*)out, (const f16*)table, ids, H, V);
+  if (out_dtype == MLORA_F16) hipLaunchKernelGGL(embed_kernel<elt>, dim3(T), dim3(ROW_THREADS), 0, s, (elt*)out, (const elt*)table, ids, H, V);
+  else hipLaunchKernelGGL(embed_kernel<float>, dim3(T), dim3(ROW_THREADS), 0, s, (float*)out, (const elt*)table, ids, H, V);
   return mlora_launch_status("embed");
 }
 

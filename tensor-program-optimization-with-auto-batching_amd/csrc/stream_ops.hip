@@ -1,0 +1,233 @@
+// Row operators of decoders whose fp32 residual stream is normed by one number and carries a per-layer token input.
+// Compiled for every element type.
+#include "common.h"
+
+namespace {
+
+constexpr int SN_THREADS = 256;
+
+__device__ __forceinline__ float sn_block_sum(float v, float* lds) {
+  v = wave_sum(v);
+  if ((threadIdx.x & 63) == 0) lds[threadIdx.x >> 6] = v;
+  __syncthreads();
+  float s = 0.f;
+#pragma unroll
+  for (int w = 0; w < SN_THREADS / WAVE; ++w) s += lds[w];
+  return s;
+}
+
+struct StreamNorm {
+  float* x;               // [T, Hp] residual stream, columns H..Hp-1 zero
+  int H, Hp;
+  float eps, gain;
+  const float* part;      // n_part blocks [T, Hp] of partial sums still to be added to x, in order
+  int n_part;
+  size_t part_stride;
+  const float* y;         // [T, Hp] branch: x += y / rms(y) * yw
+  const elt* yw;          // [Hp]
+  elt* out_frag;          // the normed row in fragment order (16-bit element types) ...
+  int frag_tt;
+  elt* out_row;           // ... and / or row-major [T, Hp]
+};
+
+// x += parts; x += y / rms(y) * yw; out = x / rms(x) * gain.  One workgroup per row, the row in registers.
+template <int VPT>
+__global__ __launch_bounds__(SN_THREADS) void stream_norm_kernel(StreamNorm a) {
+  __shared__ float lds[2][SN_THREADS / WAVE];
+  const int row = blockIdx.x;
+  float* xr = a.x + (size_t)row * a.Hp;
+  f32x4 v[VPT];
+#pragma unroll
+  for (int i = 0; i < VPT; ++i) {
+    const int c = (threadIdx.x + i * SN_THREADS) * 4;
+    v[i] = c < a.Hp ? *reinterpret_cast<const f32x4*>(xr + c) : f32x4{0.f, 0.f, 0.f, 0.f};
+  }
+  for (int q = 0; q < a.n_part; ++q) {
+    const float* pr = a.part + q * a.part_stride + (size_t)row * a.Hp;
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+      const int c = (threadIdx.x + i * SN_THREADS) * 4;
+      if (c < a.Hp) v[i] += *reinterpret_cast<const f32x4*>(pr + c);
+    }
+  }
+  if (a.y) {
+    const float* yr = a.y + (size_t)row * a.Hp;
+    f32x4 b[VPT];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+      const int c = (threadIdx.x + i * SN_THREADS) * 4;
+      b[i] = c < a.Hp ? *reinterpret_cast<const f32x4*>(yr + c) : f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int e = 0; e < 4; ++e) ss = fmaf(b[i][e], b[i][e], ss);
+    }
+    const float inv = 1.f / sqrtf(sn_block_sum(ss, lds[0]) / (float)a.H + a.eps);
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+      const int c = (threadIdx.x + i * SN_THREADS) * 4;
+      if (c < a.Hp) {
+        const eltx4 w = *reinterpret_cast<const eltx4*>(a.yw + c);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[i][e] += b[i][e] * inv * (float)w[e];
+      }
+    }
+  }
+  if (a.y || a.n_part) {
+#pragma unroll
+    for (int i = 0; i < VPT; ++i) {
+      const int c = (threadIdx.x + i * SN_THREADS) * 4;
+      if (c < a.Hp) *reinterpret_cast<f32x4*>(xr + c) = v[i];
+    }
+  }
+  if (!a.out_frag && !a.out_row) return;
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < VPT; ++i)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ss = fmaf(v[i][e], v[i][e], ss);
+  const float s = a.gain / sqrtf(sn_block_sum(ss, lds[1]) / (float)a.H + a.eps);
+#pragma unroll
+  for (int i = 0; i < VPT; ++i) {
+    const int c = (threadIdx.x + i * SN_THREADS) * 4;
+    if (c >= a.Hp) continue;
+    eltx4 o;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) o[e] = (elt)(v[i][e] * s);
+    if (a.out_frag) *reinterpret_cast<eltx4*>(a.out_frag + frag_offset(row, c, a.frag_tt)) = o;
+    if (a.out_row) *reinterpret_cast<eltx4*>(a.out_row + (size_t)row * a.Hp + c) = o;
+  }
+}
+
+__device__ __forceinline__ float gelu_tanh(float z) {
+  return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+}
+
+#ifndef MLORA_ELT_F32
+constexpr int TG_WAVES = 8;
+// out[t, n] = gelu(sum_k W[n, k] x[t, k]) * table[id_t, col0 + n] for n < dim, 0 for the padding rows, in fragment order.
+// x is the fp32 residual stream with its pending partial sums, rounded to the element type on the way into the matrix
+// cores.  A workgroup takes 16 tokens x 16 NT rows, its waves split K.
+template <int NT>
+__global__ __launch_bounds__(TG_WAVES* WAVE) void token_gate_kernel(elt* __restrict__ out, int frag_tt, const float* __restrict__ x,
+                                                                   const float* __restrict__ part, int n_part, size_t part_stride,
+                                                                   const elt* __restrict__ Wp, const elt* __restrict__ table, int ld_table,
+                                                                   int col0, int dim, const int32_t* __restrict__ ids, int V, int T, int K, int N) {
+  __shared__ f32x4 red[TG_WAVES][NT][WAVE];
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
+  const int KB = K / 32, tiles = N / 16;
+  const int nt0 = blockIdx.x * NT, t0 = blockIdx.y * 16;
+  int t = t0 + (lane & 15);
+  t = t < T ? t : T - 1;
+  const size_t xo = (size_t)t * K + (lane >> 4) * 8;
+  f32x4 acc[NT];
+#pragma unroll
+  for (int i = 0; i < NT; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int ks = wave; ks < KB; ks += TG_WAVES) {
+    eltx8 a[NT];
+#pragma unroll
+    for (int i = 0; i < NT; ++i) {
+      const int nt = nt0 + i < tiles ? nt0 + i : tiles - 1;
+      a[i] = ld8(Wp + ((size_t)nt * KB + ks) * 512 + lane * 8);
+    }
+    f32x4 lo = *reinterpret_cast<const f32x4*>(x + xo + ks * 32), hi = *reinterpret_cast<const f32x4*>(x + xo + ks * 32 + 4);
+    for (int q = 0; q < n_part; ++q) {
+      const float* p = part + q * part_stride + xo + ks * 32;
+      lo += *reinterpret_cast<const f32x4*>(p);
+      hi += *reinterpret_cast<const f32x4*>(p + 4);
+    }
+    eltx8 b;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      b[e] = (elt)lo[e];
+      b[4 + e] = (elt)hi[e];
+    }
+#pragma unroll
+    for (int i = 0; i < NT; ++i) acc[i] = mfma_16x16x32(a[i], b, acc[i]);
+  }
+#pragma unroll
+  for (int i = 0; i < NT; ++i) red[wave][i][lane] = acc[i];
+  __syncthreads();
+  for (int e = threadIdx.x; e < NT * WAVE; e += TG_WAVES * WAVE) {
+    const int i = e >> 6, sl = e & 63;
+    const int tt = t0 + (sl & 15), n = (nt0 + i) * 16 + (sl >> 4) * 4;
+    if (tt >= T || n >= N) continue;
+    f32x4 s = red[0][i][sl];
+#pragma unroll
+    for (int w = 1; w < TG_WAVES; ++w) s += red[w][i][sl];
+    const int id = ids[tt];
+    const bool ok = id >= 0 && id < V;
+    eltx4 o;
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      const float ev = ok && n + q < dim ? (float)table[(size_t)id * ld_table + col0 + n + q] : 0.f;
+      o[q] = (elt)(gelu_tanh(s[q]) * ev);
+    }
+    *reinterpret_cast<eltx4*>(out + frag_offset(tt, n, frag_tt)) = o;
+  }
+}
+#endif
+
+// the same product behind a separate linear: out[t, n] = gelu(z[t, n]) * table[id_t, col0 + n], row-major
+__global__ __launch_bounds__(256) void token_gate_mul_kernel(elt* __restrict__ out, const elt* __restrict__ z, const elt* __restrict__ table,
+                                                             int ld_table, int col0, int dim, const int32_t* __restrict__ ids, int V, int T, int N) {
+  const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+  if (i >= (size_t)T * N) return;
+  const int t = (int)(i / N), n = (int)(i % N);
+  const int id = ids[t];
+  const float ev = id >= 0 && id < V && n < dim ? (float)table[(size_t)id * ld_table + col0 + n] : 0.f;
+  out[i] = (elt)(gelu_tanh((float)z[i]) * ev);
+}
+
+}  // namespace
+
+extern "C" int mlora_stream_norm(void* out_frag, void* out_row, float* x, const float* part, int n_part, const float* branch,
+                                 const void* branch_w, float eps, float gain, int T, int H, int Hp, void* stream) {
+  MLORA_CHECK(x && T >= 0 && H > 0 && Hp >= H && Hp % 32 == 0 && Hp <= 16384, MLORA_ERR_UNSUPPORTED,
+              "stream_norm: need 0 < H <= Hp <= 16384, Hp %% 32 == 0 (T=%d H=%d Hp=%d)", T, H, Hp);
+  MLORA_CHECK((n_part == 0 || part) && n_part >= 0 && (!branch || branch_w), MLORA_ERR_INVALID, "stream_norm: null pointer");
+  MLORA_CHECK(!out_frag || sizeof(elt) == 2, MLORA_ERR_UNSUPPORTED, "stream_norm: fragment order is for 16-bit elements");
+  if (T == 0) return MLORA_OK;
+  StreamNorm a;
+  a.x = x; a.H = H; a.Hp = Hp; a.eps = eps; a.gain = gain;
+  a.part = part; a.n_part = n_part; a.part_stride = (size_t)T * Hp;
+  a.y = branch; a.yw = (const elt*)branch_w;
+  a.out_frag = (elt*)out_frag; a.frag_tt = mlora_frag_tiles(T); a.out_row = (elt*)out_row;
+  hipStream_t s = (hipStream_t)stream;
+  if (Hp <= 2048) hipLaunchKernelGGL(stream_norm_kernel<2>, dim3(T), dim3(SN_THREADS), 0, s, a);
+  else if (Hp <= 4096) hipLaunchKernelGGL(stream_norm_kernel<4>, dim3(T), dim3(SN_THREADS), 0, s, a);
+  else if (Hp <= 8192) hipLaunchKernelGGL(stream_norm_kernel<8>, dim3(T), dim3(SN_THREADS), 0, s, a);
+  else hipLaunchKernelGGL(stream_norm_kernel<16>, dim3(T), dim3(SN_THREADS), 0, s, a);
+  return mlora_launch_status("stream_norm");
+}
+
+#ifndef MLORA_ELT_F32
+extern "C" int mlora_token_gate(void* out_frag, const float* x, const float* part, int n_part, const void* Wp, const void* table,
+                                int ld_table, int col0, int dim, const int32_t* ids, int V, int T, int K, int N, void* stream) {
+  MLORA_CHECK(out_frag && x && Wp && table && ids && (n_part == 0 || part), MLORA_ERR_INVALID, "token_gate: null pointer");
+  MLORA_CHECK(T >= 0 && K > 0 && K % 32 == 0 && N > 0 && N % 32 == 0 && dim > 0 && dim <= N && col0 >= 0 && col0 + dim <= ld_table && V > 0 &&
+                  ceil_div(T, 16) <= 65535,
+              MLORA_ERR_UNSUPPORTED, "token_gate: need K %% 32 == 0, N %% 32 == 0, dim <= N (T=%d K=%d N=%d dim=%d)", T, K, N, dim);
+  if (T == 0) return MLORA_OK;
+  hipStream_t s = (hipStream_t)stream;
+  const size_t ps = (size_t)T * K;
+#define MLORA_TG(NT)                                                                                                                     \
+  hipLaunchKernelGGL(token_gate_kernel<NT>, dim3(ceil_div(N, 16 * NT), ceil_div(T, 16)), dim3(TG_WAVES * WAVE), 0, s, (elt*)out_frag,    \
+                     mlora_frag_tiles(T), x, part, n_part, ps, (const elt*)Wp, (const elt*)table, ld_table, col0, dim, ids, V, T, K, N)
+  if (T <= 256) MLORA_TG(1);
+  else if (N <= 32) MLORA_TG(2);
+  else MLORA_TG(4);
+#undef MLORA_TG
+  return mlora_launch_status("token_gate");
+}
+#endif
+
+extern "C" int mlora_token_gate_mul(void* out, const void* z, const void* table, int ld_table, int col0, int dim, const int32_t* ids, int V,
+                                    int T, int N, void* stream) {
+  MLORA_CHECK(out && z && table && ids, MLORA_ERR_INVALID, "token_gate_mul: null pointer");
+  MLORA_CHECK(T >= 0 && N > 0 && dim > 0 && dim <= N && col0 >= 0 && col0 + dim <= ld_table && V > 0 && (size_t)T * N / 256 < 0x7fffffffULL,
+              MLORA_ERR_UNSUPPORTED, "token_gate_mul: bad shape T=%d N=%d dim=%d", T, N, dim);
+  if (T == 0) return MLORA_OK;
+  hipLaunchKernelGGL(token_gate_mul_kernel, dim3((unsigned)(((size_t)T * N + 255) / 256)), dim3(256), 0, (hipStream_t)stream, (elt*)out,
+                     (const elt*)z, (const elt*)table, ld_table, col0, dim, ids, V, T, N);
+  return mlora_launch_status("token_gate_mul");
+}

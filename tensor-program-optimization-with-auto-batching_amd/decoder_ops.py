@@ -1,0 +1,180 @@
+"""Operators of include/mlora_decoder.h, and the choice of layout that goes with an element type: bfloat16 works on
+fragment-ordered activations and packed weights, fp32 on plain row-major tensors.  No CPU path.
+"""
+from __future__ import annotations
+
+import torch
+
+from . import ops
+from ._lib import ACT_NONE, ACT_RELU2, FRAG, MOE_DOWN, MOE_UP, ROWMAJOR   # noqa: F401
+from .ops import FragActivation, PackedWeight, _dev, _stream, check, lib_of
+
+
+def pad32(n: int) -> int:
+    return -(-n // 32) * 32
+
+
+def padded(w: torch.Tensor, *shape) -> torch.Tensor:
+    """`w` with zeros behind its rows / columns up to `shape`."""
+    if tuple(w.shape) == tuple(shape):
+        return w
+    out = torch.zeros(shape, dtype=w.dtype, device=w.device)
+    out[tuple(slice(0, n) for n in w.shape)] = w
+    return out
+
+
+def weight(w: torch.Tensor):
+    """A linear weight [N, K] (K % 32 == 0) in the form the linears of its type take."""
+    return w.contiguous() if w.dtype == torch.float32 else PackedWeight(w.contiguous())
+
+
+def activation(T: int, K: int, dtype, device):
+    """An activation block [T, K] in the order the linears of its type read."""
+    if dtype == torch.float32:
+        return torch.empty((T, K), dtype=dtype, device=device)
+    return FragActivation(T, K, device, dtype=dtype)
+
+
+def _wptr(w) -> int:
+    return w.data.data_ptr() if isinstance(w, PackedWeight) else _dev(w)
+
+
+def _ptr(t) -> int:
+    return None if t is None else t.data_ptr()
+
+
+def stream_norm(x, H, eps, gain=1.0, parts=None, branch=None, out=None, out_row=None):
+    """x [T, Hp] fp32 (+= pending K-split partials, += branch[0] / rms * branch[1], in place); out (FragActivation) and / or
+    out_row [T, Hp] = x / rms(x) * gain.  H: columns that count."""
+    if out is None and out_row is None and parts is None and branch is None:
+        return
+    T, Hp = x.shape
+    dt = out.dtype if out is not None else out_row.dtype if out_row is not None else branch[1].dtype if branch is not None else torch.bfloat16
+    check(lib_of(dt).mlora_stream_norm(out.data.data_ptr() if out is not None else None, _ptr(out_row), _dev(x, torch.float32),
+                                       _ptr(parts.part) if parts is not None else None, parts.ks - 1 if parts is not None else 0,
+                                       _ptr(branch[0]) if branch is not None else None, _ptr(branch[1]) if branch is not None else None,
+                                       float(eps), float(gain), T, H, Hp, _stream()), dt)
+
+
+def token_gate(x, W, table, col0, dim, ids, parts=None):
+    """gelu_tanh(W x) * table[ids, col0 : col0 + dim] (x: residual stream [T, Hp] fp32 with pending partials) as the
+    activation of the following linear, its width W's padded row count."""
+    T, Hp = x.shape
+    N, K = W.shape
+    V, ld = table.shape
+    if K != Hp or ids.shape != (T,):
+        raise ValueError(f"token_gate: x{tuple(x.shape)} W{tuple(W.shape)} ids{tuple(ids.shape)}")
+    out = activation(T, N, W.dtype, x.device)
+    L = lib_of(W.dtype)
+    if W.dtype == torch.float32:
+        z = ops.linear(x, W)
+        check(L.mlora_token_gate_mul(_dev(out), _dev(z), _dev(table, W.dtype), ld, col0, dim, _dev(ids, torch.int32), V, T, N, _stream()), W.dtype)
+        return out
+    check(L.mlora_token_gate(out.data.data_ptr(), _dev(x, torch.float32), _ptr(parts.part) if parts is not None else None,
+                             parts.ks - 1 if parts is not None else 0, _wptr(W), _dev(table, W.dtype), ld, col0, dim, _dev(ids, torch.int32),
+                             V, T, K, N, _stream()), W.dtype)
+    return out
+
+
+def clipglu_mul(gate_up, scale, limit, alpha, out):
+    """The clipped gated product of gate_up [T, 2I] (gate columns first) into `out` (activation [T, I])."""
+    T, I2 = gate_up.shape
+    dt = gate_up.dtype
+    frag = isinstance(out, FragActivation)
+    p = _dev(gate_up)
+    check(lib_of(dt).mlora_clipglu_mul(out.data.data_ptr() if frag else _dev(out), FRAG if frag else ROWMAJOR, p,
+                                       p + I2 // 2 * gate_up.element_size(), I2, T, I2 // 2, scale, limit, alpha, _stream()), dt)
+    return out
+
+
+def gate_up_clipglu(x, W, W_il, scale, limit, alpha, out):
+    """clipped gated product of x @ W.T (W [2I, K], gate rows first; W_il: its tiles interleaved) into `out` - the product as
+    the epilogue of the linear where a kernel has that, else behind it."""
+    T, K = x.shape
+    I2 = W.shape[0]
+    if isinstance(x, FragActivation):
+        L = lib_of(x.dtype)
+        args = (T, K, I2 // 2, scale, limit, alpha, _stream())
+        if T <= 64:
+            check(L.mlora_gemv_frag_clipglu(out.data.data_ptr(), x.data.data_ptr(), W_il.data.data_ptr(), *args), x.dtype)
+            return out
+        if L.mlora_gemm_frag_preferred(T, K, I2):
+            check(L.mlora_linear_frag_clipglu(out.data.data_ptr(), x.data.data_ptr(), W.data.data_ptr(), *args), x.dtype)
+            return out
+    return clipglu_mul(ops.linear(x, W), scale, limit, alpha, out)
+
+
+def head_linear(x, ldx, head_x, W, heads, T, K, N, out, ldy, head_y, alpha=1.0):
+    """out[t, h] = alpha * W[h] x[t, h]: x a tensor with row stride ldx and head stride head_x (elements), W the heads'
+    [N, K] matrices stacked, out likewise or a FragActivation [T, heads * head_y]."""
+    dt = x.dtype
+    frag = isinstance(out, FragActivation)
+    check(lib_of(dt).mlora_head_linear(out.data.data_ptr() if frag else out.data_ptr(), FRAG if frag else ROWMAJOR, ldy, head_y, x.data_ptr(),
+                                       ldx, head_x, _wptr(W), heads, T, K, N, alpha, _stream()), dt)
+    return out
+
+
+def latent_prep(q, pages, qkv, off_rot, off_c, off_kr, gain, c_norm, eps, block_table, tok_seq, tok_pos, cos, sin, H, R, rot):
+    n_seq, max_blocks = block_table.shape
+    T, ld = qkv.shape
+    check(lib_of(qkv.dtype).mlora_latent_prep(_dev(q, qkv.dtype), _dev(pages, qkv.dtype), _dev(qkv), ld, off_rot, off_c, off_kr, gain, _ptr(c_norm),
+                                              eps, _dev(block_table, torch.int32), max_blocks, _dev(tok_seq, torch.int32),
+                                              _dev(tok_pos, torch.int32), _dev(cos, torch.float32), _dev(sin, torch.float32), cos.shape[0], T, H, R,
+                                              rot, pages.shape[0], n_seq, _stream()), qkv.dtype)
+
+
+def latent_attn(q, pages, block_table, tok_seq, tok_pos, sink, scale, R, rot, max_ctx, out=None, splits=None):
+    """Causal attention of q [T, H, blocks * 32] over the latent pages -> [T, H, pad32(R)].  max_ctx: the longest context of
+    the call (chooses the number of context shares)."""
+    T, H, _ = q.shape
+    n_seq, max_blocks = block_table.shape
+    L = lib_of(q.dtype)
+    if splits is None:
+        splits = L.mlora_latent_attn_splits(T, H, max_ctx)
+    out = torch.empty((T, H, pad32(R)), dtype=q.dtype, device=q.device) if out is None else out
+    nb = L.mlora_latent_attn_workspace_bytes(T, H, R, splits)
+    ws = torch.empty(nb // 4, dtype=torch.float32, device=q.device) if nb else None
+    check(L.mlora_latent_attn(_dev(out), _dev(q), _dev(pages, q.dtype), _dev(block_table, torch.int32), max_blocks, _dev(tok_seq, torch.int32),
+                              _dev(tok_pos, torch.int32), _ptr(sink), scale, T, H, R, rot, pages.shape[0], n_seq, splits, _ptr(ws), nb, _stream()),
+          q.dtype)
+    return out
+
+
+def moe_route(logits, bias, scale, top, dtype):
+    """logits [T, >= E] fp32, bias [E] fp32 -> (pick [T, top] int32, weight [T, top] fp32)."""
+    T, ld = logits.shape
+    E = bias.shape[0]
+    pick = torch.empty((T, top), dtype=torch.int32, device=logits.device)
+    w = torch.empty((T, top), dtype=torch.float32, device=logits.device)
+    check(lib_of(dtype).mlora_moe_route(_dev(pick), _dev(w), _dev(logits, torch.float32), ld, _dev(bias, torch.float32), scale, T, E, top, _stream()),
+          dtype)
+    return pick, w
+
+
+class MoePlan:
+    """The (token, choice) entries of a routing sorted by expert and cut into tiles."""
+
+    def __init__(self, pick, E, dtype):
+        self.T, self.top = pick.shape
+        L, dev = lib_of(dtype), pick.device
+        self.tile_rows = L.mlora_moe_tile_rows(self.T, E, self.top)
+        self.max_tiles = L.mlora_moe_max_tiles(self.T, E, self.top)
+        i32 = lambda n: torch.empty(n, dtype=torch.int32, device=dev)
+        self.perm, self.tiles, self.n_tiles = i32(self.T * self.top), i32(4 * self.max_tiles), i32(1)
+        check(L.mlora_moe_plan(self.perm.data_ptr(), self.tiles.data_ptr(), self.n_tiles.data_ptr(), _dev(pick, torch.int32), self.T, E, self.top,
+                               _stream()), dtype)
+
+
+def moe_linear(x, W, plan, N, K, stage, act=ACT_NONE, alpha=1.0):
+    """Expert linears over a plan: stage MOE_UP: x [T, K] token rows -> place rows [T * top, N]; MOE_DOWN: place rows ->
+    entry rows.  W: the experts' [N, K] matrices stacked."""
+    y = torch.empty((plan.T * plan.top, N), dtype=x.dtype, device=x.device)
+    check(lib_of(x.dtype).mlora_moe_linear(_dev(y), _dev(x), _wptr(W), plan.perm.data_ptr(), plan.tiles.data_ptr(), plan.n_tiles.data_ptr(),
+                                           plan.tile_rows, plan.max_tiles, plan.T, K, N, plan.top, stage, act, alpha, _stream()), x.dtype)
+    return y
+
+
+def moe_combine(x, y, w):
+    """x [T, N] fp32 += sum over the choices of w * y (entry rows)."""
+    T, top = w.shape
+    check(lib_of(y.dtype).mlora_moe_combine(_dev(x, torch.float32), _dev(y), _dev(w, torch.float32), T, top, x.shape[1], _stream()), y.dtype)

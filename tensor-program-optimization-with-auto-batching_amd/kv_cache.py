@@ -1,4 +1,4 @@
-"""Paged KV cache: host-side page bookkeeping around the HIP attention kernels.
+"""Paged caches: host-side page bookkeeping around the HIP attention kernels.
 
 Keeps the host protocol of the reference's cache object
 (`tvm/llama_auto_batcher/llama_exec_graph.py:41-46,66,75-79,85,121-127`):
@@ -8,7 +8,9 @@ with RoPE applied inside the cache operator (`llama_for_causal_lm.py:148-174`: r
 scale 1, no sliding window).  Keys are stored already rotated, which is equivalent to rotating them at
 read time and saves the per-step re-rotation of the whole context.
 
-Device layout per layer: k [n_pages, Hkv, 16, D], v [n_pages, Hkv, D, 16] (fp16), one int32 block table
+A finished sequence gives its pages and its slot back with free_sequence(sid).
+
+Device layout of PagedKVCache per layer: k [n_pages, Hkv, 16, D], v [n_pages, Hkv, D, 16] (fp16), one int32 block table
 [max_seqs, max_blocks], fp32 RoPE tables [max_pos, D/2].
 """
 from __future__ import annotations
@@ -28,22 +30,15 @@ def rope_tables(head_dim: int, theta: float, max_pos: int):
     return np.cos(ang).astype(np.float32), np.sin(ang).astype(np.float32)
 
 
-class PagedKVCache:
-    def __init__(self, n_layers, n_pages, n_kv_heads, head_dim, max_seqs, max_blocks, rope_theta, max_pos,
-                 device="cuda:0", free_pages=None, page_size=PAGE):
+class PageTable:
+    """The host side of a paged cache: which pages of the pool belong to which sequence, and the protocol of a forward
+    pass.  What lies in a page is up to the subclass."""
+
+    def __init__(self, n_pages, max_seqs, max_blocks, max_pos, device, free_pages=None, page_size=PAGE):
         if page_size != PAGE:
             raise ValueError(f"page_size must be {PAGE}")
-        self.n_layers, self.n_pages, self.Hkv, self.D = n_layers, n_pages, n_kv_heads, head_dim
-        self.max_seqs, self.max_blocks, self.max_pos = max_seqs, max_blocks, max_pos
+        self.n_pages, self.max_seqs, self.max_blocks, self.max_pos = n_pages, max_seqs, max_blocks, max_pos
         self.device = torch.device(device)
-        if head_dim % 32:
-            raise ValueError("head_dim must be a multiple of 32")
-        # keys in matrix-core fragment order: element (token, d) of a page at [d // 32, (d % 32) // 8, token, d % 8]
-        self.k = torch.zeros((n_layers, n_pages, n_kv_heads, head_dim // 32, 4, PAGE, 8), dtype=torch.float16, device=self.device)
-        self.v = torch.zeros((n_layers, n_pages, n_kv_heads, head_dim, PAGE), dtype=torch.float16, device=self.device)
-        cos, sin = rope_tables(head_dim, rope_theta, max_pos)
-        self.rope_cos = torch.from_numpy(cos).to(self.device)
-        self.rope_sin = torch.from_numpy(sin).to(self.device)
         self.free = list(range(n_pages)) if free_pages is None else [int(p) for p in free_pages]
         if sorted(self.free) != list(range(n_pages)):
             raise ValueError("free_pages must be a permutation of range(n_pages)")
@@ -51,23 +46,30 @@ class PagedKVCache:
         self.table_h = np.full((max_seqs, max_blocks), -1, dtype=np.int32)
         self.lens = {}          # sid -> committed length
         self.slot = {}          # sid -> row of the block table
+        self.free_slots = list(range(max_seqs))
         self.block_table = torch.from_numpy(self.table_h.copy()).to(self.device)
         self._dirty = False
         self._cur = None
-
-    def k_rowmajor(self, layer: int) -> torch.Tensor:
-        """The layer's rotated keys as [n_pages, Hkv, 16, D] (a copy, for inspection)."""
-        k = self.k[layer]
-        return k.permute(0, 1, 4, 2, 3, 5).reshape(self.n_pages, self.Hkv, PAGE, self.D).contiguous()
 
     # ------------------------------------------------------------------ protocol
     def add_sequence(self, sid):
         if sid in self.slot:
             raise ValueError(f"sequence with id {sid} has already been added")
-        if len(self.slot) >= self.max_seqs:
+        if not self.free_slots:
             raise RuntimeError("paged KV cache: no sequence slot left")
-        self.slot[sid] = len(self.slot)
+        self.slot[sid] = self.free_slots.pop(0)
         self.lens[sid] = 0
+
+    def free_sequence(self, sid):
+        """Give back the pages and the slot of a finished sequence."""
+        if self._cur is not None:
+            raise RuntimeError("free_sequence between begin_forward and end_forward")
+        row = self.slot.pop(sid)
+        del self.lens[sid]
+        self.free.extend(int(p) for p in self.table_h[row] if p >= 0)
+        self.table_h[row] = -1
+        self.free_slots.insert(0, row)
+        self._dirty = True
 
     def begin_forward(self, seq_ids, append_lens, device_meta=None):
         """Reserve pages for the appended tokens and stage the per-token (sequence, position) arrays."""
@@ -107,6 +109,37 @@ class PagedKVCache:
             ctx = None
         self._cur = (list(seq_ids), list(append_lens), decode, tok_seq, tok_pos, ctx)
 
+    def end_forward(self):
+        seq_ids, append_lens = self._cur[0], self._cur[1]
+        for sid, n in zip(seq_ids, append_lens):
+            self.lens[sid] += n
+        self._cur = None
+
+    # ------------------------------------------------------------------ helpers
+    def pages_of(self, sid):
+        row = self.table_h[self.slot[sid]]
+        return row[row >= 0].tolist()
+
+
+class PagedKVCache(PageTable):
+    def __init__(self, n_layers, n_pages, n_kv_heads, head_dim, max_seqs, max_blocks, rope_theta, max_pos,
+                 device="cuda:0", free_pages=None, page_size=PAGE):
+        super().__init__(n_pages, max_seqs, max_blocks, max_pos, device, free_pages, page_size)
+        self.n_layers, self.Hkv, self.D = n_layers, n_kv_heads, head_dim
+        if head_dim % 32:
+            raise ValueError("head_dim must be a multiple of 32")
+        # keys in matrix-core fragment order: element (token, d) of a page at [d // 32, (d % 32) // 8, token, d % 8]
+        self.k = torch.zeros((n_layers, n_pages, n_kv_heads, head_dim // 32, 4, PAGE, 8), dtype=torch.float16, device=self.device)
+        self.v = torch.zeros((n_layers, n_pages, n_kv_heads, head_dim, PAGE), dtype=torch.float16, device=self.device)
+        cos, sin = rope_tables(head_dim, rope_theta, max_pos)
+        self.rope_cos = torch.from_numpy(cos).to(self.device)
+        self.rope_sin = torch.from_numpy(sin).to(self.device)
+
+    def k_rowmajor(self, layer: int) -> torch.Tensor:
+        """The layer's rotated keys as [n_pages, Hkv, 16, D] (a copy, for inspection)."""
+        k = self.k[layer]
+        return k.permute(0, 1, 4, 2, 3, 5).reshape(self.n_pages, self.Hkv, PAGE, self.D).contiguous()
+
     def attention_with_fused_qkv(self, layer, qkv, n_q_heads, out=None, frag=False, o_shrink=None):
         """qkv [T, Hq + 2 Hkv, D] (or [T, (Hq + 2 Hkv) * D]) fp16, token-major in begin_forward order.
         Rotates q in place, appends rotated k and v, attends causally; returns [T, Hq * D] fp16
@@ -127,18 +160,46 @@ class PagedKVCache:
         return ops.paged_attn_prefill(qkv, self.k[layer], self.v[layer], self.block_table, tok_seq, tok_pos,
                                       n_q_heads, self.Hkv, self.D, out=out, frag=frag)
 
-    def end_forward(self):
-        seq_ids, append_lens = self._cur[0], self._cur[1]
-        for sid, n in zip(seq_ids, append_lens):
-            self.lens[sid] += n
-        self._cur = None
-
-    # ------------------------------------------------------------------ helpers
-    def pages_of(self, sid):
-        row = self.table_h[self.slot[sid]]
-        return row[row >= 0].tolist()
-
     def kv_bytes_read_per_step(self, seq_ids):
         """Algorithmic K+V bytes one decode step reads for these sequences, all layers."""
         per_pos = self.n_layers * 2 * self.Hkv * self.D * 2
         return int(sum(self.lens[s] + 1 for s in seq_ids)) * per_pos
+
+class PagedLatentCache(PageTable):
+    """Pages of latent attention: per layer one vector per token, the normed latent and the rotated key part, in the page
+    layout of latent_attention.hip.  A layer may read another layer's pages instead of having its own."""
+
+    def __init__(self, layers, n_pages, max_seqs, max_blocks, max_pos, dtype, device="cuda:0", free_pages=None, page_size=PAGE):
+        """layers: per layer (kv_rank, rot_dim, rotation, owner): owner is the layer whose pages this one reads (itself,
+        if it has its own); rotation: rotary.Rotation."""
+        super().__init__(n_pages, max_seqs, max_blocks, max_pos, device, free_pages, page_size)
+        self.dtype = dtype
+        self.owner = [o for *_, o in layers]
+        self.pages = []
+        self.rope = []
+        tables = {}
+        for l, (rank, rot_dim, rotation, o) in enumerate(layers):
+            blocks = -(-rank // 32) + -(-rot_dim // 32)
+            # padding between and behind the two parts is read by the matrix cores: it stays zero
+            self.pages.append(torch.zeros((n_pages, blocks, 4, PAGE, 8), dtype=dtype, device=self.device) if o == l else self.pages[o])
+            key = (rotation, rot_dim)
+            if key not in tables:
+                tables[key] = tuple(torch.from_numpy(t).to(self.device) for t in rotation.tables(rot_dim, max_pos))
+            self.rope.append(tables[key])
+
+    def latents(self, layer, sid):
+        """The cached vectors [length, blocks * 32] of a sequence (a copy, for inspection)."""
+        n = self.lens[sid]
+        p = self.pages[layer][torch.tensor(self.pages_of(sid), device=self.device, dtype=torch.int64)]
+        return p.permute(0, 3, 1, 2, 4).reshape(-1, p.shape[1] * 32)[:n].contiguous()
+
+    def latent_attention(self, layer, qkv, att, out=None):
+        """The mixer of `layer` behind its input projection: qkv [T, att.proj_rows] in begin_forward order (att:
+        latent_attention.LatentAttention) -> the heads' outputs, concatenated (`out`: an activation of att.out_cols
+        columns)."""
+        if self._cur is None:
+            raise RuntimeError("latent_attention outside begin_forward/end_forward")
+        seq_ids, append_lens, _, tok_seq, tok_pos, _ = self._cur
+        max_ctx = max(self.lens[s] + n for s, n in zip(seq_ids, append_lens))
+        return att.attend(qkv, self.pages[layer], self.block_table, tok_seq, tok_pos, *self.rope[layer], max_ctx=max_ctx,
+                          store=self.owner[layer] == layer, out=out)

@@ -20,6 +20,7 @@ import torch
 
 from . import ops
 from .kv_cache import PagedKVCache
+from .model_base import CausalLM
 from .synth import LINEARS, LlamaShape, linear_dims
 
 
@@ -53,7 +54,10 @@ class LoraType:
         self.tables[(layer, proj)] = (A.contiguous(), B.contiguous())
 
 
-class LlamaForCausalLM:
+class LlamaForCausalLM(CausalLM):
+    dtypes = ("float16",)
+    native_step = True
+
     def __init__(self, shape: LlamaShape, device="cuda:0"):
         self.shape = shape
         self.device = torch.device(device)
@@ -109,6 +113,27 @@ class LlamaForCausalLM:
                 for proj in spec.targets:
                     lt.add(l, proj, lw[f"layers.{l}.{proj}.lora_A.a{tid}"], lw[f"layers.{l}.{proj}.lora_B.a{tid}"])
             m.add_lora_type(lt)
+        return m
+
+    @classmethod
+    def from_weights(cls, config: dict, tensors, dtype=torch.float16, device="cuda:0"):
+        """config: a config.json of a Llama checkpoint; tensors(name) -> tensor."""
+        heads = config["num_attention_heads"]
+        shape = LlamaShape(hidden_size=config["hidden_size"], intermediate_size=config["intermediate_size"], num_attention_heads=heads,
+                           num_key_value_heads=config.get("num_key_value_heads") or heads, num_hidden_layers=config["num_hidden_layers"],
+                           head_dim=config.get("head_dim") or config["hidden_size"] // heads, vocab_size=config["vocab_size"],
+                           rms_norm_eps=config["rms_norm_eps"], rope_theta=config.get("rope_theta", 10000.0))
+        if config.get("rope_scaling"):
+            raise ValueError("rope_scaling is not supported")
+        m = cls(shape, device)
+        for l in range(shape.num_hidden_layers):
+            n = f"model.layers.{l}."
+            w = {p: tensors(f"{n}self_attn.{p}.weight") for p in ("q_proj", "k_proj", "v_proj", "o_proj")}
+            w.update({p: tensors(f"{n}mlp.{p}.weight") for p in ("gate_proj", "up_proj", "down_proj")})
+            w.update({p: tensors(f"{n}{p}.weight") for p in ("input_layernorm", "post_attention_layernorm")})
+            m.load_layer(l, w)
+        embed = tensors("model.embed_tokens.weight")
+        m.load_head(embed, embed if config.get("tie_word_embeddings") else tensors("lm_head.weight"), tensors("model.norm.weight"))
         return m
 
     def interleaved_gate_up(self):
@@ -207,11 +232,7 @@ class LlamaForCausalLM:
         """Same arguments as the reference's VM function (`llama_for_causal_lm.py:148-174`).  The pool holds
         ceil(max_total_seq_len / page_size) + max_batch_size pages (one partial page per sequence)."""
         s = self.shape
-        n_pages = -(-max_total_seq_len // page_size) + max_batch_size
-        if free_pages is not None:
-            n_pages = len(free_pages)
-        max_seq_len = max_seq_len or min(max_total_seq_len, n_pages * page_size)
-        max_blocks = -(-max_seq_len // page_size)
+        n_pages, max_blocks = self._cache_geometry(max_batch_size, max_total_seq_len, page_size, free_pages, max_seq_len)
         return PagedKVCache(s.num_hidden_layers, n_pages, s.num_key_value_heads, s.head_dim, max_seqs=max_batch_size,
                             max_blocks=max_blocks, rope_theta=s.rope_theta, max_pos=max_blocks * page_size,
                             device=self.device, free_pages=free_pages, page_size=page_size)
@@ -493,16 +514,6 @@ class LlamaForCausalLM:
             out[tid] = full if host else torch.from_numpy(full).to(self.device)
         return out
 
-    def _last_rows(self, kv):
-        lens = kv._cur[1]
-        return torch.from_numpy(np.cumsum(lens).astype(np.int64) - 1).to(self.device)
-
-    def prefill_no_adapter(self, h, kv):
-        return self.forward(h, kv, None, self._last_rows(kv)), kv
-
-    def decode_no_adapter(self, h, kv):
-        return self.forward(h, kv, None), kv
-
     def prefill_a(self, tid, h, kv, wids):
         """Prefill of the sequences announced to kv.begin_forward; wids: one weight id per sequence
         (the reference prefills one sequence per call: wids [1])."""
@@ -523,8 +534,6 @@ class LlamaForCausalLM:
 
     def __getitem__(self, name: str):
         """Entry points by the reference's VM function names."""
-        if name in ("embed", "create_paged_kv_cache", "prefill_no_adapter", "decode_no_adapter"):
-            return getattr(self, name)
         m = re.fullmatch(r"(prefill|decode)_a(\d+)", name)
         if m:
             tid = int(m.group(2))
@@ -537,7 +546,7 @@ class LlamaForCausalLM:
             for t in tids:
                 self._check_tid(t)
             return lambda h, kv, *params: self.mixed_decode(tids, h, kv, *params)
-        raise KeyError(f"unknown entry point {name}")
+        return super().__getitem__(name)
 
     def _check_tid(self, tid):
         if not 0 <= tid < len(self.lora_types):

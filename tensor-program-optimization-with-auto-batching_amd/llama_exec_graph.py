@@ -174,6 +174,9 @@ class LlamaExecGraph(ExecGraph):
         while seqs:
             method, params = self.seq_info.get_decode_method(seqs)
             if getattr(self.exec_config, "native_decode", False):
+                if not self.vm.native_step:               # a model without the C decode step: graph-replayed operators
+                    seqs = self._decode_session(seqs, outputs, method, params)
+                    continue
                 dense = len(seqs) <= 64 and self._dense_ok(method)       # the dense shrink serves at most 64 sequences
                 seqs = self._decode_native(seqs, outputs, method, params, dense) if dense or not method.startswith("mixed_decode") \
                     else self._decode_session(seqs, outputs, method, params)

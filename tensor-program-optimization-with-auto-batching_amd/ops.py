@@ -7,7 +7,19 @@ from __future__ import annotations
 
 import torch
 
-from ._lib import F16, F32, ROWMAJOR, FRAG, STORE, ACCUMULATE, check, lib
+from . import _lib
+from ._lib import F16, F32, ROWMAJOR, FRAG, STORE, ACCUMULATE, lib
+
+_LIB_OF = {torch.float16: "float16", torch.bfloat16: "bfloat16", torch.float32: "float32"}
+
+
+def lib_of(dtype: torch.dtype):
+    """The kernel library whose element type is `dtype`."""
+    return lib(_LIB_OF[dtype])
+
+
+def check(code: int, dtype: torch.dtype = torch.float16) -> None:
+    _lib.check(code, _LIB_OF[dtype])
 
 
 def _stream() -> int:
@@ -25,20 +37,20 @@ def _dev(t: torch.Tensor, dtype=None, name="tensor") -> int:
 
 
 def _dt(t: torch.Tensor) -> int:
-    if t.dtype == torch.float16:
+    if t.dtype in (torch.float16, torch.bfloat16):
         return F16
     if t.dtype == torch.float32:
         return F32
-    raise TypeError(f"expected float16 or float32, got {t.dtype}")
+    raise TypeError(f"expected a 16-bit float type or float32, got {t.dtype}")
 
 
 class FragActivation:
-    """A [T, K] fp16 activation block stored in matrix-core fragment order (MLORA_FRAG)."""
+    """A [T, K] 16-bit activation block stored in matrix-core fragment order (MLORA_FRAG)."""
 
-    def __init__(self, T: int, K: int, device, data: torch.Tensor = None):
+    def __init__(self, T: int, K: int, device, data: torch.Tensor = None, dtype: torch.dtype = torch.float16):
         self.T, self.K = T, K
-        n = lib().mlora_frag_activation_elems(T, K)
-        self.data = torch.empty(n, dtype=torch.float16, device=device) if data is None else data
+        n = lib_of(dtype if data is None else data.dtype).mlora_frag_activation_elems(T, K)
+        self.data = torch.empty(n, dtype=dtype, device=device) if data is None else data
         if self.data.numel() < n:
             raise ValueError("FragActivation: buffer too small")
 
@@ -50,18 +62,31 @@ class FragActivation:
     def device(self):
         return self.data.device
 
+    @property
+    def dtype(self):
+        return self.data.dtype
+
+    def _tiles(self) -> int:
+        return 1 if self.T <= 16 else (2 if self.T <= 32 else (4 if self.T <= 64 else -(-self.T // 16)))
+
+    def columns(self, k0: int, K: int) -> "FragActivation":
+        """Columns k0 .. k0 + K - 1 as a block of their own (multiples of 32: whole k-blocks, contiguous in this order)."""
+        if k0 % 32 or K % 32 or k0 + K > self.K:
+            raise ValueError("FragActivation.columns: whole 32-column blocks")
+        return FragActivation(self.T, K, self.device, self.data[k0 * 16 * self._tiles():])
+
     @classmethod
     def pack(cls, x: torch.Tensor, out: "FragActivation" = None):
-        """Row-major [T, K] fp16 (unit inner stride) -> fragment order."""
+        """Row-major [T, K] (unit inner stride) -> fragment order."""
         T, K = x.shape
-        out = cls(T, K, x.device) if out is None else out
+        out = cls(T, K, x.device, dtype=x.dtype) if out is None else out
         ld = x.stride(0) if T > 1 else max(K, x.stride(0))
-        check(lib().mlora_pack_activation(out.data.data_ptr(), x.data_ptr(), ld, T, K, _stream()))
+        check(lib_of(x.dtype).mlora_pack_activation(out.data.data_ptr(), x.data_ptr(), ld, T, K, _stream()), x.dtype)
         return out
 
     def unpack(self) -> torch.Tensor:
         """Back to row-major [T, K] (host-side index arithmetic on the device tensor; for tests)."""
-        TT = 1 if self.T <= 16 else (2 if self.T <= 32 else (4 if self.T <= 64 else -(-self.T // 16)))
+        TT = self._tiles()
         v = self.data[: TT * 16 * self.K].view(self.K // 32, TT, 4, 16, 8)
         return v.permute(1, 3, 0, 2, 4).reshape(TT * 16, self.K)[: self.T].contiguous()
 
@@ -263,18 +288,23 @@ def write_tensor_part(X, Y, ids, out=None):
 
 
 class PackedWeight:
-    """A [N, K] fp16 weight stored in matrix-core fragment order (see mlora_pack_weight)."""
+    """A [N, K] 16-bit weight stored in matrix-core fragment order (see mlora_pack_weight)."""
 
     def __init__(self, W: torch.Tensor):
         N, K = W.shape
         self.N, self.K = N, K
-        n = lib().mlora_packed_weight_elems(N, K)
-        self.data = torch.empty(n, dtype=torch.float16, device=W.device)
-        check(lib().mlora_pack_weight(_dev(self.data), _dev(W, torch.float16, "W"), N, K, _stream()))
+        L = lib_of(W.dtype)
+        n = L.mlora_packed_weight_elems(N, K)
+        self.data = torch.empty(n, dtype=W.dtype, device=W.device)
+        check(L.mlora_pack_weight(_dev(self.data), _dev(W, name="W"), N, K, _stream()), W.dtype)
 
     @property
     def shape(self):
         return (self.N, self.K)
+
+    @property
+    def dtype(self):
+        return self.data.dtype
 
     def unpack(self) -> torch.Tensor:
         """Back to row-major [N, K] (index arithmetic on the device tensor)."""
@@ -283,9 +313,10 @@ class PackedWeight:
         return v.permute(0, 3, 1, 2, 4).reshape(nt * 16, self.K)[: self.N].contiguous()
 
 
-def linear(x, W, out=None, out_dtype=torch.float16, accumulate=False, kernel="auto"):
-    """y (=|+=) x @ W.T.  x [T,K] f16 (row stride may exceed K) or a FragActivation, W [N,K] f16 or a
-    PackedWeight.  accumulate=True adds into the fp32 tensor `out`.  kernel: "auto" | "gemv" | "gemm"."""
+def linear(x, W, out=None, out_dtype=None, accumulate=False, kernel="auto"):
+    """y (=|+=) x @ W.T.  x [T,K] (row stride may exceed K) or a FragActivation, W [N,K] of the same type or a
+    PackedWeight; f16, bf16 (fragment order or packed) or f32 (plain); y has their type unless out_dtype says f32.  accumulate=True adds into the fp32 tensor `out`.  kernel: "auto" | "gemv" | "gemm"."""
+    out_dtype = out_dtype or W.dtype
     if isinstance(x, FragActivation):
         return _linear_frag(x, W, out, out_dtype, accumulate)
     T, K = x.shape
@@ -297,8 +328,8 @@ def linear(x, W, out=None, out_dtype=torch.float16, accumulate=False, kernel="au
         if out is None:
             out = torch.empty((0, N), dtype=torch.float32 if accumulate else out_dtype, device=x.device)
         return out
-    if not x.is_cuda or x.dtype != torch.float16 or x.stride(1) != 1:
-        raise ValueError("linear: x must be a GPU fp16 tensor with unit inner stride")
+    if not x.is_cuda or x.dtype != W.dtype or x.stride(1) != 1:
+        raise ValueError("linear: x must be a GPU tensor of the weight's type with unit inner stride")
     ldx = x.stride(0) if T > 1 else max(K, x.stride(0))
     if out is None:
         if accumulate:
@@ -307,18 +338,18 @@ def linear(x, W, out=None, out_dtype=torch.float16, accumulate=False, kernel="au
     if out.shape != (T, N):
         raise ValueError(f"linear: out{tuple(out.shape)} expected {(T, N)}")
     if packed:
-        fn = {"auto": lib().mlora_linear_packed, "gemv": lib().mlora_gemv_packed, "gemm": lib().mlora_gemm_packed}[kernel]
+        fn = getattr(lib_of(W.dtype), {"auto": "mlora_linear_packed", "gemv": "mlora_gemv_packed", "gemm": "mlora_gemm_packed"}[kernel])
         wptr = W.data.data_ptr()
     else:
-        fn = {"auto": lib().mlora_linear, "gemv": lib().mlora_gemv, "gemm": lib().mlora_gemm}[kernel]
-        wptr = _dev(W, torch.float16, "W")
-    check(fn(_dev(out), _dt(out), ACCUMULATE if accumulate else STORE, x.data_ptr(), ldx, wptr, T, K, N, _stream()))
+        fn = getattr(lib_of(W.dtype), {"auto": "mlora_linear", "gemv": "mlora_gemv", "gemm": "mlora_gemm"}[kernel])
+        wptr = _dev(W, name="W")
+    check(fn(_dev(out), _dt(out), ACCUMULATE if accumulate else STORE, x.data_ptr(), ldx, wptr, T, K, N, _stream()), W.dtype)
     return out
 
 
 def _linear_frag(x, W, out, out_dtype, accumulate):
-    if not isinstance(W, PackedWeight):
-        raise TypeError("a fragment-ordered activation needs a PackedWeight")
+    if not isinstance(W, PackedWeight) or W.dtype != x.dtype:
+        raise TypeError("a fragment-ordered activation needs a PackedWeight of its type")
     T, K = x.shape
     N, K2 = W.shape
     if K2 != K:
@@ -329,8 +360,8 @@ def _linear_frag(x, W, out, out_dtype, accumulate):
         out = torch.empty((T, N), dtype=out_dtype, device=x.device)
     if out.shape != (T, N):
         raise ValueError(f"linear: out{tuple(out.shape)} expected {(T, N)}")
-    check(lib().mlora_linear_frag(_dev(out), _dt(out), ACCUMULATE if accumulate else STORE, x.data.data_ptr(),
-                                  W.data.data_ptr(), T, K, N, _stream()))
+    check(lib_of(W.dtype).mlora_linear_frag(_dev(out), _dt(out), ACCUMULATE if accumulate else STORE, x.data.data_ptr(),
+                                            W.data.data_ptr(), T, K, N, _stream()), W.dtype)
     return out
 
 
@@ -467,11 +498,12 @@ def linear_acc_ksplit(x: FragActivation, W: PackedWeight, resid: torch.Tensor, w
     N, K2 = W.shape
     if K2 != K or resid.shape != (T, N) or resid.dtype != torch.float32:
         raise ValueError(f"linear_acc_ksplit: x{x.shape} W{W.shape} resid{tuple(resid.shape)}")
-    ks = lib().mlora_gemv_ksplit(T, K, N + riding_rows) if ws is not None else 1
-    if ks > 1 and ws.numel() * 4 < lib().mlora_gemv_ksplit_bytes(T, N, ks):
+    L = lib_of(W.dtype)
+    ks = L.mlora_gemv_ksplit(T, K, N + riding_rows) if ws is not None else 1
+    if ks > 1 and ws.numel() * 4 < L.mlora_gemv_ksplit_bytes(T, N, ks):
         ks = 1
-    check(lib().mlora_gemv_frag_acc_ksplit(_dev(resid, torch.float32), None, _dev(ws, torch.float32) if ks > 1 else None, ks,
-                                           x.data.data_ptr(), W.data.data_ptr(), T, K, N, 0, None, None, 0, None, 0, 0, _stream()))
+    check(L.mlora_gemv_frag_acc_ksplit(_dev(resid, torch.float32), None, _dev(ws, torch.float32) if ks > 1 else None, ks,
+                                       x.data.data_ptr(), W.data.data_ptr(), T, K, N, 0, None, None, 0, None, 0, 0, _stream()), W.dtype)
     return KSplitParts(ws, ks, N) if ks > 1 else None
 
 
@@ -539,7 +571,7 @@ def embed(table, ids, out_dtype=torch.float32, out=None):
         out = torch.empty((T, H), dtype=out_dtype, device=table.device)
     if T == 0:
         return out
-    check(lib().mlora_embed(_dev(out), _dt(out), _dev(table, torch.float16), _dev(ids, torch.int32), T, H, V, _stream()))
+    check(lib_of(table.dtype).mlora_embed(_dev(out), _dt(out), _dev(table), _dev(ids, torch.int32), T, H, V, _stream()), table.dtype)
     return out
 
 
@@ -549,7 +581,7 @@ def argmax(logits, out=None):
         out = torch.empty((B,), dtype=torch.int32, device=logits.device)
     if B == 0:
         return out
-    check(lib().mlora_argmax(_dev(out, torch.int32), _dev(logits, torch.float32), B, V, _stream()))
+    check(_lib.loaded().mlora_argmax(_dev(out, torch.int32), _dev(logits, torch.float32), B, V, _stream()))
     return out
 
 
