@@ -526,6 +526,130 @@ def bench_c1_generate(args, synth, llama):
     print(json.dumps(out))
 
 
+SAFOLORN_SIZES = {      # layers like a real model's: width, heads, feed-forward, experts (number, chosen, width), token input
+    "w2048": dict(width=2048, heads=16, ff=5632, experts=(64, 6, 1408), side=128),
+    "w4096": dict(width=4096, heads=32, ff=11008, experts=(32, 4, 2752), side=256),
+}
+SAFOLORN_LAYERS = 4     # two dense, two with experts; the last two read the second one's latents
+
+
+def safolorn_model(size):
+    """Random-weight Safolorn of one of SAFOLORN_SIZES (weights drawn on the GPU, tensor by tensor)."""
+    import torch
+    c = SAFOLORN_SIZES[size]
+    E, top, eff = c["experts"]
+    yarn = {"factor": 4.0, "original": 2048, "fast": 32.0, "slow": 1.0}
+    layers = []
+    for l in range(SAFOLORN_LAYERS):
+        mixer = {"heads": c["heads"], "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5,
+                 "rot": {"base": 10000.0, "dims": 64, "scaling": yarn}}
+        if l >= 2:
+            mixer["kv_from"] = 1
+        mlp = {"kind": "dense", "ff": c["ff"], "limit": 7.0} if l % 2 == 0 else \
+              {"kind": "moe", "expert": {"ff": eff}, "router": {"experts": E, "top": top}}
+        layers.append({"type": "latent_attention", "mixer": mixer, "mlp": mlp})
+    cfg = {"architecture": "Safolorn", "vocab": 32000, "width": c["width"], "norm": {"eps": 1e-5}, "token_side": {"dim": c["side"]}, "layers": layers}
+    W, H = c["width"], c["heads"]
+    gen = torch.Generator(device="cuda:0").manual_seed(0)
+
+    def tensors(name):
+        leaf = name.split(".", 1)[1] if name[0] == "l" and name[1].isdigit() else name
+        shape = {"norm1": (), "norm2": (), "final.norm": (), "embed": (32000, W), "side.embed": (32000, c["side"] * SAFOLORN_LAYERS),
+                 "head": (32000, W), "mix.q": (H * 192, W), "mix.dkv": (576, W), "mix.dkv.norm": (512,), "mix.uk": (H * 128, 512),
+                 "mix.uv": (H * 128, 512), "mix.sink": (H,), "mix.o": (W, H * 128), "mlp.gate": (c["ff"], W), "mlp.up": (c["ff"], W),
+                 "mlp.down": (W, c["ff"]), "mlp.router": (E, W), "mlp.router.b": (E,), "side.gate": (c["side"], W),
+                 "side.proj": (W, c["side"]), "side.norm": (W,)}.get(leaf) or ((eff, W) if leaf.endswith("up") else (W, eff) if leaf.endswith("down") else ())
+        if "norm" in leaf:
+            return torch.ones(shape, dtype=torch.bfloat16, device="cuda:0")
+        return (torch.randn(shape, generator=gen, device="cuda:0") * shape[-1] ** -0.5).to(torch.bfloat16)
+
+    return _mod("registry").model_class(cfg).from_weights(cfg, tensors)
+
+
+def safolorn_llama(size, synth, llama):
+    """The Llama model of the same width, heads, dense feed-forward and depth, without adapters."""
+    c = SAFOLORN_SIZES[size]
+    shape = synth.LlamaShape(hidden_size=c["width"], intermediate_size=c["ff"], num_attention_heads=c["heads"], num_key_value_heads=c["heads"],
+                             num_hidden_layers=SAFOLORN_LAYERS, head_dim=c["width"] // c["heads"], vocab_size=32000)
+    return llama.LlamaForCausalLM.from_synthetic(0, shape, [], "cuda:0")
+
+
+def time_prefill(model, B, P, warmup, steps):
+    """Seconds of one pass over B prompts of P tokens."""
+    import torch
+    kv = model.create_paged_kv_cache(B, B * P, P, 16, max_seq_len=P)
+    tokens = torch.randint(0, 32000, (B * P,), dtype=torch.int32)
+    for b in range(B):
+        kv.add_sequence(b)
+
+    def step():
+        for b in range(B):
+            kv.lens[b] = 0
+        kv.begin_forward(list(range(B)), [P] * B)
+        model["prefill_no_adapter"](model.embed(tokens), kv)
+        kv.end_forward()
+
+    for _ in range(warmup):
+        step()
+    torch.cuda.synchronize()
+    t0 = time.perf_counter()
+    for _ in range(steps):
+        step()
+    torch.cuda.synchronize()
+    return (time.perf_counter() - t0) / steps
+
+
+def time_decode(model, B, ctx, warmup, steps):
+    """Seconds of one graph-replayed greedy step of B requests at context `ctx` (cache filled with random values)."""
+    import torch
+    dsm = _mod("decode_session")
+    blocks = -(-(ctx + warmup + steps + 2) // 16)
+    kv = model.create_paged_kv_cache(B, B * blocks * 16, ctx, 16, free_pages=np.random.default_rng(0).permutation(B * blocks), max_seq_len=blocks * 16)
+    for t in ([t for l in range(len(model.layers)) for t in (kv.k[l], kv.v[l])] if hasattr(kv, "k") else kv.pages):
+        t.normal_()
+    for b in range(B):
+        kv.add_sequence(b)
+    kv.begin_forward(list(range(B)), [ctx] * B)
+    kv.end_forward()
+    first = np.arange(B, dtype=np.int32)
+    sess = dsm.NativeDecodeSession(model, kv, list(range(B)), None, first) if model.native_step else \
+        dsm.DecodeSession(model, kv, list(range(B)), {}, first, use_graph=True)
+    for _ in range(max(warmup, 3)):
+        sess.step()
+    torch.cuda.synchronize()
+    t0 = time.perf_counter()
+    for _ in range(steps):
+        sess.step()
+    torch.cuda.synchronize()
+    return (time.perf_counter() - t0) / steps
+
+
+def bench_safolorn(args, synth, llama):
+    """Prefill and decode throughput of Safolorn layers at sizes like a real model's (bfloat16, random weights), beside the
+    Llama model of the same width, heads, dense feed-forward and depth (fp16)."""
+    import torch
+    rows = []
+    for size in SAFOLORN_SIZES:
+        for kind in ("safolorn", "llama"):
+            model = safolorn_model(size) if kind == "safolorn" else safolorn_llama(size, synth, llama)
+            r = {"size": size, "model": kind}
+            for B, P in ((8, 512), (1, 4096)):
+                r[f"prefill_{B}x{P}_tok_s"] = B * P / time_prefill(model, B, P, 2, max(2, args.steps // 8))
+            for B, ctx in ((1, 512), (32, 512), (128, 2048)):
+                r[f"decode_b{B}_ctx{ctx}_tok_s"] = B / time_decode(model, B, ctx, args.warmup, args.steps)
+            rows.append(r)
+            print(json.dumps(r), file=sys.stderr, flush=True)
+            del model
+            torch.cuda.empty_cache()
+    key = "decode_b32_ctx512_tok_s"
+    print(json.dumps({
+        "metric": "decode tok/s, Safolorn layers of width 4096, 32 requests at context 512", "value": rows[2][key], "unit": "tok/s", "n_gpus": 1,
+        "steps": args.steps, "warmup": args.warmup, "ms_per_step": 32e3 / rows[2][key], "higher_is_better": True, "scaling": "weak",
+        "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+        "config": {"sizes": SAFOLORN_SIZES, "layers": SAFOLORN_LAYERS, "host_loop": "hipGraph replay of the operators (Llama: of mlora_decode_step)"},
+        "rows": rows}))
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -534,9 +658,10 @@ def main():
     ap.add_argument("--layers", type=int, default=32, help="model depth (32 = the benchmark configuration)")
     ap.add_argument("--batch", type=int, default=32,
                     help="c3_decode: concurrent requests (32 = the benchmark configuration; up to 64 run the native step)")
-    ap.add_argument("--workload", default="c3_decode", choices=["c3_decode", "c4_prefill", "c5_decode", "c1_generate"],
+    ap.add_argument("--workload", default="c3_decode", choices=["c3_decode", "c4_prefill", "c5_decode", "c1_generate", "safolorn"],
                     help="c3_decode is the benchmark the metric is quoted on; the other two time the prefill and the "
-                         "256-request stress configurations with the same harness")
+                         "256-request stress configurations with the same harness; safolorn: prefill and decode of "
+                         "Safolorn layers beside Llama layers of the same size")
     ap.add_argument("--shape", default="llama2_7b", choices=["llama2_7b", "llama31_8b"],
                     help="c3_decode: model shape (llama2_7b = the benchmark configuration; llama31_8b = the reference's default "
                          "model: grouped-query attention, 8 kv heads, vocabulary 128256)")
@@ -571,6 +696,8 @@ def main():
         return bench_c4_prefill(args, synth, llama)
     if args.workload == "c5_decode":
         return bench_c5_decode(args, synth, llama)
+    if args.workload == "safolorn":
+        return bench_safolorn(args, synth, llama)
     if args.workload == "c1_generate":
         return bench_c1_generate(args, synth, llama)
     if args.probe:

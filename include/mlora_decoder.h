@@ -29,16 +29,17 @@ int mlora_token_gate(void* out_frag, const float* x, const float* part, int n_pa
 int mlora_token_gate_mul(void* out, const void* z, const void* table, int ld_table, int col0, int dim, const int32_t* ids, int V, int T, int N,
                          void* stream);
 
-/* Latent attention (layouts at the top of latent_attention.hip).  mlora_latent_prep takes the token's projections
- * qkv [T, ld] times `gain`: rotates the heads' query parts (columns off_rot .. + H rot) into q [T, H, NB 32], and, with c_norm,
- * norms the latent (off_c .. + R), rotates the shared key part (off_kr .. + rot) and stores both in the token's page slot.
- * mlora_head_linear: y[t, h] = alpha W[h] . x[t, h].  mlora_latent_attn: causal softmax over the sequence's pages with
- * scores (q . cached) * scale and, with `sink`, exp(sink[h]) in the denominator; out [T, H, ceil32(R)].  splits > 1 needs
- * a workspace. */
-int mlora_latent_prep(void* q, void* cache, const void* qkv, int ld, int off_rot, int off_c, int off_kr, float gain, const void* c_norm,
-                      float eps, const int32_t* block_table, int max_blocks, const int32_t* tok_seq, const int32_t* tok_pos,
-                      const float* rope_cos, const float* rope_sin, int max_pos, int T, int H, int R, int rot, int n_pages, int n_seq,
-                      void* stream);
+/* Latent attention (layouts at the top of latent_attention.hip).  mlora_latent_prep takes the token's projections qkv [T, ld]:
+ * rotates the heads' query parts (columns off_rot .. + H rot) into the rows q + (t H + h) q_ld + q_off, padded to whole blocks of
+ * 32, and, with c_norm, norms `gain` times the latent (off_c .. + R), rotates `gain` times the shared key part
+ * (off_kr .. + rot) and stores both in the token's page slot.
+ * mlora_head_linear: y[t, h] = alpha W[h] . x[t, h].  mlora_latent_attn: causal softmax over the sequence's pages with scores
+ * (q . cached) * scale, q [T, H, NB 32], and, with `sink`, exp(sink[h]) in the denominator; out [T, H, ceil32(R)].
+ * splits > 1 needs a workspace. */
+int mlora_latent_prep(void* q, int q_ld, int q_off, void* cache, const void* qkv, int ld, int off_rot, int off_c, int off_kr, float gain,
+                      const void* c_norm, float eps, const int32_t* block_table, int max_blocks, const int32_t* tok_seq,
+                      const int32_t* tok_pos, const float* rope_cos, const float* rope_sin, int max_pos, int T, int H, int R, int rot,
+                      int n_pages, int n_seq, void* stream);
 int mlora_head_linear(void* y, int y_layout, long ldy, long head_y, const void* x, long ldx, long head_x, const void* W, int heads, int T,
                       int K, int N, float alpha, void* stream);
 int mlora_latent_attn_splits(int T, int H, int max_ctx);
@@ -46,6 +47,20 @@ size_t mlora_latent_attn_workspace_bytes(int T, int H, int R, int splits);
 int mlora_latent_attn(void* out, const void* q, const void* cache, const int32_t* block_table, int max_blocks, const int32_t* tok_seq,
                       const int32_t* tok_pos, const float* sink, float scale, int T, int H, int R, int rot, int n_pages, int n_seq,
                       int splits, void* workspace, size_t workspace_bytes, void* stream);
+
+/* The same attention for prompts (bfloat16 library): makes the heads' keys and values of whole contexts in scratch memory and
+ * attends over those.  phys [pages]: the cache pages of the contexts one after the other, each context padded with -1 to a
+ * multiple of four pages; tiles [n_tiles][4] int32 = {first token, tokens (at most mlora_latent_prefill_tile_tokens), first
+ * scratch page of its context, position of the first token}, one sequence each.  q [T, ld_q]: the heads' unrotated query parts, each
+ * padded to 32 columns; q_rot [T, H, ceil32(rot)]; uk packed [H ceil32(dim), ceil32(R)], uv packed [H ceil32(vdim), ceil32(R)];
+ * out [T, H ceil32(vdim)]. */
+int mlora_latent_prefill_tile_tokens(void);
+int mlora_latent_prefill_served(int dim, int rot, int vdim);
+size_t mlora_latent_prefill_scratch_elems(int pages, int H, int dim, int rot, int vdim);
+int mlora_latent_prefill(void* out, int out_layout, int ld_out, const void* q, int ld_q, const void* q_rot, const void* cache,
+                         const int32_t* phys, int pages, const int32_t* tiles, int n_tiles, const void* uk, const void* uv, const float* sink,
+                         float scale, int T, int H, int R, int dim, int rot, int vdim, int n_pages, void* scratch, size_t scratch_elems,
+                         void* stream);
 
 /* Mixture of experts.  mlora_moe_route: z = scale logits[t] + bias, the `top` largest per token (lower index on ties), softmax
  * over those.  mlora_moe_plan sorts the (token, choice) entries by expert into tiles {expert, first place, places, 0} of

@@ -122,11 +122,15 @@ DECODER_SIGNATURES = {
     "mlora_stream_norm": (_i, [_p, _p, _p, _p, _i, _p, _p, _f, _f, _i, _i, _i, _p]),
     "mlora_token_gate": (_i, [_p, _p, _p, _i, _p, _p, _i, _i, _i, _p, _i, _i, _i, _i, _p]),
     "mlora_token_gate_mul": (_i, [_p, _p, _p, _i, _i, _i, _p, _i, _i, _i, _p]),
-    "mlora_latent_prep": (_i, [_p, _p, _p, _i, _i, _i, _i, _f, _p, _f, _p, _i, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _p]),
+    "mlora_latent_prep": (_i, [_p, _i, _i, _p, _p, _i, _i, _i, _i, _f, _p, _f, _p, _i, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _p]),
     "mlora_head_linear": (_i, [_p, _i, _l, _l, _p, _l, _l, _p, _i, _i, _i, _i, _f, _p]),
     "mlora_latent_attn_splits": (_i, [_i, _i, _i]),
     "mlora_latent_attn_workspace_bytes": (_z, [_i, _i, _i, _i]),
     "mlora_latent_attn": (_i, [_p, _p, _p, _p, _i, _p, _p, _p, _f, _i, _i, _i, _i, _i, _i, _i, _p, _z, _p]),
+    "mlora_latent_prefill_tile_tokens": (_i, []),
+    "mlora_latent_prefill_served": (_i, [_i, _i, _i]),
+    "mlora_latent_prefill_scratch_elems": (_z, [_i, _i, _i, _i, _i]),
+    "mlora_latent_prefill": (_i, [_p, _i, _i, _p, _i, _p, _p, _p, _i, _p, _i, _p, _p, _p, _f, _i, _i, _i, _i, _i, _i, _i, _p, _z, _p]),
     "mlora_moe_route": (_i, [_p, _p, _p, _i, _p, _f, _i, _i, _i, _p]),
     "mlora_moe_tile_rows": (_i, [_i, _i, _i]),
     "mlora_moe_max_tiles": (_i, [_i, _i, _i]),
@@ -134,6 +138,10 @@ DECODER_SIGNATURES = {
     "mlora_moe_linear": (_i, [_p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _f, _p]),
     "mlora_moe_combine": (_i, [_p, _p, _p, _i, _i, _i, _p]),
 }
+
+# ... and those that the fp32 library does not have
+MATRIX_CORE_ONLY = ("mlora_token_gate", "mlora_latent_prefill", "mlora_latent_prefill_tile_tokens", "mlora_latent_prefill_served",
+                    "mlora_latent_prefill_scratch_elems")
 
 _libs = {}
 
@@ -155,7 +163,7 @@ def lib(dtype: str = "float16") -> C.CDLL:
         l = C.CDLL(path)
         table = SIGNATURES if dtype == "float16" else {**{n: v for n, v in SIGNATURES.items() if hasattr(l, n)}, **DECODER_SIGNATURES}
         if dtype == "float32":
-            table.pop("mlora_token_gate")              # a matrix-core kernel
+            table = {n: v for n, v in table.items() if n not in MATRIX_CORE_ONLY}
         for name, (res, args) in table.items():
             fn = getattr(l, name)
             fn.restype = res

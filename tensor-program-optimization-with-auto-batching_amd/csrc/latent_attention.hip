@@ -9,6 +9,8 @@
 // latent takes the first RB = ceil(kv_rank / 32) blocks, the rotated part the following ones, padding is zero.
 // There is no second copy for the values: the matrix cores transpose a page's fragments by a product with the identity.
 // Query rows: [T, H, NB * 32] in the same order.
+#include <type_traits>
+
 #include "common.h"
 
 namespace {
@@ -32,30 +34,31 @@ struct LatentPrep {
   const float* cos;         // [max_pos, rot / 2]
   const float* sin;
   int max_pos, H, R, rot, RB, NB;
-  elt* q;                   // [T, H, NB * 32]: the rotated part is written here
+  elt* q;                   // the rotated query parts: row (t, h) at (t H + h) q_ld + q_off, padded to whole blocks
+  int q_ld, q_off;
 };
 
-// One workgroup per token: rotates the heads' query parts into the query rows, norms the latent, rotates the shared key
-// part and stores both in the token's page slot.  Neighbouring elements (2 i, 2 i + 1) turn by the table's angle i.
+// One workgroup per token: rotates the heads' query parts into the query rows (their `gain` is left to the scores' scale),
+// norms the latent, rotates the shared key part and stores both in the token's page slot.  Neighbouring elements (2 i, 2 i + 1) turn by the table's angle i.
 __global__ __launch_bounds__(256) void latent_prep_kernel(LatentPrep a) {
   __shared__ float red[4];
   const int t = blockIdx.x;
   const int seq = a.tok_seq[t], pos = a.tok_pos[t];
   if (seq < 0 || seq >= a.n_seq || pos < 0 || pos >= a.max_pos || pos / PAGE >= a.max_blocks) return;   // uniform
   const elt* row = a.qkv + (size_t)t * a.ld;
-  const int half = a.rot / 2, qd = a.NB * 32, rp = (a.NB - a.RB) * 32;
+  const int half = a.rot / 2, rp = (a.NB - a.RB) * 32;
   const float* cp = a.cos + (size_t)pos * half;
   const float* sp = a.sin + (size_t)pos * half;
-  elt* q = a.q + (size_t)t * a.H * qd + a.RB * 32;
+  elt* q = a.q + (size_t)t * a.H * a.q_ld + a.q_off;
   for (int i = threadIdx.x; i < a.H * (rp / 2); i += 256) {
     const int h = i / (rp / 2), k = i - h * (rp / 2);
     float u = 0.f, v = 0.f;
     if (k < half) {
-      const float x1 = (float)row[a.off_rot + h * a.rot + 2 * k] * a.gain, x2 = (float)row[a.off_rot + h * a.rot + 2 * k + 1] * a.gain;
+      const float x1 = (float)row[a.off_rot + h * a.rot + 2 * k], x2 = (float)row[a.off_rot + h * a.rot + 2 * k + 1];
       u = x1 * cp[k] - x2 * sp[k];
       v = x2 * cp[k] + x1 * sp[k];
     }
-    *reinterpret_cast<eltx2*>(q + (size_t)h * qd + 2 * k) = eltx2{(elt)u, (elt)v};
+    *reinterpret_cast<eltx2*>(q + (size_t)h * a.q_ld + 2 * k) = eltx2{(elt)u, (elt)v};
   }
   if (!a.c_norm) return;
   const int page = a.block_table[(size_t)seq * a.max_blocks + pos / PAGE];
@@ -273,6 +276,293 @@ __global__ __launch_bounds__(128) void latent_merge_kernel(LatentAttn a) {
   }
 }
 
+// ---------------------------------------------------------------------------------------------
+// Prompts: with many queries per key it is cheaper to make the heads' keys and values once than to work on the latents
+// (dim + rot_dim + vdim products per score instead of 2 kv_rank + rot_dim).  The keys and values of the contexts of a pass are
+// written to scratch memory in the order the matrix cores read them, one context after the other, each padded to whole
+// blocks of 64 keys with zeros:
+//   K [H, pages, KN, 512]      a page's fragments (16 tokens x 32 dims), as in a cache page
+//   V [H, pages / 2, VB, 512]  16 dims x 32 tokens: lane (dim % 16, g) holds tokens 4 g .. + 3 of the even, then of the odd page
+//   R [pages, KR, 512]         the rotated key part, shared by the heads
+// ---------------------------------------------------------------------------------------------
+struct LatentExpand {
+  elt* k;
+  elt* v;
+  elt* r;
+  const elt* cache;
+  const int32_t* phys;      // [pages] cache page of a scratch page, -1: padding
+  const elt* uk;            // packed [H * KN * 32, RB * 32]
+  const elt* uv;            // packed [H * VB * 16, RB * 32]
+  int pages, n_pages, H, RB, KR, KN, VB;
+  int kb_blocks, vb_blocks; // workgroups along x that make keys, then values; one more copies R
+};
+
+// a wave makes 64 rows (of W_uk or W_uv) x 4 pages
+__global__ __launch_bounds__(256) void latent_expand_kernel(LatentExpand a) {
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
+  const int pg0 = blockIdx.y * 4, NB = a.RB + a.KR;
+  int page[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    page[j] = a.phys[pg0 + j];
+    if (page[j] >= a.n_pages) page[j] = -1;
+  }
+  const eltx8 zero = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
+  int bx = blockIdx.x;
+  if (bx >= a.kb_blocks + a.vb_blocks) {
+    for (int i = threadIdx.x; i < 4 * a.KR * 64; i += 256) {
+      const int j = i / (a.KR * 64), o = i - j * (a.KR * 64);
+      const int pj = a.phys[pg0 + j];
+      st8(a.r + ((size_t)(pg0 + j) * a.KR * 64 + o) * 8,
+          pj >= 0 && pj < a.n_pages ? ld8(a.cache + (size_t)pj * NB * 512 + a.RB * 512 + o * 8) : zero);
+    }
+    return;
+  }
+  const bool val = bx >= a.kb_blocks;                                // uniform
+  if (val) bx -= a.kb_blocks;
+  const int tiles = val ? a.H * a.VB : a.H * a.KN * 2;
+  const int nt0 = (bx * 4 + wave) * 4;
+  if (nt0 >= tiles) return;
+  const elt* wp[4];
+  const elt* cp[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    wp[i] = (val ? a.uv : a.uk) + (size_t)(nt0 + i < tiles ? nt0 + i : tiles - 1) * a.RB * 512 + lane * 8;
+    cp[i] = a.cache + (size_t)(page[i] >= 0 ? page[i] : 0) * NB * 512 + lane * 8;
+  }
+  f32x4 acc[4][4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+  auto products = [&](auto V) {
+    eltx8 w[4], c[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      w[i] = ld8(wp[i]);
+      c[i] = ld8(cp[i]);
+    }
+    for (int kb = 1; kb <= a.RB; ++kb) {
+      const int kc = kb < a.RB ? kb : 0;                             // the last prefetch wraps to a valid address and is discarded
+      eltx8 wn[4], cn[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        wn[i] = ld8(wp[i] + kc * 512);
+        cn[i] = ld8(cp[i] + kc * 512);
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[i][j] = decltype(V)::value ? mfma_16x16x32(c[j], w[i], acc[i][j]) : mfma_16x16x32(w[i], c[j], acc[i][j]);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        w[i] = wn[i];
+        c[i] = cn[i];
+      }
+    }
+  };
+  if (val) products(std::true_type());
+  else products(std::false_type());
+  const int r16 = lane & 15, g = lane >> 4;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int nt = nt0 + i;
+    if (nt >= tiles) continue;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const f32x4 s = page[j] >= 0 ? acc[i][j] : f32x4{0.f, 0.f, 0.f, 0.f};
+      const eltx4 o = eltx4{(elt)s[0], (elt)s[1], (elt)s[2], (elt)s[3]};
+      if (val) {                                                     // s[r] = token 4 g + r, dim r16 of the tile
+        const int h = nt / a.VB, db = nt - h * a.VB, p = pg0 + j;
+        *reinterpret_cast<eltx4*>(a.v + (((size_t)h * (a.pages / 2) + p / 2) * a.VB + db) * 512 + lane * 8 + (p & 1) * 4) = o;
+      } else {                                                       // s[r] = dim 4 g + r of the tile, token r16
+        const int h = nt / (2 * a.KN), d = (nt - h * 2 * a.KN) * 16 + g * 4;
+        *reinterpret_cast<eltx4*>(a.k + (((size_t)h * a.pages + pg0 + j) * a.KN + (d >> 5)) * 512 + ((d >> 3) & 3) * 128 + r16 * 8 + (d & 7)) = o;
+      }
+    }
+  }
+}
+
+struct LatentPrefill {
+  elt* out;                 // [T, H * VB * 16], row-major (frag_tt == 0: row stride ld_out) or in fragment order
+  int frag_tt, ld_out;
+  const elt* q;             // [T, ld_q]: the heads' unrotated query parts at h * KN * 32
+  int ld_q;
+  const elt* qr;            // [T, H, KR * 32]: their rotated parts
+  const elt* k;
+  const elt* v;
+  const elt* r;
+  const int4* tiles;        // {first token, tokens, first scratch page, position of the first token}, long key ranges first
+  const float* sink;
+  float scale;
+  int H, pages, KN, KR, VB;
+};
+
+// Four waves own up to 128 consecutive queries of one head of one sequence, a wave 32 of them as two 16-query tiles.  Keys are
+// walked in blocks of 64: K and V go from scratch memory straight into LDS, double buffered, one bare barrier per block.
+// S^T = K . Q^T, softmax state per lane (its own query column), O^T += V^T . P^T with P as hi + lo halves.
+// KB = KN + KR and VB bound the register arrays; EXACT: they are the sizes themselves.
+constexpr int LP_WAVES = 4;
+constexpr int LP_QT = 2;
+constexpr int LP_TOK = LP_WAVES * LP_QT * 16;
+template <int KB_, int VB_, bool EXACT>
+__global__ __launch_bounds__(LP_WAVES* WAVE, 2) void latent_prefill_kernel(LatentPrefill a) {
+  extern __shared__ __align__(16) elt lsm[];                         // [2][4 KB + 2 VB][512]
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
+  const int qi = lane & 15, g = lane >> 4;
+  const int KN = a.KN, KR = a.KR, KB = EXACT ? KB_ : KN + KR, VB = EXACT ? VB_ : a.VB;
+  const int PIECES = 4 * KB + 2 * VB;                                // 1 KiB pieces of a key block
+  const int h = blockIdx.x;
+  const int4 tile = a.tiles[blockIdx.y];
+  const int wq = wave * LP_QT * 16;                                  // this wave's first query of the tile
+  eltx8 qf[LP_QT][KB_];
+#pragma unroll
+  for (int u = 0; u < LP_QT; ++u) {
+    const int i = wq + u * 16 + qi;
+    const size_t t = tile.x + (i < tile.y ? i : tile.y - 1);
+#pragma unroll
+    for (int kb = 0; kb < KB_; ++kb) {
+      qf[u][kb] = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
+      if (kb < KB) qf[u][kb] = kb < KN ? ld8(a.q + t * a.ld_q + (h * KN + kb) * 32 + g * 8) : ld8(a.qr + (t * a.H + h) * (KR * 32) + (kb - KN) * 32 + g * 8);
+    }
+  }
+  const float c2 = a.scale * 1.44269504088896340736f;                // softmax in base 2
+  float m[LP_QT], l[LP_QT];
+  f32x4 O[LP_QT][VB_];
+#pragma unroll
+  for (int u = 0; u < LP_QT; ++u) {
+    m[u] = -INFINITY;
+    l[u] = 0.f;
+#pragma unroll
+    for (int db = 0; db < VB_; ++db) O[u][db] = f32x4{0.f, 0.f, 0.f, 0.f};
+  }
+  const int last = tile.w + tile.y - 1;                              // position of the tile's last query
+  const int nblk = last / 64 + 1;
+  const elt* kh = a.k + ((size_t)h * a.pages + tile.z) * KN * 512 + lane * 8;
+  const elt* vh = a.v + ((size_t)h * (a.pages / 2) + tile.z / 2) * VB * 512 + lane * 8;
+  const elt* rh = a.r + (size_t)tile.z * KR * 512 + lane * 8;
+  // piece i of a block: page p = i / KB, fragment i % KB of it for i < 4 KB; then the pairs' V pieces
+  auto issue = [&](int b) {
+    elt* dst = lsm + (b & 1) * PIECES * 512;
+    for (int i = wave; i < PIECES; i += LP_WAVES) {                  // uniform
+      const elt* src;
+      if (i < 4 * KB) {
+        const int p = i / KB, f = i - p * KB;
+        src = f < KN ? kh + ((size_t)(4 * b + p) * KN + f) * 512 : rh + ((size_t)(4 * b + p) * KR + f - KN) * 512;
+      } else {
+        src = vh + ((size_t)(2 * b) * VB + i - 4 * KB) * 512;
+      }
+      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)src,
+                                       (__attribute__((address_space(3))) void*)(dst + i * 512), 16, 0, 0);
+    }
+  };
+  issue(0);
+  for (int b = 0; b < nblk; ++b) {
+    asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");      // this wave's pieces of block b have landed, its reads of b - 1 are done
+    bare_barrier();
+    if (b + 1 < nblk) issue(b + 1);                                  // into the buffer of block b - 1
+    const elt* ks = lsm + (b & 1) * PIECES * 512 + lane * 8;
+    const elt* vs = ks + 4 * KB * 512;
+    bool act[LP_QT];                                                 // uniform: the 16-query tile exists and reaches the block
+#pragma unroll
+    for (int u = 0; u < LP_QT; ++u) {
+      const int i1 = wq + u * 16 + 15 < tile.y - 1 ? wq + u * 16 + 15 : tile.y - 1;
+      act[u] = wq + u * 16 < tile.y && tile.w + i1 >= b * 64;
+    }
+    if (!act[0] && !act[1]) continue;
+    f32x4 st[LP_QT][4];                                              // st[u][p][r] = S[key 4 g + r of page p][query qi of tile u]
+#pragma unroll
+    for (int p = 0; p < 4; ++p) {
+#pragma unroll
+      for (int u = 0; u < LP_QT; ++u) st[u][p] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int kb = 0; kb < KB_; ++kb) {
+        if (EXACT || kb < KB) {
+          const eltx8 kf = ld8(ks + (p * KB + kb) * 512);
+#pragma unroll
+          for (int u = 0; u < LP_QT; ++u) st[u][p] = mfma_16x16x32(kf, qf[u][kb], st[u][p]);
+        }
+      }
+    }
+    eltx8 ph[LP_QT][2], pl[LP_QT][2];
+#pragma unroll
+    for (int u = 0; u < LP_QT; ++u) {
+      const int lim = tile.w + wq + u * 16 + qi - b * 64 - 4 * g;    // key (p, r) of this lane is visible while 16 p + r <= lim
+      float pm = -INFINITY;
+#pragma unroll
+      for (int p = 0; p < 4; ++p) st[u][p] *= c2;
+      if (tile.w + wq + u * 16 < b * 64 + 63) {                      // uniform: the block crosses the tile's diagonal
+#pragma unroll
+        for (int p = 0; p < 4; ++p)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) st[u][p][r] = p * 16 + r <= lim ? st[u][p][r] : -INFINITY;
+      }
+#pragma unroll
+      for (int p = 0; p < 4; ++p)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) pm = fmaxf(pm, st[u][p][r]);
+      pm = fmaxf(pm, __shfl_xor(pm, 16, WAVE));
+      pm = fmaxf(pm, __shfl_xor(pm, 32, WAVE));
+      const float mn = fmaxf(m[u], pm);
+      if (__any(mn > m[u])) {                                        // uniform
+        const float alpha = m[u] == -INFINITY ? 0.f : exp2f(m[u] - mn);
+        l[u] *= alpha;
+#pragma unroll
+        for (int db = 0; db < VB_; ++db) O[u][db] *= alpha;
+        m[u] = mn;
+      }
+      const float mm = mn == -INFINITY ? 0.f : mn;                   // a query that sees nothing of this block yet (m stays -inf)
+      float ps = 0.f;
+#pragma unroll
+      for (int p = 0; p < 4; ++p)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const float e = __builtin_amdgcn_exp2f(st[u][p][r] - mm);
+          ps += e;
+          const elt hi = (elt)e;
+          ph[u][p >> 1][(p & 1) * 4 + r] = hi;
+          pl[u][p >> 1][(p & 1) * 4 + r] = (elt)(e - (float)hi);
+        }
+      l[u] += ps;
+    }
+#pragma unroll
+    for (int j = 0; j < 2; ++j)
+#pragma unroll
+      for (int db = 0; db < VB_; ++db) {
+        if (EXACT || db < VB) {
+          const eltx8 vf = ld8(vs + (j * VB + db) * 512);
+#pragma unroll
+          for (int u = 0; u < LP_QT; ++u) {
+            O[u][db] = mfma_16x16x32(vf, ph[u][j], O[u][db]);
+            O[u][db] = mfma_16x16x32(vf, pl[u][j], O[u][db]);        // O^T[dim 16 db + 4 g + r][query qi of tile u]
+          }
+        }
+      }
+  }
+  const float sk = a.sink ? a.sink[h] * 1.44269504088896340736f : -INFINITY;
+#pragma unroll
+  for (int u = 0; u < LP_QT; ++u) {
+    float L = l[u];
+    L += __shfl_xor(L, 16, WAVE);
+    L += __shfl_xor(L, 32, WAVE);
+    const int i = wq + u * 16 + qi;
+    if (i >= tile.y) continue;
+    const float M = fmaxf(m[u], sk);
+    const float f = exp2f(m[u] - M);
+    const float inv = f / (L * f + (sk == -INFINITY ? 0.f : exp2f(sk - M)));
+    const int t = tile.x + i;
+#pragma unroll
+    for (int db = 0; db < VB_; ++db) {
+      if (EXACT || db < VB) {
+        const int col = (h * VB + db) * 16 + 4 * g;
+        elt* p = a.frag_tt ? a.out + frag_offset(t, col, a.frag_tt) : a.out + (size_t)t * a.ld_out + col;
+        *reinterpret_cast<eltx4*>(p) =
+            eltx4{(elt)(O[u][db][0] * inv), (elt)(O[u][db][1] * inv), (elt)(O[u][db][2] * inv), (elt)(O[u][db][3] * inv)};
+      }
+    }
+  }
+}
+
 // y[t, h] = alpha * W[h] . x[t, h] per head: W[h] packed [N, K], N % 16 == 0.  A wave owns 16 NI rows x 16 TJ tokens.
 template <int NI, int TJ>
 __global__ __launch_bounds__(256) void head_linear_kernel(elt* __restrict__ y, long ldy, long hy, int frag_tt, const elt* __restrict__ x, long ldx,
@@ -404,7 +694,7 @@ int launch_latent_attn(const LatentAttn& a, hipStream_t s) {
 
 }  // namespace
 
-extern "C" int mlora_latent_prep(void* q, void* cache, const void* qkv, int ld, int off_rot, int off_c, int off_kr, float gain, const void* c_norm,
+extern "C" int mlora_latent_prep(void* q, int q_ld, int q_off, void* cache, const void* qkv, int ld, int off_rot, int off_c, int off_kr, float gain, const void* c_norm,
                                  float eps, const int32_t* block_table, int max_blocks, const int32_t* tok_seq, const int32_t* tok_pos,
                                  const float* rope_cos, const float* rope_sin, int max_pos, int T, int H, int R, int rot, int n_pages, int n_seq,
                                  void* stream) {
@@ -418,6 +708,9 @@ extern "C" int mlora_latent_prep(void* q, void* cache, const void* qkv, int ld, 
   a.c_norm = (const elt*)c_norm; a.cache = (elt*)cache; a.block_table = block_table; a.max_blocks = max_blocks; a.n_pages = n_pages;
   a.n_seq = n_seq; a.tok_seq = tok_seq; a.tok_pos = tok_pos; a.cos = rope_cos; a.sin = rope_sin; a.max_pos = max_pos;
   a.H = H; a.R = R; a.rot = rot; a.RB = ceil_div(R, 32); a.NB = a.RB + ceil_div(rot, 32); a.q = (elt*)q;
+  a.q_ld = q_ld; a.q_off = q_off;
+  MLORA_CHECK(q_off >= 0 && q_off % 2 == 0 && q_ld % 2 == 0 && q_off + (a.NB - a.RB) * 32 <= q_ld, MLORA_ERR_INVALID,
+              "latent_prep: query rows of %d with the rotated part at %d", q_ld, q_off);
   hipLaunchKernelGGL(latent_prep_kernel, dim3(T), dim3(256), 0, (hipStream_t)stream, a);
   return mlora_launch_status("latent_prep");
 }
@@ -501,5 +794,64 @@ extern "C" int mlora_head_linear(void* y, int y_layout, long ldy, long head_y, c
   else MLORA_HL(4, 4);
 #undef MLORA_HL
   return mlora_launch_status("head_linear");
+}
+#endif
+
+#ifndef MLORA_ELT_F32
+template <int KB, int VB, bool EXACT>
+static int launch_latent_prefill(const LatentPrefill& a, int n_tiles, hipStream_t s) {
+  constexpr size_t cap = (size_t)2 * (4 * KB + 2 * VB) * 512 * sizeof(elt);
+  static const hipError_t configured =               // the attribute is per kernel, set once per process, by one thread
+      hipFuncSetAttribute((const void*)latent_prefill_kernel<KB, VB, EXACT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)cap);
+  if (configured != hipSuccess) return mlora_set_error(MLORA_ERR_LAUNCH, "latent_prefill: cannot reserve %zu bytes of LDS", cap);
+  const size_t lds = (size_t)2 * (4 * (a.KN + a.KR) + 2 * a.VB) * 512 * sizeof(elt);
+  hipLaunchKernelGGL((latent_prefill_kernel<KB, VB, EXACT>), dim3(a.H, n_tiles), dim3(LP_WAVES * WAVE), lds, s, a);
+  return MLORA_OK;
+}
+
+extern "C" int mlora_latent_prefill_tile_tokens(void) { return LP_TOK; }
+
+extern "C" int mlora_latent_prefill_served(int dim, int rot, int vdim) {
+  return dim > 0 && rot > 0 && vdim > 0 && ceil_div(dim, 32) + ceil_div(rot, 32) <= 6 && ceil_div(vdim, 32) <= 4;
+}
+
+// elements of scratch memory for `pages` scratch pages
+extern "C" size_t mlora_latent_prefill_scratch_elems(int pages, int H, int dim, int rot, int vdim) {
+  if (pages <= 0 || H <= 0) return 0;
+  return (size_t)pages * 512 * ((size_t)H * (ceil_div(dim, 32) + ceil_div(vdim, 32)) + ceil_div(rot, 32));
+}
+
+extern "C" int mlora_latent_prefill(void* out, int out_layout, int ld_out, const void* q, int ld_q, const void* q_rot, const void* cache,
+                                    const int32_t* phys, int pages, const int32_t* tiles, int n_tiles, const void* uk, const void* uv,
+                                    const float* sink, float scale, int T, int H, int R, int dim, int rot, int vdim, int n_pages, void* scratch,
+                                    size_t scratch_elems, void* stream) {
+  MLORA_CHECK(out && q && q_rot && cache && phys && tiles && uk && uv && scratch, MLORA_ERR_INVALID, "latent_prefill: null pointer");
+  MLORA_CHECK(mlora_latent_prefill_served(dim, rot, vdim) && H > 0 && H <= 65535 && R > 0 && n_pages > 0, MLORA_ERR_UNSUPPORTED,
+              "latent_prefill: dim=%d rot=%d vdim=%d not served", dim, rot, vdim);
+  MLORA_CHECK(pages > 0 && pages % 4 == 0 && pages / 4 <= 65535 && n_tiles > 0 && n_tiles <= 65535 && T > 0 && ld_q % 8 == 0 &&
+                  (((uintptr_t)q | (uintptr_t)q_rot | (uintptr_t)scratch | (uintptr_t)tiles) & 15) == 0,
+              MLORA_ERR_UNSUPPORTED, "latent_prefill: pages=%d must be a multiple of 4, operands aligned", pages);
+  MLORA_CHECK(scratch_elems >= mlora_latent_prefill_scratch_elems(pages, H, dim, rot, vdim), MLORA_ERR_WORKSPACE, "latent_prefill: scratch too small");
+  LatentExpand e;
+  e.KN = ceil_div(dim, 32); e.KR = ceil_div(rot, 32); e.VB = ceil_div(vdim, 32) * 2; e.RB = ceil_div(R, 32);
+  e.H = H; e.pages = pages; e.n_pages = n_pages;
+  e.k = (elt*)scratch;
+  e.v = e.k + (size_t)H * pages * e.KN * 512;
+  e.r = e.v + (size_t)H * (pages / 2) * e.VB * 512;
+  e.cache = (const elt*)cache; e.phys = phys; e.uk = (const elt*)uk; e.uv = (const elt*)uv;
+  e.kb_blocks = ceil_div(H * e.KN * 2, 16);
+  e.vb_blocks = ceil_div(H * e.VB, 16);
+  hipStream_t s = (hipStream_t)stream;
+  hipLaunchKernelGGL(latent_expand_kernel, dim3(e.kb_blocks + e.vb_blocks + 1, pages / 4), dim3(256), 0, s, e);
+  LatentPrefill a;
+  a.out = (elt*)out; a.frag_tt = out_layout == MLORA_FRAG ? mlora_frag_tiles(T) : 0; a.ld_out = ld_out;
+  a.q = (const elt*)q; a.ld_q = ld_q; a.qr = (const elt*)q_rot; a.k = e.k; a.v = e.v; a.r = e.r; a.tiles = (const int4*)tiles;
+  a.sink = sink; a.scale = scale; a.H = H; a.pages = pages; a.KN = e.KN; a.KR = e.KR; a.VB = e.VB;
+  const int KB = e.KN + e.KR;
+  int rc;
+  if (KB == 6 && e.VB == 8) rc = launch_latent_prefill<6, 8, true>(a, n_tiles, s);
+  else if (KB <= 3 && e.VB <= 4) rc = launch_latent_prefill<3, 4, false>(a, n_tiles, s);
+  else rc = launch_latent_prefill<6, 8, false>(a, n_tiles, s);
+  return rc ? rc : mlora_launch_status("latent_prefill");
 }
 #endif

@@ -114,13 +114,53 @@ def head_linear(x, ldx, head_x, W, heads, T, K, N, out, ldy, head_y, alpha=1.0):
     return out
 
 
-def latent_prep(q, pages, qkv, off_rot, off_c, off_kr, gain, c_norm, eps, block_table, tok_seq, tok_pos, cos, sin, H, R, rot):
+def latent_prep(q, q_off, pages, qkv, off_rot, off_c, off_kr, gain, c_norm, eps, block_table, tok_seq, tok_pos, cos, sin, H, R, rot):
+    """Rotates the query parts of qkv into q [T, H, q_ld] at column q_off and stores latent and key part (c_norm given)."""
     n_seq, max_blocks = block_table.shape
     T, ld = qkv.shape
-    check(lib_of(qkv.dtype).mlora_latent_prep(_dev(q, qkv.dtype), _dev(pages, qkv.dtype), _dev(qkv), ld, off_rot, off_c, off_kr, gain, _ptr(c_norm),
-                                              eps, _dev(block_table, torch.int32), max_blocks, _dev(tok_seq, torch.int32),
+    check(lib_of(qkv.dtype).mlora_latent_prep(_dev(q, qkv.dtype), q.shape[2], q_off, _dev(pages, qkv.dtype), _dev(qkv), ld, off_rot, off_c, off_kr,
+                                              gain, _ptr(c_norm), eps, _dev(block_table, torch.int32), max_blocks, _dev(tok_seq, torch.int32),
                                               _dev(tok_pos, torch.int32), _dev(cos, torch.float32), _dev(sin, torch.float32), cos.shape[0], T, H, R,
                                               rot, pages.shape[0], n_seq, _stream()), qkv.dtype)
+
+
+class PrefillPlan:
+    """Contexts and query tiles of a pass for `latent_prefill`: per sequence (cache pages of its whole context, tokens that
+    the pass appends, context length after it), in pass order."""
+
+    def __init__(self, seqs, device):
+        L = lib_of(torch.bfloat16)
+        n = L.mlora_latent_prefill_tile_tokens()
+        phys, tiles, t0 = [], [], 0
+        for pages, new, ctx in seqs:
+            base = len(phys)
+            used = -(-ctx // 16)
+            phys += list(pages[:used]) + [-1] * (-used % 4)
+            tiles += [(t0 + i, min(n, new - i), base, ctx - new + i) for i in range(0, new, n)]
+            t0 += new
+        tiles.sort(key=lambda t: -(t[1] + t[3]))                     # the longest key ranges start first
+        self.T, self.pages, self.n_tiles = t0, len(phys), len(tiles)
+        both = torch.tensor([x for t in tiles for x in t] + phys, dtype=torch.int32).to(device)
+        self.tiles, self.phys = both[: 4 * len(tiles)], both[4 * len(tiles):]
+
+
+def latent_prefill_served(dim, rot, vdim) -> bool:
+    return bool(lib_of(torch.bfloat16).mlora_latent_prefill_served(dim, rot, vdim))
+
+
+def latent_prefill(plan, q, q_rot, pages, uk, uv, sink, scale, R, dim, rot, vdim, out):
+    """Attention of a pass over keys and values made from the latents; q [T, ld] (unrotated query parts, each padded to 32
+    columns), q_rot [T, H, pad32(rot)]; out: FragActivation or tensor [T, H * pad32(vdim)]."""
+    T, H, _ = q_rot.shape
+    L = lib_of(q.dtype)
+    n = L.mlora_latent_prefill_scratch_elems(plan.pages, H, dim, rot, vdim)
+    scratch = torch.empty(n, dtype=q.dtype, device=q.device)
+    frag = isinstance(out, FragActivation)
+    check(L.mlora_latent_prefill(out.data.data_ptr() if frag else _dev(out, q.dtype), FRAG if frag else ROWMAJOR, out.shape[1], _dev(q), q.shape[1],
+                                 _dev(q_rot, q.dtype), _dev(pages, q.dtype), plan.phys.data_ptr(), plan.pages, plan.tiles.data_ptr(), plan.n_tiles,
+                                 _wptr(uk), _wptr(uv), _ptr(sink), scale, T, H, R, dim, rot, vdim, pages.shape[0], scratch.data_ptr(), n, _stream()),
+          q.dtype)
+    return out
 
 
 def latent_attn(q, pages, block_table, tok_seq, tok_pos, sink, scale, R, rot, max_ctx, out=None, splits=None):

@@ -19,6 +19,7 @@ import numpy as np
 import torch
 
 from . import ops
+from .decoder_ops import PrefillPlan
 
 PAGE = 16
 
@@ -186,6 +187,7 @@ class PagedLatentCache(PageTable):
             if key not in tables:
                 tables[key] = tuple(torch.from_numpy(t).to(self.device) for t in rotation.tables(rot_dim, max_pos))
             self.rope.append(tables[key])
+        self._plan = None
 
     def latents(self, layer, sid):
         """The cached vectors [length, blocks * 32] of a sequence (a copy, for inspection)."""
@@ -199,7 +201,12 @@ class PagedLatentCache(PageTable):
         columns)."""
         if self._cur is None:
             raise RuntimeError("latent_attention outside begin_forward/end_forward")
-        seq_ids, append_lens, _, tok_seq, tok_pos, _ = self._cur
-        max_ctx = max(self.lens[s] + n for s, n in zip(seq_ids, append_lens))
-        return att.attend(qkv, self.pages[layer], self.block_table, tok_seq, tok_pos, *self.rope[layer], max_ctx=max_ctx,
-                          store=self.owner[layer] == layer, out=out)
+        seq_ids, append_lens, decode, tok_seq, tok_pos, _ = self._cur
+        ctx = [self.lens[s] + n for s, n in zip(seq_ids, append_lens)]
+        plan = None
+        if not decode and att.prompt_form_pays(list(zip(append_lens, ctx))):
+            if self._plan is None or self._plan[0] is not self._cur:         # one plan per pass serves all its layers
+                self._plan = (self._cur, PrefillPlan([(self.pages_of(s), n, c) for s, n, c in zip(seq_ids, append_lens, ctx)], self.device))
+            plan = self._plan[1]
+        return att.attend(qkv, self.pages[layer], self.block_table, tok_seq, tok_pos, *self.rope[layer], max_ctx=max(ctx),
+                          store=self.owner[layer] == layer, plan=plan, out=out)

@@ -92,6 +92,26 @@ def test_portions_and_token_by_token(sizes, dt):
     assert agrees(got, want, dt)
 
 
+@pytest.mark.parametrize("name", list(C.CONFIGS))
+@pytest.mark.parametrize("prompt_form", [True, False])
+def test_both_forms_of_the_attention(name, prompt_form, monkeypatch):
+    """The prompt form and the lifted form, each forced for all passes that are no decode steps, portions and batches included."""
+    cfg = C.CONFIGS[name]
+    P, m = build(cfg, B16, 9, sharp=2.0)
+    att = load_pkg("latent_attention").LatentAttention
+    calls = []
+    monkeypatch.setattr(att, "prompt_form_pays", lambda self, seqs: calls.append(prompt_form and self.uk is not None) or calls[-1])
+    a, b = toks(cfg, 150, 1), toks(cfg, 77, 2)
+    kv = cache(m, free_pages=list(np.random.default_rng(0).permutation(40)))
+    ga = [run(m, kv, [("a", a[:50])])[0]]
+    x, y = run(m, kv, [("b", b[:70]), ("a", a[50:149])])
+    ga.append(y)
+    gb = [x] + [run(m, kv, [("b", b[i:j])])[0] for i, j in ((70, 72), (72, 77))]
+    ga.append(run(m, kv, [("a", a[149:])])[0])
+    assert any(calls) == prompt_form
+    assert agrees(np.concatenate(ga), R.forward(a, cfg, P), B16) and agrees(np.concatenate(gb), R.forward(b, cfg, P), B16)
+
+
 @pytest.mark.parametrize("dt", [F32, B16])
 def test_batches_of_unequal_requests(dt):
     cfg = C.CONFIGS["odd"]

@@ -91,7 +91,7 @@ def test_decoder_header_and_libraries_agree():
         b.ensure(dt)
         lib = ctypes.CDLL(lm.LIB_PATHS[dt])
         missing = [n for n in names if not hasattr(lib, n)]
-        assert missing == ([] if dt == "bfloat16" else ["mlora_token_gate"])
+        assert missing == ([] if dt == "bfloat16" else sorted(lm.MATRIX_CORE_ONLY))
 
 
 def test_decoder_argument_validation():
@@ -113,6 +113,9 @@ def test_decoder_argument_validation():
         for T, E, top in ((1, 6, 2), (40, 6, 2), (1000, 64, 8)):
             rows = lib.mlora_moe_tile_rows(T, E, top)
             assert lib.mlora_moe_max_tiles(T, E, top) >= -(-T * top // rows)
+    lp = lambda pages=4, dim=64, elems=1 << 30, sc=16: b.mlora_latent_prefill(16, 0, 64, 16, 64, 16, 16, 16, pages, 16, 1, 16, 16, None, 0.1, 8, 2, 64, dim, 16,
+                                                                              64, 8, sc, elems, None)
+    assert lp(pages=5) == -2 and lp(dim=256) == -2 and lp(elems=8) == -3 and lp(sc=None) == -1
     assert b.mlora_moe_linear(16, 16, 16, 16, 16, 16, 32, 4, 4, 32, 32, 2, 0, 0, 1.0, None) == -2
 
 

@@ -205,6 +205,44 @@ def test_latent_attention_single_keys_far_and_at_page_borders(D, dt):
     assert err(got[..., :rank], attn_want(lat, q, [0] * len(toks), [p for _, p in toks], None, 1.0, rank)) < tol(dt, b16=6e-3)
 
 
+@pytest.mark.parametrize("H,rank,dim,rot,vdim", [(1, 32, 32, 8, 32), (3, 72, 40, 24, 48), (4, 512, 128, 64, 128), (2, 96, 100, 16, 64), (5, 64, 16, 40, 100)])
+@pytest.mark.parametrize("scale,layout", [(1.0, "frag"), (-0.7, "rows")])
+def test_latent_prefill(D, ops, H, rank, dim, rot, vdim, scale, layout):
+    """Keys and values made from the latents: whole prompts, portions in the middle of one, several sequences, scattered pages;
+    sharp scores, so that a key too many or too few shows."""
+    parts = [(200, 200), (5, 5), (130, 517), (1, 64), (33, 65), (2, 18)]          # (new tokens, context after them)
+    dt = torch.bfloat16
+    lat, pages, bt, rng = latent_case(D, dt, [c for _, c in parts], H, rank, rot, seed=H)
+    dp, vp, rp = D.pad32(dim), D.pad32(vdim), D.pad32(rank)
+    T = sum(n for n, _ in parts)
+    uk, uv = rnd(rng, H, dim, rank, std=2 * rank ** -0.5), rnd(rng, H, vdim, rank, std=rank ** -0.5)
+    qkv = torch.zeros((T, D.pad32(H * dp + 7)), dtype=dt, device=DEV)
+    qn = rnd(rng, T, H, dim)
+    qkv[:, : H * dp] = D.padded(qn, T, H, dp).reshape(T, H * dp).to(dt)
+    qr = rnd(rng, T, H, rot, std=0.5)
+    sink = rng.normal(1.0, 1.0, H).astype(np.float32)
+    pl = [[int(p) for p in bt[i + 1].tolist() if p >= 0] for i in range(len(parts))]
+    plan = D.PrefillPlan([(pl[i], n, c) for i, (n, c) in enumerate(parts)], DEV)
+    out = ops.FragActivation(T, H * vp, DEV, dtype=dt) if layout == "frag" else torch.empty((T, H * vp), dtype=dt, device=DEV)
+    D.latent_prefill(plan, qkv, D.padded(qr, T, H, D.pad32(rot)).to(dt), pages, D.weight(D.padded(uk, H, dp, rp).reshape(H * dp, rp).to(dt)),
+                     D.weight(D.padded(uv, H, vp, rp).reshape(H * vp, rp).to(dt)), torch.from_numpy(sink).to(DEV), scale, rank, dim, rot, vdim, out)
+    torch.cuda.synchronize()
+    got = f64(rows_of(out)).reshape(T, H, vp)
+    bf = lambda a: torch.from_numpy(a).to(dt).double().numpy()
+    want, t = np.zeros((T, H, vdim)), 0
+    for i, (n, c) in enumerate(parts):
+        for h in range(H):
+            k, v = bf(lat[i][:, :rank] @ f64(uk)[h].T), bf(lat[i][:, :rank] @ f64(uv)[h].T)   # stored in 16 bits
+            for j in range(n):
+                pos = c - n + j
+                s = (k[: pos + 1] @ f64(qn)[t + j, h] + lat[i][: pos + 1, rank:] @ f64(qr)[t + j, h]) * scale
+                want[t + j, h] = R.sink_softmax(s, sink[h]) @ v[: pos + 1]
+        t += n
+    # a key whose 16-bit rounding falls to the other side moves a sharp softmax a little
+    e = np.abs(got[..., :vdim] - want) / np.abs(want).max()
+    assert np.quantile(e, 0.999) < 1e-2 and e.max() < 6e-2 and np.abs(got[..., vdim:]).max(initial=0) == 0
+
+
 @pytest.mark.parametrize("dt", DTYPES)
 @pytest.mark.parametrize("scaling", [None, C.YARN])
 def test_latent_prep(D, dt, scaling):
@@ -223,15 +261,15 @@ def test_latent_prep(D, dt, scaling):
     q = torch.full((T, H, D.pad32(rank) + 32), 9.0, dtype=dt, device=DEV)
     off = H * dp
     before = pages.clone()
-    D.latent_prep(q, pages, qkv, off, off + H * rot, off + H * rot + rank, 1.25, None, 1e-5, bt, torch.from_numpy(seq).to(DEV), torch.from_numpy(pos).to(DEV),
+    D.latent_prep(q, D.pad32(rank), pages, qkv, off, off + H * rot, off + H * rot + rank, 1.25, None, 1e-5, bt, torch.from_numpy(seq).to(DEV), torch.from_numpy(pos).to(DEV),
                   cos, sin, H, rank, rot)
     torch.cuda.synchronize()
     assert torch.equal(pages, before)                     # a layer that reads another layer's latents stores nothing
-    D.latent_prep(q, pages, qkv, off, off + H * rot, off + H * rot + rank, 1.25, w, 1e-5, bt, torch.from_numpy(seq).to(DEV), torch.from_numpy(pos).to(DEV),
+    D.latent_prep(q, D.pad32(rank), pages, qkv, off, off + H * rot, off + H * rot + rank, 1.25, w, 1e-5, bt, torch.from_numpy(seq).to(DEV), torch.from_numpy(pos).to(DEV),
                   cos, sin, H, rank, rot)
     torch.cuda.synchronize()
     x = 1.25 * f64(qkv)
-    wq = R.rotate(x[:, off:off + H * rot].reshape(T, H, rot), pos, c)
+    wq = R.rotate(f64(qkv)[:, off:off + H * rot].reshape(T, H, rot), pos, c)     # the gain is left to the scores' scale
     assert err(q[..., D.pad32(rank):D.pad32(rank) + rot], wq) < tol(dt, b16=5e-3)
     assert float(q[..., D.pad32(rank) + rot:].abs().sum()) == 0 and bool((q[..., :D.pad32(rank)] == 9.0).all())
     cw = R.rms(x[:, off + H * rot:off + H * rot + rank], 1e-5) * f64(w)
