@@ -16,16 +16,16 @@ extern "C" {
 #endif
 
 /* Residual stream x [T, Hp] fp32 (columns H..Hp-1 zero): x += the n_part blocks part[q][T][Hp], in order; with a branch
- * x += branch / rms(branch) * branch_w; then, where an output is given, out = x / rms(x) * gain, rms over the H columns with
- * eps inside the root; in fragment order and / or row-major [T, Hp]. */
+ * x += branch / rms(branch) * branch_w; then, where an output is given, out = x / rms(x) * gain (with `raw`: x itself), rms
+ * over the H columns with eps inside the root; in fragment order and / or row-major [T, Hp]. */
 int mlora_stream_norm(void* out_frag, void* out_row, float* x, const float* part, int n_part, const float* branch, const void* branch_w,
-                      float eps, float gain, int T, int H, int Hp, void* stream);
+                      float eps, float gain, int raw, int T, int H, int Hp, void* stream);
 
 /* Per-layer token input: out[t, n] = gelu_tanh(W[n] . x[t]) * table[ids[t], col0 + n] for n < dim, 0 for dim <= n < N.
- * mlora_token_gate takes the residual stream (with pending partial sums, as above), W packed [N, K], and writes fragment
- * order; mlora_token_gate_mul takes the product z [T, N] of a separate linear. */
-int mlora_token_gate(void* out_frag, const float* x, const float* part, int n_part, const void* Wp, const void* table, int ld_table, int col0,
-                     int dim, const int32_t* ids, int V, int T, int K, int N, void* stream);
+ * mlora_token_gate takes x [T, K] and writes out in fragment order, W packed [N, K]; mlora_token_gate_mul takes the product
+ * z [T, N] of a separate linear, row-major. */
+int mlora_token_gate(void* out_frag, const void* xf, const void* Wp, const void* table, int ld_table, int col0, int dim, const int32_t* ids,
+                     int V, int T, int K, int N, void* stream);
 int mlora_token_gate_mul(void* out, const void* z, const void* table, int ld_table, int col0, int dim, const int32_t* ids, int V, int T, int N,
                          void* stream);
 
@@ -66,8 +66,8 @@ int mlora_latent_prefill(void* out, int out_layout, int ld_out, const void* q, i
  * over those.  mlora_moe_plan sorts the (token, choice) entries by expert into tiles {expert, first place, places, 0} of
  * mlora_moe_tile_rows places (at most mlora_moe_max_tiles of them).  mlora_moe_linear multiplies tile by tile with the
  * experts' weights (one [N, K] block each): stage UP reads token rows x [T, K] and writes place rows, stage DOWN reads place
- * rows and writes entry rows; `act` is applied to alpha times the product.  mlora_moe_combine: x[t] += sum over the
- * choices of weight * row. */
+ * rows and writes entry rows; `act` is applied to alpha times the product.  mlora_moe_combine: x[t] += the n_part blocks
+ * part[q][T][N], then the sum over the choices of weight * row; out_frag (or NULL): the result in fragment order. */
 #define MLORA_ACT_NONE  0
 #define MLORA_ACT_RELU2 1   /* max(v, 0)^2 */
 #define MLORA_MOE_UP    0
@@ -79,7 +79,8 @@ int mlora_moe_max_tiles(int T, int E, int top);
 int mlora_moe_plan(int32_t* perm, int32_t* tiles, int32_t* n_tiles, const int32_t* pick, int T, int E, int top, void* stream);
 int mlora_moe_linear(void* y, const void* x, const void* W, const int32_t* perm, const int32_t* tiles, const int32_t* n_tiles, int tile_rows,
                      int max_tiles, int T, int K, int N, int top, int stage, int act, float alpha, void* stream);
-int mlora_moe_combine(float* x, const void* y, const float* weight, int T, int top, int N, void* stream);
+int mlora_moe_combine(float* x, const float* part, int n_part, const void* y, const float* weight, int T, int top, int N, void* out_frag,
+                      void* stream);
 
 #ifdef __cplusplus
 }

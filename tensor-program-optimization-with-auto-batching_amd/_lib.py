@@ -119,8 +119,8 @@ SIGNATURES["mlora_decode_step"] = (_i, [C.POINTER(DecodePlan), _p])
 
 # mirrors include/mlora_decoder.h (the bfloat16 and fp32 libraries)
 DECODER_SIGNATURES = {
-    "mlora_stream_norm": (_i, [_p, _p, _p, _p, _i, _p, _p, _f, _f, _i, _i, _i, _p]),
-    "mlora_token_gate": (_i, [_p, _p, _p, _i, _p, _p, _i, _i, _i, _p, _i, _i, _i, _i, _p]),
+    "mlora_stream_norm": (_i, [_p, _p, _p, _p, _i, _p, _p, _f, _f, _i, _i, _i, _i, _p]),
+    "mlora_token_gate": (_i, [_p, _p, _p, _p, _i, _i, _i, _p, _i, _i, _i, _i, _p]),
     "mlora_token_gate_mul": (_i, [_p, _p, _p, _i, _i, _i, _p, _i, _i, _i, _p]),
     "mlora_latent_prep": (_i, [_p, _i, _i, _p, _p, _i, _i, _i, _i, _f, _p, _f, _p, _i, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _p]),
     "mlora_head_linear": (_i, [_p, _i, _l, _l, _p, _l, _l, _p, _i, _i, _i, _i, _f, _p]),
@@ -136,7 +136,7 @@ DECODER_SIGNATURES = {
     "mlora_moe_max_tiles": (_i, [_i, _i, _i]),
     "mlora_moe_plan": (_i, [_p, _p, _p, _p, _i, _i, _i, _p]),
     "mlora_moe_linear": (_i, [_p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _f, _p]),
-    "mlora_moe_combine": (_i, [_p, _p, _p, _i, _i, _i, _p]),
+    "mlora_moe_combine": (_i, [_p, _p, _i, _p, _p, _i, _i, _i, _p, _p]),
 }
 
 # ... and those that the fp32 library does not have

@@ -115,8 +115,9 @@ __device__ __forceinline__ int latent_ctx(const LatentAttn& a, int t, int& seq) 
 template <int NRB, int NW>
 __global__ __launch_bounds__(NW * WAVE, 2) void latent_attn_kernel(LatentAttn a) {
   extern __shared__ __align__(16) char smem_raw[];
-  elt* qs = reinterpret_cast<elt*>(smem_raw);                        // [NB][64][8] query fragments
-  float* sacc = reinterpret_cast<float*>(qs + a.NB * 512);           // [NW][16][68]
+  const int RBp = a.chunks * NRB, KR = a.NB - a.RB, KRp = KR > 2 ? KR : 2;   // blocks in LDS: the latent's, the rotated part's
+  elt* qs = reinterpret_cast<elt*>(smem_raw);                        // [RBp + KRp][64][8] query fragments, zero where there is no block
+  float* sacc = reinterpret_cast<float*>(qs + (RBp + KRp) * 512);    // [NW][16][68]
   __shared__ float sm[NW][16], sl[NW][16];
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
   const int col = lane & 15, g = lane >> 4;
@@ -134,10 +135,11 @@ __global__ __launch_bounds__(NW * WAVE, 2) void latent_attn_kernel(LatentAttn a)
   const int32_t* __restrict__ bt = a.block_table + (size_t)seq * a.max_blocks;
   const int qd = a.NB * 32;
 
-  for (int i = threadIdx.x; i < a.NB * 64; i += NW * WAVE) {
-    const int kb = i >> 6, l = i & 63, h = hg * 16 + (l & 15);
+  for (int i = threadIdx.x; i < (RBp + KRp) * 64; i += NW * WAVE) {
+    const int slot = i >> 6, l = i & 63, h = hg * 16 + (l & 15);
+    const int kb = slot < RBp ? slot : slot - RBp + a.RB;
     eltx8 v = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
-    if (h < a.H) v = ld8(a.q + ((size_t)t * a.H + h) * qd + kb * 32 + (l >> 4) * 8);
+    if (h < a.H && (slot < RBp ? kb < a.RB : kb < a.NB)) v = ld8(a.q + ((size_t)t * a.H + h) * qd + kb * 32 + (l >> 4) * 8);
     st8(qs + i * 8, v);
   }
   // the identity's columns 0..15 and 16..31 as the B operand: lane (column col, k-group g) holds k = 8 g .. 8 g + 7
@@ -154,65 +156,110 @@ __global__ __launch_bounds__(NW * WAVE, 2) void latent_attn_kernel(LatentAttn a)
 #pragma unroll
   for (int db = 0; db < 2 * NRB; ++db) O[db] = f32x4{0.f, 0.f, 0.f, 0.f};
 
-  for (int pg = p0 + wave; pg < p1; pg += NW) {
+  // the cache page of the context's page pg (page 0 for one outside the cache: every key of it is masked)
+  auto page_of = [&](int pg, bool& ok) {
     const int page = bt[pg];
-    if (page < 0 || page >= a.n_pages) continue;                     // wave-uniform
-    const elt* kp = a.cache + (size_t)page * a.NB * 512 + lane * 8;
-    eltx8 kf[NRB];
+    ok = page >= 0 && page < a.n_pages;
+    return a.cache + (size_t)(ok ? page : 0) * a.NB * 512 + lane * 8;
+  };
+  eltx8 kf[NRB], rf[2];
+  bool ok = false, ok_next = false;
+  const elt* kp = a.cache;
+  if (p0 + wave < p1) {
+    kp = page_of(p0 + wave, ok);
 #pragma unroll
-    for (int b = 0; b < NRB; ++b) {
-      const int kb = b0 + b < a.RB ? b0 + b : a.RB - 1;
-      kf[b] = ld8(kp + kb * 512);
+    for (int b = 0; b < NRB; ++b) kf[b] = ld8(kp + (b0 + b < a.RB ? b0 + b : a.RB - 1) * 512);
+#pragma unroll
+    for (int r = 0; r < 2; ++r) rf[r] = ld8(kp + (r < KR ? a.RB + r : a.RB) * 512);
+  }
+  for (int pg = p0 + wave; pg < p1; pg += NW) {
+    // the next page's fragments are requested one by one as this page's are done with
+    const elt* kn = page_of(pg + NW < p1 ? pg + NW : pg, ok_next);
+    // two chains of products: st[r] = S[token 4 g + r][head col].  A block that does not exist meets zero queries.
+    f32x4 st = mfma_16x16x32(rf[0], ld8(qs + (RBp * 64 + lane) * 8), f32x4{0.f, 0.f, 0.f, 0.f});
+    f32x4 st1 = mfma_16x16x32(rf[1], ld8(qs + ((RBp + 1) * 64 + lane) * 8), f32x4{0.f, 0.f, 0.f, 0.f});
+    rf[0] = ld8(kn + a.RB * 512);
+    rf[1] = ld8(kn + (KR > 1 ? a.RB + 1 : a.RB) * 512);
+#pragma unroll
+    for (int b = 0; b < NRB; b += 2) {
+      st = mfma_16x16x32(kf[b], ld8(qs + ((b0 + b) * 64 + lane) * 8), st);
+      st1 = mfma_16x16x32(kf[b + 1], ld8(qs + ((b0 + b + 1) * 64 + lane) * 8), st1);
     }
-    f32x4 st = f32x4{0.f, 0.f, 0.f, 0.f};                            // st[r] = S[token 4 g + r][head col]
-    for (int kb = a.RB; kb < a.NB; ++kb) st = mfma_16x16x32(ld8(kp + kb * 512), ld8(qs + (kb * 64 + lane) * 8), st);
+    for (int r = 2; r < KR; ++r) st = mfma_16x16x32(ld8(kp + (a.RB + r) * 512), ld8(qs + ((RBp + r) * 64 + lane) * 8), st);
     if (a.chunks > 1)                                                // the latent's blocks outside this chunk
       for (int kb = 0; kb < a.RB; ++kb)
         if (kb < b0 || kb >= b0 + NRB) st = mfma_16x16x32(ld8(kp + kb * 512), ld8(qs + (kb * 64 + lane) * 8), st);
-#pragma unroll
-    for (int b = 0; b < NRB; ++b)
-      if (b0 + b < a.RB) st = mfma_16x16x32(kf[b], ld8(qs + ((b0 + b) * 64 + lane) * 8), st);   // uniform
+    st += st1;
 
     float pm = -INFINITY;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      st[r] = pg * PAGE + 4 * g + r >= ctx ? -INFINITY : st[r] * a.scale;
+      st[r] = !ok || pg * PAGE + 4 * g + r >= ctx ? -INFINITY : st[r] * a.scale;
       pm = fmaxf(pm, st[r]);
     }
     pm = fmaxf(pm, __shfl_xor(pm, 16, WAVE));
     pm = fmaxf(pm, __shfl_xor(pm, 32, WAVE));
-    const float m_new = fmaxf(m, pm);                                // finite: the first token of a visited page is < ctx
-    const float alpha = __expf(m - m_new);
+    const float m_new = fmaxf(m, pm);
+    if (__any(m_new > m)) {                                          // uniform: the maximum rarely moves after the first pages
+      const float alpha = m == -INFINITY ? 0.f : __expf(m - m_new);
+      l *= alpha;
+#pragma unroll
+      for (int db = 0; db < 2 * NRB; ++db) O[db] *= alpha;
+      m = m_new;
+    }
+    const float mm = m == -INFINITY ? 0.f : m;
     eltx8 pa;
     float ps = 0.f;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const float p = __expf(st[r] - m_new);
+      const float p = __expf(st[r] - mm);
       ps += p;
       const elt hi = (elt)p;
       pa[r] = hi;
       pa[4 + r] = (elt)(p - (float)hi);
     }
-    l = l * alpha + ps;                                              // the lane's share of its column's sum
-    m = m_new;
+    l += ps;                                                         // the lane's share of its column's sum
 #pragma unroll
     for (int b = 0; b < NRB; ++b) {
-      if (b0 + b < a.RB) {                                           // uniform
-        const f32x4 t0 = mfma_16x16x32(kf[b], id0, f32x4{0.f, 0.f, 0.f, 0.f}), t1 = mfma_16x16x32(kf[b], id1, f32x4{0.f, 0.f, 0.f, 0.f});
-        const eltx8 v0 = eltx8{(elt)t0[0], (elt)t0[1], (elt)t0[2], (elt)t0[3], (elt)t0[0], (elt)t0[1], (elt)t0[2], (elt)t0[3]};
-        const eltx8 v1 = eltx8{(elt)t1[0], (elt)t1[1], (elt)t1[2], (elt)t1[3], (elt)t1[0], (elt)t1[1], (elt)t1[2], (elt)t1[3]};
-        O[2 * b] *= alpha;
-        O[2 * b + 1] *= alpha;
-        O[2 * b] = mfma_16x16x32(v0, pa, O[2 * b]);                  // O^T[dim 32 b + 4 g + r][head col]
-        O[2 * b + 1] = mfma_16x16x32(v1, pa, O[2 * b + 1]);
-      }
+      const f32x4 t0 = mfma_16x16x32(kf[b], id0, f32x4{0.f, 0.f, 0.f, 0.f}), t1 = mfma_16x16x32(kf[b], id1, f32x4{0.f, 0.f, 0.f, 0.f});
+      asm volatile("" ::: "memory");                                 // not earlier: the request goes into the registers just read
+      kf[b] = ld8(kn + (b0 + b < a.RB ? b0 + b : a.RB - 1) * 512);
+      const eltx4 h0 = eltx4{(elt)t0[0], (elt)t0[1], (elt)t0[2], (elt)t0[3]}, h1 = eltx4{(elt)t1[0], (elt)t1[1], (elt)t1[2], (elt)t1[3]};
+      O[2 * b] = mfma_16x16x32(eltx8{h0[0], h0[1], h0[2], h0[3], h0[0], h0[1], h0[2], h0[3]}, pa, O[2 * b]);   // O^T[dim 32 b + 4 g + r][head col]
+      O[2 * b + 1] = mfma_16x16x32(eltx8{h1[0], h1[1], h1[2], h1[3], h1[0], h1[1], h1[2], h1[3]}, pa, O[2 * b + 1]);
     }
+    kp = kn;
+    ok = ok_next;
   }
   l += __shfl_xor(l, 16, WAVE);
   l += __shfl_xor(l, 32, WAVE);
   if (g == 0) {
     sm[wave][col] = m;
     sl[wave][col] = l;
+  }
+  __syncthreads();
+  // per head, once: what every wave's sums are multiplied with, and (M, L)
+  if (threadIdx.x < 16) {
+    const int hc = threadIdx.x, h = hg * 16 + hc;
+    const float sk = a.splits == 1 && a.sink && h < a.H ? a.sink[h] : -INFINITY;
+    float M = sk, L = 0.f;
+#pragma unroll
+    for (int w = 0; w < NW; ++w) M = fmaxf(M, sm[w][hc]);
+    if (sk != -INFINITY) L = __expf(sk - M);
+    float f[NW];
+#pragma unroll
+    for (int w = 0; w < NW; ++w) {
+      f[w] = sm[w][hc] == -INFINITY ? 0.f : __expf(sm[w][hc] - M);
+      L += sl[w][hc] * f[w];
+    }
+    const float inv = a.splits > 1 ? 1.f : L > 0.f ? 1.f / L : 0.f;
+#pragma unroll
+    for (int w = 0; w < NW; ++w) sm[w][hc] = f[w] * inv;
+    if (a.splits > 1 && h < a.H && b0 == 0) {
+      const size_t r = ((size_t)split * a.T + t) * a.H + h;
+      a.part_ml[2 * r] = M;
+      a.part_ml[2 * r + 1] = L;
+    }
   }
 #pragma unroll
   for (int c = 0; c < NRB; c += 2) {                                 // 64 dims
@@ -222,32 +269,16 @@ __global__ __launch_bounds__(NW * WAVE, 2) void latent_attn_kernel(LatentAttn a)
       for (int u = 0; u < 4; ++u)
         if (2 * c + u < 2 * NRB) *reinterpret_cast<f32x4*>(sacc + (wave * 16 + col) * 68 + u * 16 + 4 * g) = O[(2 * c + u) % (2 * NRB)];
       __syncthreads();
-      for (int e = threadIdx.x; e < 16 * 64; e += NW * WAVE) {
-        const int hc = e >> 6, dd = e & 63, h = hg * 16 + hc, d = (b0 + c) * 32 + dd;
+      for (int e = threadIdx.x; e < 16 * 16; e += NW * WAVE) {
+        const int hc = e >> 4, dd = (e & 15) * 4, h = hg * 16 + hc, d = (b0 + c) * 32 + dd;
         if (h >= a.H || d >= a.RB * 32 || d >= (b0 + NRB) * 32) continue;
-        float M = sm[0][hc];
+        f32x4 o = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int w = 1; w < NW; ++w) M = fmaxf(M, sm[w][hc]);
-        const float sk = a.sink ? a.sink[h] : -INFINITY;
-        if (a.splits == 1) M = fmaxf(M, sk);
-        float L = 0.f, o = 0.f;
-#pragma unroll
-        for (int w = 0; w < NW; ++w) {
-          const float f = sm[w][hc] == -INFINITY ? 0.f : __expf(sm[w][hc] - M);
-          L += sl[w][hc] * f;
-          o += sacc[(w * 16 + hc) * 68 + dd] * f;
-        }
-        if (a.splits == 1) {
-          if (sk != -INFINITY) L += __expf(sk - M);
-          a.out[((size_t)t * a.H + h) * (a.RB * 32) + d] = (elt)(L > 0.f ? o / L : 0.f);
-        } else {
-          const size_t r = ((size_t)split * a.T + t) * a.H + h;
-          a.part_o[r * (a.RB * 32) + d] = o;
-          if (d == 0) {
-            a.part_ml[2 * r] = M;
-            a.part_ml[2 * r + 1] = L;
-          }
-        }
+        for (int w = 0; w < NW; ++w) o += *reinterpret_cast<const f32x4*>(sacc + (w * 16 + hc) * 68 + dd) * sm[w][hc];
+        if (a.splits == 1)
+          *reinterpret_cast<eltx4*>(a.out + ((size_t)t * a.H + h) * (a.RB * 32) + d) = eltx4{(elt)o[0], (elt)o[1], (elt)o[2], (elt)o[3]};
+        else
+          *reinterpret_cast<f32x4*>(a.part_o + (((size_t)split * a.T + t) * a.H + h) * (a.RB * 32) + d) = o;
       }
     }
   }
@@ -680,7 +711,8 @@ __global__ __launch_bounds__(256) void latent_attn_f32_kernel(LatentAttn a) {
 #ifndef MLORA_ELT_F32
 template <int NRB, int NW>
 int launch_latent_attn(const LatentAttn& a, hipStream_t s) {
-  const size_t lds = (size_t)a.NB * 1024 + (size_t)NW * 16 * 68 * sizeof(float);
+  const int kr = a.NB - a.RB;
+  const size_t lds = (size_t)(a.chunks * NRB + (kr > 2 ? kr : 2)) * 1024 + (size_t)NW * 16 * 68 * sizeof(float);
   static const hipError_t configured =               // the attribute is per kernel, set once per process, by one thread
       hipFuncSetAttribute((const void*)latent_attn_kernel<NRB, NW>, hipFuncAttributeMaxDynamicSharedMemorySize, 96 * 1024);
   if (configured != hipSuccess || lds > 96 * 1024)
@@ -722,8 +754,8 @@ extern "C" int mlora_latent_attn_splits(int T, int H, int max_ctx) {
 #else
   if (T <= 0 || H <= 0 || max_ctx <= 0) return 1;
   const long wgs = (long)T * ceil_div(H, 16);
-  int s = (int)(512 / wgs);                                       // two workgroups per compute unit ...
-  const int by_ctx = max_ctx / (8 * PAGE);                        // ... of at least two pages per wave
+  int s = (int)(256 / wgs);                                       // a workgroup per compute unit ...
+  const int by_ctx = max_ctx / (8 * PAGE);                        // ... of at least one page per wave
   if (s > by_ctx) s = by_ctx;
   if (s > 32) s = 32;
   return s < 1 ? 1 : s;
@@ -762,10 +794,10 @@ extern "C" int mlora_latent_attn(void* out, const void* q, const void* cache, co
   a.chunks = ceil_div(a.RB, nrb);
   a.n_inner = ceil_div(H, 16) * a.chunks;
   int e;
-  if (nrb == 2) e = launch_latent_attn<2, 4>(a, s);
-  else if (nrb == 4) e = launch_latent_attn<4, 4>(a, s);
-  else if (nrb == 8) e = launch_latent_attn<8, 4>(a, s);
-  else e = launch_latent_attn<16, 4>(a, s);
+  if (nrb == 2) e = launch_latent_attn<2, 8>(a, s);
+  else if (nrb == 4) e = launch_latent_attn<4, 8>(a, s);
+  else if (nrb == 8) e = launch_latent_attn<8, 8>(a, s);
+  else e = launch_latent_attn<16, 8>(a, s);
   if (e) return e;
   if (splits > 1) {
     MLORA_CHECK((long)T * H <= 0x7fffffffL, MLORA_ERR_UNSUPPORTED, "latent_attn: T=%d is too many tokens", T);

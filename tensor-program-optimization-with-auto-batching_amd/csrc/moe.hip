@@ -101,11 +101,16 @@ __global__ __launch_bounds__(PL_THREADS) void moe_plan_kernel(int32_t* __restric
   }
 }
 
-// x[t, :] += sum_k weight[t, k] * y[t * top + k, :], choices in order
-__global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ x, const elt* __restrict__ y, const float* __restrict__ weight,
-                                                          int top, int N) {
+// x[t, :] += parts, then sum_k weight[t, k] * y[t * top + k, :], choices in order; out_frag: the result once more, rounded to
+// the element type, in fragment order
+__global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ x, const float* __restrict__ part, int n_part, size_t part_stride,
+                                                          const elt* __restrict__ y, const float* __restrict__ weight, int top, int N,
+                                                          elt* __restrict__ out_frag, int frag_tt) {
   const int t = blockIdx.y, c = (blockIdx.x * 256 + threadIdx.x) * 4;
   if (c >= N) return;
+  f32x4* p = reinterpret_cast<f32x4*>(x + (size_t)t * N + c);
+  f32x4 xv = *p;
+  for (int q = 0; q < n_part; ++q) xv += *reinterpret_cast<const f32x4*>(part + q * part_stride + (size_t)t * N + c);
   f32x4 s = f32x4{0.f, 0.f, 0.f, 0.f};
   for (int k = 0; k < top; ++k) {
     const float w = weight[(size_t)t * top + k];
@@ -113,8 +118,9 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ x,
 #pragma unroll
     for (int e = 0; e < 4; ++e) s[e] = fmaf(w, (float)v[e], s[e]);
   }
-  f32x4* p = reinterpret_cast<f32x4*>(x + (size_t)t * N + c);
-  *p = *p + s;
+  xv += s;
+  *p = xv;
+  if (out_frag) *reinterpret_cast<eltx4*>(out_frag + frag_offset(t, c, frag_tt)) = eltx4{(elt)xv[0], (elt)xv[1], (elt)xv[2], (elt)xv[3]};
 }
 
 #ifndef MLORA_ELT_F32
@@ -298,11 +304,14 @@ extern "C" int mlora_moe_plan(int32_t* perm, int32_t* tiles, int32_t* n_tiles, c
   return mlora_launch_status("moe_plan");
 }
 
-extern "C" int mlora_moe_combine(float* x, const void* y, const float* weight, int T, int top, int N, void* stream) {
-  MLORA_CHECK(x && y && weight, MLORA_ERR_INVALID, "moe_combine: null pointer");
-  MLORA_CHECK(T >= 0 && T <= 65535 && top > 0 && N > 0 && N % 4 == 0, MLORA_ERR_UNSUPPORTED, "moe_combine: T=%d top=%d N=%d", T, top, N);
+extern "C" int mlora_moe_combine(float* x, const float* part, int n_part, const void* y, const float* weight, int T, int top, int N,
+                                 void* out_frag, void* stream) {
+  MLORA_CHECK(x && y && weight && n_part >= 0 && (n_part == 0 || part), MLORA_ERR_INVALID, "moe_combine: null pointer");
+  MLORA_CHECK(T >= 0 && T <= 65535 && top > 0 && N > 0 && N % 4 == 0 && (!out_frag || (N % 32 == 0 && sizeof(elt) == 2)), MLORA_ERR_UNSUPPORTED,
+              "moe_combine: T=%d top=%d N=%d", T, top, N);
   if (T == 0) return MLORA_OK;
-  hipLaunchKernelGGL(moe_combine_kernel, dim3(ceil_div(N, 1024), T), dim3(256), 0, (hipStream_t)stream, x, (const elt*)y, weight, top, N);
+  hipLaunchKernelGGL(moe_combine_kernel, dim3(ceil_div(N, 1024), T), dim3(256), 0, (hipStream_t)stream, x, part, n_part, (size_t)T * N,
+                     (const elt*)y, weight, top, N, (elt*)out_frag, mlora_frag_tiles(T));
   return mlora_launch_status("moe_combine");
 }
 

@@ -28,9 +28,10 @@ struct StreamNorm {
   elt* out_frag;          // the normed row in fragment order (16-bit element types) ...
   int frag_tt;
   elt* out_row;           // ... and / or row-major [T, Hp]
+  int raw;                // the output is x itself, rounded to the element type
 };
 
-// x += parts; x += y / rms(y) * yw; out = x / rms(x) * gain.  One workgroup per row, the row in registers.
+// x += parts; x += y / rms(y) * yw; out = x / rms(x) * gain (or x).  One workgroup per row, the row in registers.
 template <int VPT>
 __global__ __launch_bounds__(SN_THREADS) void stream_norm_kernel(StreamNorm a) {
   __shared__ float lds[2][SN_THREADS / WAVE];
@@ -80,12 +81,15 @@ __global__ __launch_bounds__(SN_THREADS) void stream_norm_kernel(StreamNorm a) {
     }
   }
   if (!a.out_frag && !a.out_row) return;
-  float ss = 0.f;
+  float s = 1.f;
+  if (!a.raw) {
+    float ss = 0.f;
 #pragma unroll
-  for (int i = 0; i < VPT; ++i)
+    for (int i = 0; i < VPT; ++i)
 #pragma unroll
-    for (int e = 0; e < 4; ++e) ss = fmaf(v[i][e], v[i][e], ss);
-  const float s = a.gain / sqrtf(sn_block_sum(ss, lds[1]) / (float)a.H + a.eps);
+      for (int e = 0; e < 4; ++e) ss = fmaf(v[i][e], v[i][e], ss);
+    s = a.gain / sqrtf(sn_block_sum(ss, lds[1]) / (float)a.H + a.eps);
+  }
 #pragma unroll
   for (int i = 0; i < VPT; ++i) {
     const int c = (threadIdx.x + i * SN_THREADS) * 4;
@@ -103,46 +107,40 @@ __device__ __forceinline__ float gelu_tanh(float z) {
 }
 
 #ifndef MLORA_ELT_F32
+// out[t, n] = gelu(sum_k W[n, k] x[t, k]) * table[id_t, col0 + n] for n < dim, 0 for the padding rows; x and out in fragment
+// order.  A workgroup takes 16 tokens x 16 NT rows, its waves split K; a wave requests TG_U k-steps at a time.
 constexpr int TG_WAVES = 8;
-// out[t, n] = gelu(sum_k W[n, k] x[t, k]) * table[id_t, col0 + n] for n < dim, 0 for the padding rows, in fragment order.
-// x is the fp32 residual stream with its pending partial sums, rounded to the element type on the way into the matrix
-// cores.  A workgroup takes 16 tokens x 16 NT rows, its waves split K.
+constexpr int TG_U = 4;
 template <int NT>
-__global__ __launch_bounds__(TG_WAVES* WAVE) void token_gate_kernel(elt* __restrict__ out, int frag_tt, const float* __restrict__ x,
-                                                                   const float* __restrict__ part, int n_part, size_t part_stride,
+__global__ __launch_bounds__(TG_WAVES* WAVE) void token_gate_kernel(elt* __restrict__ out, int frag_tt, const elt* __restrict__ x,
                                                                    const elt* __restrict__ Wp, const elt* __restrict__ table, int ld_table,
                                                                    int col0, int dim, const int32_t* __restrict__ ids, int V, int T, int K, int N) {
   __shared__ f32x4 red[TG_WAVES][NT][WAVE];
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
   const int KB = K / 32, tiles = N / 16;
   const int nt0 = blockIdx.x * NT, t0 = blockIdx.y * 16;
-  int t = t0 + (lane & 15);
-  t = t < T ? t : T - 1;
-  const size_t xo = (size_t)t * K + (lane >> 4) * 8;
+  const elt* xp = x + (size_t)blockIdx.y * 512 + lane * 8;
+  const elt* wp[NT];
+#pragma unroll
+  for (int i = 0; i < NT; ++i) wp[i] = Wp + (size_t)(nt0 + i < tiles ? nt0 + i : tiles - 1) * KB * 512 + lane * 8;
   f32x4 acc[NT];
 #pragma unroll
   for (int i = 0; i < NT; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-  for (int ks = wave; ks < KB; ks += TG_WAVES) {
-    eltx8 a[NT];
+  for (int ks0 = wave; ks0 < KB; ks0 += TG_WAVES * TG_U) {
+    eltx8 a[TG_U][NT], b[TG_U];
 #pragma unroll
-    for (int i = 0; i < NT; ++i) {
-      const int nt = nt0 + i < tiles ? nt0 + i : tiles - 1;
-      a[i] = ld8(Wp + ((size_t)nt * KB + ks) * 512 + lane * 8);
-    }
-    f32x4 lo = *reinterpret_cast<const f32x4*>(x + xo + ks * 32), hi = *reinterpret_cast<const f32x4*>(x + xo + ks * 32 + 4);
-    for (int q = 0; q < n_part; ++q) {
-      const float* p = part + q * part_stride + xo + ks * 32;
-      lo += *reinterpret_cast<const f32x4*>(p);
-      hi += *reinterpret_cast<const f32x4*>(p + 4);
-    }
-    eltx8 b;
+    for (int u = 0; u < TG_U; ++u) {
+      const bool in = ks0 + u * TG_WAVES < KB;                       // uniform; past K: a valid address, zeroed
+      const int ks = in ? ks0 + u * TG_WAVES : ks0;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      b[e] = (elt)lo[e];
-      b[4 + e] = (elt)hi[e];
+      for (int i = 0; i < NT; ++i) a[u][i] = ld8(wp[i] + (size_t)ks * 512);
+      b[u] = ld8(xp + (size_t)ks * frag_tt * 512);
+      if (!in) b[u] = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
     }
 #pragma unroll
-    for (int i = 0; i < NT; ++i) acc[i] = mfma_16x16x32(a[i], b, acc[i]);
+    for (int u = 0; u < TG_U; ++u)
+#pragma unroll
+      for (int i = 0; i < NT; ++i) acc[i] = mfma_16x16x32(a[u][i], b[u], acc[i]);
   }
 #pragma unroll
   for (int i = 0; i < NT; ++i) red[wave][i][lane] = acc[i];
@@ -181,7 +179,7 @@ __global__ __launch_bounds__(256) void token_gate_mul_kernel(elt* __restrict__ o
 }  // namespace
 
 extern "C" int mlora_stream_norm(void* out_frag, void* out_row, float* x, const float* part, int n_part, const float* branch,
-                                 const void* branch_w, float eps, float gain, int T, int H, int Hp, void* stream) {
+                                 const void* branch_w, float eps, float gain, int raw, int T, int H, int Hp, void* stream) {
   MLORA_CHECK(x && T >= 0 && H > 0 && Hp >= H && Hp % 32 == 0 && Hp <= 16384, MLORA_ERR_UNSUPPORTED,
               "stream_norm: need 0 < H <= Hp <= 16384, Hp %% 32 == 0 (T=%d H=%d Hp=%d)", T, H, Hp);
   MLORA_CHECK((n_part == 0 || part) && n_part >= 0 && (!branch || branch_w), MLORA_ERR_INVALID, "stream_norm: null pointer");
@@ -191,7 +189,7 @@ extern "C" int mlora_stream_norm(void* out_frag, void* out_row, float* x, const 
   a.x = x; a.H = H; a.Hp = Hp; a.eps = eps; a.gain = gain;
   a.part = part; a.n_part = n_part; a.part_stride = (size_t)T * Hp;
   a.y = branch; a.yw = (const elt*)branch_w;
-  a.out_frag = (elt*)out_frag; a.frag_tt = mlora_frag_tiles(T); a.out_row = (elt*)out_row;
+  a.out_frag = (elt*)out_frag; a.frag_tt = mlora_frag_tiles(T); a.out_row = (elt*)out_row; a.raw = raw;
   hipStream_t s = (hipStream_t)stream;
   if (Hp <= 2048) hipLaunchKernelGGL(stream_norm_kernel<2>, dim3(T), dim3(SN_THREADS), 0, s, a);
   else if (Hp <= 4096) hipLaunchKernelGGL(stream_norm_kernel<4>, dim3(T), dim3(SN_THREADS), 0, s, a);
@@ -201,18 +199,17 @@ extern "C" int mlora_stream_norm(void* out_frag, void* out_row, float* x, const 
 }
 
 #ifndef MLORA_ELT_F32
-extern "C" int mlora_token_gate(void* out_frag, const float* x, const float* part, int n_part, const void* Wp, const void* table,
-                                int ld_table, int col0, int dim, const int32_t* ids, int V, int T, int K, int N, void* stream) {
-  MLORA_CHECK(out_frag && x && Wp && table && ids && (n_part == 0 || part), MLORA_ERR_INVALID, "token_gate: null pointer");
+extern "C" int mlora_token_gate(void* out_frag, const void* xf, const void* Wp, const void* table, int ld_table, int col0, int dim,
+                                const int32_t* ids, int V, int T, int K, int N, void* stream) {
+  MLORA_CHECK(out_frag && xf && Wp && table && ids, MLORA_ERR_INVALID, "token_gate: null pointer");
   MLORA_CHECK(T >= 0 && K > 0 && K % 32 == 0 && N > 0 && N % 32 == 0 && dim > 0 && dim <= N && col0 >= 0 && col0 + dim <= ld_table && V > 0 &&
                   ceil_div(T, 16) <= 65535,
               MLORA_ERR_UNSUPPORTED, "token_gate: need K %% 32 == 0, N %% 32 == 0, dim <= N (T=%d K=%d N=%d dim=%d)", T, K, N, dim);
   if (T == 0) return MLORA_OK;
   hipStream_t s = (hipStream_t)stream;
-  const size_t ps = (size_t)T * K;
-#define MLORA_TG(NT)                                                                                                                     \
-  hipLaunchKernelGGL(token_gate_kernel<NT>, dim3(ceil_div(N, 16 * NT), ceil_div(T, 16)), dim3(TG_WAVES * WAVE), 0, s, (elt*)out_frag,    \
-                     mlora_frag_tiles(T), x, part, n_part, ps, (const elt*)Wp, (const elt*)table, ld_table, col0, dim, ids, V, T, K, N)
+#define MLORA_TG(NT)                                                                                                                   \
+  hipLaunchKernelGGL(token_gate_kernel<NT>, dim3(ceil_div(N, 16 * NT), ceil_div(T, 16)), dim3(TG_WAVES * WAVE), 0, s, (elt*)out_frag,  \
+                     mlora_frag_tiles(T), (const elt*)xf, (const elt*)Wp, (const elt*)table, ld_table, col0, dim, ids, V, T, K, N)
   if (T <= 256) MLORA_TG(1);
   else if (N <= 32) MLORA_TG(2);
   else MLORA_TG(4);

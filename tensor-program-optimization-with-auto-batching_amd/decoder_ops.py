@@ -43,26 +43,30 @@ def _ptr(t) -> int:
     return None if t is None else t.data_ptr()
 
 
-def stream_norm(x, H, eps, gain=1.0, parts=None, branch=None, out=None, out_row=None):
+def _parts(parts):
+    """(pointer, blocks) of pending K-split partials."""
+    return (parts.part.data_ptr(), parts.ks - 1) if parts is not None else (None, 0)
+
+
+def stream_norm(x, H, eps, gain=1.0, parts=None, branch=None, out=None, out_row=None, raw=False):
     """x [T, Hp] fp32 (+= pending K-split partials, += branch[0] / rms * branch[1], in place); out (FragActivation) and / or
-    out_row [T, Hp] = x / rms(x) * gain.  H: columns that count."""
+    out_row [T, Hp] = x / rms(x) * gain, or x itself with `raw`.  H: columns that count."""
     if out is None and out_row is None and parts is None and branch is None:
         return
     T, Hp = x.shape
     dt = out.dtype if out is not None else out_row.dtype if out_row is not None else branch[1].dtype if branch is not None else torch.bfloat16
-    check(lib_of(dt).mlora_stream_norm(out.data.data_ptr() if out is not None else None, _ptr(out_row), _dev(x, torch.float32),
-                                       _ptr(parts.part) if parts is not None else None, parts.ks - 1 if parts is not None else 0,
+    check(lib_of(dt).mlora_stream_norm(out.data.data_ptr() if out is not None else None, _ptr(out_row), _dev(x, torch.float32), *_parts(parts),
                                        _ptr(branch[0]) if branch is not None else None, _ptr(branch[1]) if branch is not None else None,
-                                       float(eps), float(gain), T, H, Hp, _stream()), dt)
+                                       float(eps), float(gain), int(raw), T, H, Hp, _stream()), dt)
 
 
-def token_gate(x, W, table, col0, dim, ids, parts=None):
-    """gelu_tanh(W x) * table[ids, col0 : col0 + dim] (x: residual stream [T, Hp] fp32 with pending partials) as the
-    activation of the following linear, its width W's padded row count."""
-    T, Hp = x.shape
+def token_gate(x, W, table, col0, dim, ids):
+    """gelu_tanh(W x) * table[ids, col0 : col0 + dim] (x: an activation) as the activation of the following linear, its width
+    W's padded row count."""
+    T = x.shape[0]
     N, K = W.shape
     V, ld = table.shape
-    if K != Hp or ids.shape != (T,):
+    if x.shape[1] != K or ids.shape != (T,):
         raise ValueError(f"token_gate: x{tuple(x.shape)} W{tuple(W.shape)} ids{tuple(ids.shape)}")
     out = activation(T, N, W.dtype, x.device)
     L = lib_of(W.dtype)
@@ -70,8 +74,7 @@ def token_gate(x, W, table, col0, dim, ids, parts=None):
         z = ops.linear(x, W)
         check(L.mlora_token_gate_mul(_dev(out), _dev(z), _dev(table, W.dtype), ld, col0, dim, _dev(ids, torch.int32), V, T, N, _stream()), W.dtype)
         return out
-    check(L.mlora_token_gate(out.data.data_ptr(), _dev(x, torch.float32), _ptr(parts.part) if parts is not None else None,
-                             parts.ks - 1 if parts is not None else 0, _wptr(W), _dev(table, W.dtype), ld, col0, dim, _dev(ids, torch.int32),
+    check(L.mlora_token_gate(out.data.data_ptr(), x.data.data_ptr(), _wptr(W), _dev(table, W.dtype), ld, col0, dim, _dev(ids, torch.int32),
                              V, T, K, N, _stream()), W.dtype)
     return out
 
@@ -214,7 +217,9 @@ def moe_linear(x, W, plan, N, K, stage, act=ACT_NONE, alpha=1.0):
     return y
 
 
-def moe_combine(x, y, w):
-    """x [T, N] fp32 += sum over the choices of w * y (entry rows)."""
+def moe_combine(x, y, w, parts=None, out=None):
+    """x [T, N] fp32 += pending partials, then the sum over the choices of w * y (entry rows); out (FragActivation): the result
+    rounded to the element type."""
     T, top = w.shape
-    check(lib_of(y.dtype).mlora_moe_combine(_dev(x, torch.float32), _dev(y), _dev(w, torch.float32), T, top, x.shape[1], _stream()), y.dtype)
+    check(lib_of(y.dtype).mlora_moe_combine(_dev(x, torch.float32), *_parts(parts), _dev(y), _dev(w, torch.float32), T, top, x.shape[1],
+                                            out.data.data_ptr() if out is not None else None, _stream()), y.dtype)

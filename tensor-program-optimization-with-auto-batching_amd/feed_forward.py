@@ -54,11 +54,12 @@ class MoeRelu2:
         self.up = stack(w["up"], self.ffp, self.Hp)
         self.down = stack(w["down"], self.Hp, self.ffp)
 
-    def add_to(self, resid, x, x_row):
-        """resid [T, Hp] += output; x: the input as an activation, x_row: the same row-major."""
+    def add_to(self, resid, x, x_row, parts=None, out=None):
+        """resid [T, Hp] += pending partials and the output; x: the input as an activation, x_row: the same row-major; out: the
+        sum as an activation."""
         s = self.spec
         logits = ops.linear(x, self.router, out_dtype=torch.float32)
         pick, wt = D.moe_route(logits, self.bias, self.gain, s.top, self.dtype)
         plan = D.MoePlan(pick, s.experts, self.dtype)
         mid = D.moe_linear(x_row, self.up, plan, self.ffp, self.Hp, D.MOE_UP, D.ACT_RELU2, self.gain)
-        D.moe_combine(resid, D.moe_linear(mid, self.down, plan, self.Hp, self.ffp, D.MOE_DOWN), wt)
+        D.moe_combine(resid, D.moe_linear(mid, self.down, plan, self.Hp, self.ffp, D.MOE_DOWN), wt, parts, out)

@@ -181,10 +181,15 @@ class SafolornForCausalLM(CausalLM):
             else:
                 cat = kv.latent_attention(l, qkv, att)
             parts = self._add_linear(cat, L["out"], x, split)
+            xa = ops.FragActivation(*x.shape, dev, dtype=self.dtype) if frag and c.side_dim else None
             if moe is not None:
-                moe.add_to(x, n, n_row)
+                moe.add_to(x, n, n_row, parts, xa)
+                parts = None
+            elif xa is not None:
+                D.stream_norm(x, c.width, c.eps, parts=parts, out=xa, raw=True)
+                parts = None
             if c.side_dim:
-                g = D.token_gate(x, L["side_gate"], self.side_embed, l * c.side_dim, c.side_dim, ids, parts)
+                g = D.token_gate(xa if frag else x, L["side_gate"], self.side_embed, l * c.side_dim, c.side_dim, ids)
                 branch = (ops.linear(g, L["side_proj"], out_dtype=torch.float32), L["side_norm"])
             if layer_outputs is not None:
                 D.stream_norm(x, c.width, c.eps, parts=parts, branch=branch)

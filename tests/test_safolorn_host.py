@@ -99,9 +99,9 @@ def test_decoder_argument_validation():
     load_pkg("build").ensure("bfloat16"), load_pkg("build").ensure("float32")
     lm = load_pkg("_lib")
     b, f = lm.lib("bfloat16"), lm.lib("float32")
-    assert b.mlora_stream_norm(16, None, 16, None, 0, None, None, 1e-5, 1.0, 4, 100, 100, None) == -2
-    assert f.mlora_stream_norm(16, None, 16, None, 0, None, None, 1e-5, 1.0, 4, 96, 96, None) == -2
-    assert b.mlora_stream_norm(16, None, 16, None, 2, None, None, 1e-5, 1.0, 4, 96, 96, None) == -1
+    assert b.mlora_stream_norm(16, None, 16, None, 0, None, None, 1e-5, 1.0, 0, 4, 100, 100, None) == -2
+    assert f.mlora_stream_norm(16, None, 16, None, 0, None, None, 1e-5, 1.0, 0, 4, 96, 96, None) == -2
+    assert b.mlora_stream_norm(16, None, 16, None, 2, None, None, 1e-5, 1.0, 0, 4, 96, 96, None) == -1
     assert b.mlora_head_linear(16, 0, 64, 32, 16, 60, 32, 16, 2, 4, 32, 32, 1.0, None) == -2
     assert f.mlora_head_linear(16, 1, 64, 32, 16, 64, 32, 16, 2, 4, 32, 32, 1.0, None) == -2
     la = lambda lib, splits=1, ws=None, n=0: lib.mlora_latent_attn(16, 16, 16, 16, 4, 16, 16, None, 0.1, 2, 3, 72, 24, 8, 2, splits, ws, n, None)
