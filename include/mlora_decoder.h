@@ -63,10 +63,12 @@ int mlora_latent_prefill(void* out, int out_layout, int ld_out, const void* q, i
                          void* stream);
 
 /* Mixture of experts.  mlora_moe_route: z = scale logits[t] + bias, the `top` largest per token (lower index on ties), softmax
- * over those.  mlora_moe_plan sorts the (token, choice) entries by expert into tiles {expert, first place, places, 0} of
- * mlora_moe_tile_rows places (at most mlora_moe_max_tiles of them).  mlora_moe_linear multiplies tile by tile with the
- * experts' weights (one [N, K] block each): stage UP reads token rows x [T, K] and writes place rows, stage DOWN reads place
- * rows and writes entry rows; `act` is applied to alpha times the product.  mlora_moe_combine: x[t] += the n_part blocks
+ * over those.  mlora_moe_plan sorts the (token, choice) entries by expert into places - every
+ * expert's start at a multiple of 16 - and tiles {expert, first place, places, 0} of mlora_moe_tile_rows places; perm holds
+ * mlora_moe_max_places entries, tiles mlora_moe_max_tiles, n_tiles two numbers.  mlora_moe_linear multiplies tile by
+ * tile with the experts' weights (one [N, K] block each): stage UP reads token rows x [T, K] and writes places, stage DOWN reads places
+ * and writes entry rows [T top, N]; `act` is applied to alpha times the product.  Tiles of 256 places: the hidden places are in fragment
+ * order, K % 64 == 0, and UP needs a workspace of places * K elements; else places are rows.  mlora_moe_combine: x[t] += the n_part blocks
  * part[q][T][N], then the sum over the choices of weight * row; out_frag (or NULL): the result in fragment order. */
 #define MLORA_ACT_NONE  0
 #define MLORA_ACT_RELU2 1   /* max(v, 0)^2 */
@@ -76,9 +78,11 @@ int mlora_moe_route(int32_t* pick, float* weight, const float* logits, int ld, c
                     void* stream);
 int mlora_moe_tile_rows(int T, int E, int top);
 int mlora_moe_max_tiles(int T, int E, int top);
+int mlora_moe_max_places(int T, int E, int top);
 int mlora_moe_plan(int32_t* perm, int32_t* tiles, int32_t* n_tiles, const int32_t* pick, int T, int E, int top, void* stream);
 int mlora_moe_linear(void* y, const void* x, const void* W, const int32_t* perm, const int32_t* tiles, const int32_t* n_tiles, int tile_rows,
-                     int max_tiles, int T, int K, int N, int top, int stage, int act, float alpha, void* stream);
+                     int max_tiles, int places, int T, int K, int N, int top, int stage, int act, float alpha, void* workspace,
+                     size_t workspace_elems, void* stream);
 int mlora_moe_combine(float* x, const float* part, int n_part, const void* y, const float* weight, int T, int top, int N, void* out_frag,
                       void* stream);
 

@@ -134,8 +134,9 @@ DECODER_SIGNATURES = {
     "mlora_moe_route": (_i, [_p, _p, _p, _i, _p, _f, _i, _i, _i, _p]),
     "mlora_moe_tile_rows": (_i, [_i, _i, _i]),
     "mlora_moe_max_tiles": (_i, [_i, _i, _i]),
+    "mlora_moe_max_places": (_i, [_i, _i, _i]),
     "mlora_moe_plan": (_i, [_p, _p, _p, _p, _i, _i, _i, _p]),
-    "mlora_moe_linear": (_i, [_p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _f, _p]),
+    "mlora_moe_linear": (_i, [_p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _p, _z, _p]),
     "mlora_moe_combine": (_i, [_p, _p, _i, _p, _p, _i, _i, _i, _p, _p]),
 }
 

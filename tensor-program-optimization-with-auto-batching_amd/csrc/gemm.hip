@@ -12,13 +12,14 @@
 #include <type_traits>
 
 #include "common.h"
+#include "moe.h"
 
 int mlora_check_linear(const char* who, const void* y, int y_dtype, int mode, const void* x, int ldx, const void* W,
                        int T, int K, int N);
 
 namespace {
 
-enum { OUT_F16 = 0, OUT_F32 = 1, OUT_ACC_F32 = 2, OUT_SILU = 3, OUT_CLIP = 4 };   // the last two: a gated product (MLORA_GLU_*) in fragment order
+enum { OUT_F16 = 0, OUT_F32 = 1, OUT_ACC_F32 = 2, OUT_SILU = 3, OUT_CLIP = 4, OUT_RELU2 = 5 };   // OUT_SILU, OUT_CLIP: a gated product (MLORA_GLU_*), OUT_RELU2: max(alpha y, 0)^2, all in fragment order
 
 // compute units of the current device (0 if it cannot be asked), read once
 int gemm_n_cu() {
@@ -292,6 +293,15 @@ struct PPLora {
   const int32_t* blk_adapter;
 };
 
+// A grouped GEMM over a routing plan (moe.h): a token block is a tile of the plan - up to 256 places of one expert, whose
+// weights it is multiplied with.  Places are in fragment order (x_tt tiles of 16).  Results go to fragment-ordered places
+// (OUT_RELU2) or, row-major, to the entries the places stand for (OUT_F16), times alpha.
+struct PPGroup {
+  MoePlan plan;
+  size_t w_elems;
+  float alpha;
+};
+
 __device__ __forceinline__ unsigned long long uniform64(unsigned long long v) {
   const unsigned lo = __builtin_amdgcn_readfirstlane((unsigned)v), hi = __builtin_amdgcn_readfirstlane((unsigned)(v >> 32));
   return ((unsigned long long)hi << 32) | lo;
@@ -303,11 +313,12 @@ __device__ __forceinline__ unsigned long long uniform64(unsigned long long v) {
 // up tiles of the same channels, so that a lane ends up with both halves of its channels and the product never leaves
 // the registers.  LoRA deltas: slot 0 of `lo` is the gate projection, slot 1 the up projection (B == nullptr: not
 // adapted); each rides as its own extra k-steps, in which only that half of a wave's tiles is multiplied.
-// LORA = false is the plain GEMM (lo is ignored)
-template <int OUT, bool LORA>
+// LORA = false is the plain GEMM (lo is ignored); GROUPED: see PPGroup (gy is the number of tiles in use)
+template <int OUT, bool LORA, bool GROUPED = false>
 __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __restrict__ yv, const elt* __restrict__ x, int ldx, int x_tt,
                                                                    const elt* __restrict__ Wp, int T, int K, int N, int gx, int gy,
-                                                                   PPLora lo, GluArgs ga) {
+                                                                   PPLora lo, GluArgs ga, PPGroup gr = PPGroup()) {
+  if constexpr (GROUPED) gy = *gr.plan.n_tiles;
   extern __shared__ __align__(16) elt smem[];  // [PP_STAGES][PP_STAGE_ELEMS], then [PP_WAVES][PP_OUT_ELEMS]
   constexpr int NW = PP_WAVES;
   constexpr int LQ = 2 * PP_F / NW;            // fragments a wave fetches per stage (4)
@@ -320,6 +331,9 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
   const int tiles = (N + 15) / 16;
   const int I = N / 2, itiles = I / 16;        // SILU: channels and their 16-row tiles
   const int G = gridDim.x;
+  if constexpr (GROUPED) {
+    if ((int)blockIdx.x >= nb) return;         // fewer blocks than workgroups: nothing was requested yet
+  }
 
   // block number -> (weight-row block, token block)
   auto block_of = [&](int L, int& n0, int& t0) {
@@ -327,6 +341,7 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
     if ((nb & 7) == 0 && (G & 7) == 0) idx = (L & 7) * (nb >> 3) + (L >> 3);
     n0 = (idx / gy) * BN;
     t0 = (idx % gy) * (PP_F * 16);
+    if constexpr (GROUPED) t0 = __builtin_amdgcn_readfirstlane(idx % gy);      // a tile of the plan
   };
   // the LoRA part of a block: projection slot and adapter (-1: none), everything uniform
   auto lora_of = [&](int n0, int t0, int& slot) -> int {
@@ -358,6 +373,12 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
     int n0, t0;
     block_of(L < nb ? L : blockIdx.x, n0, t0); // past the last block: valid addresses, the data is never multiplied
     load_nst = KB;
+    const elt* Wb = Wp;
+    if constexpr (GROUPED) {
+      const int4 tile = gr.plan.tiles[t0];
+      Wb = Wp + __builtin_amdgcn_readfirstlane(tile.x) * gr.w_elems;
+      t0 = __builtin_amdgcn_readfirstlane(tile.y);
+    }
     if constexpr (LORA) {
       int slot;
       const int a = L < nb ? lora_of(n0, t0, slot) : -1;
@@ -403,7 +424,7 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
           nt = n0 / 16 + wave * LQ + q;
           nt = nt < tiles ? nt : tiles - 1;    // rows past N: a valid fragment, results dropped
         }
-        src[q] = Wp + (size_t)nt * KB * 512 + lane * 8;
+        src[q] = Wb + (size_t)nt * KB * 512 + lane * 8;
       }
       step = 512;
     } else if (x_tt > 0) {
@@ -544,6 +565,12 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
       for (int j = 0; j < WTF; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
     int n0, t0;
     block_of(L, n0, t0);
+    int tend = T;
+    if constexpr (GROUPED) {
+      const int4 tile = gr.plan.tiles[t0];
+      t0 = __builtin_amdgcn_readfirstlane(tile.y);
+      tend = t0 + __builtin_amdgcn_readfirstlane(tile.z);
+    }
     int nst = KB;                                      // KB and E are even (checked by the launcher): the register sets alternate
     if constexpr (LORA) {
       int slot;
@@ -585,6 +612,25 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
           *reinterpret_cast<eltx4*>((elt*)yv + ((size_t)(c >> 5) * x_tt + (t >> 4)) * 512 + ((c & 31) >> 3) * 128 + (t & 15) * 8 + (c & 7)) = o;
         }
       }
+    } else if constexpr (OUT == OUT_RELU2) {
+      // four channels of a token = one 8-byte piece of the output fragment
+#pragma unroll
+      for (int j = 0; j < WTF; ++j) {
+        const int t = t0 + (wt * WTF + j) * 16 + r16;
+        if (t >= tend) continue;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          const int c = n0 + (wn * 8 + i) * 16 + g * 4;
+          if (c >= N) continue;
+          eltx4 o;
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const float v = fmaxf(acc[i][j][r] * gr.alpha, 0.f);
+            o[r] = (elt)(v * v);
+          }
+          *reinterpret_cast<eltx4*>((elt*)yv + ((size_t)(c >> 5) * x_tt + (t >> 4)) * 512 + ((c & 31) >> 3) * 128 + (t & 15) * 8 + (c & 7)) = o;
+        }
+      }
     } else if constexpr (OUT == OUT_F16) {
       // 16 tokens x 64 columns at a time through the wave's staging buffer: D[n][t] fragments in, token rows out
 #pragma unroll
@@ -593,7 +639,8 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
         for (int h = 0; h < 2; ++h) {
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
-            const f32x4 sacc = acc[h * 4 + i][j];
+            f32x4 sacc = acc[h * 4 + i][j];
+            if constexpr (GROUPED) sacc *= gr.alpha;
             *reinterpret_cast<eltx4*>(ostage + r16 * PP_OUT_LD + i * 16 + g * 4) = eltx4{(elt)sacc[0], (elt)sacc[1], (elt)sacc[2], (elt)sacc[3]};
           }
           __builtin_amdgcn_wave_barrier();
@@ -602,16 +649,18 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
             const int c = q * 64 + lane;           // 16-byte chunk: token row c / 8, columns (c % 8) * 8 ..
             const int tr = c >> 3, cc = (c & 7) * 8;
             const int t = t0 + (wt * WTF + j) * 16 + tr;
+            int row = t;
+            if constexpr (GROUPED) row = gr.plan.perm[t < tend ? t : tend - 1];
             const int n = n0 + (wn * 8 + h * 4) * 16 + cc;
             const eltx4 lo = *reinterpret_cast<const eltx4*>(ostage + tr * PP_OUT_LD + cc);
             const eltx4 hi = *reinterpret_cast<const eltx4*>(ostage + tr * PP_OUT_LD + cc + 4);
-            if (t < T && n + 8 <= N) {
-              st8((elt*)yv + (size_t)t * N + n, eltx8{lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]});
-            } else if (t < T) {
+            if (t < tend && n + 8 <= N) {
+              st8((elt*)yv + (size_t)row * N + n, eltx8{lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]});
+            } else if (t < tend) {
 #pragma unroll
               for (int e = 0; e < 4; ++e) {
-                if (n + e < N) ((elt*)yv)[(size_t)t * N + n + e] = lo[e];
-                if (n + 4 + e < N) ((elt*)yv)[(size_t)t * N + n + 4 + e] = hi[e];
+                if (n + e < N) ((elt*)yv)[(size_t)row * N + n + e] = lo[e];
+                if (n + 4 + e < N) ((elt*)yv)[(size_t)row * N + n + 4 + e] = hi[e];
               }
             }
           }
@@ -1122,6 +1171,38 @@ extern "C" int mlora_linear_frag_silu(void* act, const void* xf, const void* Wp,
   }
   const int e = launch_gemm_pp<OUT_SILU>(act, (const elt*)xf, 0, mlora_frag_tiles(T), (const elt*)Wp, T, K, 2 * I, (hipStream_t)stream, lo);
   return e ? e : mlora_launch_status("linear_frag_silu");
+}
+#endif
+
+#ifdef MLORA_ELT_BF16
+// One expert linear over a plan of 256-place tiles: xf places in fragment order (x_tt tiles of 16), y as PPGroup says.
+template <int OUT>
+static int launch_gemm_grouped(void* y, const elt* xf, int x_tt, const elt* Wp, int K, int N, int max_tiles, const PPGroup& gr, hipStream_t s) {
+  constexpr size_t lds = ((size_t)PP_STAGES * PP_STAGE_ELEMS + (size_t)PP_WAVES * PP_OUT_ELEMS) * sizeof(elt);
+  static const hipError_t configured =
+      hipFuncSetAttribute((const void*)gemm_pp_kernel<OUT, false, true>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+  if (configured != hipSuccess)
+    return mlora_set_error(MLORA_ERR_LAUNCH, "moe_linear: cannot reserve %zu bytes of LDS: %s", lds, hipGetErrorString(configured));
+  const int gx = ceil_div(N, PP_F * 16);
+  int n_cu = gemm_n_cu();
+  if (n_cu <= 0) n_cu = 256;
+  const long nb = (long)gx * max_tiles;
+  hipLaunchKernelGGL((gemm_pp_kernel<OUT, false, true>), dim3(nb < n_cu ? (int)nb : n_cu), dim3(PP_WAVES * WAVE), lds, s, y, xf, 0, x_tt, Wp,
+                     x_tt * 16, K, N, gx, max_tiles, PPLora(), GluArgs(), gr);
+  return MLORA_OK;
+}
+
+int mlora_gemm_grouped(void* y, const void* xf, int x_tt, const void* Wp, const MoePlan& plan, int max_tiles, int K, int N, int relu2, float alpha,
+                       void* stream) {
+  MLORA_CHECK(K % 64 == 0 && N % 32 == 0 && x_tt > 0 && max_tiles > 0, MLORA_ERR_UNSUPPORTED, "moe_linear: K=%d N=%d", K, N);   // the caller's checks say more
+  PPGroup gr;
+  gr.plan = plan;
+  gr.w_elems = (size_t)N * K;
+  gr.alpha = alpha;
+  hipStream_t s = (hipStream_t)stream;
+  const int e = relu2 ? launch_gemm_grouped<OUT_RELU2>(y, (const elt*)xf, x_tt, (const elt*)Wp, K, N, max_tiles, gr, s)
+                      : launch_gemm_grouped<OUT_F16>(y, (const elt*)xf, x_tt, (const elt*)Wp, K, N, max_tiles, gr, s);
+  return e ? e : mlora_launch_status("moe_linear");
 }
 #endif
 

@@ -111,9 +111,11 @@ extern "C" int mlora_head_linear(void* y, int y_layout, long ldy, long head_y, c
 }
 
 extern "C" int mlora_moe_linear(void* y, const void* x, const void* W, const int32_t* perm, const int32_t* tiles, const int32_t* n_tiles,
-                                int tile_rows, int max_tiles, int T, int K, int N, int top, int stage, int act, float alpha, void* stream) {
+                                int tile_rows, int max_tiles, int places, int T, int K, int N, int top, int stage, int act, float alpha,
+                                void* workspace, size_t workspace_elems, void* stream) {
   MLORA_CHECK(y && x && W && perm && tiles && n_tiles && T >= 0 && K > 0 && N > 0 && top > 0 && tile_rows == FB, MLORA_ERR_INVALID,
               "moe_linear: null pointer or bad shape (tile_rows=%d)", tile_rows);
+  (void)places; (void)workspace; (void)workspace_elems;      // the matrix-core form's
   if (T == 0) return MLORA_OK;
   F32Linear a = {};
   a.y = (float*)y; a.x = (const float*)x; a.W = (const float*)W;

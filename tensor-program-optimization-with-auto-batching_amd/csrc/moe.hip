@@ -68,9 +68,9 @@ __global__ __launch_bounds__(PL_THREADS) void moe_plan_kernel(int32_t* __restric
     const int lane = threadIdx.x;
     int base = 0, tbase = 0;
     for (int e0 = 0; e0 < E; e0 += WAVE) {
-      const int c = e0 + lane < E ? count[e0 + lane] : 0;
+      const int c = e0 + lane < E ? count[e0 + lane] : 0, cp = (c + 15) & ~15;
       const int nt = (c + tile_rows - 1) / tile_rows;
-      int s = c, ts = nt;
+      int s = cp, ts = nt;
 #pragma unroll
       for (int o = 1; o < WAVE; o <<= 1) {
         const int a = __shfl_up(s, o, WAVE), b = __shfl_up(ts, o, WAVE);
@@ -80,18 +80,22 @@ __global__ __launch_bounds__(PL_THREADS) void moe_plan_kernel(int32_t* __restric
         }
       }
       if (e0 + lane < E) {
-        first[e0 + lane] = base + s - c;
+        first[e0 + lane] = base + s - cp;
         tile0[e0 + lane] = tbase + ts - nt;
       }
       base += __shfl(s, WAVE - 1, WAVE);
       tbase += __shfl(ts, WAVE - 1, WAVE);
     }
-    if (lane == 0) *n_tiles = tbase;
+    if (lane == 0) {
+      n_tiles[0] = tbase;
+      n_tiles[1] = base;
+    }
   }
   __syncthreads();
   for (int e = threadIdx.x; e < E; e += PL_THREADS) {
     const int c = count[e];
     for (int i = 0, k = 0; i < c; i += tile_rows, ++k) tiles[tile0[e] + k] = make_int4(e, first[e] + i, c - i < tile_rows ? c - i : tile_rows, 0);
+    for (int i = c; i & 15; ++i) perm[first[e] + i] = -1;
     count[e] = 0;
   }
   __syncthreads();
@@ -201,68 +205,16 @@ __global__ __launch_bounds__(MG_WAVES* WAVE) void moe_gemv_kernel(MoeLinear a, M
   }
 }
 
-// Tiles of 128 entries: a wave owns 64 entries x 64 rows, four waves 128 x 128, operands straight into registers, one k-step
-// ahead.  Blocks of one expert's rows are neighbours in the grid.
-constexpr int MM_ROWS = 128;
-__global__ __launch_bounds__(256) void moe_gemm_kernel(MoeLinear a, MoePlan plan) {
-  if ((int)blockIdx.y >= *plan.n_tiles) return;
-  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
-  const int4 tile = plan.tiles[blockIdx.y];
-  const int KB = a.K / 32, ntiles = a.N / 16;
-  const int nt0 = blockIdx.x * 8 + (wave & 1) * 4, r0 = (wave >> 1) * 64;
-  if (nt0 >= ntiles || r0 >= tile.z) return;
-  const int r16 = lane & 15, g = lane >> 4;
-  const elt* xp[4];
-  const elt* wp[4];
-#pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    const int r = r0 + j * 16 + r16;
-    const int place = tile.y + (r < tile.z ? r : tile.z - 1);
-    xp[j] = a.x + (size_t)(a.up ? plan.perm[place] / a.top : place) * a.K + g * 8;
-    const int nt = nt0 + j < ntiles ? nt0 + j : ntiles - 1;
-    wp[j] = a.W + tile.x * a.w_elems + (size_t)nt * KB * 512 + lane * 8;
-  }
-  f32x4 acc[4][4];
-#pragma unroll
-  for (int i = 0; i < 4; ++i)
-#pragma unroll
-    for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-  eltx8 w[4], b[4];
-#pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    w[i] = ld8(wp[i]);
-    b[i] = ld8(xp[i]);
-  }
-  for (int ks = 1; ks <= KB; ++ks) {
-    const int kc = ks < KB ? ks : 0;         // the last prefetch wraps to a valid address and is discarded
-    eltx8 wn[4], bn[4];
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      wn[i] = ld8(wp[i] + (size_t)kc * 512);
-      bn[i] = ld8(xp[i] + kc * 32);
-    }
-#pragma unroll
-    for (int i = 0; i < 4; ++i)
-#pragma unroll
-      for (int j = 0; j < 4; ++j) acc[i][j] = mfma_16x16x32(w[i], b[j], acc[i][j]);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      w[i] = wn[i];
-      b[i] = bn[i];
-    }
-  }
-#pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    const int r = r0 + j * 16 + r16;
-    if (r >= tile.z) continue;
-    const int p = tile.y + r;
-    elt* yr = a.y + (size_t)(a.up ? p : plan.perm[p]) * a.N;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int n = (nt0 + i) * 16 + g * 4;
-      if (n < a.N) *reinterpret_cast<eltx4*>(yr + n) = moe_out(acc[i][j], a);
-    }
-  }
+// the token rows of the places, in fragment order: a wave copies one fragment (16 places x 32 columns)
+constexpr int MM_ROWS = 256;
+__global__ __launch_bounds__(256) void moe_gather_kernel(elt* __restrict__ xf, const elt* __restrict__ x, const int32_t* __restrict__ perm,
+                                                         const int32_t* __restrict__ n_tiles, int x_tt, int K, int top) {
+  const int lane = threadIdx.x & 63, ks = blockIdx.x * 4 + (threadIdx.x >> 6), tt = blockIdx.y;
+  if (tt * 16 >= n_tiles[1] || ks * 32 >= K) return;
+  const int entry = perm[tt * 16 + (lane & 15)];
+  eltx8 v = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
+  if (entry >= 0) v = ld8(x + (size_t)(entry / top) * K + ks * 32 + (lane >> 4) * 8);
+  st8(xf + ((size_t)ks * x_tt + tt) * 512 + lane * 8, v);
 }
 #endif
 
@@ -279,7 +231,7 @@ extern "C" int mlora_moe_route(int32_t* pick, float* weight, const float* logits
   return mlora_launch_status("moe_route");
 }
 
-// rows per expert tile for this many entries (the fp32 build has one size)
+// places per expert tile for this many entries (the fp32 build has one size)
 extern "C" int mlora_moe_tile_rows(int T, int E, int top) {
 #ifdef MLORA_ELT_F32
   return 64;
@@ -288,11 +240,17 @@ extern "C" int mlora_moe_tile_rows(int T, int E, int top) {
 #endif
 }
 
-// an upper bound of the tiles of a plan, whatever the routing
+// upper bounds, whatever the routing: tiles, and places (a multiple of 16)
 extern "C" int mlora_moe_max_tiles(int T, int E, int top) {
   if (T <= 0 || E <= 0 || top <= 0) return 0;
   const long n = (long)T * top;
   return (int)(n / mlora_moe_tile_rows(T, E, top) + (n < E ? n : E));
+}
+
+extern "C" int mlora_moe_max_places(int T, int E, int top) {
+  if (T <= 0 || E <= 0 || top <= 0) return 0;
+  const long n = (long)T * top;
+  return (int)((n + 15 * (n < E ? n : E) + 15) / 16 * 16);
 }
 
 extern "C" int mlora_moe_plan(int32_t* perm, int32_t* tiles, int32_t* n_tiles, const int32_t* pick, int T, int E, int top, void* stream) {
@@ -317,20 +275,34 @@ extern "C" int mlora_moe_combine(float* x, const float* part, int n_part, const 
 
 #ifndef MLORA_ELT_F32
 extern "C" int mlora_moe_linear(void* y, const void* x, const void* W, const int32_t* perm, const int32_t* tiles, const int32_t* n_tiles,
-                                int tile_rows, int max_tiles, int T, int K, int N, int top, int stage, int act, float alpha, void* stream) {
+                                int tile_rows, int max_tiles, int places, int T, int K, int N, int top, int stage, int act, float alpha,
+                                void* workspace, size_t workspace_elems, void* stream) {
   MLORA_CHECK(y && x && W && perm && tiles && n_tiles, MLORA_ERR_INVALID, "moe_linear: null pointer");
   MLORA_CHECK(T >= 0 && K > 0 && K % 32 == 0 && N > 0 && N % 16 == 0 && top > 0 && max_tiles >= 0 && max_tiles <= 65535 &&
-                  (long)N * K < (1L << 31) && (tile_rows == 16 || tile_rows == MM_ROWS),
+                  (long)N * K < (1L << 31) && (tile_rows == 16 || tile_rows == MM_ROWS) && places % 16 == 0 && places / 16 <= 65535,
               MLORA_ERR_UNSUPPORTED, "moe_linear: need K %% 32 == 0, N %% 16 == 0 (T=%d K=%d N=%d tiles=%d)", T, K, N, max_tiles);
   if (T == 0 || max_tiles == 0) return MLORA_OK;
-  MoeLinear a;
-  a.y = (elt*)y; a.x = (const elt*)x; a.W = (const elt*)W; a.w_elems = (size_t)N * K;
-  a.K = K; a.N = N; a.top = top; a.up = stage == MLORA_MOE_UP; a.act = act; a.alpha = alpha;
   MoePlan p;
   p.perm = perm; p.tiles = (const int4*)tiles; p.n_tiles = n_tiles;
   hipStream_t s = (hipStream_t)stream;
-  if (tile_rows == 16) hipLaunchKernelGGL((moe_gemv_kernel<2, 4>), dim3(ceil_div(N, 32), max_tiles), dim3(MG_WAVES * WAVE), 0, s, a, p);
-  else hipLaunchKernelGGL(moe_gemm_kernel, dim3(ceil_div(N, 128), max_tiles), dim3(256), 0, s, a, p);
+  if (tile_rows == MM_ROWS) {
+    MLORA_CHECK(K % 64 == 0 && N % 32 == 0 && (((uintptr_t)x | (uintptr_t)y | (uintptr_t)workspace) & 15) == 0, MLORA_ERR_UNSUPPORTED,
+                "moe_linear: 256-place tiles need K %% 64 == 0, N %% 32 == 0, aligned operands (K=%d N=%d)", K, N);
+    MLORA_CHECK(act == (stage == MLORA_MOE_UP ? MLORA_ACT_RELU2 : MLORA_ACT_NONE), MLORA_ERR_UNSUPPORTED,
+                "moe_linear: over 256-place tiles the up stage squares its positive part, the down stage does not");
+    const void* xf = x;
+    if (stage == MLORA_MOE_UP) {
+      MLORA_CHECK(workspace && workspace_elems >= (size_t)places * K, MLORA_ERR_WORKSPACE, "moe_linear: workspace of %zu elements needed", (size_t)places * K);
+      hipLaunchKernelGGL(moe_gather_kernel, dim3(ceil_div(K, 128), places / 16), dim3(256), 0, s, (elt*)workspace, (const elt*)x, perm, n_tiles,
+                         places / 16, K, top);
+      xf = workspace;
+    }
+    return mlora_gemm_grouped(y, xf, places / 16, W, p, max_tiles, K, N, stage == MLORA_MOE_UP, alpha, stream);
+  }
+  MoeLinear a;
+  a.y = (elt*)y; a.x = (const elt*)x; a.W = (const elt*)W; a.w_elems = (size_t)N * K;
+  a.K = K; a.N = N; a.top = top; a.up = stage == MLORA_MOE_UP; a.act = act; a.alpha = alpha;
+  hipLaunchKernelGGL((moe_gemv_kernel<2, 4>), dim3(ceil_div(N, 32), max_tiles), dim3(MG_WAVES * WAVE), 0, s, a, p);
   return mlora_launch_status("moe_linear");
 }
 #endif

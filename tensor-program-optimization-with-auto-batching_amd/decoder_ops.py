@@ -14,6 +14,11 @@ def pad32(n: int) -> int:
     return -(-n // 32) * 32
 
 
+def pad64(n: int) -> int:
+    """Row widths: the matrix-core kernels for many tokens take K in steps of 64."""
+    return -(-n // 64) * 64
+
+
 def padded(w: torch.Tensor, *shape) -> torch.Tensor:
     """`w` with zeros behind its rows / columns up to `shape`."""
     if tuple(w.shape) == tuple(shape):
@@ -195,25 +200,29 @@ def moe_route(logits, bias, scale, top, dtype):
 
 
 class MoePlan:
-    """The (token, choice) entries of a routing sorted by expert and cut into tiles."""
+    """The (token, choice) entries of a routing sorted by expert into places and cut into tiles."""
 
     def __init__(self, pick, E, dtype):
         self.T, self.top = pick.shape
         L, dev = lib_of(dtype), pick.device
         self.tile_rows = L.mlora_moe_tile_rows(self.T, E, self.top)
         self.max_tiles = L.mlora_moe_max_tiles(self.T, E, self.top)
+        self.places = L.mlora_moe_max_places(self.T, E, self.top)
         i32 = lambda n: torch.empty(n, dtype=torch.int32, device=dev)
-        self.perm, self.tiles, self.n_tiles = i32(self.T * self.top), i32(4 * self.max_tiles), i32(1)
+        self.perm, self.tiles, self.n_tiles = i32(self.places), i32(4 * self.max_tiles), i32(2)
         check(L.mlora_moe_plan(self.perm.data_ptr(), self.tiles.data_ptr(), self.n_tiles.data_ptr(), _dev(pick, torch.int32), self.T, E, self.top,
                                _stream()), dtype)
 
 
 def moe_linear(x, W, plan, N, K, stage, act=ACT_NONE, alpha=1.0):
-    """Expert linears over a plan: stage MOE_UP: x [T, K] token rows -> place rows [T * top, N]; MOE_DOWN: place rows ->
-    entry rows.  W: the experts' [N, K] matrices stacked."""
-    y = torch.empty((plan.T * plan.top, N), dtype=x.dtype, device=x.device)
+    """Expert linears over a plan: stage MOE_UP: x [T, K] token rows -> places (rows [places, N], or those in fragment order
+    where the plan's tiles are large); MOE_DOWN: places -> entry rows [T * top, N].  W: the experts' [N, K] matrices stacked."""
+    up = stage == MOE_UP
+    y = torch.empty((plan.places if up else plan.T * plan.top, N), dtype=x.dtype, device=x.device)
+    ws = torch.empty(plan.places * K, dtype=x.dtype, device=x.device) if up and plan.tile_rows == 256 else None
     check(lib_of(x.dtype).mlora_moe_linear(_dev(y), _dev(x), _wptr(W), plan.perm.data_ptr(), plan.tiles.data_ptr(), plan.n_tiles.data_ptr(),
-                                           plan.tile_rows, plan.max_tiles, plan.T, K, N, plan.top, stage, act, alpha, _stream()), x.dtype)
+                                           plan.tile_rows, plan.max_tiles, plan.places, plan.T, K, N, plan.top, stage, act, alpha, _ptr(ws),
+                                           ws.numel() if ws is not None else 0, _stream()), x.dtype)
     return y
 
 

@@ -7,7 +7,7 @@ import torch
 
 from . import decoder_ops as D
 from . import ops
-from .decoder_ops import pad32, padded
+from .decoder_ops import pad32, pad64, padded
 
 
 @dataclasses.dataclass(frozen=True)
@@ -29,8 +29,8 @@ class ClippedGlu:
 
     def __init__(self, spec: ClippedGluSpec, w: dict, width: int, gain: float, dtype, device):
         self.spec, self.gain, self.dtype = spec, float(gain), dtype
-        Hp = pad32(width)
-        self.ffp = pad32(spec.ff)
+        Hp = pad64(width)
+        self.ffp = pad64(spec.ff)
         gu = torch.cat([padded(w[k].to(device, dtype), self.ffp, Hp) for k in ("gate", "up")])
         self.gate_up = D.weight(gu)
         self.gate_up_il = ops.interleave_gate_up(gu) if dtype != torch.float32 else None
@@ -47,7 +47,7 @@ class MoeRelu2:
     def __init__(self, spec: MoeSpec, w: dict, width: int, gain: float, dtype, device):
         """w: router [E, width], router_b [E], up: E x [ff, width], down: E x [width, ff]."""
         self.spec, self.gain, self.dtype = spec, float(gain), dtype
-        E, self.Hp, self.ffp = spec.experts, pad32(width), pad32(spec.ff)
+        E, self.Hp, self.ffp = spec.experts, pad64(width), pad64(spec.ff)
         self.router = D.weight(padded(w["router"].to(device, dtype), pad32(E), self.Hp))
         self.bias = w["router_b"].to(device, torch.float32).contiguous()
         stack = lambda ws, n, k: D.weight(torch.cat([padded(m.to(device, dtype), n, k) for m in ws]))

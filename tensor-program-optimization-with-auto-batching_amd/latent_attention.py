@@ -13,7 +13,7 @@ from typing import Optional
 import torch
 
 from . import decoder_ops as D
-from .decoder_ops import pad32, padded
+from .decoder_ops import pad32, pad64, padded
 from .rotary import Rotation
 
 
@@ -44,7 +44,7 @@ class LatentAttention:
         kv_from, dkv [kv_rank + rot_dim, width], dkv_norm [kv_rank]."""
         s, self.spec = spec, spec
         self.gain, self.eps, self.dtype = float(gain), float(eps), dtype
-        H, R, Hp = s.heads, s.kv_rank, pad32(width)
+        H, R, Hp = s.heads, s.kv_rank, pad64(width)
         self.dp, self.vp, self.rank_p = pad32(s.dim), pad32(s.vdim), pad32(R)
         self.q_cols = self.rank_p + pad32(s.rot_dim)
         self.out_cols = H * self.vp

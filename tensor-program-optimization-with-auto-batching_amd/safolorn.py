@@ -18,7 +18,7 @@ import torch
 
 from . import decoder_ops as D
 from . import ops
-from .decoder_ops import pad32, padded
+from .decoder_ops import pad32, pad64, padded
 from .feed_forward import ClippedGlu, ClippedGluSpec, MoeRelu2, MoeSpec
 from .kv_cache import PagedLatentCache
 from .latent_attention import LatentAttention, LatentSpec
@@ -64,7 +64,7 @@ class SafolornConfig:
 @dataclasses.dataclass
 class TokenHidden:
     """Residual stream of a pass with the token ids that its layers look up."""
-    x: torch.Tensor            # [T, pad32(width)] fp32
+    x: torch.Tensor            # [T, pad64(width)] fp32
     ids: torch.Tensor          # [T] int32
 
     @property
@@ -78,7 +78,7 @@ class SafolornForCausalLM(CausalLM):
     def __init__(self, config: SafolornConfig, dtype=torch.bfloat16, device="cuda:0"):
         self.config, self.dtype, self.device = config, dtype, torch.device(device)
         self.layers = []
-        self.width_p = pad32(config.width)
+        self.width_p = pad64(config.width)
         self.embed_tokens = self.side_embed = self.head = None
         self.final_gain = 1.0
 

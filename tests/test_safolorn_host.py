@@ -112,11 +112,13 @@ def test_decoder_argument_validation():
     for lib in (b, f):
         for T, E, top in ((1, 6, 2), (40, 6, 2), (1000, 64, 8)):
             rows = lib.mlora_moe_tile_rows(T, E, top)
-            assert lib.mlora_moe_max_tiles(T, E, top) >= -(-T * top // rows)
+            assert lib.mlora_moe_max_tiles(T, E, top) >= -(-T * top // rows) and lib.mlora_moe_max_places(T, E, top) >= T * top
+    ml = lambda rows=32, K=64, stage=0, act=1, ws=16, n=1 << 20: b.mlora_moe_linear(16, 16, 16, 16, 16, 16, rows, 4, 64, 4, K, 64, 2, stage, act, 1.0, ws, n,
+                                                                                     None)
+    assert ml() == -2 and ml(rows=256, K=96) == -2 and ml(rows=256, act=0) == -2 and ml(rows=256, n=64) == -3 and ml(rows=16, K=40) == -2
     lp = lambda pages=4, dim=64, elems=1 << 30, sc=16: b.mlora_latent_prefill(16, 0, 64, 16, 64, 16, 16, 16, pages, 16, 1, 16, 16, None, 0.1, 8, 2, 64, dim, 16,
                                                                               64, 8, sc, elems, None)
     assert lp(pages=5) == -2 and lp(dim=256) == -2 and lp(elems=8) == -3 and lp(sc=None) == -1
-    assert b.mlora_moe_linear(16, 16, 16, 16, 16, 16, 32, 4, 4, 32, 32, 2, 0, 0, 1.0, None) == -2
 
 
 # ------------------------------------------------------------------ the oracle by what the equations fix

@@ -290,7 +290,7 @@ def test_latent_prep(D, dt, scaling):
 def test_experts(D, ops, dt, T, E, top):
     rng = np.random.default_rng(T + E)
     Wd, ff = 72, 40
-    Hp, fp = D.pad32(Wd), D.pad32(ff)
+    Hp = D.pad64(Wd)
     P = {"x.mlp.router": f64(rnd(rng, E, Wd, std=Wd ** -0.5)), "x.mlp.router.b": f64(rnd(rng, E))}
     for e in range(E):
         P[f"x.mlp.e{e}.up"], P[f"x.mlp.e{e}.down"] = f64(rnd(rng, ff, Wd, std=Wd ** -0.5)), f64(rnd(rng, Wd, ff, std=ff ** -0.5))
@@ -311,11 +311,13 @@ def test_experts(D, ops, dt, T, E, top):
     # the plan covers every entry once, tiles hold one expert
     plan = D.MoePlan(pick, E, dt)
     torch.cuda.synchronize()
-    tiles, perm = plan.tiles.view(-1, 4).cpu().numpy()[: int(plan.n_tiles)], plan.perm.cpu().numpy()
-    assert sorted(perm) == list(range(T * top)) and int(plan.n_tiles) <= plan.max_tiles and tiles[:, 2].sum() == T * top
+    tiles, perm = plan.tiles.view(-1, 4).cpu().numpy()[: int(plan.n_tiles[0])], plan.perm.cpu().numpy()
+    used = int(plan.n_tiles[1])
+    assert used <= plan.places and used % 16 == 0 and sorted(p for p in perm[:used] if p >= 0) == list(range(T * top))
+    assert len(tiles) <= plan.max_tiles and tiles[:, 2].sum() == T * top
     flat = order.reshape(-1)
     for e, first, n, _ in tiles:
-        assert 0 < n <= plan.tile_rows and (flat[perm[first:first + n]] == e).all()
+        assert 0 < n <= plan.tile_rows and first % 16 == 0 and (flat[perm[first:first + n]] == e).all()
     # the whole block; in bf16 on the router's own fp32 logits of the rounded input, so that choices agree
     resid = rnd(rng, T, Hp)
     before, kp, sums = f64(resid), None, None
