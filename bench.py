@@ -634,7 +634,7 @@ def bench_safolorn(args, synth, llama):
             model = safolorn_model(size) if kind == "safolorn" else safolorn_llama(size, synth, llama)
             r = {"size": size, "model": kind}
             for B, P in ((8, 512), (1, 4096)):
-                r[f"prefill_{B}x{P}_tok_s"] = B * P / time_prefill(model, B, P, 2, max(2, args.steps // 8))
+                r[f"prefill_{B}x{P}_tok_s"] = B * P / time_prefill(model, B, P, 3, max(2, args.steps // 4))
             for B, ctx in ((1, 512), (32, 512), (128, 2048)):
                 r[f"decode_b{B}_ctx{ctx}_tok_s"] = B / time_decode(model, B, ctx, args.warmup, args.steps)
             rows.append(r)

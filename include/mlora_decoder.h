@@ -33,13 +33,16 @@ int mlora_token_gate_mul(void* out, const void* z, const void* table, int ld_tab
  * rotates the heads' query parts (columns off_rot .. + H rot) into the rows q + (t H + h) q_ld + q_off, padded to whole blocks of
  * 32, and, with c_norm, norms `gain` times the latent (off_c .. + R), rotates `gain` times the shared key part
  * (off_kr .. + rot) and stores both in the token's page slot.
+ * With `lift` [H ceil32(R), lift_k] (packed; bfloat16 library) the same launch lifts the unrotated query parts - the first
+ * lift_k columns per head of qkv - into columns 0 .. ceil32(R) of the rows (q_off = ceil32(R) then).
  * mlora_head_linear: y[t, h] = alpha W[h] . x[t, h].  mlora_latent_attn: causal softmax over the sequence's pages with scores
  * (q . cached) * scale, q [T, H, NB 32], and, with `sink`, exp(sink[h]) in the denominator; out [T, H, ceil32(R)].
- * splits > 1 needs a workspace. */
+ * splits > 1 needs a workspace.  mlora_latent_attn_out (splits > 1) takes the result through W_uv (packed [H vp, ceil32(R)]) in
+ * the launch that merges the splits: y [T, H vp] in either layout. */
 int mlora_latent_prep(void* q, int q_ld, int q_off, void* cache, const void* qkv, int ld, int off_rot, int off_c, int off_kr, float gain,
                       const void* c_norm, float eps, const int32_t* block_table, int max_blocks, const int32_t* tok_seq,
                       const int32_t* tok_pos, const float* rope_cos, const float* rope_sin, int max_pos, int T, int H, int R, int rot,
-                      int n_pages, int n_seq, void* stream);
+                      int n_pages, int n_seq, const void* lift, int lift_k, void* stream);
 int mlora_head_linear(void* y, int y_layout, long ldy, long head_y, const void* x, long ldx, long head_x, const void* W, int heads, int T,
                       int K, int N, float alpha, void* stream);
 int mlora_latent_attn_splits(int T, int H, int max_ctx);
@@ -47,6 +50,9 @@ size_t mlora_latent_attn_workspace_bytes(int T, int H, int R, int splits);
 int mlora_latent_attn(void* out, const void* q, const void* cache, const int32_t* block_table, int max_blocks, const int32_t* tok_seq,
                       const int32_t* tok_pos, const float* sink, float scale, int T, int H, int R, int rot, int n_pages, int n_seq,
                       int splits, void* workspace, size_t workspace_bytes, void* stream);
+int mlora_latent_attn_out(void* y, int y_layout, long ldy, const void* uv, int vp, const void* q, const void* cache, const int32_t* block_table,
+                          int max_blocks, const int32_t* tok_seq, const int32_t* tok_pos, const float* sink, float scale, int T, int H, int R,
+                          int rot, int n_pages, int n_seq, int splits, void* workspace, size_t workspace_bytes, void* stream);
 
 /* The same attention for prompts (bfloat16 library): makes the heads' keys and values of whole contexts in scratch memory and
  * attends over those.  phys [pages]: the cache pages of the contexts one after the other, each context padded with -1 to a

@@ -122,11 +122,12 @@ DECODER_SIGNATURES = {
     "mlora_stream_norm": (_i, [_p, _p, _p, _p, _i, _p, _p, _f, _f, _i, _i, _i, _i, _p]),
     "mlora_token_gate": (_i, [_p, _p, _p, _p, _i, _i, _i, _p, _i, _i, _i, _i, _p]),
     "mlora_token_gate_mul": (_i, [_p, _p, _p, _i, _i, _i, _p, _i, _i, _i, _p]),
-    "mlora_latent_prep": (_i, [_p, _i, _i, _p, _p, _i, _i, _i, _i, _f, _p, _f, _p, _i, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _p]),
+    "mlora_latent_prep": (_i, [_p, _i, _i, _p, _p, _i, _i, _i, _i, _f, _p, _f, _p, _i, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _p, _i, _p]),
     "mlora_head_linear": (_i, [_p, _i, _l, _l, _p, _l, _l, _p, _i, _i, _i, _i, _f, _p]),
     "mlora_latent_attn_splits": (_i, [_i, _i, _i]),
     "mlora_latent_attn_workspace_bytes": (_z, [_i, _i, _i, _i]),
     "mlora_latent_attn": (_i, [_p, _p, _p, _p, _i, _p, _p, _p, _f, _i, _i, _i, _i, _i, _i, _i, _p, _z, _p]),
+    "mlora_latent_attn_out": (_i, [_p, _i, _l, _p, _i, _p, _p, _p, _i, _p, _p, _p, _f, _i, _i, _i, _i, _i, _i, _i, _p, _z, _p]),
     "mlora_latent_prefill_tile_tokens": (_i, []),
     "mlora_latent_prefill_served": (_i, [_i, _i, _i]),
     "mlora_latent_prefill_scratch_elems": (_z, [_i, _i, _i, _i, _i]),
@@ -141,7 +142,7 @@ DECODER_SIGNATURES = {
 }
 
 # ... and those that the fp32 library does not have
-MATRIX_CORE_ONLY = ("mlora_token_gate", "mlora_latent_prefill", "mlora_latent_prefill_tile_tokens", "mlora_latent_prefill_served",
+MATRIX_CORE_ONLY = ("mlora_token_gate", "mlora_latent_attn_out", "mlora_latent_prefill", "mlora_latent_prefill_tile_tokens", "mlora_latent_prefill_served",
                     "mlora_latent_prefill_scratch_elems")
 
 _libs = {}

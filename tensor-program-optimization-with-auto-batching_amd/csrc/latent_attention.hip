@@ -13,6 +13,9 @@
 
 #include "common.h"
 
+// Every kernel with matrix-core products here names its waves per SIMD (two) in its launch bounds: without, the compiler
+// keeps the accumulators in the accumulation registers and has been seen to read them back before a loop's last product
+// had written them.
 namespace {
 
 constexpr int PAGE = MLORA_PAGE_SIZE;
@@ -40,9 +43,7 @@ struct LatentPrep {
 
 // One workgroup per token: rotates the heads' query parts into the query rows (their `gain` is left to the scores' scale),
 // norms the latent, rotates the shared key part and stores both in the token's page slot.  Neighbouring elements (2 i, 2 i + 1) turn by the table's angle i.
-__global__ __launch_bounds__(256) void latent_prep_kernel(LatentPrep a) {
-  __shared__ float red[4];
-  const int t = blockIdx.x;
+__device__ __forceinline__ void latent_prep(const LatentPrep& a, int t, float* __restrict__ red) {
   const int seq = a.tok_seq[t], pos = a.tok_pos[t];
   if (seq < 0 || seq >= a.n_seq || pos < 0 || pos >= a.max_pos || pos / PAGE >= a.max_blocks) return;   // uniform
   const elt* row = a.qkv + (size_t)t * a.ld;
@@ -79,6 +80,11 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(LatentPrep a) {
     *reinterpret_cast<eltx2*>(a.cache + latent_offset(page, a.NB, pos % PAGE, a.RB * 32 + 2 * k)) =
         eltx2{(elt)(x1 * cp[k] - x2 * sp[k]), (elt)(x2 * cp[k] + x1 * sp[k])};
   }
+}
+
+__global__ __launch_bounds__(256) void latent_prep_kernel(LatentPrep a) {
+  __shared__ float red[4];
+  latent_prep(a, blockIdx.x, red);
 }
 
 struct LatentAttn {
@@ -328,8 +334,9 @@ struct LatentExpand {
   int kb_blocks, vb_blocks; // workgroups along x that make keys, then values; one more copies R
 };
 
-// a wave makes 64 rows (of W_uk or W_uv) x 4 pages
-__global__ __launch_bounds__(256) void latent_expand_kernel(LatentExpand a) {
+// a wave makes 16 LE_ROWS rows (of W_uk or W_uv) x 4 pages
+constexpr int LE_ROWS = 4;
+__global__ __launch_bounds__(256, 2) void latent_expand_kernel(LatentExpand a) {
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
   const int pg0 = blockIdx.y * 4, NB = a.RB + a.KR;
   int page[4];
@@ -340,7 +347,8 @@ __global__ __launch_bounds__(256) void latent_expand_kernel(LatentExpand a) {
   }
   const eltx8 zero = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
   int bx = blockIdx.x;
-  if (bx >= a.kb_blocks + a.vb_blocks) {
+  if (bx > a.kb_blocks + a.vb_blocks) return;
+  if (bx == a.kb_blocks + a.vb_blocks) {
     for (int i = threadIdx.x; i < 4 * a.KR * 64; i += 256) {
       const int j = i / (a.KR * 64), o = i - j * (a.KR * 64);
       const int pj = a.phys[pg0 + j];
@@ -352,51 +360,48 @@ __global__ __launch_bounds__(256) void latent_expand_kernel(LatentExpand a) {
   const bool val = bx >= a.kb_blocks;                                // uniform
   if (val) bx -= a.kb_blocks;
   const int tiles = val ? a.H * a.VB : a.H * a.KN * 2;
-  const int nt0 = (bx * 4 + wave) * 4;
+  const int nt0 = (bx * 4 + wave) * LE_ROWS;
   if (nt0 >= tiles) return;
-  const elt* wp[4];
+  const elt* wp = (val ? a.uv : a.uk) + lane * 8;
+  int wo[LE_ROWS];                                                   // uniform
   const elt* cp[4];
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    wp[i] = (val ? a.uv : a.uk) + (size_t)(nt0 + i < tiles ? nt0 + i : tiles - 1) * a.RB * 512 + lane * 8;
-    cp[i] = a.cache + (size_t)(page[i] >= 0 ? page[i] : 0) * NB * 512 + lane * 8;
-  }
-  f32x4 acc[4][4];
+  for (int i = 0; i < LE_ROWS; ++i) wo[i] = (nt0 + i < tiles ? nt0 + i : tiles - 1) * a.RB * 512;
 #pragma unroll
-  for (int i = 0; i < 4; ++i)
+  for (int i = 0; i < 4; ++i) cp[i] = a.cache + (size_t)(page[i] >= 0 ? page[i] : 0) * NB * 512 + lane * 8;
+  f32x4 acc[LE_ROWS][4];
+#pragma unroll
+  for (int i = 0; i < LE_ROWS; ++i)
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
   auto products = [&](auto V) {
-    eltx8 w[4], c[4];
+    eltx8 w[LE_ROWS], c[4];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      w[i] = ld8(wp[i]);
-      c[i] = ld8(cp[i]);
-    }
+    for (int i = 0; i < LE_ROWS; ++i) w[i] = ld8(wp + wo[i]);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) c[i] = ld8(cp[i]);
     for (int kb = 1; kb <= a.RB; ++kb) {
       const int kc = kb < a.RB ? kb : 0;                             // the last prefetch wraps to a valid address and is discarded
-      eltx8 wn[4], cn[4];
+      eltx8 wn[LE_ROWS], cn[4];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        wn[i] = ld8(wp[i] + kc * 512);
-        cn[i] = ld8(cp[i] + kc * 512);
-      }
+      for (int i = 0; i < LE_ROWS; ++i) wn[i] = ld8(wp + (wo[i] + kc * 512));
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
+      for (int i = 0; i < 4; ++i) cn[i] = ld8(cp[i] + kc * 512);
+#pragma unroll
+      for (int i = 0; i < LE_ROWS; ++i)
 #pragma unroll
         for (int j = 0; j < 4; ++j) acc[i][j] = decltype(V)::value ? mfma_16x16x32(c[j], w[i], acc[i][j]) : mfma_16x16x32(w[i], c[j], acc[i][j]);
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        w[i] = wn[i];
-        c[i] = cn[i];
-      }
+      for (int i = 0; i < LE_ROWS; ++i) w[i] = wn[i];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) c[i] = cn[i];
     }
   };
   if (val) products(std::true_type());
   else products(std::false_type());
   const int r16 = lane & 15, g = lane >> 4;
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
+  for (int i = 0; i < LE_ROWS; ++i) {
     const int nt = nt0 + i;
     if (nt >= tiles) continue;
 #pragma unroll
@@ -595,51 +600,166 @@ __global__ __launch_bounds__(LP_WAVES* WAVE, 2) void latent_prefill_kernel(Laten
 }
 
 // y[t, h] = alpha * W[h] . x[t, h] per head: W[h] packed [N, K], N % 16 == 0.  A wave owns 16 NI rows x 16 TJ tokens.
+struct HeadLinear {
+  elt* y;
+  long ldy, hy;
+  int frag_tt;
+  const elt* x;
+  long ldx, hx;
+  const elt* W;
+  int T, K, N;
+  float alpha;
+};
+
 template <int NI, int TJ>
-__global__ __launch_bounds__(256) void head_linear_kernel(elt* __restrict__ y, long ldy, long hy, int frag_tt, const elt* __restrict__ x, long ldx,
-                                                          long hx, const elt* __restrict__ Wp, int T, int K, int N, float alpha) {
+__device__ __forceinline__ void head_linear(const HeadLinear& a, int bx, int by, int h) {
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
-  const int h = blockIdx.z, t0 = blockIdx.y * 16 * TJ;
-  const int KB = K / 32, tiles = N / 16, nt0 = (blockIdx.x * 4 + wave) * NI;
+  const int t0 = by * 16 * TJ;
+  const int KB = a.K / 32, tiles = a.N / 16, nt0 = (bx * 4 + wave) * NI;
   if (nt0 >= tiles) return;
   const int r16 = lane & 15, g = lane >> 4;
   const elt* wp[NI];
   const elt* xp[TJ];
 #pragma unroll
-  for (int i = 0; i < NI; ++i) wp[i] = Wp + ((size_t)h * tiles + (nt0 + i < tiles ? nt0 + i : tiles - 1)) * KB * 512 + lane * 8;
+  for (int i = 0; i < NI; ++i) wp[i] = a.W + ((size_t)h * tiles + (nt0 + i < tiles ? nt0 + i : tiles - 1)) * KB * 512 + lane * 8;
 #pragma unroll
   for (int j = 0; j < TJ; ++j) {
     const int t = t0 + j * 16 + r16;
-    xp[j] = x + (t < T ? t : T - 1) * ldx + h * hx + g * 8;
+    xp[j] = a.x + (t < a.T ? t : a.T - 1) * a.ldx + h * a.hx + g * 8;
   }
   f32x4 acc[NI][TJ];
 #pragma unroll
   for (int i = 0; i < NI; ++i)
 #pragma unroll
     for (int j = 0; j < TJ; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-  for (int ks = 0; ks < KB; ++ks) {
-    eltx8 w[NI], b[TJ];
+  constexpr int U = NI * TJ > 4 ? 1 : 4;                             // k-steps requested together
+  for (int k0 = 0; k0 < KB; k0 += U) {
+    eltx8 w[U][NI], b[U][TJ];
 #pragma unroll
-    for (int i = 0; i < NI; ++i) w[i] = ld8(wp[i] + (size_t)ks * 512);
+    for (int u = 0; u < U; ++u) {
+      const int ks = k0 + u < KB ? k0 + u : k0;                      // past K: a valid address, zeroed
 #pragma unroll
-    for (int j = 0; j < TJ; ++j) b[j] = ld8(xp[j] + ks * 32);
+      for (int i = 0; i < NI; ++i) w[u][i] = ld8(wp[i] + (size_t)ks * 512);
 #pragma unroll
-    for (int i = 0; i < NI; ++i)
+      for (int j = 0; j < TJ; ++j) {
+        b[u][j] = ld8(xp[j] + ks * 32);
+        if (k0 + u >= KB) b[u][j] = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
+      }
+    }
 #pragma unroll
-      for (int j = 0; j < TJ; ++j) acc[i][j] = mfma_16x16x32(w[i], b[j], acc[i][j]);
+    for (int u = 0; u < U; ++u)
+#pragma unroll
+      for (int i = 0; i < NI; ++i)
+#pragma unroll
+        for (int j = 0; j < TJ; ++j) acc[i][j] = mfma_16x16x32(w[u][i], b[u][j], acc[i][j]);
   }
 #pragma unroll
   for (int j = 0; j < TJ; ++j) {
     const int t = t0 + j * 16 + r16;
-    if (t >= T) continue;
+    if (t >= a.T) continue;
 #pragma unroll
     for (int i = 0; i < NI; ++i) {
       const int n = (nt0 + i) * 16 + g * 4;
-      if (n >= N) continue;
-      const f32x4 s = acc[i][j] * alpha;
-      elt* p = frag_tt ? y + frag_offset(t, (int)(h * hy) + n, frag_tt) : y + t * ldy + h * hy + n;
+      if (n >= a.N) continue;
+      const f32x4 s = acc[i][j] * a.alpha;
+      elt* p = a.frag_tt ? a.y + frag_offset(t, (int)(h * a.hy) + n, a.frag_tt) : a.y + t * a.ldy + h * a.hy + n;
       *reinterpret_cast<eltx4*>(p) = eltx4{(elt)s[0], (elt)s[1], (elt)s[2], (elt)s[3]};
     }
+  }
+}
+
+template <int NI, int TJ>
+__global__ __launch_bounds__(256, 2) void head_linear_kernel(HeadLinear a) {
+  head_linear<NI, TJ>(a, blockIdx.x, blockIdx.y, blockIdx.z);
+}
+
+// latent_prep and the lifting of the queries (which need nothing of each other) in one launch: T workgroups, then nx * ny * H
+template <int TJ>
+__global__ __launch_bounds__(256, 2) void latent_query_kernel(LatentPrep p, HeadLinear a, int nx, int ny) {
+  __shared__ float red[4];
+  int b = blockIdx.x;
+  if (b < a.T) return latent_prep(p, b, red);                        // uniform
+  b -= a.T;
+  const int bx = b % nx, r = b / nx;
+  head_linear<1, TJ>(a, bx, r % ny, r / ny);
+}
+
+// The splits of (16 tokens, head) added - with the sink's share of the denominator - and taken through W_uv in one launch:
+// the merged context vectors meet the matrix cores from LDS.  grid (H, token tiles).
+constexpr int LO_SPLITS = 32;
+constexpr int LO_WAVES = 8;
+constexpr int LO_PRE = 8;          // weight fragments of a wave's first tile that are requested ahead of the merge
+__global__ __launch_bounds__(LO_WAVES* WAVE, 2) void latent_out_kernel(LatentAttn a, HeadLinear o) {
+  extern __shared__ __align__(16) elt xs[];                          // [RB][64][8]
+  __shared__ float fs[LO_SPLITS][16], ls[LO_SPLITS][16];
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
+  const int h = blockIdx.x, t0 = blockIdx.y * 16, rd = a.RB * 32, tiles = o.N / 16;
+  const size_t n = (size_t)a.T * a.H;
+  for (int i = threadIdx.x; i < a.splits * 16; i += LO_WAVES * WAVE) {
+    const int t = t0 + (i & 15) < a.T ? t0 + (i & 15) : a.T - 1;
+    const float* ml = a.part_ml + 2 * (((size_t)(i >> 4) * a.T + t) * a.H + h);
+    fs[i >> 4][i & 15] = ml[0];
+    ls[i >> 4][i & 15] = ml[1];
+  }
+  const elt* wp = o.W + (size_t)h * tiles * a.RB * 512 + lane * 8;
+  eltx8 w[LO_PRE];
+#pragma unroll
+  for (int u = 0; u < LO_PRE; ++u) w[u] = ld8(wp + ((size_t)(wave < tiles ? wave : 0) * a.RB + (u < a.RB ? u : 0)) * 512);
+  __syncthreads();
+  if (threadIdx.x < 16) {
+    const float sk = a.sink ? a.sink[h] : -INFINITY;
+    float M = sk;
+    for (int s = 0; s < a.splits; ++s) M = fmaxf(M, fs[s][threadIdx.x]);
+    float L = sk != -INFINITY ? __expf(sk - M) : 0.f;
+    for (int s = 0; s < a.splits; ++s) {
+      const float m = fs[s][threadIdx.x], f = m == -INFINITY ? 0.f : __expf(m - M);
+      fs[s][threadIdx.x] = f;
+      L += ls[s][threadIdx.x] * f;
+    }
+    const float inv = L > 0.f ? 1.f / L : 0.f;
+    for (int s = 0; s < a.splits; ++s) fs[s][threadIdx.x] *= inv;
+  }
+  // the splits are added as they come: four splits of a thread's eight values are in flight at a time
+  for (int i0 = 0; i0 < a.RB * 64; i0 += LO_WAVES * WAVE) {
+    const int i = i0 + threadIdx.x, ic = i < a.RB * 64 ? i : 0, tk = ic & 15, t = t0 + tk < a.T ? t0 + tk : a.T - 1;
+    const float* p = a.part_o + ((size_t)t * a.H + h) * rd + (ic >> 6) * 32 + ((ic >> 4) & 3) * 8;
+    f32x4 lo = f32x4{0.f, 0.f, 0.f, 0.f}, hi = lo;
+    for (int s0 = 0; s0 < a.splits; s0 += 4) {
+      f32x4 v[4][2];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const float* ps = p + (size_t)(s0 + u < a.splits ? s0 + u : s0) * n * rd;
+        v[u][0] = *reinterpret_cast<const f32x4*>(ps);
+        v[u][1] = *reinterpret_cast<const f32x4*>(ps + 4);
+      }
+      if (i0 == 0 && s0 == 0) __syncthreads();                       // the factors
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const float f = s0 + u < a.splits ? fs[s0 + u][tk] : 0.f;
+        lo += v[u][0] * f;
+        hi += v[u][1] * f;
+      }
+    }
+    if (i < a.RB * 64)
+      st8(xs + i * 8, eltx8{(elt)lo[0], (elt)lo[1], (elt)lo[2], (elt)lo[3], (elt)hi[0], (elt)hi[1], (elt)hi[2], (elt)hi[3]});
+  }
+  __syncthreads();
+  const int r16 = lane & 15, g = lane >> 4, t = t0 + r16;
+  for (int nt = wave; nt < tiles; nt += LO_WAVES) {
+    f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int k0 = 0; k0 < a.RB; k0 += LO_PRE) {
+      if (nt != wave || k0 > 0) {                                    // uniform
+#pragma unroll
+        for (int u = 0; u < LO_PRE; ++u) w[u] = ld8(wp + ((size_t)nt * a.RB + (k0 + u < a.RB ? k0 + u : k0)) * 512);
+      }
+#pragma unroll
+      for (int u = 0; u < LO_PRE; ++u)
+        if (k0 + u < a.RB) acc = mfma_16x16x32(w[u], ld8(xs + ((k0 + u) * 64 + lane) * 8), acc);   // uniform
+    }
+    if (t >= a.T) continue;
+    const int c = nt * 16 + g * 4;
+    elt* p = o.frag_tt ? o.y + frag_offset(t, (int)(h * o.hy) + c, o.frag_tt) : o.y + t * o.ldy + h * o.hy + c;
+    *reinterpret_cast<eltx4*>(p) = eltx4{(elt)acc[0], (elt)acc[1], (elt)acc[2], (elt)acc[3]};
   }
 }
 
@@ -726,10 +846,11 @@ int launch_latent_attn(const LatentAttn& a, hipStream_t s) {
 
 }  // namespace
 
+// lift [H * RB * 32, lift_k] packed (or NULL): the unrotated query parts (columns 0.. of qkv, lift_k per head) lifted into q
 extern "C" int mlora_latent_prep(void* q, int q_ld, int q_off, void* cache, const void* qkv, int ld, int off_rot, int off_c, int off_kr, float gain, const void* c_norm,
                                  float eps, const int32_t* block_table, int max_blocks, const int32_t* tok_seq, const int32_t* tok_pos,
                                  const float* rope_cos, const float* rope_sin, int max_pos, int T, int H, int R, int rot, int n_pages, int n_seq,
-                                 void* stream) {
+                                 const void* lift, int lift_k, void* stream) {
   MLORA_CHECK(q && cache && qkv && block_table && tok_seq && tok_pos && rope_cos && rope_sin, MLORA_ERR_INVALID, "latent_prep: null pointer");
   MLORA_CHECK(T >= 0 && H > 0 && R > 0 && rot > 0 && rot % 2 == 0 && off_rot >= 0 && off_rot + H * rot <= ld && max_blocks > 0 && n_pages > 0 &&
                   n_seq > 0 && max_pos > 0 && (!c_norm || (off_c >= 0 && off_kr >= 0 && off_c + R <= ld && off_kr + rot <= ld)),
@@ -743,6 +864,26 @@ extern "C" int mlora_latent_prep(void* q, int q_ld, int q_off, void* cache, cons
   a.q_ld = q_ld; a.q_off = q_off;
   MLORA_CHECK(q_off >= 0 && q_off % 2 == 0 && q_ld % 2 == 0 && q_off + (a.NB - a.RB) * 32 <= q_ld, MLORA_ERR_INVALID,
               "latent_prep: query rows of %d with the rotated part at %d", q_ld, q_off);
+#ifndef MLORA_ELT_F32
+  if (lift) {
+    MLORA_CHECK(lift_k > 0 && lift_k % 32 == 0 && H * lift_k <= ld && ld % 8 == 0 && q_off == a.RB * 32 && q_ld % 4 == 0, MLORA_ERR_UNSUPPORTED,
+                "latent_prep: lifting needs query parts of whole 32 columns ahead of the rest (lift_k=%d ld=%d)", lift_k, ld);
+    HeadLinear l;
+    l.y = (elt*)q; l.ldy = (long)H * q_ld; l.hy = q_ld; l.frag_tt = 0;
+    l.x = (const elt*)qkv; l.ldx = ld; l.hx = lift_k; l.W = (const elt*)lift; l.T = T; l.K = lift_k; l.N = a.RB * 32; l.alpha = 1.f;
+    const int nx = ceil_div(l.N, 64), tj = T <= 16 ? 1 : T <= 32 ? 2 : 4, ny = ceil_div(T, 16 * tj);
+    const long blocks = T + (long)nx * ny * H;
+    MLORA_CHECK(blocks <= 0x7fffffffL, MLORA_ERR_UNSUPPORTED, "latent_prep: T=%d is too many tokens", T);
+    hipStream_t s = (hipStream_t)stream;
+    if (tj == 1) hipLaunchKernelGGL(latent_query_kernel<1>, dim3((unsigned)blocks), dim3(256), 0, s, a, l, nx, ny);
+    else if (tj == 2) hipLaunchKernelGGL(latent_query_kernel<2>, dim3((unsigned)blocks), dim3(256), 0, s, a, l, nx, ny);
+    else hipLaunchKernelGGL(latent_query_kernel<4>, dim3((unsigned)blocks), dim3(256), 0, s, a, l, nx, ny);
+    return mlora_launch_status("latent_prep");
+  }
+#else
+  MLORA_CHECK(!lift, MLORA_ERR_UNSUPPORTED, "latent_prep: the fp32 library lifts queries with mlora_head_linear");
+  (void)lift_k;
+#endif
   hipLaunchKernelGGL(latent_prep_kernel, dim3(T), dim3(256), 0, (hipStream_t)stream, a);
   return mlora_launch_status("latent_prep");
 }
@@ -767,10 +908,10 @@ extern "C" size_t mlora_latent_attn_workspace_bytes(int T, int H, int R, int spl
   return (size_t)splits * T * H * ((size_t)ceil_div(R, 32) * 32 + 2) * sizeof(float);
 }
 
-extern "C" int mlora_latent_attn(void* out, const void* q, const void* cache, const int32_t* block_table, int max_blocks, const int32_t* tok_seq,
-                                 const int32_t* tok_pos, const float* sink, float scale, int T, int H, int R, int rot, int n_pages, int n_seq,
-                                 int splits, void* workspace, size_t workspace_bytes, void* stream) {
-  MLORA_CHECK(out && q && cache && block_table && tok_seq && tok_pos, MLORA_ERR_INVALID, "latent_attn: null pointer");
+// o: a HeadLinear that takes the merged context vectors (nullptr: they go to `out`)
+static int latent_attn_impl(void* out, const void* q, const void* cache, const int32_t* block_table, int max_blocks, const int32_t* tok_seq,
+                            const int32_t* tok_pos, const float* sink, float scale, int T, int H, int R, int rot, int n_pages, int n_seq,
+                            int splits, void* workspace, size_t workspace_bytes, const void* o, void* stream) {
   MLORA_CHECK(T >= 0 && H > 0 && H <= 65535 && R > 0 && rot > 0 && max_blocks > 0 && n_pages > 0 && n_seq > 0 && splits >= 1, MLORA_ERR_INVALID,
               "latent_attn: bad shape T=%d H=%d R=%d rot=%d", T, H, R, rot);
   if (T == 0) return MLORA_OK;
@@ -781,6 +922,7 @@ extern "C" int mlora_latent_attn(void* out, const void* q, const void* cache, co
   a.part_o = a.part_ml = nullptr; a.n_inner = a.chunks = 1;
   hipStream_t s = (hipStream_t)stream;
 #ifdef MLORA_ELT_F32
+  (void)o; (void)workspace; (void)workspace_bytes;
   MLORA_CHECK(splits == 1 && a.NB * 128 <= 48 * 1024, MLORA_ERR_UNSUPPORTED, "latent_attn: splits=%d R=%d not served in fp32", splits, R);
   hipLaunchKernelGGL(latent_attn_f32_kernel, dim3(T, H, ceil_div(a.RB * 32, 256 * LA_DPT)), dim3(256), a.NB * 128, s, a);
 #else
@@ -801,11 +943,36 @@ extern "C" int mlora_latent_attn(void* out, const void* q, const void* cache, co
   if (e) return e;
   if (splits > 1) {
     MLORA_CHECK((long)T * H <= 0x7fffffffL, MLORA_ERR_UNSUPPORTED, "latent_attn: T=%d is too many tokens", T);
-    hipLaunchKernelGGL(latent_merge_kernel, dim3(T * H), dim3(128), 0, s, a);
+    if (o) hipLaunchKernelGGL(latent_out_kernel, dim3(H, ceil_div(T, 16)), dim3(LO_WAVES * WAVE), (size_t)a.RB * 1024, s, a, *(const HeadLinear*)o);
+    else hipLaunchKernelGGL(latent_merge_kernel, dim3(T * H), dim3(128), 0, s, a);
   }
 #endif
   return mlora_launch_status("latent_attn");
 }
+
+extern "C" int mlora_latent_attn(void* out, const void* q, const void* cache, const int32_t* block_table, int max_blocks, const int32_t* tok_seq,
+                                 const int32_t* tok_pos, const float* sink, float scale, int T, int H, int R, int rot, int n_pages, int n_seq,
+                                 int splits, void* workspace, size_t workspace_bytes, void* stream) {
+  MLORA_CHECK(out && q && cache && block_table && tok_seq && tok_pos, MLORA_ERR_INVALID, "latent_attn: null pointer");
+  return latent_attn_impl(out, q, cache, block_table, max_blocks, tok_seq, tok_pos, sink, scale, T, H, R, rot, n_pages, n_seq, splits, workspace,
+                          workspace_bytes, nullptr, stream);
+}
+
+#ifndef MLORA_ELT_F32
+extern "C" int mlora_latent_attn_out(void* y, int y_layout, long ldy, const void* uv, int vp, const void* q, const void* cache,
+                                     const int32_t* block_table, int max_blocks, const int32_t* tok_seq, const int32_t* tok_pos, const float* sink,
+                                     float scale, int T, int H, int R, int rot, int n_pages, int n_seq, int splits, void* workspace,
+                                     size_t workspace_bytes, void* stream) {
+  MLORA_CHECK(y && uv && q && cache && block_table && tok_seq && tok_pos, MLORA_ERR_INVALID, "latent_attn_out: null pointer");
+  MLORA_CHECK(splits > 1 && splits <= LO_SPLITS && vp > 0 && vp % 32 == 0 && (y_layout == MLORA_FRAG || ldy % 4 == 0) && ceil_div(T, 16) <= 65535 &&
+                  R <= 1536,
+              MLORA_ERR_UNSUPPORTED, "latent_attn_out: need 2..%d splits, vp %% 32 == 0 (splits=%d vp=%d R=%d)", LO_SPLITS, splits, vp, R);
+  HeadLinear o = {};
+  o.y = (elt*)y; o.ldy = ldy; o.hy = vp; o.frag_tt = y_layout == MLORA_FRAG ? mlora_frag_tiles(T) : 0; o.W = (const elt*)uv; o.T = T; o.N = vp;
+  return latent_attn_impl(nullptr, q, cache, block_table, max_blocks, tok_seq, tok_pos, sink, scale, T, H, R, rot, n_pages, n_seq, splits, workspace,
+                          workspace_bytes, &o, stream);
+}
+#endif
 
 #ifndef MLORA_ELT_F32
 extern "C" int mlora_head_linear(void* y, int y_layout, long ldy, long head_y, const void* x, long ldx, long head_x, const void* W, int heads, int T,
@@ -817,9 +984,11 @@ extern "C" int mlora_head_linear(void* y, int y_layout, long ldy, long head_y, c
   if (T == 0) return MLORA_OK;
   const int tt = y_layout == MLORA_FRAG ? mlora_frag_tiles(T) : 0;
   hipStream_t s = (hipStream_t)stream;
-#define MLORA_HL(NI, TJ)                                                                                                              \
-  hipLaunchKernelGGL((head_linear_kernel<NI, TJ>), dim3(ceil_div(N, 64 * NI), ceil_div(T, 16 * TJ), heads), dim3(256), 0, s, (elt*)y, \
-                     ldy, head_y, tt, (const elt*)x, ldx, head_x, (const elt*)W, T, K, N, alpha)
+  HeadLinear a;
+  a.y = (elt*)y; a.ldy = ldy; a.hy = head_y; a.frag_tt = tt; a.x = (const elt*)x; a.ldx = ldx; a.hx = head_x; a.W = (const elt*)W;
+  a.T = T; a.K = K; a.N = N; a.alpha = alpha;
+#define MLORA_HL(NI, TJ) \
+  hipLaunchKernelGGL((head_linear_kernel<NI, TJ>), dim3(ceil_div(N, 64 * NI), ceil_div(T, 16 * TJ), heads), dim3(256), 0, s, a)
   if (T <= 16) MLORA_HL(1, 1);
   else if (T <= 32) MLORA_HL(1, 2);
   else if (T <= 256) MLORA_HL(1, 4);
@@ -863,6 +1032,8 @@ extern "C" int mlora_latent_prefill(void* out, int out_layout, int ld_out, const
   MLORA_CHECK(pages > 0 && pages % 4 == 0 && pages / 4 <= 65535 && n_tiles > 0 && n_tiles <= 65535 && T > 0 && ld_q % 8 == 0 &&
                   (((uintptr_t)q | (uintptr_t)q_rot | (uintptr_t)scratch | (uintptr_t)tiles) & 15) == 0,
               MLORA_ERR_UNSUPPORTED, "latent_prefill: pages=%d must be a multiple of 4, operands aligned", pages);
+  MLORA_CHECK((long)H * (ceil_div(dim, 32) + ceil_div(vdim, 32)) * ceil_div(R, 32) * 1024 < (1L << 31), MLORA_ERR_UNSUPPORTED,
+              "latent_prefill: weights too large (H=%d R=%d)", H, R);
   MLORA_CHECK(scratch_elems >= mlora_latent_prefill_scratch_elems(pages, H, dim, rot, vdim), MLORA_ERR_WORKSPACE, "latent_prefill: scratch too small");
   LatentExpand e;
   e.KN = ceil_div(dim, 32); e.KR = ceil_div(rot, 32); e.VB = ceil_div(vdim, 32) * 2; e.RB = ceil_div(R, 32);
@@ -871,10 +1042,10 @@ extern "C" int mlora_latent_prefill(void* out, int out_layout, int ld_out, const
   e.v = e.k + (size_t)H * pages * e.KN * 512;
   e.r = e.v + (size_t)H * (pages / 2) * e.VB * 512;
   e.cache = (const elt*)cache; e.phys = phys; e.uk = (const elt*)uk; e.uv = (const elt*)uv;
-  e.kb_blocks = ceil_div(H * e.KN * 2, 16);
-  e.vb_blocks = ceil_div(H * e.VB, 16);
+  e.kb_blocks = ceil_div(H * e.KN * 2, 4 * LE_ROWS);
+  e.vb_blocks = ceil_div(H * e.VB, 4 * LE_ROWS);
   hipStream_t s = (hipStream_t)stream;
-  hipLaunchKernelGGL(latent_expand_kernel, dim3(e.kb_blocks + e.vb_blocks + 1, pages / 4), dim3(256), 0, s, e);
+  hipLaunchKernelGGL(latent_expand_kernel, dim3((e.kb_blocks + e.vb_blocks + 1 + 7) / 8 * 8, pages / 4), dim3(256), 0, s, e);   // whole eights: a weight row stays on one XCD
   LatentPrefill a;
   a.out = (elt*)out; a.frag_tt = out_layout == MLORA_FRAG ? mlora_frag_tiles(T) : 0; a.ld_out = ld_out;
   a.q = (const elt*)q; a.ld_q = ld_q; a.qr = (const elt*)q_rot; a.k = e.k; a.v = e.v; a.r = e.r; a.tiles = (const int4*)tiles;

@@ -155,7 +155,7 @@ __device__ __forceinline__ eltx4 moe_out(f32x4 s, const MoeLinear& a) {
 // of one expert, its waves split K, the partial tiles meet in LDS in wave order.
 constexpr int MG_WAVES = 8;
 template <int NT, int PIPE>
-__global__ __launch_bounds__(MG_WAVES* WAVE) void moe_gemv_kernel(MoeLinear a, MoePlan plan) {
+__global__ __launch_bounds__(MG_WAVES* WAVE, 2) void moe_gemv_kernel(MoeLinear a, MoePlan plan) {
   if ((int)blockIdx.y >= *plan.n_tiles) return;
   __shared__ f32x4 red[MG_WAVES][NT][WAVE];
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;

@@ -112,7 +112,7 @@ __device__ __forceinline__ float gelu_tanh(float z) {
 constexpr int TG_WAVES = 8;
 constexpr int TG_U = 4;
 template <int NT>
-__global__ __launch_bounds__(TG_WAVES* WAVE) void token_gate_kernel(elt* __restrict__ out, int frag_tt, const elt* __restrict__ x,
+__global__ __launch_bounds__(TG_WAVES* WAVE, 2) void token_gate_kernel(elt* __restrict__ out, int frag_tt, const elt* __restrict__ x,
                                                                    const elt* __restrict__ Wp, const elt* __restrict__ table, int ld_table,
                                                                    int col0, int dim, const int32_t* __restrict__ ids, int V, int T, int K, int N) {
   __shared__ f32x4 red[TG_WAVES][NT][WAVE];

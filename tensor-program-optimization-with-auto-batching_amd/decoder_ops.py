@@ -122,14 +122,17 @@ def head_linear(x, ldx, head_x, W, heads, T, K, N, out, ldy, head_y, alpha=1.0):
     return out
 
 
-def latent_prep(q, q_off, pages, qkv, off_rot, off_c, off_kr, gain, c_norm, eps, block_table, tok_seq, tok_pos, cos, sin, H, R, rot):
-    """Rotates the query parts of qkv into q [T, H, q_ld] at column q_off and stores latent and key part (c_norm given)."""
+def latent_prep(q, q_off, pages, qkv, off_rot, off_c, off_kr, gain, c_norm, eps, block_table, tok_seq, tok_pos, cos, sin, H, R, rot,
+                lift=None):
+    """Rotates the query parts of qkv into q [T, H, q_ld] at column q_off and stores latent and key part (c_norm given); lift:
+    also lifts the unrotated parts (the first columns of qkv) with these matrices, stacked [H * pad32(R), K per head]."""
     n_seq, max_blocks = block_table.shape
     T, ld = qkv.shape
     check(lib_of(qkv.dtype).mlora_latent_prep(_dev(q, qkv.dtype), q.shape[2], q_off, _dev(pages, qkv.dtype), _dev(qkv), ld, off_rot, off_c, off_kr,
                                               gain, _ptr(c_norm), eps, _dev(block_table, torch.int32), max_blocks, _dev(tok_seq, torch.int32),
                                               _dev(tok_pos, torch.int32), _dev(cos, torch.float32), _dev(sin, torch.float32), cos.shape[0], T, H, R,
-                                              rot, pages.shape[0], n_seq, _stream()), qkv.dtype)
+                                              rot, pages.shape[0], n_seq, _wptr(lift) if lift is not None else None,
+                                              lift.shape[1] if lift is not None else 0, _stream()), qkv.dtype)
 
 
 class PrefillPlan:
@@ -168,6 +171,27 @@ def latent_prefill(plan, q, q_rot, pages, uk, uv, sink, scale, R, dim, rot, vdim
                                  _dev(q_rot, q.dtype), _dev(pages, q.dtype), plan.phys.data_ptr(), plan.pages, plan.tiles.data_ptr(), plan.n_tiles,
                                  _wptr(uk), _wptr(uv), _ptr(sink), scale, T, H, R, dim, rot, vdim, pages.shape[0], scratch.data_ptr(), n, _stream()),
           q.dtype)
+    return out
+
+
+def latent_attn_splits(T, H, max_ctx, dtype) -> int:
+    """Shares of the context that attention over contexts up to max_ctx is cut into."""
+    return lib_of(dtype).mlora_latent_attn_splits(T, H, max_ctx)
+
+
+def latent_attn_out(q, pages, block_table, tok_seq, tok_pos, sink, scale, R, rot, splits, uv, vp, out):
+    """latent_attn over splits > 1 shares of the context, taken through the heads' W_uv (stacked [H * vp, pad32(R)]) into `out`
+    (activation [T, H * vp])."""
+    T, H, _ = q.shape
+    n_seq, max_blocks = block_table.shape
+    L = lib_of(q.dtype)
+    nb = L.mlora_latent_attn_workspace_bytes(T, H, R, splits)
+    ws = torch.empty(nb // 4, dtype=torch.float32, device=q.device)
+    frag = isinstance(out, FragActivation)
+    check(L.mlora_latent_attn_out(out.data.data_ptr() if frag else _dev(out, q.dtype), FRAG if frag else ROWMAJOR, H * vp, _wptr(uv), vp, _dev(q),
+                                  _dev(pages, q.dtype), _dev(block_table, torch.int32), max_blocks, _dev(tok_seq, torch.int32),
+                                  _dev(tok_pos, torch.int32), _ptr(sink), scale, T, H, R, rot, pages.shape[0], n_seq, splits, _ptr(ws), nb,
+                                  _stream()), q.dtype)
     return out
 
 

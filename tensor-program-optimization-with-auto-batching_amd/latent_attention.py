@@ -91,14 +91,22 @@ class LatentAttention:
             out = D.activation(T, self.out_cols, self.dtype, qkv.device)
         # the norm's gain on the queries is left to the scale of the scores
         scale = s.scale * self.gain
-        prep = lambda q, q_off: D.latent_prep(q, q_off, pages, qkv, self.off_rot, self.off_c, self.off_kr, self.gain, self.c_norm if store else None,
-                                              self.eps, block_table, tok_seq, tok_pos, cos, sin, H, s.kv_rank, s.rot_dim)
+        prep = lambda q, q_off, lift=None: D.latent_prep(q, q_off, pages, qkv, self.off_rot, self.off_c, self.off_kr, self.gain,
+                                                         self.c_norm if store else None, self.eps, block_table, tok_seq, tok_pos, cos, sin, H,
+                                                         s.kv_rank, s.rot_dim, lift)
         if plan is not None:
             q_rot = torch.empty((T, H, self.q_cols - self.rank_p), dtype=self.dtype, device=qkv.device)
             prep(q_rot, 0)
             return D.latent_prefill(plan, qkv, q_rot, pages, self.uk, self.uv, self.sink, scale, s.kv_rank, s.dim, s.rot_dim, s.vdim, out)
         q = torch.empty((T, H, self.q_cols), dtype=self.dtype, device=qkv.device)
-        prep(q, self.rank_p)
-        D.head_linear(qkv, self.proj_rows, self.dp, self.lift, H, T, self.dp, self.rank_p, q, H * self.q_cols, self.q_cols)
-        ctx = D.latent_attn(q, pages, block_table, tok_seq, tok_pos, self.sink, scale, s.kv_rank, s.rot_dim, max_ctx)
+        cached = (pages, block_table, tok_seq, tok_pos, self.sink, scale, s.kv_rank, s.rot_dim)
+        if self.dtype == torch.float32:
+            prep(q, self.rank_p)
+            D.head_linear(qkv, self.proj_rows, self.dp, self.lift, H, T, self.dp, self.rank_p, q, H * self.q_cols, self.q_cols)
+        else:
+            prep(q, self.rank_p, self.lift)
+        splits = D.latent_attn_splits(T, H, max_ctx, self.dtype)
+        if splits > 1:
+            return D.latent_attn_out(q, *cached, splits, self.uv, self.vp, out)
+        ctx = D.latent_attn(q, *cached, max_ctx, splits=splits)
         return D.head_linear(ctx, H * self.rank_p, self.rank_p, self.uv, H, T, self.rank_p, self.vp, out, self.out_cols, self.vp)

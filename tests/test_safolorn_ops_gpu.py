@@ -179,6 +179,12 @@ def test_latent_attention_decode(D, dt, H, rank, rot, sunk):
         torch.cuda.synchronize()
         assert err(got[..., :rank], want) < tol(dt, b16=5e-3), splits
         assert float(got[..., rank:].abs().sum()) == 0
+        if splits > 1:                                    # the same, merged on the way through W_uv
+            uv = rnd(rng, H, 64, rank, std=rank ** -0.5, dt=dt)
+            y = load_pkg("ops").FragActivation(len(ctxs), H * 64, DEV, dtype=dt)
+            D.latent_attn_out(*args, splits, D.weight(D.padded(uv, H, 64, D.pad32(rank)).reshape(H * 64, D.pad32(rank))), 64, y)
+            torch.cuda.synchronize()
+            assert err(y.unpack().view(-1, H, 64), np.einsum("thr,hvr->thv", want, f64(uv))) < 8e-3, splits
 
 
 @pytest.mark.parametrize("dt", DTYPES)
@@ -281,6 +287,14 @@ def test_latent_prep(D, dt, scaling):
     at = np.array([int(bt[s, p // 16]) for s, p in zip(seq, pos)])
     got = f64(rows)[at, pos % 16]
     assert np.abs(got[:, :rank] - cw).max() < tol(dt, b16=1e-2) * 2 and np.abs(got[:, D.pad32(rank):D.pad32(rank) + rot] - kw).max() < tol(dt, b16=1e-2) * 2
+    if dt == torch.bfloat16:                              # the same with the unrotated parts lifted beside it
+        W = rnd(rng, H, D.pad32(rank), dp, std=dp ** -0.5, dt=dt)
+        q2, p2 = torch.empty_like(q), before.clone()
+        D.latent_prep(q2, D.pad32(rank), p2, qkv, off, off + H * rot, off + H * rot + rank, 1.25, w, 1e-5, bt, torch.from_numpy(seq).to(DEV),
+                      torch.from_numpy(pos).to(DEV), cos, sin, H, rank, rot, D.weight(W.view(H * D.pad32(rank), dp)))
+        torch.cuda.synchronize()
+        assert torch.equal(p2, pages) and torch.equal(q2[..., D.pad32(rank):], q[..., D.pad32(rank):])
+        assert err(q2[..., :D.pad32(rank)], np.einsum("thk,hrk->thr", f64(qkv)[:, :off].reshape(T, H, dp), f64(W))) < 5e-3
     changed = (pages != before).permute(0, 3, 1, 2, 4).reshape(pages.shape[0], 16, -1).any(-1).sum()
     assert int(changed) == T                              # every token one slot, no other slot
 
