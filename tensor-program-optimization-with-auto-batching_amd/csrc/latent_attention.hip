@@ -334,11 +334,13 @@ struct LatentExpand {
   int kb_blocks, vb_blocks; // workgroups along x that make keys, then values; one more copies R
 };
 
-// a wave makes 16 LE_ROWS rows (of W_uk or W_uv) x 4 pages
+// A wave makes 16 LE_ROWS rows (of W_uk or W_uv) x 4 pages; the two halves of a workgroup take the same rows for neighbouring
+// pages, so that a weight fragment crosses from the second-level cache once for both.
 constexpr int LE_ROWS = 4;
-__global__ __launch_bounds__(256, 2) void latent_expand_kernel(LatentExpand a) {
+__global__ __launch_bounds__(512, 3) void latent_expand_kernel(LatentExpand a) {
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
-  const int pg0 = blockIdx.y * 4, NB = a.RB + a.KR;
+  const int pg0 = blockIdx.y * 8 + (wave >> 2) * 4, NB = a.RB + a.KR;
+  if (pg0 >= a.pages) return;                                        // no barrier below
   int page[4];
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
@@ -349,7 +351,7 @@ __global__ __launch_bounds__(256, 2) void latent_expand_kernel(LatentExpand a) {
   int bx = blockIdx.x;
   if (bx > a.kb_blocks + a.vb_blocks) return;
   if (bx == a.kb_blocks + a.vb_blocks) {
-    for (int i = threadIdx.x; i < 4 * a.KR * 64; i += 256) {
+    for (int i = threadIdx.x & 255; i < 4 * a.KR * 64; i += 256) {
       const int j = i / (a.KR * 64), o = i - j * (a.KR * 64);
       const int pj = a.phys[pg0 + j];
       st8(a.r + ((size_t)(pg0 + j) * a.KR * 64 + o) * 8,
@@ -360,7 +362,7 @@ __global__ __launch_bounds__(256, 2) void latent_expand_kernel(LatentExpand a) {
   const bool val = bx >= a.kb_blocks;                                // uniform
   if (val) bx -= a.kb_blocks;
   const int tiles = val ? a.H * a.VB : a.H * a.KN * 2;
-  const int nt0 = (bx * 4 + wave) * LE_ROWS;
+  const int nt0 = (bx * 4 + (wave & 3)) * LE_ROWS;
   if (nt0 >= tiles) return;
   const elt* wp = (val ? a.uv : a.uk) + lane * 8;
   int wo[LE_ROWS];                                                   // uniform
@@ -387,6 +389,7 @@ __global__ __launch_bounds__(256, 2) void latent_expand_kernel(LatentExpand a) {
       for (int i = 0; i < LE_ROWS; ++i) wn[i] = ld8(wp + (wo[i] + kc * 512));
 #pragma unroll
       for (int i = 0; i < 4; ++i) cn[i] = ld8(cp[i] + kc * 512);
+      __builtin_amdgcn_sched_barrier(0);                             // the requests go out ahead of the products
 #pragma unroll
       for (int i = 0; i < LE_ROWS; ++i)
 #pragma unroll
@@ -871,7 +874,7 @@ extern "C" int mlora_latent_prep(void* q, int q_ld, int q_off, void* cache, cons
     HeadLinear l;
     l.y = (elt*)q; l.ldy = (long)H * q_ld; l.hy = q_ld; l.frag_tt = 0;
     l.x = (const elt*)qkv; l.ldx = ld; l.hx = lift_k; l.W = (const elt*)lift; l.T = T; l.K = lift_k; l.N = a.RB * 32; l.alpha = 1.f;
-    const int nx = ceil_div(l.N, 64), tj = T <= 16 ? 1 : T <= 32 ? 2 : 4, ny = ceil_div(T, 16 * tj);
+    const int nx = ceil_div(l.N, 64), tj = T <= 16 ? 1 : T <= 256 ? 2 : 4, ny = ceil_div(T, 16 * tj);
     const long blocks = T + (long)nx * ny * H;
     MLORA_CHECK(blocks <= 0x7fffffffL, MLORA_ERR_UNSUPPORTED, "latent_prep: T=%d is too many tokens", T);
     hipStream_t s = (hipStream_t)stream;
@@ -990,8 +993,7 @@ extern "C" int mlora_head_linear(void* y, int y_layout, long ldy, long head_y, c
 #define MLORA_HL(NI, TJ) \
   hipLaunchKernelGGL((head_linear_kernel<NI, TJ>), dim3(ceil_div(N, 64 * NI), ceil_div(T, 16 * TJ), heads), dim3(256), 0, s, a)
   if (T <= 16) MLORA_HL(1, 1);
-  else if (T <= 32) MLORA_HL(1, 2);
-  else if (T <= 256) MLORA_HL(1, 4);
+  else if (T <= 256) MLORA_HL(1, 2);
   else MLORA_HL(4, 4);
 #undef MLORA_HL
   return mlora_launch_status("head_linear");
@@ -1045,7 +1047,7 @@ extern "C" int mlora_latent_prefill(void* out, int out_layout, int ld_out, const
   e.kb_blocks = ceil_div(H * e.KN * 2, 4 * LE_ROWS);
   e.vb_blocks = ceil_div(H * e.VB, 4 * LE_ROWS);
   hipStream_t s = (hipStream_t)stream;
-  hipLaunchKernelGGL(latent_expand_kernel, dim3((e.kb_blocks + e.vb_blocks + 1 + 7) / 8 * 8, pages / 4), dim3(256), 0, s, e);   // whole eights: a weight row stays on one XCD
+  hipLaunchKernelGGL(latent_expand_kernel, dim3((e.kb_blocks + e.vb_blocks + 1 + 7) / 8 * 8, ceil_div(pages, 8)), dim3(512), 0, s, e);   // whole eights: a weight row stays on one XCD
   LatentPrefill a;
   a.out = (elt*)out; a.frag_tt = out_layout == MLORA_FRAG ? mlora_frag_tiles(T) : 0; a.ld_out = ld_out;
   a.q = (const elt*)q; a.ld_q = ld_q; a.qr = (const elt*)q_rot; a.k = e.k; a.v = e.v; a.r = e.r; a.tiles = (const int4*)tiles;
