@@ -108,59 +108,71 @@ __device__ __forceinline__ float gelu_tanh(float z) {
 
 #ifndef MLORA_ELT_F32
 // out[t, n] = gelu(sum_k W[n, k] x[t, k]) * table[id_t, col0 + n] for n < dim, 0 for the padding rows; x and out in fragment
-// order.  A workgroup takes 16 tokens x 16 NT rows, its waves split K; a wave requests TG_U k-steps at a time.
+// order.  A workgroup takes 16 TT tokens x 16 NT rows, its waves split K; a wave requests TG_U k-steps at a time.
 constexpr int TG_WAVES = 8;
-constexpr int TG_U = 4;
-template <int NT>
+template <int NT, int TT, int TG_U>
 __global__ __launch_bounds__(TG_WAVES* WAVE, 2) void token_gate_kernel(elt* __restrict__ out, int frag_tt, const elt* __restrict__ x,
-                                                                   const elt* __restrict__ Wp, const elt* __restrict__ table, int ld_table,
-                                                                   int col0, int dim, const int32_t* __restrict__ ids, int V, int T, int K, int N) {
+                                                                      const elt* __restrict__ Wp, const elt* __restrict__ table, int ld_table,
+                                                                      int col0, int dim, const int32_t* __restrict__ ids, int V, int T, int K, int N) {
   __shared__ f32x4 red[TG_WAVES][NT][WAVE];
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
   const int KB = K / 32, tiles = N / 16;
-  const int nt0 = blockIdx.x * NT, t0 = blockIdx.y * 16;
-  const elt* xp = x + (size_t)blockIdx.y * 512 + lane * 8;
+  const int nt0 = blockIdx.x * NT, tt0 = blockIdx.y * TT;
+  const elt* xp[TT];
+#pragma unroll
+  for (int j = 0; j < TT; ++j) xp[j] = x + (size_t)(tt0 + j < frag_tt ? tt0 + j : frag_tt - 1) * 512 + lane * 8;
   const elt* wp[NT];
 #pragma unroll
   for (int i = 0; i < NT; ++i) wp[i] = Wp + (size_t)(nt0 + i < tiles ? nt0 + i : tiles - 1) * KB * 512 + lane * 8;
-  f32x4 acc[NT];
+  f32x4 acc[NT][TT];
 #pragma unroll
-  for (int i = 0; i < NT; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int i = 0; i < NT; ++i)
+#pragma unroll
+    for (int j = 0; j < TT; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
   for (int ks0 = wave; ks0 < KB; ks0 += TG_WAVES * TG_U) {
-    eltx8 a[TG_U][NT], b[TG_U];
+    eltx8 a[TG_U][NT], b[TG_U][TT];
 #pragma unroll
     for (int u = 0; u < TG_U; ++u) {
       const bool in = ks0 + u * TG_WAVES < KB;                       // uniform; past K: a valid address, zeroed
       const int ks = in ? ks0 + u * TG_WAVES : ks0;
 #pragma unroll
       for (int i = 0; i < NT; ++i) a[u][i] = ld8(wp[i] + (size_t)ks * 512);
-      b[u] = ld8(xp + (size_t)ks * frag_tt * 512);
-      if (!in) b[u] = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
+#pragma unroll
+      for (int j = 0; j < TT; ++j) {
+        b[u][j] = ld8(xp[j] + (size_t)ks * frag_tt * 512);
+        if (!in) b[u][j] = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
+      }
     }
 #pragma unroll
     for (int u = 0; u < TG_U; ++u)
 #pragma unroll
-      for (int i = 0; i < NT; ++i) acc[i] = mfma_16x16x32(a[u][i], b[u], acc[i]);
+      for (int i = 0; i < NT; ++i)
+#pragma unroll
+        for (int j = 0; j < TT; ++j) acc[i][j] = mfma_16x16x32(a[u][i], b[u][j], acc[i][j]);
   }
 #pragma unroll
-  for (int i = 0; i < NT; ++i) red[wave][i][lane] = acc[i];
-  __syncthreads();
-  for (int e = threadIdx.x; e < NT * WAVE; e += TG_WAVES * WAVE) {
-    const int i = e >> 6, sl = e & 63;
-    const int tt = t0 + (sl & 15), n = (nt0 + i) * 16 + (sl >> 4) * 4;
-    if (tt >= T || n >= N) continue;
-    f32x4 s = red[0][i][sl];
+  for (int j = 0; j < TT; ++j) {
+    if (j > 0) __syncthreads();
 #pragma unroll
-    for (int w = 1; w < TG_WAVES; ++w) s += red[w][i][sl];
-    const int id = ids[tt];
-    const bool ok = id >= 0 && id < V;
-    eltx4 o;
+    for (int i = 0; i < NT; ++i) red[wave][i][lane] = acc[i][j];
+    __syncthreads();
+    for (int e = threadIdx.x; e < NT * WAVE; e += TG_WAVES * WAVE) {
+      const int i = e >> 6, sl = e & 63;
+      const int t = (tt0 + j) * 16 + (sl & 15), n = (nt0 + i) * 16 + (sl >> 4) * 4;
+      if (t >= T || n >= N) continue;
+      f32x4 s = red[0][i][sl];
 #pragma unroll
-    for (int q = 0; q < 4; ++q) {
-      const float ev = ok && n + q < dim ? (float)table[(size_t)id * ld_table + col0 + n + q] : 0.f;
-      o[q] = (elt)(gelu_tanh(s[q]) * ev);
+      for (int w = 1; w < TG_WAVES; ++w) s += red[w][i][sl];
+      const int id = ids[t];
+      const bool ok = id >= 0 && id < V;
+      eltx4 o;
+#pragma unroll
+      for (int q = 0; q < 4; ++q) {
+        const float ev = ok && n + q < dim ? (float)table[(size_t)id * ld_table + col0 + n + q] : 0.f;
+        o[q] = (elt)(gelu_tanh(s[q]) * ev);
+      }
+      *reinterpret_cast<eltx4*>(out + frag_offset(t, n, frag_tt)) = o;
     }
-    *reinterpret_cast<eltx4*>(out + frag_offset(tt, n, frag_tt)) = o;
   }
 }
 #endif
@@ -207,12 +219,13 @@ extern "C" int mlora_token_gate(void* out_frag, const void* xf, const void* Wp, 
               MLORA_ERR_UNSUPPORTED, "token_gate: need K %% 32 == 0, N %% 32 == 0, dim <= N (T=%d K=%d N=%d dim=%d)", T, K, N, dim);
   if (T == 0) return MLORA_OK;
   hipStream_t s = (hipStream_t)stream;
-#define MLORA_TG(NT)                                                                                                                   \
-  hipLaunchKernelGGL(token_gate_kernel<NT>, dim3(ceil_div(N, 16 * NT), ceil_div(T, 16)), dim3(TG_WAVES * WAVE), 0, s, (elt*)out_frag,  \
-                     mlora_frag_tiles(T), (const elt*)xf, (const elt*)Wp, (const elt*)table, ld_table, col0, dim, ids, V, T, K, N)
-  if (T <= 256) MLORA_TG(1);
-  else if (N <= 32) MLORA_TG(2);
-  else MLORA_TG(4);
+#define MLORA_TG(NT, TT, U)                                                                                                        \
+  hipLaunchKernelGGL((token_gate_kernel<NT, TT, U>), dim3(ceil_div(N, 16 * NT), ceil_div(T, 16 * TT)), dim3(TG_WAVES * WAVE), 0, s, \
+                     (elt*)out_frag, mlora_frag_tiles(T), (const elt*)xf, (const elt*)Wp, (const elt*)table, ld_table, col0, dim, ids, V, T, K, N)
+  if (T <= 256) MLORA_TG(1, 1, 4);
+  else if (N <= 32) MLORA_TG(2, 1, 4);
+  else if ((long)ceil_div(N, 64) * ceil_div(T, 64) >= 256) MLORA_TG(4, 4, 2);      // a workgroup per compute unit with four token tiles
+  else MLORA_TG(4, 1, 4);
 #undef MLORA_TG
   return mlora_launch_status("token_gate");
 }

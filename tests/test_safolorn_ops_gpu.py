@@ -60,7 +60,7 @@ def test_stream_norm(D, ops, dt, T, H, Hp):
 
 
 @pytest.mark.parametrize("dt", DTYPES)
-@pytest.mark.parametrize("T,width,dim", [(1, 40, 5), (33, 104, 20), (300, 96, 40), (16, 200, 70)])
+@pytest.mark.parametrize("T,width,dim", [(1, 40, 5), (33, 104, 20), (300, 96, 20), (300, 96, 40), (4100, 72, 250), (16, 200, 70)])
 def test_token_gate(D, ops, dt, T, width, dim):
     rng = np.random.default_rng(T)
     Hp, N, V = D.pad32(width), D.pad32(dim), 50
