@@ -14,7 +14,7 @@ LIB_PATHS = {"float16": LIB_PATH, "bfloat16": os.path.join(_HERE, "libmlora_bf16
 
 F16, F32 = 0, 1          # F16: the library's own 16-bit element type (in the fp32 library: fp32)
 GLU_SILU, GLU_CLIPPED = 0, 1
-ACT_NONE, ACT_RELU2 = 0, 1
+ACT_NONE, ACT_RELU2, ACT_GLU = 0, 1, 2
 MOE_UP, MOE_DOWN = 0, 1
 ROWMAJOR, FRAG = 0, 1
 STORE, ACCUMULATE = 0, 1
@@ -117,9 +117,30 @@ class DecodePlan(C.Structure):
 
 SIGNATURES["mlora_decode_step"] = (_i, [C.POINTER(DecodePlan), _p])
 
+
+class TanhNorm(C.Structure):
+    _fields_ = [("w", _p), ("b", _p), ("alpha", _f)]
+
+
+class StreamStep(C.Structure):
+    _fields_ = [("x_out", _p), ("x", _p), ("y", _p), ("part", _p), ("rows", _p), ("out_frag", _p), ("out_row", _p), ("mu", _p), ("shift", _p),
+                ("tok_seq", _p), ("tok_pos", _p), ("tok_last", _p), ("post", TanhNorm), ("pre", TanhNorm), ("mix_stride", _l),
+                ("n_part", _i), ("top", _i), ("T", _i), ("Hp", _i), ("ld_row", _i), ("n_seq", _i), ("mult", _f), ("row_weight", _f)]
+
+
 # mirrors include/mlora_decoder.h (the bfloat16 and fp32 libraries)
 DECODER_SIGNATURES = {
     "mlora_stream_norm": (_i, [_p, _p, _p, _p, _i, _p, _p, _f, _f, _i, _i, _i, _i, _p]),
+    "mlora_stream_step": (_i, [C.POINTER(StreamStep), _p]),
+    "mlora_embed_scaled": (_i, [_p, _p, _p, _i, _p, _p, _f, _i, _i, _i, _p]),
+    "mlora_linear_ksplit_store": (_i, [_p, _p, _i, _p, _p, _i, _i, _i, _p]),
+    "mlora_time_mix": (_i, [_p, _i, _i, _p, _p, _p, _p, _i, _p, _i, _i, _p, _i, _p, _p, _p, _f, _p, _i, _p, _i, _p, _p, _i, _i, _i, _p]),
+    "mlora_tied_prep": (_i, [_p, _p, _p, _p, _i, _p, _p, _f, _f, _f, _p, _i, _p, _p, _i, _i, _i, _i, _i, _i, _p]),
+    "mlora_tied_attn_splits": (_i, [_i, _i, _i, _i]),
+    "mlora_tied_attn": (_i, [_p, _i, _p, _p, _p, _p, _i, _p, _p, _p, _f, _i, _i, _i, _i, _i, _i, _i, _p, _z, _p]),
+    "mlora_tied_prefill_served": (_i, [_i]),
+    "mlora_tied_prefill_scratch_elems": (_z, [_i, _i, _i]),
+    "mlora_tied_prefill": (_i, [_p, _i, _i, _p, _p, _p, _p, _i, _p, _i, _p, _f, _i, _i, _i, _i, _i, _p, _z, _p]),
     "mlora_token_gate": (_i, [_p, _p, _p, _p, _i, _i, _i, _p, _i, _i, _i, _i, _p]),
     "mlora_token_gate_mul": (_i, [_p, _p, _p, _i, _i, _i, _p, _i, _i, _i, _p]),
     "mlora_latent_prep": (_i, [_p, _i, _i, _p, _p, _i, _i, _i, _i, _f, _p, _f, _p, _i, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _p, _i, _p]),
@@ -137,13 +158,15 @@ DECODER_SIGNATURES = {
     "mlora_moe_max_tiles": (_i, [_i, _i, _i]),
     "mlora_moe_max_places": (_i, [_i, _i, _i]),
     "mlora_moe_plan": (_i, [_p, _p, _p, _p, _i, _i, _i, _p]),
+    "mlora_moe_table_plan": (_i, [_p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _p]),
     "mlora_moe_linear": (_i, [_p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _p, _z, _p]),
     "mlora_moe_combine": (_i, [_p, _p, _i, _p, _p, _i, _i, _i, _p, _p]),
 }
 
 # ... and those that the fp32 library does not have
 MATRIX_CORE_ONLY = ("mlora_token_gate", "mlora_latent_attn_out", "mlora_latent_prefill", "mlora_latent_prefill_tile_tokens", "mlora_latent_prefill_served",
-                    "mlora_latent_prefill_scratch_elems")
+                    "mlora_latent_prefill_scratch_elems", "mlora_tied_prefill", "mlora_tied_prefill_served", "mlora_tied_prefill_scratch_elems",
+                    "mlora_linear_ksplit_store")
 
 _libs = {}
 

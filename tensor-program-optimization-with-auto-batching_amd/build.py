@@ -16,7 +16,7 @@ from concurrent.futures import ThreadPoolExecutor
 HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 SOURCES = ["api.hip", "gather_mm.hip", "gather_mm_batch.hip", "gemv.hip", "gemm.hip", "rowops.hip", "attention.hip", "decode_step.hip"]
-DECODER_SOURCES = ["stream_ops.hip", "latent_attention.hip", "moe.hip"]
+DECODER_SOURCES = ["stream_ops.hip", "latent_attention.hip", "time_mix.hip", "moe.hip"]
 LIBS = {   # element type -> (library, sources, suffix of the objects, extra flags)
     "float16": (os.path.join(HERE, "libmlora_hip.so"), SOURCES, "", []),
     "bfloat16": (os.path.join(HERE, "libmlora_bf16.so"), ["api.hip", "gemv.hip", "gemm.hip", "rowops.hip", *DECODER_SOURCES], "_bf16",

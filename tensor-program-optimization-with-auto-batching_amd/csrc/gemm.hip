@@ -301,6 +301,7 @@ struct PPGroup {
   size_t w_elems;
   float alpha;
 };
+// With OUT_SILU the group's up stage ends in a gated product: an expert's weights are its gate rows, then its up rows.
 
 __device__ __forceinline__ unsigned long long uniform64(unsigned long long v) {
   const unsigned lo = __builtin_amdgcn_readfirstlane((unsigned)v), hi = __builtin_amdgcn_readfirstlane((unsigned)(v >> 32));
@@ -599,7 +600,7 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_pp_kernel(void* __rest
 #pragma unroll
       for (int j = 0; j < WTF; ++j) {
         const int t = t0 + (wt * WTF + j) * 16 + r16;
-        if ((t >> 4) >= x_tt) continue;                  // the token tile does not exist
+        if ((t >> 4) >= x_tt || (GROUPED && t >= tend)) continue;   // the token tile does not exist (the place is another expert's)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
           const int c = n0 + (wn * 4 + i) * 16 + g * 4;
@@ -1142,6 +1143,7 @@ extern "C" int mlora_linear_frag_lora(void* y, int y_dtype, int mode, const void
   else e = launch_gemm_pp<OUT_F16>(y, (const elt*)xf, 0, tt, (const elt*)Wp, T, K, N, s, lo);
   return e ? e : mlora_launch_status("linear_frag_lora");
 }
+#endif
 
 extern "C" int mlora_linear_frag_silu(void* act, const void* xf, const void* Wp, int T, int K, int I, const mlora_fused_lora* projs,
                                       int n_proj, const int32_t* blk_adapter, int r, void* stream) {
@@ -1172,7 +1174,6 @@ extern "C" int mlora_linear_frag_silu(void* act, const void* xf, const void* Wp,
   const int e = launch_gemm_pp<OUT_SILU>(act, (const elt*)xf, 0, mlora_frag_tiles(T), (const elt*)Wp, T, K, 2 * I, (hipStream_t)stream, lo);
   return e ? e : mlora_launch_status("linear_frag_silu");
 }
-#endif
 
 #ifdef MLORA_ELT_BF16
 // One expert linear over a plan of 256-place tiles: xf places in fragment order (x_tt tiles of 16), y as PPGroup says.
@@ -1183,7 +1184,7 @@ static int launch_gemm_grouped(void* y, const elt* xf, int x_tt, const elt* Wp, 
       hipFuncSetAttribute((const void*)gemm_pp_kernel<OUT, false, true>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
   if (configured != hipSuccess)
     return mlora_set_error(MLORA_ERR_LAUNCH, "moe_linear: cannot reserve %zu bytes of LDS: %s", lds, hipGetErrorString(configured));
-  const int gx = ceil_div(N, PP_F * 16);
+  const int gx = OUT == OUT_SILU ? ceil_div(N / 2, PP_F * 8) : ceil_div(N, PP_F * 16);
   int n_cu = gemm_n_cu();
   if (n_cu <= 0) n_cu = 256;
   const long nb = (long)gx * max_tiles;
@@ -1192,17 +1193,36 @@ static int launch_gemm_grouped(void* y, const elt* xf, int x_tt, const elt* Wp, 
   return MLORA_OK;
 }
 
-int mlora_gemm_grouped(void* y, const void* xf, int x_tt, const void* Wp, const MoePlan& plan, int max_tiles, int K, int N, int relu2, float alpha,
+int mlora_gemm_grouped(void* y, const void* xf, int x_tt, const void* Wp, const MoePlan& plan, int max_tiles, int K, int N, int act, float alpha,
                        void* stream) {
   MLORA_CHECK(K % 64 == 0 && N % 32 == 0 && x_tt > 0 && max_tiles > 0, MLORA_ERR_UNSUPPORTED, "moe_linear: K=%d N=%d", K, N);   // the caller's checks say more
   PPGroup gr;
   gr.plan = plan;
-  gr.w_elems = (size_t)N * K;
+  gr.w_elems = (size_t)N * K * (act == MLORA_ACT_GLU ? 2 : 1);
   gr.alpha = alpha;
   hipStream_t s = (hipStream_t)stream;
-  const int e = relu2 ? launch_gemm_grouped<OUT_RELU2>(y, (const elt*)xf, x_tt, (const elt*)Wp, K, N, max_tiles, gr, s)
-                      : launch_gemm_grouped<OUT_F16>(y, (const elt*)xf, x_tt, (const elt*)Wp, K, N, max_tiles, gr, s);
+  const int e = act == MLORA_ACT_GLU ? launch_gemm_grouped<OUT_SILU>(y, (const elt*)xf, x_tt, (const elt*)Wp, K, 2 * N, max_tiles, gr, s)
+                : act == MLORA_ACT_RELU2 ? launch_gemm_grouped<OUT_RELU2>(y, (const elt*)xf, x_tt, (const elt*)Wp, K, N, max_tiles, gr, s)
+                                         : launch_gemm_grouped<OUT_F16>(y, (const elt*)xf, x_tt, (const elt*)Wp, K, N, max_tiles, gr, s);
   return e ? e : mlora_launch_status("moe_linear");
+}
+#endif
+
+#ifdef MLORA_ELT_BF16
+int mlora_gemv_ksplit_store(float* y, float* part, int ks, const void* xf, const void* Wp, int T, int K, int N, void* stream);
+
+// y [T, N] fp32 = xf . Wp^T over ks K slices (mlora_gemv_ksplit): slice 0 into y, slices 1.. into part[ks - 1][T][N]
+extern "C" int mlora_linear_ksplit_store(float* y, float* part, int ks, const void* xf, const void* Wp, int T, int K, int N, void* stream) {
+  if (int e = mlora_check_linear("linear_ksplit_store", y, MLORA_F32, MLORA_STORE, xf, K, Wp, T, K, N)) return e;
+  MLORA_CHECK(ks >= 1 && ks <= 4 && (ks == 1 || part) && (K / 32) / ks >= 1 && ((uintptr_t)xf & 15) == 0, MLORA_ERR_INVALID,
+              "linear_ksplit_store: ks=%d outside 1..4, too many slices for K=%d, or no partials buffer", ks, K);
+  if (T == 0) return MLORA_OK;
+  if (T <= 64) return mlora_gemv_ksplit_store(y, part, ks, xf, Wp, T, K, N, stream);
+  if (ks == 1) return mlora_linear_frag(y, MLORA_F32, MLORA_STORE, xf, Wp, T, K, N, stream);
+  MidShape m = gemm_mid_shape(T, K, N, ks);
+  m.ksplit = ks;                               // the caller's partial buffers were sized for ks slices
+  const int e = launch_gemm_mid<OUT_F32>(y, part, N, m, (const elt*)xf, mlora_frag_tiles(T), (const elt*)Wp, T, K, N, (hipStream_t)stream);
+  return e ? e : mlora_launch_status("linear_ksplit_store");
 }
 #endif
 

@@ -721,6 +721,12 @@ extern "C" int mlora_gemv_frag_acc_ksplit(float* y, float* y2, float* part, int 
                                           ks, part);
 }
 
+// the storing form (mlora_linear_ksplit_store), T <= 64
+int mlora_gemv_ksplit_store(float* y, float* part, int ks, const void* xf, const void* Wp, int T, int K, int N, void* stream) {
+  MLORA_CHECK(ks == 1 || (K / KSTEP) / ks >= 8, MLORA_ERR_INVALID, "linear_ksplit_store: too many slices for K=%d", K);
+  return gemv_dispatch<true, true, false>(y, MLORA_F32, MLORA_STORE, xf, K, Wp, T, K, N, stream, LoraShrinkBatch(), N, nullptr, ks, part);
+}
+
 #ifndef MLORA_ELT_BF16      // the adapter kernels are fp16
 // Riders per token of the delta-carrying launch below (0: the shape is not served): a rider thread keeps at most
 // RIDE_BQ 16-byte chunks of B, the launch must be K-split (it is the split form of the kernel that carries riders),

@@ -9,6 +9,11 @@
 // latent takes the first RB = ceil(kv_rank / 32) blocks, the rotated part the following ones, padding is zero.
 // There is no second copy for the values: the matrix cores transpose a page's fragments by a product with the identity.
 // Query rows: [T, H, NB * 32] in the same order.
+//
+// Tied attention (TIED): the heads of a group share a key/value head whose values are its keys before their norm.  A page
+// holds the values v of each of the G key/value heads, [n_pages, G, RB, 4, 16, 8], and one number per token and head,
+// 1 / rms(v) [n_pages, G, 16] fp32, so that a key is (1 / rms) v w and is never stored: the norm's weight w goes to the queries,
+// the number to the scores.  A distance bias slope_h (i - j) is taken off the scores.
 #include <type_traits>
 
 #include "common.h"
@@ -100,7 +105,15 @@ struct LatentAttn {
   const float* sink;        // [H]
   float scale;
   int T, H, RB, NB, splits, n_inner, chunks;
+  const float* key_scale;   // tied: [n_pages, G, 16]
+  const float* slopes;      // tied: [H]
+  int G, gs, gt;            // tied: key/value heads, heads per group, 16-head tiles per group
+  int frag_tt;              // `out` in fragment order (tied) if > 0
 };
+
+__device__ __forceinline__ size_t latent_out_offset(const LatentAttn& a, int t, int h, int d) {
+  return a.frag_tt ? frag_offset(t, h * a.RB * 32 + d, a.frag_tt) : ((size_t)t * a.H + h) * (a.RB * 32) + d;
+}
 
 // the context a token sees: every position up to its own
 __device__ __forceinline__ int latent_ctx(const LatentAttn& a, int t, int& seq) {
@@ -118,10 +131,10 @@ __device__ __forceinline__ int latent_ctx(const LatentAttn& a, int t, int& seq) 
 //   page^T               two products with halves of the identity per 32 dims: exact
 //   O^T += page^T . P^T  P as hi + lo halves in the two halves of the k-slots, the page's values repeated in both
 // The waves' states (m, l, O) meet in LDS, 64 dims at a time.
-template <int NRB, int NW>
+template <int NRB, int NW, bool TIED = false>
 __global__ __launch_bounds__(NW * WAVE, 2) void latent_attn_kernel(LatentAttn a) {
   extern __shared__ __align__(16) char smem_raw[];
-  const int RBp = a.chunks * NRB, KR = a.NB - a.RB, KRp = KR > 2 ? KR : 2;   // blocks in LDS: the latent's, the rotated part's
+  const int RBp = a.chunks * NRB, KR = TIED ? 0 : a.NB - a.RB, KRp = TIED ? 0 : KR > 2 ? KR : 2;   // blocks in LDS: the latent's, the rotated part's
   elt* qs = reinterpret_cast<elt*>(smem_raw);                        // [RBp + KRp][64][8] query fragments, zero where there is no block
   float* sacc = reinterpret_cast<float*>(qs + (RBp + KRp) * 512);    // [NW][16][68]
   __shared__ float sm[NW][16], sl[NW][16];
@@ -133,6 +146,9 @@ __global__ __launch_bounds__(NW * WAVE, 2) void latent_attn_kernel(LatentAttn a)
   if (outer >= a.T * a.splits) return;                               // uniform
   const int t = outer / a.splits, split = outer - t * a.splits;
   const int hg = inner / a.chunks, b0 = (inner - hg * a.chunks) * NRB;
+  // the heads of the tile's columns: h0 .. h0 + hn - 1
+  const int kvh = TIED ? hg / a.gt : 0, hw = TIED ? (hg - kvh * a.gt) * 16 : hg * 16;
+  const int h0 = TIED ? kvh * a.gs + hw : hw, hn = (TIED ? a.gs : a.H) - hw;
   int seq;
   const int ctx = latent_ctx(a, t, seq);
   const int npages = (ctx + PAGE - 1) / PAGE;
@@ -142,10 +158,10 @@ __global__ __launch_bounds__(NW * WAVE, 2) void latent_attn_kernel(LatentAttn a)
   const int qd = a.NB * 32;
 
   for (int i = threadIdx.x; i < (RBp + KRp) * 64; i += NW * WAVE) {
-    const int slot = i >> 6, l = i & 63, h = hg * 16 + (l & 15);
+    const int slot = i >> 6, l = i & 63, h = h0 + (l & 15);
     const int kb = slot < RBp ? slot : slot - RBp + a.RB;
     eltx8 v = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
-    if (h < a.H && (slot < RBp ? kb < a.RB : kb < a.NB)) v = ld8(a.q + ((size_t)t * a.H + h) * qd + kb * 32 + (l >> 4) * 8);
+    if ((l & 15) < hn && (slot < RBp ? kb < a.RB : kb < a.NB)) v = ld8(a.q + ((size_t)t * a.H + h) * qd + kb * 32 + (l >> 4) * 8);
     st8(qs + i * 8, v);
   }
   // the identity's columns 0..15 and 16..31 as the B operand: lane (column col, k-group g) holds k = 8 g .. 8 g + 7
@@ -166,8 +182,15 @@ __global__ __launch_bounds__(NW * WAVE, 2) void latent_attn_kernel(LatentAttn a)
   auto page_of = [&](int pg, bool& ok) {
     const int page = bt[pg];
     ok = page >= 0 && page < a.n_pages;
-    return a.cache + (size_t)(ok ? page : 0) * a.NB * 512 + lane * 8;
+    return a.cache + ((size_t)(ok ? page : 0) * (TIED ? a.G : 1) + kvh) * a.NB * 512 + lane * 8;
   };
+  // tied: the scale of this lane's four keys of a page, and its head's slope
+  auto scale_of = [&](int pg) {
+    const int page = bt[pg];
+    return *reinterpret_cast<const f32x4*>(a.key_scale + ((size_t)(page >= 0 && page < a.n_pages ? page : 0) * a.G + kvh) * PAGE + 4 * g);
+  };
+  f32x4 ksc = f32x4{0.f, 0.f, 0.f, 0.f};
+  const float slope = TIED ? a.slopes[h0 + (col < hn ? col : 0)] : 0.f;
   eltx8 kf[NRB], rf[2];
   bool ok = false, ok_next = false;
   const elt* kp = a.cache;
@@ -175,17 +198,26 @@ __global__ __launch_bounds__(NW * WAVE, 2) void latent_attn_kernel(LatentAttn a)
     kp = page_of(p0 + wave, ok);
 #pragma unroll
     for (int b = 0; b < NRB; ++b) kf[b] = ld8(kp + (b0 + b < a.RB ? b0 + b : a.RB - 1) * 512);
+    if constexpr (TIED) {
+      ksc = scale_of(p0 + wave);
+    } else {
 #pragma unroll
-    for (int r = 0; r < 2; ++r) rf[r] = ld8(kp + (r < KR ? a.RB + r : a.RB) * 512);
+      for (int r = 0; r < 2; ++r) rf[r] = ld8(kp + (r < KR ? a.RB + r : a.RB) * 512);
+    }
   }
   for (int pg = p0 + wave; pg < p1; pg += NW) {
     // the next page's fragments are requested one by one as this page's are done with
     const elt* kn = page_of(pg + NW < p1 ? pg + NW : pg, ok_next);
     // two chains of products: st[r] = S[token 4 g + r][head col].  A block that does not exist meets zero queries.
-    f32x4 st = mfma_16x16x32(rf[0], ld8(qs + (RBp * 64 + lane) * 8), f32x4{0.f, 0.f, 0.f, 0.f});
-    f32x4 st1 = mfma_16x16x32(rf[1], ld8(qs + ((RBp + 1) * 64 + lane) * 8), f32x4{0.f, 0.f, 0.f, 0.f});
-    rf[0] = ld8(kn + a.RB * 512);
-    rf[1] = ld8(kn + (KR > 1 ? a.RB + 1 : a.RB) * 512);
+    f32x4 st = f32x4{0.f, 0.f, 0.f, 0.f}, st1 = st, ksn = st;
+    if constexpr (TIED) {
+      ksn = scale_of(pg + NW < p1 ? pg + NW : pg);
+    } else {
+      st = mfma_16x16x32(rf[0], ld8(qs + (RBp * 64 + lane) * 8), f32x4{0.f, 0.f, 0.f, 0.f});
+      st1 = mfma_16x16x32(rf[1], ld8(qs + ((RBp + 1) * 64 + lane) * 8), f32x4{0.f, 0.f, 0.f, 0.f});
+      rf[0] = ld8(kn + a.RB * 512);
+      rf[1] = ld8(kn + (KR > 1 ? a.RB + 1 : a.RB) * 512);
+    }
 #pragma unroll
     for (int b = 0; b < NRB; b += 2) {
       st = mfma_16x16x32(kf[b], ld8(qs + ((b0 + b) * 64 + lane) * 8), st);
@@ -200,7 +232,9 @@ __global__ __launch_bounds__(NW * WAVE, 2) void latent_attn_kernel(LatentAttn a)
     float pm = -INFINITY;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      st[r] = !ok || pg * PAGE + 4 * g + r >= ctx ? -INFINITY : st[r] * a.scale;
+      const int j = pg * PAGE + 4 * g + r;
+      const float sc = TIED ? fmaf(-slope, (float)(ctx - 1 - j), st[r] * a.scale * ksc[r]) : st[r] * a.scale;
+      st[r] = !ok || j >= ctx ? -INFINITY : sc;
       pm = fmaxf(pm, st[r]);
     }
     pm = fmaxf(pm, __shfl_xor(pm, 16, WAVE));
@@ -236,6 +270,7 @@ __global__ __launch_bounds__(NW * WAVE, 2) void latent_attn_kernel(LatentAttn a)
     }
     kp = kn;
     ok = ok_next;
+    ksc = ksn;
   }
   l += __shfl_xor(l, 16, WAVE);
   l += __shfl_xor(l, 32, WAVE);
@@ -246,8 +281,8 @@ __global__ __launch_bounds__(NW * WAVE, 2) void latent_attn_kernel(LatentAttn a)
   __syncthreads();
   // per head, once: what every wave's sums are multiplied with, and (M, L)
   if (threadIdx.x < 16) {
-    const int hc = threadIdx.x, h = hg * 16 + hc;
-    const float sk = a.splits == 1 && a.sink && h < a.H ? a.sink[h] : -INFINITY;
+    const int hc = threadIdx.x, h = h0 + hc;
+    const float sk = !TIED && a.splits == 1 && a.sink && hc < hn ? a.sink[h] : -INFINITY;
     float M = sk, L = 0.f;
 #pragma unroll
     for (int w = 0; w < NW; ++w) M = fmaxf(M, sm[w][hc]);
@@ -261,7 +296,7 @@ __global__ __launch_bounds__(NW * WAVE, 2) void latent_attn_kernel(LatentAttn a)
     const float inv = a.splits > 1 ? 1.f : L > 0.f ? 1.f / L : 0.f;
 #pragma unroll
     for (int w = 0; w < NW; ++w) sm[w][hc] = f[w] * inv;
-    if (a.splits > 1 && h < a.H && b0 == 0) {
+    if (a.splits > 1 && hc < hn && b0 == 0) {
       const size_t r = ((size_t)split * a.T + t) * a.H + h;
       a.part_ml[2 * r] = M;
       a.part_ml[2 * r + 1] = L;
@@ -276,13 +311,14 @@ __global__ __launch_bounds__(NW * WAVE, 2) void latent_attn_kernel(LatentAttn a)
         if (2 * c + u < 2 * NRB) *reinterpret_cast<f32x4*>(sacc + (wave * 16 + col) * 68 + u * 16 + 4 * g) = O[(2 * c + u) % (2 * NRB)];
       __syncthreads();
       for (int e = threadIdx.x; e < 16 * 16; e += NW * WAVE) {
-        const int hc = e >> 4, dd = (e & 15) * 4, h = hg * 16 + hc, d = (b0 + c) * 32 + dd;
-        if (h >= a.H || d >= a.RB * 32 || d >= (b0 + NRB) * 32) continue;
+        const int hc = e >> 4, dd = (e & 15) * 4, h = h0 + hc, d = (b0 + c) * 32 + dd;
+        if (hc >= hn || d >= a.RB * 32 || d >= (b0 + NRB) * 32) continue;
         f32x4 o = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int w = 0; w < NW; ++w) o += *reinterpret_cast<const f32x4*>(sacc + (w * 16 + hc) * 68 + dd) * sm[w][hc];
         if (a.splits == 1)
-          *reinterpret_cast<eltx4*>(a.out + ((size_t)t * a.H + h) * (a.RB * 32) + d) = eltx4{(elt)o[0], (elt)o[1], (elt)o[2], (elt)o[3]};
+          *reinterpret_cast<eltx4*>(a.out + (TIED ? latent_out_offset(a, t, h, d) : ((size_t)t * a.H + h) * (a.RB * 32) + d)) =
+              eltx4{(elt)o[0], (elt)o[1], (elt)o[2], (elt)o[3]};
         else
           *reinterpret_cast<f32x4*>(a.part_o + (((size_t)split * a.T + t) * a.H + h) * (a.RB * 32) + d) = o;
       }
@@ -309,7 +345,7 @@ __global__ __launch_bounds__(128) void latent_merge_kernel(LatentAttn a) {
       const float m = a.part_ml[2 * (s * n + th)];
       if (m != -INFINITY) o += *reinterpret_cast<const f32x4*>(a.part_o + (s * n + th) * rd + d) * __expf(m - M);
     }
-    *reinterpret_cast<eltx4*>(a.out + (size_t)th * rd + d) = eltx4{(elt)(o[0] * inv), (elt)(o[1] * inv), (elt)(o[2] * inv), (elt)(o[3] * inv)};
+    *reinterpret_cast<eltx4*>(a.out + latent_out_offset(a, th / a.H, h, d)) = eltx4{(elt)(o[0] * inv), (elt)(o[1] * inv), (elt)(o[2] * inv), (elt)(o[3] * inv)};
   }
 }
 
@@ -435,6 +471,8 @@ struct LatentPrefill {
   const float* sink;
   float scale;
   int H, pages, KN, KR, VB;
+  const float* slopes;      // tied: [H]
+  int gs;                   // tied: heads per key/value head
 };
 
 // Four waves own up to 128 consecutive queries of one head of one sequence, a wave 32 of them as two 16-query tiles.  Keys are
@@ -444,12 +482,13 @@ struct LatentPrefill {
 constexpr int LP_WAVES = 4;
 constexpr int LP_QT = 2;
 constexpr int LP_TOK = LP_WAVES * LP_QT * 16;
-template <int KB_, int VB_, bool EXACT>
+// TIED: the heads of a group read one K and V (no rotated part), and a distance bias is taken off the scores.
+template <int KB_, int VB_, bool EXACT, bool TIED = false>
 __global__ __launch_bounds__(LP_WAVES* WAVE, 2) void latent_prefill_kernel(LatentPrefill a) {
   extern __shared__ __align__(16) elt lsm[];                         // [2][4 KB + 2 VB][512]
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
   const int qi = lane & 15, g = lane >> 4;
-  const int KN = a.KN, KR = a.KR, KB = EXACT ? KB_ : KN + KR, VB = EXACT ? VB_ : a.VB;
+  const int KN = TIED && EXACT ? KB_ : a.KN, KR = TIED ? 0 : a.KR, KB = EXACT ? KB_ : KN + KR, VB = EXACT ? VB_ : a.VB;
   const int PIECES = 4 * KB + 2 * VB;                                // 1 KiB pieces of a key block
   const int h = blockIdx.x;
   const int4 tile = a.tiles[blockIdx.y];
@@ -477,8 +516,10 @@ __global__ __launch_bounds__(LP_WAVES* WAVE, 2) void latent_prefill_kernel(Laten
   }
   const int last = tile.w + tile.y - 1;                              // position of the tile's last query
   const int nblk = last / 64 + 1;
-  const elt* kh = a.k + ((size_t)h * a.pages + tile.z) * KN * 512 + lane * 8;
-  const elt* vh = a.v + ((size_t)h * (a.pages / 2) + tile.z / 2) * VB * 512 + lane * 8;
+  const int kvh = TIED ? h / a.gs : h;
+  const float slope = TIED ? a.slopes[h] * 1.44269504088896340736f : 0.f;
+  const elt* kh = a.k + ((size_t)kvh * a.pages + tile.z) * KN * 512 + lane * 8;
+  const elt* vh = a.v + ((size_t)kvh * (a.pages / 2) + tile.z / 2) * VB * 512 + lane * 8;
   const elt* rh = a.r + (size_t)tile.z * KR * 512 + lane * 8;
   // piece i of a block: page p = i / KB, fragment i % KB of it for i < 4 KB; then the pairs' V pieces
   auto issue = [&](int b) {
@@ -529,7 +570,13 @@ __global__ __launch_bounds__(LP_WAVES* WAVE, 2) void latent_prefill_kernel(Laten
       const int lim = tile.w + wq + u * 16 + qi - b * 64 - 4 * g;    // key (p, r) of this lane is visible while 16 p + r <= lim
       float pm = -INFINITY;
 #pragma unroll
-      for (int p = 0; p < 4; ++p) st[u][p] *= c2;
+      for (int p = 0; p < 4; ++p) {
+        st[u][p] *= c2;
+        if constexpr (TIED) {
+#pragma unroll
+          for (int r = 0; r < 4; ++r) st[u][p][r] = fmaf(-slope, (float)(lim - p * 16 - r), st[u][p][r]);
+        }
+      }
       if (tile.w + wq + u * 16 < b * 64 + 63) {                      // uniform: the block crosses the tile's diagonal
 #pragma unroll
         for (int p = 0; p < 4; ++p)
@@ -780,13 +827,15 @@ __global__ __launch_bounds__(256) void latent_attn_f32_kernel(LatentAttn a) {
   const int ctx = latent_ctx(a, t, seq), qd = a.NB * 32, rd = a.RB * 32;
   const int32_t* bt = a.block_table + (size_t)seq * a.max_blocks;
   for (int d = threadIdx.x; d < qd; d += 256) fsm[d] = a.q[((size_t)t * a.H + h) * qd + d];
+  const int kvh = h / a.gs;                       // one key/value head unless tied
+  const float slope = a.slopes ? a.slopes[h] : 0.f;
   float m = a.sink ? a.sink[h] : -INFINITY, l = a.sink ? 1.f : 0.f, o[LA_DPT] = {};
   for (int j0 = 0; j0 < ctx; j0 += LA_KEYS) {
     __syncthreads();
     if (threadIdx.x < LA_KEYS / PAGE) {
       const int pg = j0 / PAGE + threadIdx.x;
       const int page = pg * PAGE < ctx ? bt[pg] : -1;
-      pgs[threadIdx.x] = page < a.n_pages ? page : -1;
+      pgs[threadIdx.x] = page >= 0 && page < a.n_pages ? page * a.G + kvh : -1;
     }
     __syncthreads();
     const int j = j0 + threadIdx.x, page = pgs[threadIdx.x / PAGE];
@@ -798,6 +847,8 @@ __global__ __launch_bounds__(256) void latent_attn_f32_kernel(LatentAttn a) {
 #pragma unroll
         for (int e = 0; e < 8; ++e) acc = fmaf(kp[(size_t)b * 128 + e], fsm[b * 8 + e], acc);
       s = acc * a.scale;
+      if (a.key_scale) s *= a.key_scale[(size_t)page * PAGE + j % PAGE];
+      if (a.slopes) s = fmaf(-slope, (float)(ctx - 1 - j), s);
     }
     float mx = wave_max(s);
     if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = mx;
@@ -832,18 +883,114 @@ __global__ __launch_bounds__(256) void latent_attn_f32_kernel(LatentAttn a) {
 #endif
 
 #ifndef MLORA_ELT_F32
-template <int NRB, int NW>
+template <int NRB, int NW, bool TIED = false>
 int launch_latent_attn(const LatentAttn& a, hipStream_t s) {
   const int kr = a.NB - a.RB;
-  const size_t lds = (size_t)(a.chunks * NRB + (kr > 2 ? kr : 2)) * 1024 + (size_t)NW * 16 * 68 * sizeof(float);
+  const size_t lds = (size_t)(a.chunks * NRB + (TIED ? 0 : kr > 2 ? kr : 2)) * 1024 + (size_t)NW * 16 * 68 * sizeof(float);
   static const hipError_t configured =               // the attribute is per kernel, set once per process, by one thread
-      hipFuncSetAttribute((const void*)latent_attn_kernel<NRB, NW>, hipFuncAttributeMaxDynamicSharedMemorySize, 96 * 1024);
+      hipFuncSetAttribute((const void*)latent_attn_kernel<NRB, NW, TIED>, hipFuncAttributeMaxDynamicSharedMemorySize, 96 * 1024);
   if (configured != hipSuccess || lds > 96 * 1024)
     return mlora_set_error(MLORA_ERR_UNSUPPORTED, "latent_attn: cannot reserve %zu bytes of LDS", lds);
   const long outer = ((long)a.T * a.splits + 7) / 8 * 8;
   if (outer * a.n_inner > 0x7fffffffL) return mlora_set_error(MLORA_ERR_UNSUPPORTED, "latent_attn: T=%d is too many tokens", a.T);
-  hipLaunchKernelGGL((latent_attn_kernel<NRB, NW>), dim3((unsigned)(outer * a.n_inner)), dim3(NW * WAVE), lds, s, a);
+  hipLaunchKernelGGL((latent_attn_kernel<NRB, NW, TIED>), dim3((unsigned)(outer * a.n_inner)), dim3(NW * WAVE), lds, s, a);
   return MLORA_OK;
+}
+#endif
+
+// ---------------------------------------------------------------------------------------------
+// Tied attention
+// ---------------------------------------------------------------------------------------------
+struct TiedPrep {
+  const float* y;           // [T, ld]: projections without their biases, the H query heads' and then the G key/value heads' D columns each
+  int ld;
+  const float* bias;        // [(H + G) D]
+  const float* q_norm;      // [D]: the queries' norm weight (times that of the keys, where the keys go without)
+  float eps, temp_coef, temp_every;
+  elt* q;                   // [T, H, RB * 32]
+  elt* cache;
+  float* key_scale;
+  const int32_t* block_table;
+  int max_blocks, n_pages, n_seq;
+  const int32_t* tok_seq;
+  const int32_t* tok_pos;
+  int T, H, G, D, RB;
+};
+
+constexpr int TP_VPT = 8;      // columns per lane: heads of up to 512
+// One wave per (token, head): adds the bias; a query is normed and takes its temperature, a value goes to the token's page slot
+// with the reciprocal of its root mean square.
+__global__ __launch_bounds__(256) void tied_prep_kernel(TiedPrep a) {
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int hh = blockIdx.y * 4 + wave, t = blockIdx.x;
+  if (hh >= a.H + a.G) return;                                       // no barrier below
+  const int seq = a.tok_seq[t], pos = a.tok_pos[t], Dp = a.RB * 32;
+  float v[TP_VPT], ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < TP_VPT; ++i) {
+    const int d = lane + i * WAVE;
+    v[i] = d < a.D ? a.y[(size_t)t * a.ld + hh * a.D + d] + a.bias[hh * a.D + d] : 0.f;
+    ss = fmaf(v[i], v[i], ss);
+  }
+  const float inv = 1.f / sqrtf(wave_sum(ss) / (float)a.D + a.eps);
+  if (hh < a.H) {
+    float f = inv;
+    if (a.temp_every > 0.f) f *= fmaf(a.temp_coef, logf(floorf((float)(pos + 1) / a.temp_every) + 1.f), 1.f);
+    elt* q = a.q + ((size_t)t * a.H + hh) * Dp;
+#pragma unroll
+    for (int i = 0; i < TP_VPT; ++i) {
+      const int d = lane + i * WAVE;
+      if (d < Dp) q[d] = (elt)(d < a.D ? v[i] * f * a.q_norm[d] : 0.f);
+    }
+    return;
+  }
+  if (seq < 0 || seq >= a.n_seq || pos < 0 || pos / PAGE >= a.max_blocks) return;
+  const int page = a.block_table[(size_t)seq * a.max_blocks + pos / PAGE];
+  if (page < 0 || page >= a.n_pages) return;
+  const int pg = page * a.G + hh - a.H;
+#pragma unroll
+  for (int i = 0; i < TP_VPT; ++i) {
+    const int d = lane + i * WAVE;
+    if (d < Dp) a.cache[latent_offset(pg, a.RB, pos % PAGE, d)] = (elt)v[i];
+  }
+  if (lane == 0) a.key_scale[(size_t)pg * PAGE + pos % PAGE] = inv;
+}
+
+#ifndef MLORA_ELT_F32
+// The keys (normed, without the weight, which the queries carry) and the transposed values of whole contexts in the scratch
+// layouts of the prompt form, K [G, pages, RB, 512] and V [G, pages / 2, 2 RB, 512]: one workgroup per (pair of pages, key/value head).
+__global__ __launch_bounds__(256) void tied_expand_kernel(elt* __restrict__ k, elt* __restrict__ v, const elt* __restrict__ cache,
+                                                          const float* __restrict__ key_scale, const int32_t* __restrict__ phys, int pages,
+                                                          int n_pages, int G, int RB) {
+  const int pp = blockIdx.x, kvh = blockIdx.y;
+  int pg[2];
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    pg[j] = phys[2 * pp + j];
+    pg[j] = pg[j] >= 0 && pg[j] < n_pages ? pg[j] * G + kvh : -1;
+  }
+  for (int i = threadIdx.x; i < 2 * RB * 64; i += 256) {             // keys: a page's fragments, each token's row scaled
+    const int j = i / (RB * 64), o = i - j * (RB * 64);
+    eltx8 x = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
+    if (pg[j] >= 0) {
+      const float s = key_scale[(size_t)pg[j] * PAGE + (o & 15)];
+      x = ld8(cache + (size_t)pg[j] * RB * 512 + o * 8);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[e] = (elt)((float)x[e] * s);
+    }
+    st8(k + (((size_t)kvh * pages + 2 * pp + j) * RB * 64 + o) * 8, x);
+  }
+  for (int i = threadIdx.x; i < 2 * RB * 64; i += 256) {             // values: 16 dims x 32 tokens per fragment
+    const int db = i >> 6, l = i & 63, d = db * 16 + (l & 15), g = l >> 4;
+    eltx8 x = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
+#pragma unroll
+    for (int j = 0; j < 2; ++j)
+      if (pg[j] >= 0) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) x[j * 4 + r] = cache[latent_offset(pg[j], RB, 4 * g + r, d)];
+      }
+    st8(v + (((size_t)kvh * (pages / 2) + pp) * 2 * RB * 64 + i) * 8, x);
+  }
 }
 #endif
 
@@ -918,7 +1065,8 @@ static int latent_attn_impl(void* out, const void* q, const void* cache, const i
   MLORA_CHECK(T >= 0 && H > 0 && H <= 65535 && R > 0 && rot > 0 && max_blocks > 0 && n_pages > 0 && n_seq > 0 && splits >= 1, MLORA_ERR_INVALID,
               "latent_attn: bad shape T=%d H=%d R=%d rot=%d", T, H, R, rot);
   if (T == 0) return MLORA_OK;
-  LatentAttn a;
+  LatentAttn a = {};
+  a.G = 1; a.gs = H;
   a.out = (elt*)out; a.q = (const elt*)q; a.cache = (const elt*)cache; a.block_table = block_table; a.max_blocks = max_blocks;
   a.n_pages = n_pages; a.n_seq = n_seq; a.tok_seq = tok_seq; a.tok_pos = tok_pos; a.sink = sink; a.scale = scale;
   a.T = T; a.H = H; a.RB = ceil_div(R, 32); a.NB = a.RB + ceil_div(rot, 32); a.splits = splits;
@@ -1001,14 +1149,14 @@ extern "C" int mlora_head_linear(void* y, int y_layout, long ldy, long head_y, c
 #endif
 
 #ifndef MLORA_ELT_F32
-template <int KB, int VB, bool EXACT>
+template <int KB, int VB, bool EXACT, bool TIED = false>
 static int launch_latent_prefill(const LatentPrefill& a, int n_tiles, hipStream_t s) {
   constexpr size_t cap = (size_t)2 * (4 * KB + 2 * VB) * 512 * sizeof(elt);
   static const hipError_t configured =               // the attribute is per kernel, set once per process, by one thread
-      hipFuncSetAttribute((const void*)latent_prefill_kernel<KB, VB, EXACT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)cap);
+      hipFuncSetAttribute((const void*)latent_prefill_kernel<KB, VB, EXACT, TIED>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)cap);
   if (configured != hipSuccess) return mlora_set_error(MLORA_ERR_LAUNCH, "latent_prefill: cannot reserve %zu bytes of LDS", cap);
   const size_t lds = (size_t)2 * (4 * (a.KN + a.KR) + 2 * a.VB) * 512 * sizeof(elt);
-  hipLaunchKernelGGL((latent_prefill_kernel<KB, VB, EXACT>), dim3(a.H, n_tiles), dim3(LP_WAVES * WAVE), lds, s, a);
+  hipLaunchKernelGGL((latent_prefill_kernel<KB, VB, EXACT, TIED>), dim3(a.H, n_tiles), dim3(LP_WAVES * WAVE), lds, s, a);
   return MLORA_OK;
 }
 
@@ -1048,7 +1196,7 @@ extern "C" int mlora_latent_prefill(void* out, int out_layout, int ld_out, const
   e.vb_blocks = ceil_div(H * e.VB, 4 * LE_ROWS);
   hipStream_t s = (hipStream_t)stream;
   hipLaunchKernelGGL(latent_expand_kernel, dim3((e.kb_blocks + e.vb_blocks + 1 + 7) / 8 * 8, ceil_div(pages, 8)), dim3(512), 0, s, e);   // whole eights: a weight row stays on one XCD
-  LatentPrefill a;
+  LatentPrefill a = {};
   a.out = (elt*)out; a.frag_tt = out_layout == MLORA_FRAG ? mlora_frag_tiles(T) : 0; a.ld_out = ld_out;
   a.q = (const elt*)q; a.ld_q = ld_q; a.qr = (const elt*)q_rot; a.k = e.k; a.v = e.v; a.r = e.r; a.tiles = (const int4*)tiles;
   a.sink = sink; a.scale = scale; a.H = H; a.pages = pages; a.KN = e.KN; a.KR = e.KR; a.VB = e.VB;
@@ -1058,5 +1206,109 @@ extern "C" int mlora_latent_prefill(void* out, int out_layout, int ld_out, const
   else if (KB <= 3 && e.VB <= 4) rc = launch_latent_prefill<3, 4, false>(a, n_tiles, s);
   else rc = launch_latent_prefill<6, 8, false>(a, n_tiles, s);
   return rc ? rc : mlora_launch_status("latent_prefill");
+}
+#endif
+
+// ---------------------------------------------------------------------------------------------
+// Tied attention
+// ---------------------------------------------------------------------------------------------
+extern "C" int mlora_tied_prep(void* q, void* cache, float* key_scale, const float* y, int ld, const float* bias, const float* q_norm, float eps,
+                               float temp_coef, float temp_every, const int32_t* block_table, int max_blocks, const int32_t* tok_seq,
+                               const int32_t* tok_pos, int T, int H, int G, int D, int n_pages, int n_seq, void* stream) {
+  MLORA_CHECK(q && cache && key_scale && y && bias && q_norm && block_table && tok_seq && tok_pos, MLORA_ERR_INVALID, "tied_prep: null pointer");
+  MLORA_CHECK(T >= 0 && H > 0 && G > 0 && H % G == 0 && D > 0 && D <= WAVE * TP_VPT && ld >= (H + G) * D && max_blocks > 0 && n_pages > 0 && n_seq > 0 &&
+                  (long)n_pages * G <= 0x7fffffffL && ceil_div(H + G, 4) <= 65535,
+              MLORA_ERR_UNSUPPORTED, "tied_prep: need whole groups of heads of at most %d columns (T=%d H=%d G=%d D=%d)", WAVE * TP_VPT, T, H, G, D);
+  if (T == 0) return MLORA_OK;
+  TiedPrep a;
+  a.y = y; a.ld = ld; a.bias = bias; a.q_norm = q_norm; a.eps = eps; a.temp_coef = temp_coef; a.temp_every = temp_every; a.q = (elt*)q;
+  a.cache = (elt*)cache; a.key_scale = key_scale; a.block_table = block_table; a.max_blocks = max_blocks; a.n_pages = n_pages; a.n_seq = n_seq;
+  a.tok_seq = tok_seq; a.tok_pos = tok_pos; a.T = T; a.H = H; a.G = G; a.D = D; a.RB = ceil_div(D, 32);
+  hipLaunchKernelGGL(tied_prep_kernel, dim3(T, ceil_div(H + G, 4)), dim3(256), 0, (hipStream_t)stream, a);
+  return mlora_launch_status("tied_prep");
+}
+
+extern "C" int mlora_tied_attn_splits(int T, int H, int G, int max_ctx) {
+#ifdef MLORA_ELT_F32
+  return 1;
+#else
+  if (T <= 0 || G <= 0 || H < G || max_ctx <= 0) return 1;
+  const long wgs = (long)T * G * ceil_div(H / G, 16);
+  int s = (int)(512 / wgs);                                       // two workgroups per compute unit ...
+  const int by_ctx = max_ctx / (8 * PAGE);                        // ... of at least one page per wave
+  if (s > by_ctx) s = by_ctx;
+  if (s > 32) s = 32;
+  return s < 1 ? 1 : s;
+#endif
+}
+
+extern "C" int mlora_tied_attn(void* out, int out_layout, const void* q, const void* cache, const float* key_scale, const int32_t* block_table,
+                               int max_blocks, const int32_t* tok_seq, const int32_t* tok_pos, const float* slopes, float scale, int T, int H, int G,
+                               int D, int n_pages, int n_seq, int splits, void* workspace, size_t workspace_bytes, void* stream) {
+  MLORA_CHECK(out && q && cache && key_scale && slopes && block_table && tok_seq && tok_pos, MLORA_ERR_INVALID, "tied_attn: null pointer");
+  MLORA_CHECK(T >= 0 && H > 0 && H <= 65535 && G > 0 && H % G == 0 && D > 0 && D <= 512 && max_blocks > 0 && n_pages > 0 && n_seq > 0 && splits >= 1 &&
+                  (long)n_pages * G <= 0x7fffffffL && (out_layout == MLORA_ROWMAJOR || sizeof(elt) == 2),
+              MLORA_ERR_UNSUPPORTED, "tied_attn: bad shape T=%d H=%d G=%d D=%d", T, H, G, D);
+  if (T == 0) return MLORA_OK;
+  LatentAttn a = {};
+  a.out = (elt*)out; a.q = (const elt*)q; a.cache = (const elt*)cache; a.block_table = block_table; a.max_blocks = max_blocks;
+  a.n_pages = n_pages; a.n_seq = n_seq; a.tok_seq = tok_seq; a.tok_pos = tok_pos; a.scale = scale; a.T = T; a.H = H;
+  a.RB = a.NB = ceil_div(D, 32); a.splits = splits; a.key_scale = key_scale; a.slopes = slopes; a.G = G; a.gs = H / G; a.gt = ceil_div(H / G, 16);
+  a.frag_tt = out_layout == MLORA_FRAG ? mlora_frag_tiles(T) : 0; a.chunks = 1;
+  hipStream_t s = (hipStream_t)stream;
+#ifdef MLORA_ELT_F32
+  (void)workspace; (void)workspace_bytes;
+  MLORA_CHECK(splits == 1, MLORA_ERR_UNSUPPORTED, "tied_attn: splits=%d not served in fp32", splits);
+  hipLaunchKernelGGL(latent_attn_f32_kernel, dim3(T, H, ceil_div(a.RB * 32, 256 * LA_DPT)), dim3(256), a.NB * 128, s, a);
+#else
+  if (splits > 1) {
+    MLORA_CHECK(workspace && workspace_bytes >= mlora_latent_attn_workspace_bytes(T, H, D, splits), MLORA_ERR_WORKSPACE,
+                "tied_attn: workspace of %zu bytes needed", mlora_latent_attn_workspace_bytes(T, H, D, splits));
+    MLORA_CHECK((long)T * H <= 0x7fffffffL, MLORA_ERR_UNSUPPORTED, "tied_attn: T=%d is too many tokens", T);
+    a.part_o = (float*)workspace;
+    a.part_ml = a.part_o + (size_t)splits * T * H * a.RB * 32;
+  }
+  a.n_inner = G * a.gt;
+  int e;
+  if (a.RB <= 2) e = launch_latent_attn<2, 8, true>(a, s);
+  else if (a.RB <= 4) e = launch_latent_attn<4, 8, true>(a, s);
+  else if (a.RB <= 8) e = launch_latent_attn<8, 8, true>(a, s);
+  else e = launch_latent_attn<16, 8, true>(a, s);
+  if (e) return e;
+  if (splits > 1) hipLaunchKernelGGL(latent_merge_kernel, dim3(T * H), dim3(128), 0, s, a);
+#endif
+  return mlora_launch_status("tied_attn");
+}
+
+#ifndef MLORA_ELT_F32
+extern "C" int mlora_tied_prefill_served(int D) { return D > 0 && D <= 128; }
+
+extern "C" size_t mlora_tied_prefill_scratch_elems(int pages, int G, int D) {
+  if (pages <= 0 || G <= 0 || D <= 0) return 0;
+  return (size_t)pages * G * ceil_div(D, 32) * 1024;
+}
+
+extern "C" int mlora_tied_prefill(void* out, int out_layout, int ld_out, const void* q, const void* cache, const float* key_scale, const int32_t* phys,
+                                  int pages, const int32_t* tiles, int n_tiles, const float* slopes, float scale, int T, int H, int G, int D,
+                                  int n_pages, void* scratch, size_t scratch_elems, void* stream) {
+  MLORA_CHECK(out && q && cache && key_scale && phys && tiles && slopes && scratch, MLORA_ERR_INVALID, "tied_prefill: null pointer");
+  MLORA_CHECK(mlora_tied_prefill_served(D) && H > 0 && H <= 65535 && G > 0 && H % G == 0 && n_pages > 0 && (long)n_pages * G <= 0x7fffffffL,
+              MLORA_ERR_UNSUPPORTED, "tied_prefill: H=%d G=%d D=%d not served", H, G, D);
+  MLORA_CHECK(pages > 0 && pages % 4 == 0 && n_tiles > 0 && n_tiles <= 65535 && T > 0 && (((uintptr_t)q | (uintptr_t)scratch | (uintptr_t)tiles) & 15) == 0,
+              MLORA_ERR_UNSUPPORTED, "tied_prefill: pages=%d must be a multiple of 4, operands aligned", pages);
+  MLORA_CHECK(scratch_elems >= mlora_tied_prefill_scratch_elems(pages, G, D), MLORA_ERR_WORKSPACE, "tied_prefill: scratch too small");
+  hipStream_t s = (hipStream_t)stream;
+  LatentPrefill a = {};
+  a.KN = ceil_div(D, 32); a.KR = 0; a.VB = 2 * a.KN; a.H = H; a.pages = pages; a.gs = H / G;
+  elt* k = (elt*)scratch;
+  elt* v = k + (size_t)G * pages * a.KN * 512;
+  hipLaunchKernelGGL(tied_expand_kernel, dim3(pages / 2, G), dim3(256), 0, s, k, v, (const elt*)cache, key_scale, phys, pages, n_pages, G, a.KN);
+  a.out = (elt*)out; a.frag_tt = out_layout == MLORA_FRAG ? mlora_frag_tiles(T) : 0; a.ld_out = ld_out;
+  a.q = (const elt*)q; a.ld_q = H * a.KN * 32; a.k = k; a.v = v; a.r = k; a.tiles = (const int4*)tiles; a.scale = scale; a.slopes = slopes;
+  int rc;
+  if (a.KN == 4) rc = launch_latent_prefill<4, 8, true, true>(a, n_tiles, s);
+  else if (a.KN == 2) rc = launch_latent_prefill<2, 4, true, true>(a, n_tiles, s);
+  else rc = launch_latent_prefill<4, 8, false, true>(a, n_tiles, s);
+  return rc ? rc : mlora_launch_status("tied_prefill");
 }
 #endif

@@ -9,5 +9,5 @@ struct MoePlan {
   const int32_t* n_tiles;   // device: tiles in use, then places in use (a multiple of 16)
 };
 
-int mlora_gemm_grouped(void* y, const void* xf, int x_tt, const void* Wp, const MoePlan& plan, int max_tiles, int K, int N, int relu2, float alpha,
+int mlora_gemm_grouped(void* y, const void* xf, int x_tt, const void* Wp, const MoePlan& plan, int max_tiles, int K, int N, int act, float alpha,
                        void* stream);

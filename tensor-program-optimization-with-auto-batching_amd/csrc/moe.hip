@@ -55,14 +55,31 @@ __global__ __launch_bounds__(RT_WAVES* WAVE) void moe_route_kernel(int32_t* __re
 constexpr int PL_THREADS = 1024;
 constexpr int PL_MAX_E = RT_MAX_E;
 
-// Counting sort of the entries by expert, one workgroup.  The order of an expert's entries among themselves may differ
-// from run to run; nothing depends on it (every row of a tile is computed by itself).
+// The experts of a pass's entries: chosen by a router, or looked up by token id.
+struct PlanSource {
+  const int32_t* pick;      // [n] ...
+  const int32_t* table;     // ... or, if given, [layers, V, top]
+  const int32_t* ids;       // [n / top]
+  int V, top, E;
+  __device__ __forceinline__ int operator()(int i) const {
+    if (!table) return pick[i];
+    const int t = i / top, id = ids[t];
+    const int e = table[((size_t)blockIdx.x * V + (id >= 0 && id < V ? id : 0)) * top + i - t * top];
+    return e >= 0 && e < E ? e : 0;
+  }
+};
+
+// Counting sort of the entries by expert, one workgroup (per layer, with tables).  The order of an expert's entries among
+// themselves may differ from run to run; nothing depends on it (every row of a tile is computed by itself).
 __global__ __launch_bounds__(PL_THREADS) void moe_plan_kernel(int32_t* __restrict__ perm, int4* __restrict__ tiles, int32_t* __restrict__ n_tiles,
-                                                              const int32_t* __restrict__ pick, int n, int E, int tile_rows) {
+                                                              PlanSource pick, int n, int E, int tile_rows, int perm_stride, int tiles_stride) {
   __shared__ int count[PL_MAX_E], first[PL_MAX_E], tile0[PL_MAX_E];
+  perm += (size_t)blockIdx.x * perm_stride;
+  tiles += (size_t)blockIdx.x * tiles_stride;
+  n_tiles += 2 * blockIdx.x;
   for (int e = threadIdx.x; e < E; e += PL_THREADS) count[e] = 0;
   __syncthreads();
-  for (int i = threadIdx.x; i < n; i += PL_THREADS) atomicAdd(&count[pick[i]], 1);
+  for (int i = threadIdx.x; i < n; i += PL_THREADS) atomicAdd(&count[pick(i)], 1);
   __syncthreads();
   if (threadIdx.x < WAVE) {                 // one wave scans, 64 experts at a time
     const int lane = threadIdx.x;
@@ -100,7 +117,7 @@ __global__ __launch_bounds__(PL_THREADS) void moe_plan_kernel(int32_t* __restric
   }
   __syncthreads();
   for (int i = threadIdx.x; i < n; i += PL_THREADS) {
-    const int e = pick[i];
+    const int e = pick(i);
     perm[first[e] + atomicAdd(&count[e], 1)] = i;
   }
 }
@@ -154,13 +171,15 @@ __device__ __forceinline__ eltx4 moe_out(f32x4 s, const MoeLinear& a) {
 // Tiles of 16 entries (a decode step: a few tokens per expert): the weights are what is read.  A workgroup takes 16 NT rows
 // of one expert, its waves split K, the partial tiles meet in LDS in wave order.
 constexpr int MG_WAVES = 8;
-template <int NT, int PIPE>
+// GLU: the weights are gate rows, then up rows (a.N of each); a workgroup takes NT / 2 tiles of both and stores their product.
+template <int NT, int PIPE, bool GLU = false>
 __global__ __launch_bounds__(MG_WAVES* WAVE, 2) void moe_gemv_kernel(MoeLinear a, MoePlan plan) {
   if ((int)blockIdx.y >= *plan.n_tiles) return;
   __shared__ f32x4 red[MG_WAVES][NT][WAVE];
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
   const int4 tile = plan.tiles[blockIdx.y];
-  const int KB = a.K / 32, ntiles = a.N / 16, nt0 = blockIdx.x * NT;
+  constexpr int NO = GLU ? NT / 2 : NT;       // row tiles of the output
+  const int KB = a.K / 32, ntiles = a.N / 16, nt0 = blockIdx.x * NO;
   const int i16 = lane & 15;
   const int place = tile.y + (i16 < tile.z ? i16 : tile.z - 1);
   const int entry = plan.perm[place];
@@ -168,7 +187,10 @@ __global__ __launch_bounds__(MG_WAVES* WAVE, 2) void moe_gemv_kernel(MoeLinear a
   const elt* wp = a.W + tile.x * a.w_elems + lane * 8;
   int woff[NT];
 #pragma unroll
-  for (int i = 0; i < NT; ++i) woff[i] = (nt0 + i < ntiles ? nt0 + i : ntiles - 1) * KB * 512;
+  for (int i = 0; i < NT; ++i) {
+    const int nt = nt0 + (GLU ? i >> 1 : i);
+    woff[i] = ((nt < ntiles ? nt : ntiles - 1) + (GLU && (i & 1) ? ntiles : 0)) * KB * 512;
+  }
   f32x4 acc[NT];
 #pragma unroll
   for (int i = 0; i < NT; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -193,14 +215,27 @@ __global__ __launch_bounds__(MG_WAVES* WAVE, 2) void moe_gemv_kernel(MoeLinear a
 #pragma unroll
   for (int i = 0; i < NT; ++i) red[wave][i][lane] = acc[i];
   __syncthreads();
-  for (int e = threadIdx.x; e < NT * WAVE; e += MG_WAVES * WAVE) {
+  for (int e = threadIdx.x; e < NO * WAVE; e += MG_WAVES * WAVE) {
     const int i = e >> 6, sl = e & 63, row = sl & 15;
     const int n = (nt0 + i) * 16 + (sl >> 4) * 4;
     if (row >= tile.z || n >= a.N) continue;
+    const int p = tile.y + row;
+    if constexpr (GLU) {
+      f32x4 sg = red[0][2 * i][sl], su = red[0][2 * i + 1][sl];
+#pragma unroll
+      for (int q = 1; q < MG_WAVES; ++q) {
+        sg += red[q][2 * i][sl];
+        su += red[q][2 * i + 1][sl];
+      }
+      eltx4 o;
+#pragma unroll
+      for (int q = 0; q < 4; ++q) o[q] = (elt)glu<MLORA_GLU_SILU>(sg[q], su[q], GluArgs());
+      *reinterpret_cast<eltx4*>(a.y + (size_t)p * a.N + n) = o;
+      continue;
+    }
     f32x4 s = red[0][i][sl];
 #pragma unroll
     for (int q = 1; q < MG_WAVES; ++q) s += red[q][i][sl];
-    const int p = tile.y + row;
     *reinterpret_cast<eltx4*>(a.y + (size_t)(a.up ? p : plan.perm[p]) * a.N + n) = moe_out(s, a);
   }
 }
@@ -257,9 +292,21 @@ extern "C" int mlora_moe_plan(int32_t* perm, int32_t* tiles, int32_t* n_tiles, c
   MLORA_CHECK(perm && tiles && n_tiles && pick && ((uintptr_t)tiles & 15) == 0, MLORA_ERR_INVALID, "moe_plan: null or unaligned pointer");
   MLORA_CHECK(T > 0 && E > 0 && E <= PL_MAX_E && top > 0 && (long)T * top < 0x7fffffffL, MLORA_ERR_UNSUPPORTED,
               "moe_plan: need experts <= %d (T=%d E=%d top=%d)", PL_MAX_E, T, E, top);
-  hipLaunchKernelGGL(moe_plan_kernel, dim3(1), dim3(PL_THREADS), 0, (hipStream_t)stream, perm, (int4*)tiles, n_tiles, pick, T * top, E,
-                     mlora_moe_tile_rows(T, E, top));
+  const PlanSource src = {pick, nullptr, nullptr, 0, top, E};
+  hipLaunchKernelGGL(moe_plan_kernel, dim3(1), dim3(PL_THREADS), 0, (hipStream_t)stream, perm, (int4*)tiles, n_tiles, src, T * top, E,
+                     mlora_moe_tile_rows(T, E, top), 0, 0);
   return mlora_launch_status("moe_plan");
+}
+
+extern "C" int mlora_moe_table_plan(int32_t* perm, int32_t* tiles, int32_t* n_tiles, const int32_t* table, const int32_t* ids, int layers, int V, int T,
+                                    int E, int top, void* stream) {
+  MLORA_CHECK(perm && tiles && n_tiles && table && ids && ((uintptr_t)tiles & 15) == 0, MLORA_ERR_INVALID, "moe_table_plan: null or unaligned pointer");
+  MLORA_CHECK(layers > 0 && V > 0 && T > 0 && E > 0 && E <= PL_MAX_E && top > 0 && (long)T * top < 0x7fffffffL, MLORA_ERR_UNSUPPORTED,
+              "moe_table_plan: need experts <= %d (layers=%d V=%d T=%d E=%d top=%d)", PL_MAX_E, layers, V, T, E, top);
+  const PlanSource src = {nullptr, table, ids, V, top, E};
+  hipLaunchKernelGGL(moe_plan_kernel, dim3(layers), dim3(PL_THREADS), 0, (hipStream_t)stream, perm, (int4*)tiles, n_tiles, src, T * top, E,
+                     mlora_moe_tile_rows(T, E, top), mlora_moe_max_places(T, E, top), mlora_moe_max_tiles(T, E, top));
+  return mlora_launch_status("moe_table_plan");
 }
 
 extern "C" int mlora_moe_combine(float* x, const float* part, int n_part, const void* y, const float* weight, int T, int top, int N,
@@ -279,8 +326,9 @@ extern "C" int mlora_moe_linear(void* y, const void* x, const void* W, const int
                                 void* workspace, size_t workspace_elems, void* stream) {
   MLORA_CHECK(y && x && W && perm && tiles && n_tiles, MLORA_ERR_INVALID, "moe_linear: null pointer");
   MLORA_CHECK(T >= 0 && K > 0 && K % 32 == 0 && N > 0 && N % 16 == 0 && top > 0 && max_tiles >= 0 && max_tiles <= 65535 &&
-                  (long)N * K < (1L << 31) && (tile_rows == 16 || tile_rows == MM_ROWS) && places % 16 == 0 && places / 16 <= 65535,
+                  (long)N * K < (1L << (act == MLORA_ACT_GLU ? 30 : 31)) && (tile_rows == 16 || tile_rows == MM_ROWS) && places % 16 == 0 && places / 16 <= 65535,
               MLORA_ERR_UNSUPPORTED, "moe_linear: need K %% 32 == 0, N %% 16 == 0 (T=%d K=%d N=%d tiles=%d)", T, K, N, max_tiles);
+  MLORA_CHECK(act != MLORA_ACT_GLU || (stage == MLORA_MOE_UP && alpha == 1.f), MLORA_ERR_UNSUPPORTED, "moe_linear: a gated product is the up stage's, unscaled");
   if (T == 0 || max_tiles == 0) return MLORA_OK;
   MoePlan p;
   p.perm = perm; p.tiles = (const int4*)tiles; p.n_tiles = n_tiles;
@@ -288,8 +336,8 @@ extern "C" int mlora_moe_linear(void* y, const void* x, const void* W, const int
   if (tile_rows == MM_ROWS) {
     MLORA_CHECK(K % 64 == 0 && N % 32 == 0 && (((uintptr_t)x | (uintptr_t)y | (uintptr_t)workspace) & 15) == 0, MLORA_ERR_UNSUPPORTED,
                 "moe_linear: 256-place tiles need K %% 64 == 0, N %% 32 == 0, aligned operands (K=%d N=%d)", K, N);
-    MLORA_CHECK(act == (stage == MLORA_MOE_UP ? MLORA_ACT_RELU2 : MLORA_ACT_NONE), MLORA_ERR_UNSUPPORTED,
-                "moe_linear: over 256-place tiles the up stage squares its positive part, the down stage does not");
+    MLORA_CHECK(stage == MLORA_MOE_UP ? act != MLORA_ACT_NONE : act == MLORA_ACT_NONE, MLORA_ERR_UNSUPPORTED,
+                "moe_linear: over 256-place tiles the up stage ends with its activation, the down stage has none");
     const void* xf = x;
     if (stage == MLORA_MOE_UP) {
       MLORA_CHECK(workspace && workspace_elems >= (size_t)places * K, MLORA_ERR_WORKSPACE, "moe_linear: workspace of %zu elements needed", (size_t)places * K);
@@ -297,12 +345,13 @@ extern "C" int mlora_moe_linear(void* y, const void* x, const void* W, const int
                          places / 16, K, top);
       xf = workspace;
     }
-    return mlora_gemm_grouped(y, xf, places / 16, W, p, max_tiles, K, N, stage == MLORA_MOE_UP, alpha, stream);
+    return mlora_gemm_grouped(y, xf, places / 16, W, p, max_tiles, K, N, act, alpha, stream);
   }
   MoeLinear a;
-  a.y = (elt*)y; a.x = (const elt*)x; a.W = (const elt*)W; a.w_elems = (size_t)N * K;
+  a.y = (elt*)y; a.x = (const elt*)x; a.W = (const elt*)W; a.w_elems = (size_t)N * K * (act == MLORA_ACT_GLU ? 2 : 1);
   a.K = K; a.N = N; a.top = top; a.up = stage == MLORA_MOE_UP; a.act = act; a.alpha = alpha;
-  hipLaunchKernelGGL((moe_gemv_kernel<2, 4>), dim3(ceil_div(N, 32), max_tiles), dim3(MG_WAVES * WAVE), 0, s, a, p);
+  if (act == MLORA_ACT_GLU) hipLaunchKernelGGL((moe_gemv_kernel<2, 4, true>), dim3(N / 16, max_tiles), dim3(MG_WAVES * WAVE), 0, s, a, p);
+  else hipLaunchKernelGGL((moe_gemv_kernel<2, 4>), dim3(ceil_div(N, 32), max_tiles), dim3(MG_WAVES * WAVE), 0, s, a, p);
   return mlora_launch_status("moe_linear");
 }
 #endif

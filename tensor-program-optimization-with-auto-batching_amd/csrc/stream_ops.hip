@@ -1,5 +1,5 @@
-// Row operators of decoders whose fp32 residual stream is normed by one number and carries a per-layer token input.
-// Compiled for every element type.
+// Row operators of decoders with an fp32 residual stream: the one-number norm and a per-layer token input; the elementwise
+// norm ahead of and behind a sublayer, with the mixes of neighbouring tokens.  Compiled for every element type.
 #include "common.h"
 
 namespace {
@@ -188,6 +188,118 @@ __global__ __launch_bounds__(256) void token_gate_mul_kernel(elt* __restrict__ o
   out[i] = (elt)(gelu_tanh((float)z[i]) * ev);
 }
 
+// ---------------------------------------------------------------------------------------------
+// The residual stream of a decoder whose norms are elementwise, dt(v) = tanh(alpha v) w + b:
+//   x' = x + mult post(branch),  branch = y + parts + row_weight * (entry rows of the token)
+//   h  = pre(x'), written once, or as the mixes h + (h_prev - h) mu_s of a token and the one before it in its sequence
+// No row statistics are needed, so the previous token's h is computed again instead of being exchanged.
+// ---------------------------------------------------------------------------------------------
+__device__ __forceinline__ f32x4 ld4f(const elt* p) {
+  const eltx4 v = *reinterpret_cast<const eltx4*>(p);
+  return f32x4{(float)v[0], (float)v[1], (float)v[2], (float)v[3]};
+}
+
+struct TanhNorm {
+  f32x4 w, b;
+  float alpha;
+  bool on;
+  __device__ __forceinline__ TanhNorm(const mlora_tanh_norm& n, int c) : alpha(n.alpha), on(n.w != nullptr) {
+    w = on ? ld4f((const elt*)n.w + c) : f32x4{1.f, 1.f, 1.f, 1.f};
+    b = on ? ld4f((const elt*)n.b + c) : f32x4{0.f, 0.f, 0.f, 0.f};
+  }
+  __device__ __forceinline__ f32x4 operator()(f32x4 v) const {
+    if (!on) return v;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = fmaf(tanhf(alpha * v[e]), w[e], b[e]);
+    return v;
+  }
+};
+
+// one token's four columns of x + mult post(branch)
+__device__ __forceinline__ f32x4 step_row(const mlora_stream_step_args& a, const TanhNorm& post, int t, int c) {
+  const size_t o = (size_t)t * a.Hp + c;
+  f32x4 x = a.x ? *reinterpret_cast<const f32x4*>(a.x + o) : f32x4{0.f, 0.f, 0.f, 0.f};
+  if (!a.y && !a.rows) return x;
+  f32x4 v = a.y ? *reinterpret_cast<const f32x4*>(a.y + o) : f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int q = 0; q < a.n_part; ++q) v += *reinterpret_cast<const f32x4*>(a.part + (size_t)q * a.T * a.Hp + o);
+  if (a.rows) {
+    f32x4 s = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int k = 0; k < a.top; ++k) s += ld4f((const elt*)a.rows + ((size_t)t * a.top + k) * a.Hp + c);
+    v += s * a.row_weight;
+  }
+  v = post(v);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) x[e] = fmaf(a.mult, v[e], x[e]);
+  return x;
+}
+
+constexpr int ST_THREADS = 128;
+constexpr int ST_MIX = 5;
+// A thread takes four columns of `rows` consecutive tokens.
+template <bool SHIFT>
+__global__ __launch_bounds__(ST_THREADS) void stream_step_kernel(mlora_stream_step_args a, int rows, int frag_tt) {
+  const int c = (blockIdx.x * ST_THREADS + threadIdx.x) * 4;
+  if (c >= a.Hp) return;
+  const TanhNorm post(a.post, c), pre(a.pre, c);
+  const bool out = a.out_frag || a.out_row;
+  f32x4 mu[SHIFT ? ST_MIX : 1], prev = f32x4{0.f, 0.f, 0.f, 0.f};
+  int prev_seq = -1;                                                 // whose h `prev` is
+  if constexpr (SHIFT) {
+#pragma unroll
+    for (int s = 0; s < ST_MIX; ++s) mu[s] = ld4f((const elt*)a.mu + (size_t)s * a.Hp + c);
+  }
+  const int t0 = blockIdx.y * rows, t1 = t0 + rows < a.T ? t0 + rows : a.T;
+  for (int t = t0; t < t1; ++t) {
+    const f32x4 x = step_row(a, post, t, c);
+    if (a.x_out) *reinterpret_cast<f32x4*>(a.x_out + (size_t)t * a.Hp + c) = x;
+    if (!out) continue;
+    const f32x4 h = pre(x);
+    if constexpr (SHIFT) {
+      const int seq = a.tok_seq[t], pos = a.tok_pos[t];
+      const bool live = seq >= 0 && seq < a.n_seq;
+      if (pos <= 0) prev = f32x4{0.f, 0.f, 0.f, 0.f};
+      else if (t > 0 && a.tok_seq[t - 1] == seq) {
+        if (prev_seq < 0) prev = pre(step_row(a, post, t - 1, c));   // the token before belongs to another workgroup
+      } else prev = live ? *reinterpret_cast<const f32x4*>(a.shift + (size_t)seq * a.Hp + c) : f32x4{0.f, 0.f, 0.f, 0.f};
+      if (live && (t == 0 || a.tok_seq[t - 1] != seq)) {
+        // the sequence's first token of the pass read the state; it also leaves the last one's h there
+        int last = a.tok_last ? a.tok_last[t] : t;
+        last = last < a.T ? last : a.T - 1;
+        *reinterpret_cast<f32x4*>(a.shift + (size_t)seq * a.Hp + c) = last > t ? pre(step_row(a, post, last, c)) : h;
+      }
+#pragma unroll
+      for (int s = 0; s < ST_MIX; ++s) {
+        eltx4 o;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o[e] = (elt)fmaf(prev[e] - h[e], mu[s][e], h[e]);
+        if (a.out_frag) *reinterpret_cast<eltx4*>((elt*)a.out_frag + s * (size_t)a.mix_stride + frag_offset(t, c, frag_tt)) = o;
+        if (a.out_row) *reinterpret_cast<eltx4*>((elt*)a.out_row + s * (size_t)a.mix_stride + (size_t)t * a.ld_row + c) = o;
+      }
+      prev = h;
+      prev_seq = 0;
+    } else {
+      const eltx4 o = eltx4{(elt)h[0], (elt)h[1], (elt)h[2], (elt)h[3]};
+      if (a.out_frag) *reinterpret_cast<eltx4*>((elt*)a.out_frag + frag_offset(t, c, frag_tt)) = o;
+      if (a.out_row) *reinterpret_cast<eltx4*>((elt*)a.out_row + (size_t)t * a.ld_row + c) = o;
+    }
+  }
+}
+
+// x = table[id] * scale in fp32, and the same rounded, in fragment order or with a row stride of its own
+__global__ __launch_bounds__(256) void embed_scaled_kernel(float* __restrict__ x, elt* __restrict__ out_frag, int frag_tt, elt* __restrict__ out_row,
+                                                           int ld_row, const elt* __restrict__ table, const int32_t* __restrict__ ids, float scale,
+                                                           int H, int V) {
+  const int t = blockIdx.y, c = (blockIdx.x * 256 + threadIdx.x) * 4;
+  if (c >= H) return;
+  const int id = ids[t];
+  f32x4 v = f32x4{0.f, 0.f, 0.f, 0.f};
+  if (id >= 0 && id < V) v = ld4f(table + (size_t)id * H + c) * scale;
+  *reinterpret_cast<f32x4*>(x + (size_t)t * H + c) = v;
+  const eltx4 o = eltx4{(elt)v[0], (elt)v[1], (elt)v[2], (elt)v[3]};
+  if (out_frag) *reinterpret_cast<eltx4*>(out_frag + frag_offset(t, c, frag_tt)) = o;
+  if (out_row) *reinterpret_cast<eltx4*>(out_row + (size_t)t * ld_row + c) = o;
+}
+
 }  // namespace
 
 extern "C" int mlora_stream_norm(void* out_frag, void* out_row, float* x, const float* part, int n_part, const float* branch,
@@ -240,4 +352,39 @@ extern "C" int mlora_token_gate_mul(void* out, const void* z, const void* table,
   hipLaunchKernelGGL(token_gate_mul_kernel, dim3((unsigned)(((size_t)T * N + 255) / 256)), dim3(256), 0, (hipStream_t)stream, (elt*)out,
                      (const elt*)z, (const elt*)table, ld_table, col0, dim, ids, V, T, N);
   return mlora_launch_status("token_gate_mul");
+}
+
+extern "C" int mlora_stream_step(const mlora_stream_step_args* args, void* stream) {
+  MLORA_CHECK(args, MLORA_ERR_INVALID, "stream_step: null pointer");
+  const mlora_stream_step_args& a = *args;
+  MLORA_CHECK(a.T >= 0 && a.Hp > 0 && a.Hp % 32 == 0 && a.n_part >= 0 && a.T <= 65535 * 8, MLORA_ERR_UNSUPPORTED,
+              "stream_step: need Hp %% 32 == 0 (T=%d Hp=%d)", a.T, a.Hp);
+  MLORA_CHECK((a.x || a.y || a.rows) && (a.n_part == 0 || (a.part && a.y)) && (!a.rows || a.top > 0) && (!a.post.w || a.post.b) && (!a.pre.w || a.pre.b),
+              MLORA_ERR_INVALID, "stream_step: null pointer");
+  MLORA_CHECK(!a.out_frag || sizeof(elt) == 2, MLORA_ERR_UNSUPPORTED, "stream_step: fragment order is for 16-bit elements");
+  MLORA_CHECK(!a.out_row || (a.ld_row >= a.Hp && a.ld_row % 4 == 0), MLORA_ERR_INVALID, "stream_step: row stride %d", a.ld_row);
+  if (a.mu)
+    MLORA_CHECK(a.shift && a.tok_seq && a.tok_pos && a.n_seq > 0 && (a.out_frag || a.out_row) && (!(a.y || a.rows) || a.x_out != a.x), MLORA_ERR_INVALID,
+                "stream_step: the mixes need the state, the tokens' sequences and a stream that is not updated in place");
+  if (a.T == 0) return MLORA_OK;
+  hipStream_t s = (hipStream_t)stream;
+  const int cols = ceil_div(a.Hp, ST_THREADS * 4), tt = mlora_frag_tiles(a.T);
+  int rows = 1;
+  while (rows < 8 && (long)cols * ceil_div(a.T, 2 * rows) >= 2048) rows *= 2;
+  while (ceil_div(a.T, rows) > 65535) rows *= 2;
+  const dim3 grid(cols, ceil_div(a.T, rows));
+  if (a.mu) hipLaunchKernelGGL(stream_step_kernel<true>, grid, dim3(ST_THREADS), 0, s, a, rows, tt);
+  else hipLaunchKernelGGL(stream_step_kernel<false>, grid, dim3(ST_THREADS), 0, s, a, rows, tt);
+  return mlora_launch_status("stream_step");
+}
+
+extern "C" int mlora_embed_scaled(float* x, void* out_frag, void* out_row, int ld_row, const void* table, const int32_t* ids, float scale, int T, int H,
+                                  int V, void* stream) {
+  MLORA_CHECK(x && table && ids, MLORA_ERR_INVALID, "embed_scaled: null pointer");
+  MLORA_CHECK(T >= 0 && T <= 65535 && H > 0 && H % 32 == 0 && V > 0 && (!out_frag || sizeof(elt) == 2) && (!out_row || (ld_row >= H && ld_row % 4 == 0)),
+              MLORA_ERR_UNSUPPORTED, "embed_scaled: need H %% 32 == 0 (T=%d H=%d V=%d)", T, H, V);
+  if (T == 0) return MLORA_OK;
+  hipLaunchKernelGGL(embed_scaled_kernel, dim3(ceil_div(H, 1024), T), dim3(256), 0, (hipStream_t)stream, x, (elt*)out_frag, mlora_frag_tiles(T),
+                     (elt*)out_row, ld_row, (const elt*)table, ids, scale, H, V);
+  return mlora_launch_status("embed_scaled");
 }

@@ -3,10 +3,12 @@ fragment-ordered activations and packed weights, fp32 on plain row-major tensors
 """
 from __future__ import annotations
 
+import ctypes
+
 import torch
 
 from . import ops
-from ._lib import ACT_NONE, ACT_RELU2, FRAG, MOE_DOWN, MOE_UP, ROWMAJOR   # noqa: F401
+from ._lib import ACT_GLU, ACT_NONE, ACT_RELU2, FRAG, MOE_DOWN, MOE_UP, ROWMAJOR, StreamStep   # noqa: F401
 from .ops import FragActivation, PackedWeight, _dev, _stream, check, lib_of
 
 
@@ -65,6 +67,106 @@ def stream_norm(x, H, eps, gain=1.0, parts=None, branch=None, out=None, out_row=
                                        float(eps), float(gain), int(raw), T, H, Hp, _stream()), dt)
 
 
+def embed_scaled(table, ids, scale, out=None):
+    """table[ids] * scale in fp32; out: an activation that takes the same in the table's type."""
+    V, H = table.shape
+    T = ids.numel()
+    x = torch.empty((T, H), dtype=torch.float32, device=table.device)
+    frag = out.data.data_ptr() if isinstance(out, FragActivation) else None
+    row, ld = (out.data_ptr(), out.stride(0)) if isinstance(out, torch.Tensor) else (None, 0)
+    check(lib_of(table.dtype).mlora_embed_scaled(_dev(x), frag, row, ld, _dev(table), _dev(ids, torch.int32), scale, T, H, V, _stream()), table.dtype)
+    return x
+
+
+class ElementwiseNorm:
+    """tanh(alpha v) w + b, without statistics (weights [Hp], zero behind the width)."""
+
+    def __init__(self, w, b, alpha, width_p, dtype, device):
+        self.w, self.b = (padded(t.to(device, dtype), width_p).contiguous() for t in (w, b))
+        self.alpha = float(alpha)
+
+    def fill(self, f):
+        f.w, f.b, f.alpha = self.w.data_ptr(), self.b.data_ptr(), self.alpha
+
+
+class ResidualStream:
+    """The fp32 stream x [T, Hp] of a pass with a branch that is still to be added: x + mult post(branch), where the branch is
+    a sum of K-split partials and of entry rows of a mixture of experts.  Every step of a sublayer is one launch that adds
+    what is pending and norms for the next sublayer."""
+
+    def __init__(self, x, dtype, mult=1.0):
+        self.x, self.dtype, self.mult = x, dtype, float(mult)
+        self.shape, self.device = x.shape, x.device
+        self.spare = None
+        self.pending = None           # (y or None, KSplitParts or None, rows or None, row weight, norm or None, replaces x)
+
+    def branch(self, y, parts=None, norm=None, rows=None, row_weight=1.0):
+        assert self.pending is None
+        self.pending = (y, parts, rows, row_weight, norm, False)
+
+    def replace(self, y, parts=None):
+        """x becomes y (+ its partials)."""
+        assert self.pending is None
+        self.pending = (y, parts, None, 1.0, None, True)
+
+    def step(self, norm=None, out=None, out_row=None, mu=None, shift=None, tokens=None):
+        """Adds what is pending; out (FragActivation) and / or out_row (rows, any stride): norm(x), or x itself without norm.
+        mu [5, Hp], shift (state), tokens = (sequence, position, last token or None) per token: five mixes, stacked in out /
+        out_row."""
+        if out is None and out_row is None and self.pending is None:
+            return
+        T, Hp = self.shape
+        a = StreamStep(T=T, Hp=Hp, x=self.x.data_ptr(), mult=self.mult, row_weight=1.0)
+        keep = None
+        if self.pending is not None:
+            y, parts, rows, a.row_weight, post, new = keep = self.pending
+            if y is not None:
+                a.y = _dev(y, torch.float32)
+            if parts is not None:
+                a.part, a.n_part = parts.part.data_ptr(), parts.ks - 1
+            if rows is not None:
+                a.rows, a.top = _dev(rows, self.dtype), rows.shape[0] // T
+            if post is not None:
+                post.fill(a.post)
+            if new:
+                a.x, a.mult = None, 1.0
+            x = self.x
+            if mu is not None or new:                     # a neighbour reads the old stream
+                if self.spare is None:
+                    self.spare = torch.empty_like(self.x)
+                x, self.spare = self.spare, self.x
+            a.x_out = x.data_ptr()
+            self.x, self.pending = x, None
+        if norm is not None:
+            norm.fill(a.pre)
+        if out is not None:
+            a.out_frag, a.mix_stride = out.data.data_ptr(), out.data.numel() // 5
+        if out_row is not None:
+            a.out_row, a.ld_row = out_row.data_ptr(), out_row.stride(-2)
+            if mu is not None:
+                a.mix_stride = out_row.stride(0)
+        if mu is not None:
+            seq, pos, last = tokens
+            a.mu, a.shift, a.n_seq = _dev(mu, self.dtype), _dev(shift, torch.float32), shift.shape[0]
+            a.tok_seq, a.tok_pos, a.tok_last = _dev(seq, torch.int32), _dev(pos, torch.int32), _ptr(last)
+        check(lib_of(self.dtype).mlora_stream_step(ctypes.byref(a), _stream()), self.dtype)
+        del keep
+
+
+def linear_sum(x, W, split=True):
+    """x @ W.T as (y fp32, K-split partials still to be added to it, or None)."""
+    if not split or not isinstance(x, FragActivation):
+        return ops.linear(x, W, out_dtype=torch.float32), None
+    T, K = x.shape
+    N = W.shape[0]
+    L = lib_of(W.dtype)
+    ks = L.mlora_gemv_ksplit(T, K, N)
+    y = torch.empty((T, N), dtype=torch.float32, device=x.device)
+    part = torch.empty((ks - 1) * T * N, dtype=torch.float32, device=x.device) if ks > 1 else None
+    check(L.mlora_linear_ksplit_store(y.data_ptr(), _ptr(part), ks, x.data.data_ptr(), W.data.data_ptr(), T, K, N, _stream()), W.dtype)
+    return y, ops.KSplitParts(part, ks, N) if ks > 1 else None
+
+
 def token_gate(x, W, table, col0, dim, ids):
     """gelu_tanh(W x) * table[ids, col0 : col0 + dim] (x: an activation) as the activation of the following linear, its width
     W's padded row count."""
@@ -110,6 +212,94 @@ def gate_up_clipglu(x, W, W_il, scale, limit, alpha, out):
             check(L.mlora_linear_frag_clipglu(out.data.data_ptr(), x.data.data_ptr(), W.data.data_ptr(), *args), x.dtype)
             return out
     return clipglu_mul(ops.linear(x, W), scale, limit, alpha, out)
+
+
+def silu_mul(gate_up, out):
+    """silu(gate) * up of gate_up [T, 2I] (gate columns first) into `out` (activation [T, I])."""
+    T, I2 = gate_up.shape
+    dt = gate_up.dtype
+    frag = isinstance(out, FragActivation)
+    p = _dev(gate_up)
+    check(lib_of(dt).mlora_silu_mul(out.data.data_ptr() if frag else _dev(out), FRAG if frag else ROWMAJOR, p, p + I2 // 2 * gate_up.element_size(), I2,
+                                    T, I2 // 2, _stream()), dt)
+    return out
+
+
+def gate_up_silu(x, W, W_il, out):
+    """silu(gate) * up of x @ W.T (W [2I, K], gate rows first; W_il: its tiles interleaved) into `out` - the product as the
+    epilogue of the linear where a kernel has that, else behind it."""
+    T, K = x.shape
+    I2 = W.shape[0]
+    if isinstance(x, FragActivation):
+        L = lib_of(x.dtype)
+        if T <= 64:
+            check(L.mlora_gemv_frag_silu(out.data.data_ptr(), x.data.data_ptr(), W_il.data.data_ptr(), T, K, I2 // 2, _stream()), x.dtype)
+            return out
+        if L.mlora_gemm_frag_preferred(T, K, I2):
+            check(L.mlora_linear_frag_silu(out.data.data_ptr(), x.data.data_ptr(), W.data.data_ptr(), T, K, I2 // 2, None, 0, None, 0, _stream()),
+                  x.dtype)
+            return out
+    return silu_mul(ops.linear(x, W), out)
+
+
+def time_mix(r, k, v, g, z, R, w2t, w0, u, norm, eps, state, segs, tok_seq, tok_pos, out):
+    """The recurrence of time mixing (csrc/time_mix.hip) over a pass: r, k, v, g [T, ld], z [T, >= R] fp32, state [n, H, D, D] fp32
+    (updated), segs [n][4] int32 or None (a decode step) -> out, an activation [T, H * D rounded up]."""
+    T, ld = r.shape
+    n_seq, H, D, _ = state.shape
+    frag = isinstance(out, FragActivation)
+    check(lib_of(r.dtype).mlora_time_mix(out.data.data_ptr() if frag else _dev(out, r.dtype), FRAG if frag else ROWMAJOR, out.shape[1],
+                                         _dev(r), _dev(k, r.dtype), _dev(v, r.dtype), _dev(g, r.dtype), ld, _dev(z, torch.float32), z.shape[1], R,
+                                         _dev(w2t, r.dtype), w2t.shape[1], _dev(w0, torch.float32), _dev(u, torch.float32), _dev(norm, r.dtype), eps,
+                                         _dev(state, torch.float32), n_seq, _ptr(segs), T if segs is None else segs.shape[0],
+                                         _dev(tok_seq, torch.int32), _dev(tok_pos, torch.int32), T, H, D, _stream()), r.dtype)
+    return out
+
+
+def tied_prep(q, pages, key_scale, y, bias, q_norm, eps, temp, block_table, tok_seq, tok_pos, H, G, dim):
+    """Queries [T, H, pad32(dim)] from the projections y [T, >= (H + G) dim] fp32, and their values and key scales into the pages.
+    temp: (coefficient, every) of the queries' temperature, or None."""
+    n_seq, max_blocks = block_table.shape
+    T, ld = y.shape
+    coef, every = temp or (0.0, 0.0)
+    check(lib_of(q.dtype).mlora_tied_prep(_dev(q), _dev(pages, q.dtype), _dev(key_scale, torch.float32), _dev(y, torch.float32), ld,
+                                          _dev(bias, torch.float32), _dev(q_norm, torch.float32), eps, coef, every, _dev(block_table, torch.int32),
+                                          max_blocks, _dev(tok_seq, torch.int32), _dev(tok_pos, torch.int32), T, H, G, dim, pages.shape[0], n_seq,
+                                          _stream()), q.dtype)
+
+
+def tied_attn(q, pages, key_scale, block_table, tok_seq, tok_pos, slopes, scale, G, dim, max_ctx, out, splits=None):
+    """Causal attention over pages whose values are its keys -> out, an activation [T, H * pad32(dim)]."""
+    T, H, _ = q.shape
+    n_seq, max_blocks = block_table.shape
+    L = lib_of(q.dtype)
+    if splits is None:
+        splits = L.mlora_tied_attn_splits(T, H, G, max_ctx)
+    nb = L.mlora_latent_attn_workspace_bytes(T, H, dim, splits)
+    ws = torch.empty(nb // 4, dtype=torch.float32, device=q.device) if nb else None
+    frag = isinstance(out, FragActivation)
+    check(L.mlora_tied_attn(out.data.data_ptr() if frag else _dev(out, q.dtype), FRAG if frag else ROWMAJOR, _dev(q), _dev(pages, q.dtype),
+                            _dev(key_scale, torch.float32), _dev(block_table, torch.int32), max_blocks, _dev(tok_seq, torch.int32),
+                            _dev(tok_pos, torch.int32), _dev(slopes, torch.float32), scale, T, H, G, dim, pages.shape[0], n_seq, splits, _ptr(ws), nb,
+                            _stream()), q.dtype)
+    return out
+
+
+def tied_prefill_served(dim) -> bool:
+    return bool(lib_of(torch.bfloat16).mlora_tied_prefill_served(dim))
+
+
+def tied_prefill(plan, q, pages, key_scale, slopes, scale, G, dim, out):
+    """The same for a pass over prompts (plan: PrefillPlan), with keys and transposed values laid out in scratch memory."""
+    T, H, _ = q.shape
+    L = lib_of(q.dtype)
+    n = L.mlora_tied_prefill_scratch_elems(plan.pages, G, dim)
+    scratch = torch.empty(n, dtype=q.dtype, device=q.device)
+    frag = isinstance(out, FragActivation)
+    check(L.mlora_tied_prefill(out.data.data_ptr() if frag else _dev(out, q.dtype), FRAG if frag else ROWMAJOR, out.shape[1], _dev(q),
+                               _dev(pages, q.dtype), _dev(key_scale, torch.float32), plan.phys.data_ptr(), plan.pages, plan.tiles.data_ptr(), plan.n_tiles,
+                               _dev(slopes, torch.float32), scale, T, H, G, dim, pages.shape[0], scratch.data_ptr(), n, _stream()), q.dtype)
+    return out
 
 
 def head_linear(x, ldx, head_x, W, heads, T, K, N, out, ldy, head_y, alpha=1.0):
@@ -227,15 +417,35 @@ class MoePlan:
     """The (token, choice) entries of a routing sorted by expert into places and cut into tiles."""
 
     def __init__(self, pick, E, dtype):
-        self.T, self.top = pick.shape
-        L, dev = lib_of(dtype), pick.device
-        self.tile_rows = L.mlora_moe_tile_rows(self.T, E, self.top)
-        self.max_tiles = L.mlora_moe_max_tiles(self.T, E, self.top)
-        self.places = L.mlora_moe_max_places(self.T, E, self.top)
-        i32 = lambda n: torch.empty(n, dtype=torch.int32, device=dev)
-        self.perm, self.tiles, self.n_tiles = i32(self.places), i32(4 * self.max_tiles), i32(2)
-        check(L.mlora_moe_plan(self.perm.data_ptr(), self.tiles.data_ptr(), self.n_tiles.data_ptr(), _dev(pick, torch.int32), self.T, E, self.top,
-                               _stream()), dtype)
+        self._sizes(*pick.shape, E, dtype)
+        self.perm, self.tiles, self.n_tiles = self._room(1, pick.device)
+        check(lib_of(dtype).mlora_moe_plan(self.perm.data_ptr(), self.tiles.data_ptr(), self.n_tiles.data_ptr(), _dev(pick, torch.int32), self.T, E,
+                                           self.top, _stream()), dtype)
+
+    def _sizes(self, T, top, E, dtype):
+        L = lib_of(dtype)
+        self.T, self.top = T, top
+        self.tile_rows = L.mlora_moe_tile_rows(T, E, top)
+        self.max_tiles = L.mlora_moe_max_tiles(T, E, top)
+        self.places = L.mlora_moe_max_places(T, E, top)
+
+    def _room(self, layers, dev):
+        return tuple(torch.empty(layers * n, dtype=torch.int32, device=dev) for n in (self.places, 4 * self.max_tiles, 2))
+
+    @classmethod
+    def of_tables(cls, tables, ids, E, dtype):
+        """Plans of all layers whose experts are looked up by token id (tables [layers, V, top] int32) in one launch."""
+        n, V, top = tables.shape
+        T = ids.numel()
+        plans = [cls.__new__(cls) for _ in range(n)]
+        for p in plans:
+            p._sizes(T, top, E, dtype)
+        room = plans[0]._room(n, ids.device)
+        check(lib_of(dtype).mlora_moe_table_plan(*(r.data_ptr() for r in room), _dev(tables, torch.int32), _dev(ids, torch.int32), n, V, T, E, top,
+                                                 _stream()), dtype)
+        for p, perm, tiles, n_tiles in zip(plans, *(r.view(n, -1) for r in room)):
+            p.perm, p.tiles, p.n_tiles = perm, tiles, n_tiles
+        return plans
 
 
 def moe_linear(x, W, plan, N, K, stage, act=ACT_NONE, alpha=1.0):

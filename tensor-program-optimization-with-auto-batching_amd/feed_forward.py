@@ -1,7 +1,8 @@
-"""Feed-forward blocks: a dense one with a clipped gated product, and a mixture of experts."""
+"""Feed-forward blocks: a dense one with a clipped gated product, and mixtures of experts, routed by a router or by token id."""
 from __future__ import annotations
 
 import dataclasses
+from typing import Optional
 
 import torch
 
@@ -22,6 +23,20 @@ class MoeSpec:
     ff: int
     experts: int
     top: int
+
+
+@dataclasses.dataclass(frozen=True)
+class TableMoeSpec:
+    """Experts by token id, each of weight 1 / top, and a shared expert of width `shared` (None: none)."""
+    ff: int
+    experts: int
+    top: int
+    shared: Optional[int] = None
+
+    @classmethod
+    def from_config(cls, c: dict) -> "TableMoeSpec":
+        shared = c.get("shared")
+        return cls(int(c["expert"]["ff"]), int(c["router"]["experts"]), int(c["router"]["top"]), int(shared["ff"]) if shared else None)
 
 
 class ClippedGlu:
@@ -63,3 +78,64 @@ class MoeRelu2:
         plan = D.MoePlan(pick, s.experts, self.dtype)
         mid = D.moe_linear(x_row, self.up, plan, self.ffp, self.Hp, D.MOE_UP, D.ACT_RELU2, self.gain)
         D.moe_combine(resid, D.moe_linear(mid, self.down, plan, self.Hp, self.ffp, D.MOE_DOWN), wt, parts, out)
+
+
+class SiluGlu:
+    """down(silu(gate h) * up h)."""
+
+    def __init__(self, w: dict, ff: int, width: int, dtype, device):
+        Hp, self.ffp, self.dtype = pad64(width), pad64(ff), dtype
+        gu = torch.cat([padded(w[k].to(device, dtype), self.ffp, Hp) for k in ("gate", "up")])
+        self.gate_up = D.weight(gu)
+        self.gate_up_il = ops.interleave_gate_up(gu) if dtype != torch.float32 else None
+        self.down = D.weight(padded(w["down"].to(device, dtype), Hp, self.ffp))
+
+    def hidden(self, x):
+        return D.gate_up_silu(x, self.gate_up, self.gate_up_il, D.activation(x.shape[0], self.ffp, self.dtype, x.device))
+
+
+class TableMoe:
+    """Experts down(silu(gate h) * up h) chosen by token id, and a shared one for every token."""
+
+    def __init__(self, spec: TableMoeSpec, w: dict, width: int, dtype, device):
+        """w: table [V, top], gate, up: E x [ff, width], down: E x [width, ff], shared: the same three, if there is one."""
+        self.spec, self.dtype = spec, dtype
+        self.Hp, self.ffp = pad64(width), pad64(spec.ff)
+        self.table = w["table"].to(device, torch.int32).contiguous()
+        if self.table.shape[1] != spec.top or int(self.table.min()) < 0 or int(self.table.max()) >= spec.experts:
+            raise ValueError(f"expert table {tuple(self.table.shape)}: entries outside 0..{spec.experts - 1}, or not {spec.top} per token")
+        cut = lambda m, n, k: padded(m.to(device, dtype), n, k)
+        # per expert its gate rows, then its up rows
+        self.gate_up = D.weight(torch.cat([cut(m, self.ffp, self.Hp) for g, u in zip(w["gate"], w["up"]) for m in (g, u)]))
+        self.down = D.weight(torch.cat([cut(m, self.Hp, self.ffp) for m in w["down"]]))
+        self.shared = SiluGlu(w["shared"], spec.shared, width, dtype, device) if spec.shared else None
+
+    def __call__(self, x, x_row, plan, split):
+        """x: the input as an activation, x_row: the same row-major -> (entry rows [T * top, Hp] of weight 1 / top, shared output fp32 or
+        None, its pending partials)."""
+        if self.dtype == torch.float32:
+            gu = D.moe_linear(x_row, self.gate_up, plan, 2 * self.ffp, self.Hp, D.MOE_UP)
+            mid = D.silu_mul(gu, torch.empty((gu.shape[0], self.ffp), dtype=gu.dtype, device=gu.device))
+        else:
+            mid = D.moe_linear(x_row, self.gate_up, plan, self.ffp, self.Hp, D.MOE_UP, D.ACT_GLU)
+        rows = D.moe_linear(mid, self.down, plan, self.Hp, self.ffp, D.MOE_DOWN)
+        if self.shared is None:
+            return rows, None, None
+        return (rows, *D.linear_sum(self.shared.hidden(x), self.shared.down, split))
+
+
+class TableRouting:
+    """The routing of a pass: which expert a token takes depends on its id alone, so the plans of all layers are made at once."""
+
+    def __init__(self, blocks: dict, dtype):
+        """blocks: layer -> TableMoe."""
+        self.dtype, self.groups = dtype, {}
+        for l, b in blocks.items():
+            self.groups.setdefault((b.spec.experts, b.spec.top), []).append(l)
+        self.tables = {k: torch.stack([blocks[l].table for l in ls]).contiguous() for k, ls in self.groups.items()}
+
+    def plans(self, ids):
+        out = {}
+        for (E, top), layers in self.groups.items():
+            out.update(zip(layers, D.MoePlan.of_tables(self.tables[E, top], ids, E, self.dtype)))
+        return out

@@ -166,6 +166,7 @@ class PagedKVCache(PageTable):
         per_pos = self.n_layers * 2 * self.Hkv * self.D * 2
         return int(sum(self.lens[s] + 1 for s in seq_ids)) * per_pos
 
+
 class PagedLatentCache(PageTable):
     """Pages of latent attention: per layer one vector per token, the normed latent and the rotated key part, in the page
     layout of latent_attention.hip.  A layer may read another layer's pages instead of having its own."""
@@ -210,3 +211,74 @@ class PagedLatentCache(PageTable):
             plan = self._plan[1]
         return att.attend(qkv, self.pages[layer], self.block_table, tok_seq, tok_pos, *self.rope[layer], max_ctx=max(ctx),
                           store=self.owner[layer] == layer, plan=plan, out=out)
+
+
+class PagedStateCache(PageTable):
+    """What the layers of a model with recurrent and attention layers keep per sequence, one entry per layer run (a layer that
+    runs several times has one for every pass): pages of tied attention, or a state per slot.  A slot needs no clearing:
+    kernels start a sequence's state from zero at its position 0."""
+
+    def __init__(self, runs, width_p, n_pages, max_seqs, max_blocks, max_pos, dtype, device="cuda:0", free_pages=None, page_size=PAGE):
+        """runs: per layer run the mixer's spec (TiedSpec or TimeMixSpec); width_p: columns of the residual stream."""
+        super().__init__(n_pages, max_seqs, max_blocks, max_pos, device, free_pages, page_size)
+        self.dtype = dtype
+        self.entries = []
+        zeros = lambda *shape, dt=torch.float32: torch.zeros(shape, dtype=dt, device=self.device)
+        for s in runs:
+            if hasattr(s, "kv_heads"):
+                # pages [n_pages, G, dim / 32, 4, 16, 8] of values, and one key scale per token and head
+                self.entries.append((zeros(n_pages, s.kv_heads, -(-s.dim // 32), 4, PAGE, 8, dt=dtype), zeros(n_pages, s.kv_heads, PAGE)))
+            else:
+                # matrix states, and the previous token's normed row
+                self.entries.append((zeros(max_seqs, s.heads, s.dim, s.dim), zeros(max_seqs, width_p)))
+        self._meta = None
+
+    def values(self, run, sid):
+        """The cached values [length, G, columns] of a sequence (a copy, for inspection)."""
+        p = self.entries[run][0][torch.tensor(self.pages_of(sid), device=self.device, dtype=torch.int64)]
+        return p.permute(0, 4, 1, 2, 3, 5).reshape(-1, p.shape[1], p.shape[2] * 32)[: self.lens[sid]].contiguous()
+
+    def state(self, run, sid):
+        """The matrix states [H, D, D] of a sequence (a view)."""
+        return self.entries[run][0][self.slot[sid]]
+
+    def shift(self, run):
+        """The previous tokens' rows [slots, columns] of a recurrent layer run."""
+        return self.entries[run][1]
+
+    def _pass(self):
+        """Of the current pass, made once for all its layers: {"last": the last token of every token's sequence, "segs": [n][4]
+        {slot, first token, tokens, position}} - both None in a decode step - and the plan of its prompt form, if taken."""
+        if self._cur is None:
+            raise RuntimeError("outside begin_forward/end_forward")
+        if self._meta is None or self._meta[0] is not self._cur:
+            seq_ids, lens, decode = self._cur[:3]
+            m = {"last": None, "segs": None, "plan": None}
+            if not decode:
+                ends = np.cumsum(lens)
+                segs = [(self.slot[s], e - n, n, self.lens[s]) for s, n, e in zip(seq_ids, lens, ends)]
+                both = np.concatenate([np.asarray(segs, dtype=np.int32).reshape(-1), np.repeat(ends - 1, lens).astype(np.int32)])
+                both = torch.from_numpy(both).to(self.device)
+                m["segs"], m["last"] = both[: 4 * len(segs)].view(-1, 4), both[4 * len(segs):]
+            self._meta = (self._cur, m)
+        return self._meta[1]
+
+    def token_meta(self):
+        """(sequence, position, last token of its sequence in the pass) per token."""
+        return self._cur[3], self._cur[4], self._pass()["last"]
+
+    def time_mix(self, run, mixes, mixer):
+        """The recurrence of a layer run on the five mixes of the pass (mixer: time_mix.TimeMix)."""
+        return mixer.run(mixes, self.entries[run][0], self._pass()["segs"], self._cur[3], self._cur[4])
+
+    def tied_attention(self, run, y, att):
+        """The attention of a layer run behind its input projection y (att: tied_attention.TiedAttention)."""
+        m = self._pass()
+        seq_ids, append_lens, decode, tok_seq, tok_pos, _ = self._cur
+        seqs = [(n, self.lens[s] + n) for s, n in zip(seq_ids, append_lens)]
+        plan = None
+        if not decode and att.prompt_form_pays(seqs):
+            if m["plan"] is None:
+                m["plan"] = PrefillPlan([(self.pages_of(s), n, c) for s, (n, c) in zip(seq_ids, seqs)], self.device)
+            plan = m["plan"]
+        return att.attend(y, *self.entries[run], self.block_table, tok_seq, tok_pos, max_ctx=max(c for _, c in seqs), plan=plan)

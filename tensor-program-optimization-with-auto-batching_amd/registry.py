@@ -14,6 +14,7 @@ from safetensors import safe_open
 MODELS = {                    # architecture -> (module, class)
     "LlamaForCausalLM": ("llama", "LlamaForCausalLM"),
     "Safolorn": ("safolorn", "SafolornForCausalLM"),
+    "Dinasun": ("dinasun", "DinasunForCausalLM"),
 }
 
 

@@ -1,0 +1,63 @@
+"""Time mixing: a linear recurrence over a matrix state per head, with a decay per key channel that depends on the token.
+
+Every projection reads its own mix of the token's row and the previous token's.  The equations stand in csrc/time_mix.hip.
+"""
+from __future__ import annotations
+
+import dataclasses
+
+import torch
+
+from . import decoder_ops as D
+from . import ops
+from .decoder_ops import pad32, pad64, padded
+
+MIXES = ("r", "k", "v", "g", "w")
+
+
+@dataclasses.dataclass(frozen=True)
+class TimeMixSpec:
+    heads: int
+    dim: int
+
+    @classmethod
+    def from_config(cls, c: dict) -> "TimeMixSpec":
+        return cls(int(c["heads"]), int(c["dim"]))
+
+
+class TimeMix:
+    """Weights of one layer in kernel order."""
+
+    def __init__(self, spec: TimeMixSpec, w: dict, width: int, eps: float, dtype, device):
+        """w: mu.r .. mu.w [width], r, k, v, g [H dim, width], w1 [rank, width], w2 [H dim, rank], w0 [H dim], u [H, dim],
+        norm [H dim], o [width, H dim]."""
+        self.spec, self.eps, self.dtype = spec, float(eps), dtype
+        cols, Hp = spec.heads * spec.dim, pad64(width)
+        self.out_cols = pad64(cols)
+        t = lambda n: w[n].to(device, dtype)
+        self.mu = torch.stack([padded(t("mu." + s), Hp) for s in MIXES]).contiguous()
+        self.proj = {s: D.weight(padded(t(s), self.out_cols, Hp)) for s in "rkvg"}
+        self.rank = w["w1"].shape[0]
+        self.w1 = D.weight(padded(t("w1"), pad32(self.rank), Hp))
+        self.w2t = padded(t("w2").t(), self.rank, self.out_cols).contiguous()
+        self.w0 = w["w0"].to(device, torch.float32).contiguous()
+        self.u = w["u"].to(device, torch.float32).reshape(-1).contiguous()
+        self.norm = t("norm").contiguous()
+        self.o = D.weight(padded(t("o"), Hp, self.out_cols))
+
+    def mixes(self, T, width_p, device):
+        """Room for the five mixes of a pass: (what a stream step fills as out or out_row, the five activations)."""
+        if self.dtype == torch.float32:
+            rows = torch.empty((len(MIXES), T, width_p), dtype=self.dtype, device=device)
+            return {"out_row": rows}, list(rows)
+        n = ops.lib_of(self.dtype).mlora_frag_activation_elems(T, width_p)
+        data = torch.empty(len(MIXES) * n, dtype=self.dtype, device=device)
+        acts = [ops.FragActivation(T, width_p, device, data[i * n:(i + 1) * n]) for i in range(len(MIXES))]
+        return {"out": ops.FragActivation(T, width_p, device, data)}, acts
+
+    def run(self, mixes, state, segs, tok_seq, tok_pos):
+        """mixes: the five activations -> the gated outputs of the heads, an activation of out_cols columns; updates state."""
+        r, k, v, g = (ops.linear(m, self.proj[s]) for m, s in zip(mixes, "rkvg"))
+        z = ops.linear(mixes[4], self.w1, out_dtype=torch.float32)
+        out = D.activation(r.shape[0], self.out_cols, self.dtype, r.device)
+        return D.time_mix(r, k, v, g, z, self.rank, self.w2t, self.w0, self.u, self.norm, self.eps, state, segs, tok_seq, tok_pos, out)
