@@ -566,6 +566,47 @@ def safolorn_model(size):
     return _mod("registry").model_class(cfg).from_weights(cfg, tensors)
 
 
+DINASUN_SIZES = {       # as above: width, attention heads (key/value heads), time-mixing heads of 64, experts and the shared one's width
+    "w2048": dict(width=2048, heads=16, kv_heads=4, mix_heads=32, rank=64, experts=(64, 6, 1408), shared=2816),
+    "w4096": dict(width=4096, heads=32, kv_heads=8, mix_heads=64, rank=64, experts=(32, 4, 2752), shared=5504),
+}
+
+
+def dinasun_model(size):
+    """Random-weight Dinasun of one of DINASUN_SIZES: time mixing, attention twice over (a loop), time mixing - four layer runs,
+    each with experts."""
+    import torch
+    c = DINASUN_SIZES[size]
+    E, top, eff = c["experts"]
+    mlp = {"kind": "moe", "expert": {"ff": eff}, "router": {"experts": E, "top": top}, "shared": {"ff": c["shared"]}}
+    mix = {"type": "wkv", "mixer": {"heads": c["mix_heads"], "dim": 64}, "mlp": mlp}
+    att = {"type": "attention", "mlp": mlp, "mixer": {"heads": c["heads"], "kv_heads": c["kv_heads"], "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                                                      "q_temp": {"coef": 0.3, "every": 1024}}}
+    cfg = {"architecture": "Dinasun", "vocab": 32000, "width": c["width"], "norm": {"eps": 1e-5}, "embedding": {"scale": 8.0}, "residual_mult": 0.5,
+           "layers": [mix, att, mix], "loop": {"start": 1, "stop": 2, "times": 2}}
+    W, HD, R, Q, G = c["width"], c["mix_heads"] * 64, c["rank"], c["heads"] * 128, c["kv_heads"] * 128
+    gen = torch.Generator(device="cuda:0").manual_seed(0)
+
+    def tensors(name):
+        leaf = name.split(".", 1)[1] if name[0] == "l" and name[1].isdigit() else name
+        if leaf == "mlp.table":
+            return torch.rand((32000, E), generator=gen, device="cuda:0").topk(top, -1).indices.to(torch.int32)
+        if leaf.endswith(".alpha"):
+            return torch.tensor(0.5, device="cuda:0")
+        att = name.startswith("l1.")
+        shape = {"embed": (32000, W), "loop.in": (W, 2 * W), "mix.q": (Q, W), "mix.q.b": (Q,), "mix.k.b": (G,), "mix.q.norm": (128,),
+                 "mix.k.norm": (128,), "mix.k": (G if att else HD, W), "mix.o": (W, Q if att else HD), "mix.w1": (R, W), "mix.w2": (HD, R), "mix.w0": (HD,),
+                 "mix.u": (c["mix_heads"], 64), "mix.norm": (HD,)}.get(leaf)
+        if shape is None:
+            ff = c["shared"] if ".shared." in leaf else eff
+            shape = (W, ff) if leaf.endswith(".down") else (ff, W) if leaf.startswith("mlp.") else (HD, W) if leaf in ("mix.r", "mix.v", "mix.g") else (W,)
+        if "norm" in leaf and not leaf.endswith(".b"):
+            return torch.ones(shape, dtype=torch.bfloat16, device="cuda:0")
+        return (torch.randn(shape, generator=gen, device="cuda:0") * shape[-1] ** -0.5).to(torch.bfloat16)
+
+    return _mod("registry").model_class(cfg).from_weights(cfg, tensors)
+
+
 def safolorn_llama(size, synth, llama):
     """The Llama model of the same width, heads, dense feed-forward and depth, without adapters."""
     c = SAFOLORN_SIZES[size]
@@ -605,7 +646,8 @@ def time_decode(model, B, ctx, warmup, steps):
     dsm = _mod("decode_session")
     blocks = -(-(ctx + warmup + steps + 2) // 16)
     kv = model.create_paged_kv_cache(B, B * blocks * 16, ctx, 16, free_pages=np.random.default_rng(0).permutation(B * blocks), max_seq_len=blocks * 16)
-    for t in ([t for l in range(len(model.layers)) for t in (kv.k[l], kv.v[l])] if hasattr(kv, "k") else kv.pages):
+    for t in ([t for l in range(len(model.layers)) for t in (kv.k[l], kv.v[l])] if hasattr(kv, "k") else
+              kv.pages if hasattr(kv, "pages") else [t for e in kv.entries for t in e]):
         t.normal_()
     for b in range(B):
         kv.add_sequence(b)
@@ -624,14 +666,16 @@ def time_decode(model, B, ctx, warmup, steps):
     return (time.perf_counter() - t0) / steps
 
 
-def bench_safolorn(args, synth, llama):
-    """Prefill and decode throughput of Safolorn layers at sizes like a real model's (bfloat16, random weights), beside the
-    Llama model of the same width, heads, dense feed-forward and depth (fp16)."""
+def bench_design(args, synth, llama, design):
+    """Prefill and decode throughput of a design's layers at sizes like a real model's (bfloat16, random weights), beside the
+    Llama model of the same width, heads, dense feed-forward and depth (fp16); Dinasun's also beside Safolorn's."""
     import torch
     rows = []
+    kinds = {"safolorn": ("safolorn", "llama"), "dinasun": ("dinasun", "safolorn", "llama")}[design]
     for size in SAFOLORN_SIZES:
-        for kind in ("safolorn", "llama"):
-            model = safolorn_model(size) if kind == "safolorn" else safolorn_llama(size, synth, llama)
+        for kind in kinds:
+            model = {"dinasun": lambda: dinasun_model(size), "safolorn": lambda: safolorn_model(size),
+                     "llama": lambda: safolorn_llama(size, synth, llama)}[kind]()
             r = {"size": size, "model": kind}
             for B, P in ((8, 512), (1, 4096)):
                 r[f"prefill_{B}x{P}_tok_s"] = B * P / time_prefill(model, B, P, 3, max(2, args.steps // 4))
@@ -641,12 +685,12 @@ def bench_safolorn(args, synth, llama):
             print(json.dumps(r), file=sys.stderr, flush=True)
             del model
             torch.cuda.empty_cache()
-    key = "decode_b32_ctx512_tok_s"
+    value = next(r for r in rows if r["size"] == "w4096" and r["model"] == design)["decode_b32_ctx512_tok_s"]
     print(json.dumps({
-        "metric": "decode tok/s, Safolorn layers of width 4096, 32 requests at context 512", "value": rows[2][key], "unit": "tok/s", "n_gpus": 1,
-        "steps": args.steps, "warmup": args.warmup, "ms_per_step": 32e3 / rows[2][key], "higher_is_better": True, "scaling": "weak",
+        "metric": f"decode tok/s, {design.capitalize()} layers of width 4096, 32 requests at context 512", "value": value, "unit": "tok/s", "n_gpus": 1,
+        "steps": args.steps, "warmup": args.warmup, "ms_per_step": 32e3 / value, "higher_is_better": True, "scaling": "weak",
         "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
-        "config": {"sizes": SAFOLORN_SIZES, "layers": SAFOLORN_LAYERS, "host_loop": "hipGraph replay of the operators (Llama: of mlora_decode_step)"},
+        "config": {"sizes": SAFOLORN_SIZES if design == "safolorn" else DINASUN_SIZES, "layers": SAFOLORN_LAYERS, "host_loop": "hipGraph replay of the operators (Llama: of mlora_decode_step)"},
         "rows": rows}))
 
 
@@ -658,10 +702,10 @@ def main():
     ap.add_argument("--layers", type=int, default=32, help="model depth (32 = the benchmark configuration)")
     ap.add_argument("--batch", type=int, default=32,
                     help="c3_decode: concurrent requests (32 = the benchmark configuration; up to 64 run the native step)")
-    ap.add_argument("--workload", default="c3_decode", choices=["c3_decode", "c4_prefill", "c5_decode", "c1_generate", "safolorn"],
+    ap.add_argument("--workload", default="c3_decode", choices=["c3_decode", "c4_prefill", "c5_decode", "c1_generate", "safolorn", "dinasun"],
                     help="c3_decode is the benchmark the metric is quoted on; the other two time the prefill and the "
-                         "256-request stress configurations with the same harness; safolorn: prefill and decode of "
-                         "Safolorn layers beside Llama layers of the same size")
+                         "256-request stress configurations with the same harness; safolorn, dinasun: prefill and decode of "
+                         "that design's layers beside Llama layers of the same size")
     ap.add_argument("--shape", default="llama2_7b", choices=["llama2_7b", "llama31_8b"],
                     help="c3_decode: model shape (llama2_7b = the benchmark configuration; llama31_8b = the reference's default "
                          "model: grouped-query attention, 8 kv heads, vocabulary 128256)")
@@ -696,8 +740,8 @@ def main():
         return bench_c4_prefill(args, synth, llama)
     if args.workload == "c5_decode":
         return bench_c5_decode(args, synth, llama)
-    if args.workload == "safolorn":
-        return bench_safolorn(args, synth, llama)
+    if args.workload in ("safolorn", "dinasun"):
+        return bench_design(args, synth, llama, args.workload)
     if args.workload == "c1_generate":
         return bench_c1_generate(args, synth, llama)
     if args.probe:
