@@ -74,12 +74,25 @@ int mlora_embed_scaled(float* x, void* out_frag, void* out_row, int ld_row, cons
                        void* stream);
 
 /* Time mixing (equations at the top of time_mix.hip): a recurrence per head over a matrix state, its decay, the norm of the
- * heads' outputs and their gate.  r, k, v, g [T, ld]; z [T, ld_z] fp32, R columns (before the tanh); w2t [R, ld_w2]; w0, u fp32 and norm,
+ * heads' outputs and their gate.  r, k, v, g [T, ld]; z [T, ld_z] fp32, R columns (before the tanh); w2 [H * D, ld_w2], zero behind R; w0, u fp32 and norm,
  * each [H * D]; state [n_seq, H, D, D] fp32, updated.  segs [n_segs][4] int32 = {slot, first token, tokens, position of the first
  * token}; NULL: every token is a segment of its own (n_segs = T; a decode step).  y [T, ld_y], ld_y = H * D rounded up, zero behind H * D. */
 int mlora_time_mix(void* y, int y_layout, int ld_y, const void* r, const void* k, const void* v, const void* g, int ld, const float* z, int ld_z,
-                   int R, const void* w2t, int ld_w2, const float* w0, const float* u, const void* norm, float eps, float* state, int n_seq,
+                   int R, const void* w2, int ld_w2, const float* w0, const float* u, const void* norm, float eps, float* state, int n_seq,
                    const int32_t* segs, int n_segs, const int32_t* tok_seq, const int32_t* tok_pos, int T, int H, int D, void* stream);
+
+/* The same for prompts (bfloat16 library), in chunks on the matrix cores.  zp [T, 3, ld_zp]: tanh of the decay's low-rank projection as
+ * the sum of three elements (mlora_tanh_parts: out [T, 3, N] from xf [T, K] and packed W [N, K]); w2 [H * D, ld_zp].  ranges [n_ranges][8]
+ * int32 = {slot, first token, tokens, position of the first token, scratch state it starts from (-1: the slot's), scratch state that
+ * takes what it adds (-1: none), whether it is its sequence's last, 0}: ranges of a sequence run side by side; a sequence of several
+ * ranges has one scratch state per range and an entry in seqs [n_seqs][4] = {slot, position of its first token, first scratch state,
+ * ranges}.  scratch: n_states * H * D * (D + 1) floats. */
+int mlora_tanh_parts(void* out, const void* xf, const void* Wp, int T, int K, int N, void* stream);
+int mlora_time_mix_prompt_served(int D);
+int mlora_time_mix_prompt(void* y, int y_layout, int ld_y, const void* r, const void* k, const void* v, const void* g, int ld, const void* zp, int ld_zp,
+                          const void* w2, const float* w0, const float* u, const void* norm, float eps, float* state, int n_seq,
+                          const int32_t* ranges, int n_ranges, const int32_t* seqs, int n_seqs, float* scratch, size_t scratch_floats, int n_states,
+                          int T, int H, int D, void* stream);
 
 /* Latent attention (layouts at the top of latent_attention.hip).  mlora_latent_prep takes the token's projections qkv [T, ld]:
  * rotates the heads' query parts (columns off_rot .. + H rot) into the rows q + (t H + h) q_ld + q_off, padded to whole blocks of

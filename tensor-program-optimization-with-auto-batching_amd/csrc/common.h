@@ -76,6 +76,16 @@ __device__ __forceinline__ float wave_max(float v) {
   return v;
 }
 
+// A value of another lane of the wave's row of 16: lane i gets lane i - N's (the first N get 0), or everyone gets lane N's
+template <int N>
+__device__ __forceinline__ float row_shr(float v) {
+  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x110 + N, 0xf, 0xf, true));
+}
+template <int N>
+__device__ __forceinline__ float row_lane(float v) {
+  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x150 + N, 0xf, 0xf, false));
+}
+
 // 16-byte global load of 8 fp16 values
 __device__ __forceinline__ f16x8 ld8(const f16* p) { return *reinterpret_cast<const f16x8*>(p); }
 __device__ __forceinline__ void st8(f16* p, f16x8 v) { *reinterpret_cast<f16x8*>(p) = v; }

@@ -571,10 +571,12 @@ __global__ __launch_bounds__(LP_WAVES* WAVE, 2) void latent_prefill_kernel(Laten
       float pm = -INFINITY;
 #pragma unroll
       for (int p = 0; p < 4; ++p) {
-        st[u][p] *= c2;
         if constexpr (TIED) {
+          const float off = slope * (float)(p * 16 - lim);           // minus the slope times the distance of the lane's first key of the page
 #pragma unroll
-          for (int r = 0; r < 4; ++r) st[u][p][r] = fmaf(-slope, (float)(lim - p * 16 - r), st[u][p][r]);
+          for (int r = 0; r < 4; ++r) st[u][p][r] = fmaf(st[u][p][r], c2, off + slope * r);
+        } else {
+          st[u][p] *= c2;
         }
       }
       if (tile.w + wq + u * 16 < b * 64 + 63) {                      // uniform: the block crosses the tile's diagonal
@@ -917,31 +919,46 @@ struct TiedPrep {
   int T, H, G, D, RB;
 };
 
-constexpr int TP_VPT = 8;      // columns per lane: heads of up to 512
-// One wave per (token, head): adds the bias; a query is normed and takes its temperature, a value goes to the token's page slot
-// with the reciprocal of its root mean square.
+constexpr int TP_MAX_D = 512;
+// LN lanes per (token, head), eight columns each: adds the bias; a query is normed and takes its temperature, a value goes to the
+// token's page slot with the reciprocal of its root mean square.  VEC: whole eights of columns, 16-byte aligned.
+template <int LN, bool VEC>
 __global__ __launch_bounds__(256) void tied_prep_kernel(TiedPrep a) {
-  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  const int hh = blockIdx.y * 4 + wave, t = blockIdx.x;
-  if (hh >= a.H + a.G) return;                                       // no barrier below
+  const int d = (threadIdx.x % LN) * 8, hh = blockIdx.y * (256 / LN) + threadIdx.x / LN, t = blockIdx.x;
+  if (hh >= a.H + a.G) return;                                       // whole groups of LN lanes; no barrier below
   const int seq = a.tok_seq[t], pos = a.tok_pos[t], Dp = a.RB * 32;
-  float v[TP_VPT], ss = 0.f;
+  const float* yp = a.y + (size_t)t * a.ld + hh * a.D + d;
+  const float* bp = a.bias + hh * a.D + d;
+  f32x4 v[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}}, w[2] = {v[0], v[0]};
+  if constexpr (VEC) {
+    if (d < a.D) {
 #pragma unroll
-  for (int i = 0; i < TP_VPT; ++i) {
-    const int d = lane + i * WAVE;
-    v[i] = d < a.D ? a.y[(size_t)t * a.ld + hh * a.D + d] + a.bias[hh * a.D + d] : 0.f;
-    ss = fmaf(v[i], v[i], ss);
+      for (int i = 0; i < 2; ++i) {
+        v[i] = *reinterpret_cast<const f32x4*>(yp + 4 * i) + *reinterpret_cast<const f32x4*>(bp + 4 * i);
+        w[i] = *reinterpret_cast<const f32x4*>(a.q_norm + d + 4 * i);
+      }
+    }
+  } else {
+#pragma unroll
+    for (int e = 0; e < 8; ++e)
+      if (d + e < a.D) {
+        v[e >> 2][e & 3] = yp[e] + bp[e];
+        w[e >> 2][e & 3] = a.q_norm[d + e];
+      }
   }
-  const float inv = 1.f / sqrtf(wave_sum(ss) / (float)a.D + a.eps);
+  float ss = 0.f;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) ss = fmaf(v[e >> 2][e & 3], v[e >> 2][e & 3], ss);
+#pragma unroll
+  for (int o = LN / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, WAVE);
+  const float inv = 1.f / sqrtf(ss / (float)a.D + a.eps);
+  eltx8 o;
   if (hh < a.H) {
     float f = inv;
     if (a.temp_every > 0.f) f *= fmaf(a.temp_coef, logf(floorf((float)(pos + 1) / a.temp_every) + 1.f), 1.f);
-    elt* q = a.q + ((size_t)t * a.H + hh) * Dp;
 #pragma unroll
-    for (int i = 0; i < TP_VPT; ++i) {
-      const int d = lane + i * WAVE;
-      if (d < Dp) q[d] = (elt)(d < a.D ? v[i] * f * a.q_norm[d] : 0.f);
-    }
+    for (int e = 0; e < 8; ++e) o[e] = (elt)(v[e >> 2][e & 3] * f * w[e >> 2][e & 3]);
+    if (d < Dp) st8(a.q + ((size_t)t * a.H + hh) * Dp + d, o);
     return;
   }
   if (seq < 0 || seq >= a.n_seq || pos < 0 || pos / PAGE >= a.max_blocks) return;
@@ -949,11 +966,18 @@ __global__ __launch_bounds__(256) void tied_prep_kernel(TiedPrep a) {
   if (page < 0 || page >= a.n_pages) return;
   const int pg = page * a.G + hh - a.H;
 #pragma unroll
-  for (int i = 0; i < TP_VPT; ++i) {
-    const int d = lane + i * WAVE;
-    if (d < Dp) a.cache[latent_offset(pg, a.RB, pos % PAGE, d)] = (elt)v[i];
-  }
-  if (lane == 0) a.key_scale[(size_t)pg * PAGE + pos % PAGE] = inv;
+  for (int e = 0; e < 8; ++e) o[e] = (elt)v[e >> 2][e & 3];
+  if (d < Dp) st8(a.cache + latent_offset(pg, a.RB, pos % PAGE, d), o);
+  if (d == 0) a.key_scale[(size_t)pg * PAGE + pos % PAGE] = inv;
+}
+
+template <int LN>
+void launch_tied_prep(const TiedPrep& a, hipStream_t s) {
+  const dim3 grid(a.T, ceil_div(a.H + a.G, 256 / LN));
+  if (a.D % 8 == 0 && a.ld % 4 == 0 && (((uintptr_t)a.y | (uintptr_t)a.bias | (uintptr_t)a.q_norm) & 15) == 0)
+    hipLaunchKernelGGL((tied_prep_kernel<LN, true>), grid, dim3(256), 0, s, a);
+  else
+    hipLaunchKernelGGL((tied_prep_kernel<LN, false>), grid, dim3(256), 0, s, a);
 }
 
 #ifndef MLORA_ELT_F32
@@ -1216,15 +1240,20 @@ extern "C" int mlora_tied_prep(void* q, void* cache, float* key_scale, const flo
                                float temp_coef, float temp_every, const int32_t* block_table, int max_blocks, const int32_t* tok_seq,
                                const int32_t* tok_pos, int T, int H, int G, int D, int n_pages, int n_seq, void* stream) {
   MLORA_CHECK(q && cache && key_scale && y && bias && q_norm && block_table && tok_seq && tok_pos, MLORA_ERR_INVALID, "tied_prep: null pointer");
-  MLORA_CHECK(T >= 0 && H > 0 && G > 0 && H % G == 0 && D > 0 && D <= WAVE * TP_VPT && ld >= (H + G) * D && max_blocks > 0 && n_pages > 0 && n_seq > 0 &&
+  MLORA_CHECK(T >= 0 && H > 0 && G > 0 && H % G == 0 && D > 0 && D <= TP_MAX_D && ld >= (H + G) * D && max_blocks > 0 && n_pages > 0 && n_seq > 0 &&
                   (long)n_pages * G <= 0x7fffffffL && ceil_div(H + G, 4) <= 65535,
-              MLORA_ERR_UNSUPPORTED, "tied_prep: need whole groups of heads of at most %d columns (T=%d H=%d G=%d D=%d)", WAVE * TP_VPT, T, H, G, D);
+              MLORA_ERR_UNSUPPORTED, "tied_prep: need whole groups of heads of at most %d columns (T=%d H=%d G=%d D=%d)", TP_MAX_D, T, H, G, D);
   if (T == 0) return MLORA_OK;
   TiedPrep a;
   a.y = y; a.ld = ld; a.bias = bias; a.q_norm = q_norm; a.eps = eps; a.temp_coef = temp_coef; a.temp_every = temp_every; a.q = (elt*)q;
   a.cache = (elt*)cache; a.key_scale = key_scale; a.block_table = block_table; a.max_blocks = max_blocks; a.n_pages = n_pages; a.n_seq = n_seq;
   a.tok_seq = tok_seq; a.tok_pos = tok_pos; a.T = T; a.H = H; a.G = G; a.D = D; a.RB = ceil_div(D, 32);
-  hipLaunchKernelGGL(tied_prep_kernel, dim3(T, ceil_div(H + G, 4)), dim3(256), 0, (hipStream_t)stream, a);
+  hipStream_t s = (hipStream_t)stream;
+  if (D <= 32) launch_tied_prep<4>(a, s);
+  else if (D <= 64) launch_tied_prep<8>(a, s);
+  else if (D <= 128) launch_tied_prep<16>(a, s);
+  else if (D <= 256) launch_tied_prep<32>(a, s);
+  else launch_tied_prep<64>(a, s);
   return mlora_launch_status("tied_prep");
 }
 

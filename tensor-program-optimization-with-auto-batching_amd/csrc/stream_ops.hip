@@ -107,13 +107,52 @@ __device__ __forceinline__ float gelu_tanh(float z) {
 }
 
 #ifndef MLORA_ELT_F32
-// out[t, n] = gelu(sum_k W[n, k] x[t, k]) * table[id_t, col0 + n] for n < dim, 0 for the padding rows; x and out in fragment
-// order.  A workgroup takes 16 TT tokens x 16 NT rows, its waves split K; a wave requests TG_U k-steps at a time.
+// What becomes of four rows n .. n + 3 of a token's narrow product s = W x:
+//   token gate: out[t, n] = gelu(s) * table[id_t, col0 + n] for n < dim, 0 for the padding rows, in fragment order
+struct TokenGate {
+  elt* out;
+  const elt* table;
+  int ld_table, col0, dim;
+  const int32_t* ids;
+  int V;
+  __device__ __forceinline__ void operator()(int t, int n, f32x4 s, int frag_tt) const {
+    const int id = ids[t];
+    const bool ok = id >= 0 && id < V;
+    eltx4 o;
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      const float ev = ok && n + q < dim ? (float)table[(size_t)id * ld_table + col0 + n + q] : 0.f;
+      o[q] = (elt)(gelu_tanh(s[q]) * ev);
+    }
+    *reinterpret_cast<eltx4*>(out + frag_offset(t, n, frag_tt)) = o;
+  }
+};
+//   tanh(s) in full precision as the sum of three elements, out [T][3][N]
+struct TanhParts {
+  elt* out;
+  int N;
+  __device__ __forceinline__ void operator()(int t, int n, f32x4 s, int) const {
+    eltx4 o[3];
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      float v = tanhf(s[q]);
+#pragma unroll
+      for (int p = 0; p < 3; ++p) {
+        o[p][q] = (elt)v;
+        v -= (float)o[p][q];
+      }
+    }
+#pragma unroll
+    for (int p = 0; p < 3; ++p) *reinterpret_cast<eltx4*>(out + ((size_t)t * 3 + p) * N + n) = o[p];
+  }
+};
+
+// The narrow product of a token block: x in fragment order, W packed.  A workgroup takes 16 TT tokens x 16 NT rows, its waves split
+// K; a wave requests TG_U k-steps at a time.
 constexpr int TG_WAVES = 8;
-template <int NT, int TT, int TG_U>
-__global__ __launch_bounds__(TG_WAVES* WAVE, 2) void token_gate_kernel(elt* __restrict__ out, int frag_tt, const elt* __restrict__ x,
-                                                                      const elt* __restrict__ Wp, const elt* __restrict__ table, int ld_table,
-                                                                      int col0, int dim, const int32_t* __restrict__ ids, int V, int T, int K, int N) {
+template <int NT, int TT, int TG_U, typename END>
+__global__ __launch_bounds__(TG_WAVES* WAVE, 2) void token_gate_kernel(END end, int frag_tt, const elt* __restrict__ x, const elt* __restrict__ Wp, int T,
+                                                                      int K, int N) {
   __shared__ f32x4 red[TG_WAVES][NT][WAVE];
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
   const int KB = K / 32, tiles = N / 16;
@@ -163,17 +202,21 @@ __global__ __launch_bounds__(TG_WAVES* WAVE, 2) void token_gate_kernel(elt* __re
       f32x4 s = red[0][i][sl];
 #pragma unroll
       for (int w = 1; w < TG_WAVES; ++w) s += red[w][i][sl];
-      const int id = ids[t];
-      const bool ok = id >= 0 && id < V;
-      eltx4 o;
-#pragma unroll
-      for (int q = 0; q < 4; ++q) {
-        const float ev = ok && n + q < dim ? (float)table[(size_t)id * ld_table + col0 + n + q] : 0.f;
-        o[q] = (elt)(gelu_tanh(s[q]) * ev);
-      }
-      *reinterpret_cast<eltx4*>(out + frag_offset(t, n, frag_tt)) = o;
+      end(t, n, s, frag_tt);
     }
   }
+}
+
+template <typename END>
+void launch_narrow(const END& end, const void* xf, const void* Wp, int T, int K, int N, hipStream_t s) {
+#define MLORA_TG(NT, TT, U)                                                                                                                    \
+  hipLaunchKernelGGL((token_gate_kernel<NT, TT, U, END>), dim3(ceil_div(N, 16 * NT), ceil_div(T, 16 * TT)), dim3(TG_WAVES * WAVE), 0, s, end, \
+                     mlora_frag_tiles(T), (const elt*)xf, (const elt*)Wp, T, K, N)
+  if (T <= 256) MLORA_TG(1, 1, 4);
+  else if (N <= 32) MLORA_TG(2, 1, 4);
+  else if ((long)ceil_div(N, 64) * ceil_div(T, 64) >= 256) MLORA_TG(4, 4, 2);      // a workgroup per compute unit with four token tiles
+  else MLORA_TG(4, 1, 4);
+#undef MLORA_TG
 }
 #endif
 
@@ -199,6 +242,18 @@ __device__ __forceinline__ f32x4 ld4f(const elt* p) {
   return f32x4{(float)v[0], (float)v[1], (float)v[2], (float)v[3]};
 }
 
+// tanh to fp32 accuracy on the fast reciprocal and exponential: 1 - 2 / (exp(2 |x|) + 1), and its series where that cancels
+__device__ __forceinline__ float tanh_f(float x) {
+#ifdef MLORA_ELT_F32
+  return tanhf(x);
+#else
+  const float a = fabsf(x), x2 = x * x;
+  const float big = fmaf(-2.f, __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(a * 2.88539008177792681472f)), 1.f);
+  const float small = fmaf(x2 * x, fmaf(x2, fmaf(x2, fmaf(x2, 62.f / 2835.f, -17.f / 315.f), 2.f / 15.f), -1.f / 3.f), x);
+  return a < 0.25f ? small : copysignf(big, x);
+#endif
+}
+
 struct TanhNorm {
   f32x4 w, b;
   float alpha;
@@ -210,7 +265,7 @@ struct TanhNorm {
   __device__ __forceinline__ f32x4 operator()(f32x4 v) const {
     if (!on) return v;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) v[e] = fmaf(tanhf(alpha * v[e]), w[e], b[e]);
+    for (int e = 0; e < 4; ++e) v[e] = fmaf(tanh_f(alpha * v[e]), w[e], b[e]);
     return v;
   }
 };
@@ -285,6 +340,143 @@ __global__ __launch_bounds__(ST_THREADS) void stream_step_kernel(mlora_stream_st
   }
 }
 
+#ifndef MLORA_ELT_F32
+struct F8 {
+  f32x4 v[2];
+};
+__device__ __forceinline__ F8 ld8f(const float* p) { return F8{{*reinterpret_cast<const f32x4*>(p), *reinterpret_cast<const f32x4*>(p + 4)}}; }
+struct TanhNorm8 {          // weights as elements: they stay in registers over many tokens
+  eltx8 w, b;
+  float alpha;
+  bool on;
+  __device__ __forceinline__ TanhNorm8(const mlora_tanh_norm& n, int c) : alpha(n.alpha), on(n.w != nullptr) {
+    w = b = eltx8{0, 0, 0, 0, 0, 0, 0, 0};
+    if (on) {
+      w = ld8((const elt*)n.w + c);
+      b = ld8((const elt*)n.b + c);
+    }
+  }
+  __device__ __forceinline__ F8 operator()(F8 x) const {
+    if (!on) return x;                                               // uniform
+#pragma unroll
+    for (int e = 0; e < 8; ++e) x.v[e >> 2][e & 3] = fmaf(tanh_f(alpha * x.v[e >> 2][e & 3]), (float)w[e], (float)b[e]);
+    return x;
+  }
+};
+
+// one token's eight columns of x + mult post(branch)
+__device__ __forceinline__ F8 step_row8(const mlora_stream_step_args& a, const TanhNorm8& post, int t, int c) {
+  const size_t o = (size_t)t * a.Hp + c;
+  F8 x = F8{{f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}}}, v = x;
+  if (a.x) x = ld8f(a.x + o);
+  if (!a.y && !a.rows) return x;
+  if (a.y) v = ld8f(a.y + o);
+  for (int q = 0; q < a.n_part; ++q) {
+    const F8 p = ld8f(a.part + (size_t)q * a.T * a.Hp + o);
+    v.v[0] += p.v[0];
+    v.v[1] += p.v[1];
+  }
+  if (a.rows) {
+    const elt* rp = (const elt*)a.rows + (size_t)t * a.top * a.Hp + c;
+    F8 s = F8{{f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}}};
+    for (int k0 = 0; k0 < a.top; k0 += 4) {                          // four rows are requested together
+      eltx8 r[4];
+#pragma unroll
+      for (int k = 0; k < 4; ++k) r[k] = ld8(rp + (size_t)(k0 + k < a.top ? k0 + k : k0) * a.Hp);
+#pragma unroll
+      for (int k = 0; k < 4; ++k) {
+        const float f = k0 + k < a.top ? 1.f : 0.f;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) s.v[e >> 2][e & 3] = fmaf(f, (float)r[k][e], s.v[e >> 2][e & 3]);
+      }
+    }
+    v.v[0] += s.v[0] * a.row_weight;
+    v.v[1] += s.v[1] * a.row_weight;
+  }
+  v = post(v);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) x.v[e >> 2][e & 3] = fmaf(a.mult, v.v[e >> 2][e & 3], x.v[e >> 2][e & 3]);
+  return x;
+}
+
+// The same with outputs in fragment order: a wave takes 32 columns of `tiles` tiles of 16 tokens - lane (token q16, columns
+// 8 g ..) - so that it reads whole lines of the stream and writes whole fragments, and a token's neighbour is the lane beside it.
+template <bool SHIFT>
+__global__ __launch_bounds__(256) void stream_step_tile_kernel(mlora_stream_step_args a, int tiles, int frag_tt) {
+  const int lane = threadIdx.x & 63, q16 = lane & 15, g = lane >> 4;
+  const int ks = blockIdx.x * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), c = ks * 32 + g * 8;
+  if (ks * 32 >= a.Hp) return;                                       // uniform; no barrier below
+  const TanhNorm8 post(a.post, c), pre(a.pre, c);
+  eltx8 mu[SHIFT ? ST_MIX : 1];
+  if constexpr (SHIFT) {
+#pragma unroll
+    for (int s = 0; s < ST_MIX; ++s) mu[s] = ld8((const elt*)a.mu + (size_t)s * a.Hp + c);
+  }
+  F8 carry = F8{{f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}}};      // the row ahead of the tile
+  bool carried = false;                                              // uniform
+  const int tile0 = blockIdx.y * tiles;
+  for (int i = 0; i < tiles; ++i) {
+    const int t0 = (tile0 + i) * 16, t = t0 + q16;
+    if (t0 >= a.T) return;                                           // uniform
+    const bool in = t < a.T;
+    const int tc = in ? t : a.T - 1;
+    const F8 x = step_row8(a, post, tc, c);
+    if (a.x_out && in) {
+      f32x4* p = reinterpret_cast<f32x4*>(a.x_out + (size_t)t * a.Hp + c);
+      p[0] = x.v[0];
+      p[1] = x.v[1];
+    }
+    const F8 h = pre(x);
+    elt* fp = (elt*)a.out_frag + ((size_t)ks * frag_tt + tile0 + i) * 512 + g * 128 + q16 * 8;   // exists also for the tile's tokens behind T
+    if constexpr (SHIFT) {
+      const int seq = a.tok_seq[tc], pos = a.tok_pos[tc];
+      const int seq_p = tc > 0 ? a.tok_seq[tc - 1] : -1;
+      const bool live = in && seq >= 0 && seq < a.n_seq, cont = tc > 0 && seq_p == seq;
+      F8 prev;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const float p = row_shr<1>(h.v[e >> 2][e & 3]);
+        prev.v[e >> 2][e & 3] = q16 > 0 ? p : carry.v[e >> 2][e & 3];
+      }
+      if (in && q16 == 0 && cont && pos > 0 && !carried) prev = pre(step_row8(a, post, t - 1, c));     // it belongs to another workgroup
+      if (in && !cont && pos > 0) {
+        prev = F8{{f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}}};
+        if (live) prev = ld8f(a.shift + (size_t)seq * a.Hp + c);
+      }
+      if (pos <= 0) prev = F8{{f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}}};
+      if (live && !cont) {
+        // the sequence's first token of the pass read the state; it also leaves the last one's row there
+        int last = a.tok_last ? a.tok_last[t] : t;
+        last = last < a.T ? last : a.T - 1;
+        const F8 l = last > t ? pre(step_row8(a, post, last, c)) : h;
+        f32x4* p = reinterpret_cast<f32x4*>(a.shift + (size_t)seq * a.Hp + c);
+        p[0] = l.v[0];
+        p[1] = l.v[1];
+      }
+#pragma unroll
+      for (int s = 0; s < ST_MIX; ++s) {
+        eltx8 o;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          const float hv = h.v[e >> 2][e & 3];
+          o[e] = (elt)fmaf(prev.v[e >> 2][e & 3] - hv, (float)mu[s][e], hv);
+        }
+        st8(fp + s * (size_t)a.mix_stride, o);
+      }
+#pragma unroll
+      for (int e = 0; e < 8; ++e) carry.v[e >> 2][e & 3] = row_lane<15>(h.v[e >> 2][e & 3]);
+      carried = true;
+    } else {
+      eltx8 o;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) o[e] = (elt)h.v[e >> 2][e & 3];
+      st8(fp, o);
+      if (a.out_row && in) st8((elt*)a.out_row + (size_t)t * a.ld_row + c, o);
+    }
+  }
+}
+#endif
+
 // x = table[id] * scale in fp32, and the same rounded, in fragment order or with a row stride of its own
 __global__ __launch_bounds__(256) void embed_scaled_kernel(float* __restrict__ x, elt* __restrict__ out_frag, int frag_tt, elt* __restrict__ out_row,
                                                            int ld_row, const elt* __restrict__ table, const int32_t* __restrict__ ids, float scale,
@@ -330,16 +522,17 @@ extern "C" int mlora_token_gate(void* out_frag, const void* xf, const void* Wp, 
                   ceil_div(T, 16) <= 65535,
               MLORA_ERR_UNSUPPORTED, "token_gate: need K %% 32 == 0, N %% 32 == 0, dim <= N (T=%d K=%d N=%d dim=%d)", T, K, N, dim);
   if (T == 0) return MLORA_OK;
-  hipStream_t s = (hipStream_t)stream;
-#define MLORA_TG(NT, TT, U)                                                                                                        \
-  hipLaunchKernelGGL((token_gate_kernel<NT, TT, U>), dim3(ceil_div(N, 16 * NT), ceil_div(T, 16 * TT)), dim3(TG_WAVES * WAVE), 0, s, \
-                     (elt*)out_frag, mlora_frag_tiles(T), (const elt*)xf, (const elt*)Wp, (const elt*)table, ld_table, col0, dim, ids, V, T, K, N)
-  if (T <= 256) MLORA_TG(1, 1, 4);
-  else if (N <= 32) MLORA_TG(2, 1, 4);
-  else if ((long)ceil_div(N, 64) * ceil_div(T, 64) >= 256) MLORA_TG(4, 4, 2);      // a workgroup per compute unit with four token tiles
-  else MLORA_TG(4, 1, 4);
-#undef MLORA_TG
+  launch_narrow(TokenGate{(elt*)out_frag, (const elt*)table, ld_table, col0, dim, ids, V}, xf, Wp, T, K, N, (hipStream_t)stream);
   return mlora_launch_status("token_gate");
+}
+
+extern "C" int mlora_tanh_parts(void* out, const void* xf, const void* Wp, int T, int K, int N, void* stream) {
+  MLORA_CHECK(out && xf && Wp, MLORA_ERR_INVALID, "tanh_parts: null pointer");
+  MLORA_CHECK(T >= 0 && K > 0 && K % 32 == 0 && N > 0 && N % 32 == 0 && ceil_div(T, 16) <= 65535, MLORA_ERR_UNSUPPORTED,
+              "tanh_parts: need K %% 32 == 0, N %% 32 == 0 (T=%d K=%d N=%d)", T, K, N);
+  if (T == 0) return MLORA_OK;
+  launch_narrow(TanhParts{(elt*)out, N}, xf, Wp, T, K, N, (hipStream_t)stream);
+  return mlora_launch_status("tanh_parts");
 }
 #endif
 
@@ -368,7 +561,20 @@ extern "C" int mlora_stream_step(const mlora_stream_step_args* args, void* strea
                 "stream_step: the mixes need the state, the tokens' sequences and a stream that is not updated in place");
   if (a.T == 0) return MLORA_OK;
   hipStream_t s = (hipStream_t)stream;
-  const int cols = ceil_div(a.Hp, ST_THREADS * 4), tt = mlora_frag_tiles(a.T);
+  const int tt = mlora_frag_tiles(a.T);
+#ifndef MLORA_ELT_F32
+  if (a.out_frag && !(a.mu && a.out_row) && a.ld_row % 8 == 0) {
+    const int cb = ceil_div(a.Hp, 128), nt = ceil_div(a.T, 16);
+    int tiles = 1;
+    while (tiles < 8 && (long)cb * ceil_div(nt, 2 * tiles) >= 1024) tiles *= 2;
+    while (ceil_div(nt, tiles) > 65535) tiles *= 2;
+    const dim3 grid(cb, ceil_div(nt, tiles));
+    if (a.mu) hipLaunchKernelGGL(stream_step_tile_kernel<true>, grid, dim3(256), 0, s, a, tiles, tt);
+    else hipLaunchKernelGGL(stream_step_tile_kernel<false>, grid, dim3(256), 0, s, a, tiles, tt);
+    return mlora_launch_status("stream_step");
+  }
+#endif
+  const int cols = ceil_div(a.Hp, ST_THREADS * 4);
   int rows = 1;
   while (rows < 8 && (long)cols * ceil_div(a.T, 2 * rows) >= 2048) rows *= 2;
   while (ceil_div(a.T, rows) > 65535) rows *= 2;

@@ -242,7 +242,7 @@ def gate_up_silu(x, W, W_il, out):
     return silu_mul(ops.linear(x, W), out)
 
 
-def time_mix(r, k, v, g, z, R, w2t, w0, u, norm, eps, state, segs, tok_seq, tok_pos, out):
+def time_mix(r, k, v, g, z, R, w2, w0, u, norm, eps, state, segs, tok_seq, tok_pos, out):
     """The recurrence of time mixing (csrc/time_mix.hip) over a pass: r, k, v, g [T, ld], z [T, >= R] fp32, state [n, H, D, D] fp32
     (updated), segs [n][4] int32 or None (a decode step) -> out, an activation [T, H * D rounded up]."""
     T, ld = r.shape
@@ -250,9 +250,53 @@ def time_mix(r, k, v, g, z, R, w2t, w0, u, norm, eps, state, segs, tok_seq, tok_
     frag = isinstance(out, FragActivation)
     check(lib_of(r.dtype).mlora_time_mix(out.data.data_ptr() if frag else _dev(out, r.dtype), FRAG if frag else ROWMAJOR, out.shape[1],
                                          _dev(r), _dev(k, r.dtype), _dev(v, r.dtype), _dev(g, r.dtype), ld, _dev(z, torch.float32), z.shape[1], R,
-                                         _dev(w2t, r.dtype), w2t.shape[1], _dev(w0, torch.float32), _dev(u, torch.float32), _dev(norm, r.dtype), eps,
+                                         _dev(w2, r.dtype), w2.shape[1], _dev(w0, torch.float32), _dev(u, torch.float32), _dev(norm, r.dtype), eps,
                                          _dev(state, torch.float32), n_seq, _ptr(segs), T if segs is None else segs.shape[0],
                                          _dev(tok_seq, torch.int32), _dev(tok_pos, torch.int32), T, H, D, _stream()), r.dtype)
+    return out
+
+
+class TimeMixPlan:
+    """Ranges of a pass for `time_mix_prompt`: segs, per sequence (slot, first token, tokens, position of the first); tokens: of a
+    range (chosen by the size of the pass)."""
+
+    def __init__(self, segs, heads, device, tokens=None):
+        if tokens is None:                                           # about four workgroups per compute unit
+            tokens = min(max(1 << max(sum(n for _, _, n, _ in segs) * heads // 1024, 1).bit_length() - 1, 64), 256)
+        ranges, seqs, self.n_states = [], [], 0
+        for slot, first, n, pos in segs:
+            parts = -(-n // tokens)
+            if parts > 1:
+                seqs.append((slot, pos, self.n_states, parts))
+            for c in range(parts):
+                at, end = c * tokens, c == parts - 1
+                ranges.append((slot, first + at, min(tokens, n - at), pos + at, self.n_states + c if parts > 1 else -1, -1 if end else self.n_states + c, int(end), 0))
+            if parts > 1:
+                self.n_states += parts
+        self.n_ranges, self.n_seqs = len(ranges), len(seqs)
+        both = torch.tensor([x for t in (*ranges, *seqs) for x in t], dtype=torch.int32).to(device)
+        self.ranges, self.seqs = both[: 8 * len(ranges)], both[8 * len(ranges):]
+
+
+def time_mix_prompt_served(dim) -> bool:
+    return bool(lib_of(torch.bfloat16).mlora_time_mix_prompt_served(dim))
+
+
+def time_mix_prompt(plan, r, k, v, g, mix, w1, w2, w0, u, norm, eps, state, out):
+    """time_mix for a pass over prompts; mix: the activation that the decay's low-rank projection w1 takes."""
+    T, ld = r.shape
+    n_seq, H, D, _ = state.shape
+    L = lib_of(r.dtype)
+    N = w1.shape[0]
+    zp = torch.empty((T, 3, N), dtype=r.dtype, device=r.device)
+    check(L.mlora_tanh_parts(zp.data_ptr(), mix.data.data_ptr(), _wptr(w1), T, mix.shape[1], N, _stream()), r.dtype)
+    n = plan.n_states * H * D * (D + 1)
+    scratch = torch.empty(n, dtype=torch.float32, device=r.device) if n else None
+    frag = isinstance(out, FragActivation)
+    check(L.mlora_time_mix_prompt(out.data.data_ptr() if frag else _dev(out, r.dtype), FRAG if frag else ROWMAJOR, out.shape[1], _dev(r), _dev(k, r.dtype),
+                                  _dev(v, r.dtype), _dev(g, r.dtype), ld, zp.data_ptr(), N, _dev(w2, r.dtype), _dev(w0, torch.float32),
+                                  _dev(u, torch.float32), _dev(norm, r.dtype), eps, _dev(state, torch.float32), n_seq, plan.ranges.data_ptr(),
+                                  plan.n_ranges, plan.seqs.data_ptr(), plan.n_seqs, _ptr(scratch), n, plan.n_states, T, H, D, _stream()), r.dtype)
     return out
 
 

@@ -19,7 +19,7 @@ import numpy as np
 import torch
 
 from . import ops
-from .decoder_ops import PrefillPlan
+from .decoder_ops import PrefillPlan, TimeMixPlan
 
 PAGE = 16
 
@@ -248,15 +248,15 @@ class PagedStateCache(PageTable):
 
     def _pass(self):
         """Of the current pass, made once for all its layers: {"last": the last token of every token's sequence, "segs": [n][4]
-        {slot, first token, tokens, position}} - both None in a decode step - and the plan of its prompt form, if taken."""
+        {slot, first token, tokens, position}} - both None in a decode step - and the plans of the prompt forms, once taken."""
         if self._cur is None:
             raise RuntimeError("outside begin_forward/end_forward")
         if self._meta is None or self._meta[0] is not self._cur:
             seq_ids, lens, decode = self._cur[:3]
-            m = {"last": None, "segs": None, "plan": None}
+            m = {"last": None, "segs": None, "plan": None, "ranges": {}, "host": None}
             if not decode:
                 ends = np.cumsum(lens)
-                segs = [(self.slot[s], e - n, n, self.lens[s]) for s, n, e in zip(seq_ids, lens, ends)]
+                m["host"] = segs = [(self.slot[s], int(e) - n, n, self.lens[s]) for s, n, e in zip(seq_ids, lens, ends)]
                 both = np.concatenate([np.asarray(segs, dtype=np.int32).reshape(-1), np.repeat(ends - 1, lens).astype(np.int32)])
                 both = torch.from_numpy(both).to(self.device)
                 m["segs"], m["last"] = both[: 4 * len(segs)].view(-1, 4), both[4 * len(segs):]
@@ -269,7 +269,12 @@ class PagedStateCache(PageTable):
 
     def time_mix(self, run, mixes, mixer):
         """The recurrence of a layer run on the five mixes of the pass (mixer: time_mix.TimeMix)."""
-        return mixer.run(mixes, self.entries[run][0], self._pass()["segs"], self._cur[3], self._cur[4])
+        m, plan, heads = self._pass(), None, mixer.spec.heads
+        if m["host"] is not None and mixer.prompt_form:
+            if heads not in m["ranges"]:
+                m["ranges"][heads] = TimeMixPlan(m["host"], heads, self.device)
+            plan = m["ranges"][heads]
+        return mixer.run(mixes, self.entries[run][0], m["segs"], self._cur[3], self._cur[4], plan)
 
     def tied_attention(self, run, y, att):
         """The attention of a layer run behind its input projection y (att: tied_attention.TiedAttention)."""

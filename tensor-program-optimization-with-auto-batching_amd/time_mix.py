@@ -39,11 +39,12 @@ class TimeMix:
         self.proj = {s: D.weight(padded(t(s), self.out_cols, Hp)) for s in "rkvg"}
         self.rank = w["w1"].shape[0]
         self.w1 = D.weight(padded(t("w1"), pad32(self.rank), Hp))
-        self.w2t = padded(t("w2").t(), self.rank, self.out_cols).contiguous()
+        self.w2 = padded(t("w2"), cols, pad32(self.rank)).contiguous()
         self.w0 = w["w0"].to(device, torch.float32).contiguous()
         self.u = w["u"].to(device, torch.float32).reshape(-1).contiguous()
         self.norm = t("norm").contiguous()
         self.o = D.weight(padded(t("o"), Hp, self.out_cols))
+        self.prompt_form = dtype != torch.float32 and D.time_mix_prompt_served(spec.dim)
 
     def mixes(self, T, width_p, device):
         """Room for the five mixes of a pass: (what a stream step fills as out or out_row, the five activations)."""
@@ -55,9 +56,13 @@ class TimeMix:
         acts = [ops.FragActivation(T, width_p, device, data[i * n:(i + 1) * n]) for i in range(len(MIXES))]
         return {"out": ops.FragActivation(T, width_p, device, data)}, acts
 
-    def run(self, mixes, state, segs, tok_seq, tok_pos):
-        """mixes: the five activations -> the gated outputs of the heads, an activation of out_cols columns; updates state."""
+    def run(self, mixes, state, segs, tok_seq, tok_pos, plan=None):
+        """mixes: the five activations -> the gated outputs of the heads, an activation of out_cols columns; updates state.
+        segs: the sequences of the pass (None: a decode step); plan: a TimeMixPlan of the pass for the prompt form."""
         r, k, v, g = (ops.linear(m, self.proj[s]) for m, s in zip(mixes, "rkvg"))
-        z = ops.linear(mixes[4], self.w1, out_dtype=torch.float32)
         out = D.activation(r.shape[0], self.out_cols, self.dtype, r.device)
-        return D.time_mix(r, k, v, g, z, self.rank, self.w2t, self.w0, self.u, self.norm, self.eps, state, segs, tok_seq, tok_pos, out)
+        rest = (self.w2, self.w0, self.u, self.norm, self.eps, state)
+        if plan is not None:
+            return D.time_mix_prompt(plan, r, k, v, g, mixes[4], self.w1, *rest, out)
+        z = ops.linear(mixes[4], self.w1, out_dtype=torch.float32)
+        return D.time_mix(r, k, v, g, z, self.rank, *rest, segs, tok_seq, tok_pos, out)

@@ -124,7 +124,15 @@ def mix_case(D, rng, dt, T, H, Dm, Rk):
     u, norm = rnd(rng, H * Dm), rnd(rng, H * Dm, dt=dt)
     w = np.exp(-np.exp(np.tanh(f64(z)[:, :Rk]) @ f64(w2).T + f64(w0)))
     cut = lambda a: f64(a)[:, : H * Dm].reshape(T, H, Dm)
-    return t, z, D.padded(w2.t(), Rk, ld).contiguous(), w0, u, norm, (cut(t["r"]), cut(t["k"]), cut(t["v"]), w.reshape(T, H, Dm)), f64(u).reshape(H, Dm)
+    return t, z, D.padded(w2, H * Dm, D.pad32(Rk)).contiguous(), w0, u, norm, (cut(t["r"]), cut(t["k"]), cut(t["v"]), w.reshape(T, H, Dm)), f64(u).reshape(H, Dm)
+
+
+def mix_prompt(D, ops, plan, t, z, Rk, *rest):
+    """The prompt form on given projections: the low-rank product is with the identity."""
+    n = z.shape[1]
+    eye = torch.zeros((n, n), dtype=torch.bfloat16, device=DEV)
+    eye[:Rk, :Rk] = torch.eye(Rk)
+    return D.time_mix_prompt(plan, t["r"], t["k"], t["v"], t["g"], ops.FragActivation.pack(z.to(torch.bfloat16)), D.weight(eye), *rest)
 
 
 def mix_want(ref, u, gate, norm, H, Dm, eps, S):
@@ -143,7 +151,7 @@ def test_time_mix(D, ops, dt, H, Dm, Rk, case):
     segs = MIX_SEGS[case]
     rng = np.random.default_rng(H * Dm + case)
     T, n = sum(c for c, _ in segs), len(segs)
-    t, z, w2t, w0, u, norm, ref, uu = mix_case(D, rng, dt, T, H, Dm, Rk)
+    t, z, w2, w0, u, norm, ref, uu = mix_case(D, rng, dt, T, H, Dm, Rk)
     slots = rng.permutation(n + 1)[:n]
     state0 = rnd(rng, n + 1, H, Dm, Dm, std=3.0)
     state = state0.clone()
@@ -152,7 +160,7 @@ def test_time_mix(D, ops, dt, H, Dm, Rk, case):
     decode = all(c == 1 for c, _ in segs)
     seg = None if decode else i32([(s, a, c, p) for s, a, (c, p) in zip(slots, starts, segs)])
     seq, pos = np.repeat(slots, [c for c, _ in segs]), np.concatenate([p + np.arange(c) for c, p in segs])
-    D.time_mix(t["r"], t["k"], t["v"], t["g"], z, Rk, w2t, w0, u, norm, 1e-4, state, seg, i32(seq), i32(pos), out)
+    D.time_mix(t["r"], t["k"], t["v"], t["g"], z, Rk, w2, w0, u, norm, 1e-4, state, seg, i32(seq), i32(pos), out)
     torch.cuda.synchronize()
     got = rows_of(out)
     assert float(got[:, H * Dm:].abs().sum()) == 0
@@ -165,20 +173,47 @@ def test_time_mix(D, ops, dt, H, Dm, Rk, case):
     assert torch.equal(state[idle], state0[idle])
 
 
+@pytest.mark.parametrize("H,Dm,Rk", [(3, 24, 5), (1, 64, 70), (2, 40, 16), (2, 128, 33), (1, 30, 8), (4, 64, 64), (2, 16, 130), (1, 100, 20)])
+@pytest.mark.parametrize("case", range(len(MIX_SEGS)))
+@pytest.mark.parametrize("tokens", [None, 16, 48])
+def test_time_mix_prompt(D, ops, H, Dm, Rk, case, tokens):
+    """The chunked form: the same segments, in ranges side by side (cut where the plan cuts them, and shorter)."""
+    segs, dt = MIX_SEGS[case], torch.bfloat16
+    rng = np.random.default_rng(H * Dm + case)
+    T, n = sum(c for c, _ in segs), len(segs)
+    t, z, w2, w0, u, norm, ref, uu = mix_case(D, rng, dt, T, H, Dm, Rk)
+    slots = [int(s) for s in rng.permutation(n + 1)[:n]]
+    state0 = rnd(rng, n + 1, H, Dm, Dm, std=3.0)
+    state, out = state0.clone(), D.activation(T, D.pad64(H * Dm), dt, DEV)
+    starts = np.cumsum([0] + [c for c, _ in segs])[:-1].tolist()
+    plan = D.TimeMixPlan([(s, a, c, p) for s, a, (c, p) in zip(slots, starts, segs)], H, DEV, tokens)
+    mix_prompt(D, ops, plan, t, z, Rk, w2, w0, u, norm, 1e-4, state, out)
+    torch.cuda.synchronize()
+    got = rows_of(out)
+    assert float(got[:, H * Dm:].abs().sum()) == 0
+    for s, a, (c, p) in zip(slots, starts, segs):
+        part = [x[a:a + c] for x in ref]
+        want, S = mix_want(part, uu, f64(t["g"])[a:a + c, : H * Dm], f64(norm), H, Dm, 1e-4, f64(state0)[s] if p else None)
+        assert err(got[a:a + c, : H * Dm], want) < 6e-3, (c, p)
+        assert err(state[s], S) < 4e-5, (c, p)
+    idle = [s for s in range(n + 1) if s not in slots]
+    assert torch.equal(state[idle], state0[idle])
+
+
 @pytest.mark.parametrize("dt", DTYPES)
 @pytest.mark.parametrize("sizes", [[2], [1], [70, 3], [64], [65, 31, 128]])
 def test_time_mix_in_portions(D, ops, dt, sizes):
     """However a sequence is cut, outputs and final state are those of the whole."""
     H, Dm, Rk, T = 2, 64, 12, 300
     rng = np.random.default_rng(7)
-    t, z, w2t, w0, u, norm, ref, uu = mix_case(D, rng, dt, T, H, Dm, Rk)
+    t, z, w2, w0, u, norm, ref, uu = mix_case(D, rng, dt, T, H, Dm, Rk)
     want, S = mix_want(ref, uu, f64(t["g"])[:, : H * Dm], f64(norm), H, Dm, 1e-4, None)
     state, at, i, outs = rnd(rng, 2, H, Dm, Dm), 0, 0, []
     while at < T:
         c = min(sizes[i % len(sizes)], T - at)
         sl = lambda a: a[at:at + c].contiguous()
         out = D.activation(c, D.pad64(H * Dm), dt, DEV)
-        D.time_mix(sl(t["r"]), sl(t["k"]), sl(t["v"]), sl(t["g"]), sl(z), Rk, w2t, w0, u, norm, 1e-4, state, None if c == 1 else i32([[1, 0, c, at]]),
+        D.time_mix(sl(t["r"]), sl(t["k"]), sl(t["v"]), sl(t["g"]), sl(z), Rk, w2, w0, u, norm, 1e-4, state, None if c == 1 else i32([[1, 0, c, at]]),
                    i32([1] * c), i32(at + np.arange(c)), out)
         outs.append(rows_of(out))
         at, i = at + c, i + 1
@@ -192,23 +227,28 @@ def test_time_mix_decays_of_any_strength(D, ops, dt, w0):
     """From none (everything is kept) to total within a token: no overflow, no loss of what is kept."""
     H, Dm, Rk, T = 1, 64, 4, 400
     rng = np.random.default_rng(3)
-    t, z, w2t, _, u, norm, ref, uu = mix_case(D, rng, dt, T, H, Dm, Rk)
+    t, z, w2, _, u, norm, ref, uu = mix_case(D, rng, dt, T, H, Dm, Rk)
     w0 = torch.full((H * Dm,), w0, device=DEV) + rnd(rng, H * Dm, std=0.5)
-    w = np.exp(-np.exp(np.tanh(f64(z)[:, :Rk]) @ f64(w2t)[:, : H * Dm] + f64(w0))).reshape(T, H, Dm)
+    w = np.exp(-np.exp(np.tanh(f64(z)[:, :Rk]) @ f64(w2)[:, :Rk].T + f64(w0))).reshape(T, H, Dm)
     want, S = mix_want((*ref[:3], w), uu, f64(t["g"])[:, : H * Dm], f64(norm), H, Dm, 1e-4, None)
     state, out = rnd(rng, 1, H, Dm, Dm), D.activation(T, H * Dm, dt, DEV)
-    D.time_mix(t["r"], t["k"], t["v"], t["g"], z, Rk, w2t, w0, u, norm, 1e-4, state, i32([[0, 0, T, 0]]), i32([0] * T), i32(np.arange(T)), out)
+    D.time_mix(t["r"], t["k"], t["v"], t["g"], z, Rk, w2, w0, u, norm, 1e-4, state, i32([[0, 0, T, 0]]), i32([0] * T), i32(np.arange(T)), out)
     torch.cuda.synchronize()
     assert err(rows_of(out), want) < tol(dt, f32=2e-5, b16=6e-3) and err(state[0], S) < 2e-5
+    if dt == torch.bfloat16:
+        state, out = rnd(rng, 1, H, Dm, Dm), D.activation(T, H * Dm, dt, DEV)
+        mix_prompt(D, ops, D.TimeMixPlan([(0, 0, T, 0)], H, DEV), t, z, Rk, w2, w0, u, norm, 1e-4, state, out)
+        torch.cuda.synchronize()
+        assert err(rows_of(out), want) < 6e-3 and err(state[0], S) < 4e-5
 
 
-@pytest.mark.parametrize("dt", DTYPES)
-def test_time_mix_far_tokens(D, ops, dt):
+@pytest.mark.parametrize("dt,prompt", [(torch.float32, False), (torch.bfloat16, False), (torch.bfloat16, True)])
+def test_time_mix_far_tokens(D, ops, dt, prompt):
     """One token's key stands out in a channel of its own that hardly decays: its value comes back wherever a later token asks for
     that channel, over chunk edges and portions, and not to the tokens before it."""
     H, Dm, Rk, T = 1, 64, 4, 300
     rng = np.random.default_rng(11)
-    t, z, w2t, w0, u, norm, ref, uu = mix_case(D, rng, dt, T, H, Dm, Rk)
+    t, z, w2, w0, u, norm, ref, uu = mix_case(D, rng, dt, T, H, Dm, Rk)
     spots = [0, 1, 15, 16, 31, 32, 63, 64, 127, 128, 200]
     w0 = torch.full((H * Dm,), -3.0, device=DEV)
     w0[: len(spots)] = -12.0
@@ -227,9 +267,12 @@ def test_time_mix_far_tokens(D, ops, dt):
     state, outs = torch.zeros((1, H, Dm, Dm), device=DEV), []
     for a, b in ((0, 130), (130, 132), (132, 300)):
         out = D.activation(b - a, Dm, dt, DEV)
-        sl = lambda x: x[a:b].contiguous()
-        D.time_mix(sl(t["r"]), sl(t["k"]), sl(t["v"]), sl(t["g"]), sl(z), Rk, w2t, w0, u, norm, 1e-4, state, i32([[0, 0, b - a, a]]), i32([0] * (b - a)),
-                   i32(np.arange(a, b)), out)
+        part, zs = {s: x[a:b].contiguous() for s, x in t.items()}, z[a:b].contiguous()
+        if prompt:
+            mix_prompt(D, ops, D.TimeMixPlan([(0, 0, b - a, a)], H, DEV, 32), part, zs, Rk, w2, w0, u, norm, 1e-4, state, out)
+        else:
+            D.time_mix(*(part[s] for s in "rkvg"), zs, Rk, w2, w0, u, norm, 1e-4, state, i32([[0, 0, b - a, a]]), i32([0] * (b - a)),
+                       i32(np.arange(a, b)), out)
         outs.append(rows_of(out))
     torch.cuda.synchronize()
     got, gate = f64(torch.cat(outs)), R.silu(f64(t["g"])[:, :Dm]) * f64(norm)
