@@ -69,6 +69,11 @@ int mlora_stream_step(const mlora_stream_step_args* args, void* stream);
  * slices: the reader of y adds the ks - 1 partial blocks part[q][T][N]. */
 int mlora_linear_ksplit_store(float* y, float* part, int ks, const void* xf, const void* Wp, int T, int K, int N, void* stream);
 
+/* y [T, N_main] = xf_g . Wp^T (bfloat16 library, T <= 64), row group g = row / group_rows (a multiple of 64) of the packed weight reading
+ * the activation xf + g * x_stride; the N_ext rows behind N_main are a last group, whose result goes to y2 [T, N_ext] fp32. */
+int mlora_gemv_frag_groups(void* y, float* y2, const void* xf, long x_stride, int group_rows, const void* Wp, int T, int K, int N_main, int N_ext,
+                           void* stream);
+
 /* x [T, H] fp32 = table[ids[t]] * scale (zero for an id outside 0..V-1), and the same in elements (out_frag and / or out_row). */
 int mlora_embed_scaled(float* x, void* out_frag, void* out_row, int ld_row, const void* table, const int32_t* ids, float scale, int T, int H, int V,
                        void* stream);

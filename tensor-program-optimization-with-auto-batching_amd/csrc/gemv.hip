@@ -122,12 +122,13 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE) void lora_expand_shares_kernel(Lo
 // With SHRINK the first `shrink_blocks` workgroups of the launch do LoRA shrink units (one per wave) on the same
 // x instead of a GEMV tile: the adapter work rides in the GEMV launch and finishes long before it does.
 // An accumulating launch without shrink units may instead carry `ride_blocks` delta riders (lora_delta_ride).
-template <int NT, int TT, int OUT, bool PACKED, bool XFRAG, bool SHRINK, int PIPE = 4>   // PIPE: k-steps in flight per wave
+// GX (fragment order): the rows are groups of gx_rows (a multiple of 16 NT) that read activations of their own, gx_stride elements apart.
+template <int NT, int TT, int OUT, bool PACKED, bool XFRAG, bool SHRINK, int PIPE = 4, bool GX = false>   // PIPE: k-steps in flight per wave
 __global__ __launch_bounds__(GEMV_WAVES* WAVE, (NT * TT > 8 ? 2 : 4)) void gemv_kernel(void* __restrict__ yv, const elt* __restrict__ x, int ldx,
                                                                 const elt* __restrict__ W, int T, int K, int N,
                                                                 LoraShrinkBatch sb, int shrink_blocks, int n_main,
                                                                 float* __restrict__ y2, int ksplit, float* __restrict__ part,
-                                                                LoraDeltaRide dr, int ride_blocks, GluArgs ga) {
+                                                                LoraDeltaRide dr, int ride_blocks, GluArgs ga, int gx_rows = 0, long gx_stride = 0) {
   constexpr int TILES = NT * TT;
   constexpr int HT = TILES > 8 ? TILES / 2 : TILES;   // accumulator tiles summed per pass through LDS (64 KiB holds 8)
   constexpr bool RIDE = OUT == OUT_ACC_F32 && PACKED && XFRAG && !SHRINK;   // the launches that may carry delta riders
@@ -164,6 +165,7 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE, (NT * TT > 8 ? 2 : 4)) void gemv_
   const int r16 = lane & 15;
   const int kg = lane >> 4;
   const int n0 = bid * (16 * NT);
+  if constexpr (GX) x += (n0 / gx_rows) * gx_stride;
   const int KB = K / KSTEP;
   constexpr int WSTEP = PACKED ? 512 : KSTEP;   // elements between consecutive k-steps of one fragment stream
 
@@ -719,6 +721,39 @@ extern "C" int mlora_gemv_frag_acc_ksplit(float* y, float* y2, float* part, int 
                                            shrink_batch(xf, v_part, A, n_proj, tok_adapter, T, K, r, n_ad), N_main, y2, ks, part);
   return gemv_dispatch<true, true, false>(y, MLORA_F32, MLORA_ACCUMULATE, xf, K, Wp, T, K, N, stream, LoraShrinkBatch(), N_main, y2,
                                           ks, part);
+}
+
+template <int NT, int TT, int PIPE>
+static void launch_gemv_groups(void* y, float* y2, const elt* x, long stride, int rows, const elt* W, int T, int K, int N, int n_main, hipStream_t s) {
+  hipLaunchKernelGGL((gemv_kernel<NT, TT, OUT_F16, true, true, false, PIPE, true>), dim3(ceil_div(N, 16 * NT)), dim3(GEMV_WAVES * WAVE), 0, s, y, x, K, W, T,
+                     K, N, LoraShrinkBatch(), 0, n_main, y2, 1, (float*)nullptr, LoraDeltaRide(), 0, GluArgs(), rows, stride);
+}
+
+extern "C" int mlora_gemv_frag_groups(void* y, float* y2, const void* xf, long x_stride, int group_rows, const void* Wp, int T, int K, int N_main, int N_ext,
+                                      void* stream) {
+  if (int e = mlora_check_linear("gemv_frag_groups", y, MLORA_F16, MLORA_STORE, xf, K, Wp, T, K, N_main)) return e;
+  MLORA_CHECK(T <= 64 && group_rows > 0 && group_rows % 64 == 0 && N_main % group_rows == 0 && N_ext >= 0 && N_ext <= group_rows && N_ext % 4 == 0 &&
+                  (N_ext == 0 || y2) && x_stride % 8 == 0 && (((uintptr_t)xf | (uintptr_t)y) & 15) == 0,
+              MLORA_ERR_UNSUPPORTED, "gemv_frag_groups: T <= 64 and groups of whole 64 rows (T=%d rows=%d N_main=%d N_ext=%d)", T, group_rows, N_main, N_ext);
+  if (T == 0) return MLORA_OK;
+  hipStream_t s = (hipStream_t)stream;
+  const elt* x = (const elt*)xf;
+  const elt* W = (const elt*)Wp;
+  const int N = N_main + N_ext, tiles = ceil_div(N, 16);
+  if (tiles >= 768) {                          // the rules of gemv_dispatch
+    if (T <= 16) launch_gemv_groups<4, 1, 4>(y, y2, x, x_stride, group_rows, W, T, K, N, N_main, s);
+    else if (T <= 32) launch_gemv_groups<4, 2, 3>(y, y2, x, x_stride, group_rows, W, T, K, N, N_main, s);
+    else launch_gemv_groups<4, 4, 2>(y, y2, x, x_stride, group_rows, W, T, K, N, N_main, s);
+  } else if (tiles > 256) {
+    if (T <= 16) launch_gemv_groups<2, 1, 4>(y, y2, x, x_stride, group_rows, W, T, K, N, N_main, s);
+    else if (T <= 32) launch_gemv_groups<2, 2, 4>(y, y2, x, x_stride, group_rows, W, T, K, N, N_main, s);
+    else launch_gemv_groups<2, 4, 2>(y, y2, x, x_stride, group_rows, W, T, K, N, N_main, s);
+  } else {
+    if (T <= 16) launch_gemv_groups<1, 1, 4>(y, y2, x, x_stride, group_rows, W, T, K, N, N_main, s);
+    else if (T <= 32) launch_gemv_groups<1, 2, 4>(y, y2, x, x_stride, group_rows, W, T, K, N, N_main, s);
+    else launch_gemv_groups<1, 4, 4>(y, y2, x, x_stride, group_rows, W, T, K, N, N_main, s);
+  }
+  return mlora_launch_status("gemv_frag_groups");
 }
 
 // the storing form (mlora_linear_ksplit_store), T <= 64

@@ -14,6 +14,9 @@
 // holds the values v of each of the G key/value heads, [n_pages, G, RB, 4, 16, 8], and one number per token and head,
 // 1 / rms(v) [n_pages, G, 16] fp32, so that a key is (1 / rms) v w and is never stored: the norm's weight w goes to the queries,
 // the number to the scores.  A distance bias slope_h (i - j) is taken off the scores.
+// Normed keys have a root mean square of at most one, so a score lies within B = |scale| |q| sqrt(D) of zero, and the query's own key
+// (distance 0) scores at least -B: a key whose bias exceeds 2 B by 126 bits has a weight that fp32 holds as zero.  Pages behind that
+// reach are not read.
 #include <type_traits>
 
 #include "common.h"
@@ -107,7 +110,7 @@ struct LatentAttn {
   int T, H, RB, NB, splits, n_inner, chunks;
   const float* key_scale;   // tied: [n_pages, G, 16]
   const float* slopes;      // tied: [H]
-  int G, gs, gt;            // tied: key/value heads, heads per group, 16-head tiles per group
+  int G, gs, gt, D;         // tied: key/value heads, heads per group, 16-head tiles per group, columns of a head
   int frag_tt;              // `out` in fragment order (tied) if > 0
 };
 
@@ -122,6 +125,12 @@ __device__ __forceinline__ int latent_ctx(const LatentAttn& a, int t, int& seq) 
   if (seq < 0 || seq >= a.n_seq || ctx < 0) ctx = 0;
   if (seq < 0 || seq >= a.n_seq) seq = 0;
   return ctx < a.max_blocks * PAGE ? ctx : a.max_blocks * PAGE;
+}
+
+// tied: positions behind a query that can have a weight, given the square of its length (see above)
+__device__ __forceinline__ float tied_reach(float qq, int D, float scale, float slope) {
+  const float B = fabsf(scale) * sqrtf(qq * (float)D) * 1.02f;      // a margin for the rounding of queries and keys
+  return fminf((2.f * B + 90.f) / fmaxf(slope, 1e-30f), 1e9f) + 2.f;
 }
 
 #ifndef MLORA_ELT_F32
@@ -152,8 +161,8 @@ __global__ __launch_bounds__(NW * WAVE, 2) void latent_attn_kernel(LatentAttn a)
   int seq;
   const int ctx = latent_ctx(a, t, seq);
   const int npages = (ctx + PAGE - 1) / PAGE;
-  const int per = (npages + a.splits - 1) / a.splits;
-  const int p0 = split * per, p1 = p0 + per < npages ? p0 + per : npages;
+  int per = (npages + a.splits - 1) / a.splits;
+  int p0 = split * per, p1 = p0 + per < npages ? p0 + per : npages;
   const int32_t* __restrict__ bt = a.block_table + (size_t)seq * a.max_blocks;
   const int qd = a.NB * 32;
 
@@ -172,6 +181,23 @@ __global__ __launch_bounds__(NW * WAVE, 2) void latent_attn_kernel(LatentAttn a)
     id1[e] = (elt)(g * 8 + e == col + 16 ? 1.f : 0.f);
   }
   __syncthreads();
+  const float slope = TIED ? a.slopes[h0 + (col < hn ? col : 0)] : 0.f;
+  if constexpr (TIED) {                                              // the pages within reach of any of the heads
+    float qq = 0.f;
+    for (int s = 0; s < RBp; ++s) {
+      const eltx8 v = ld8(qs + (s * 64 + lane) * 8);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) qq = fmaf((float)v[e], (float)v[e], qq);
+    }
+    qq += __shfl_xor(qq, 16, WAVE);
+    qq += __shfl_xor(qq, 32, WAVE);
+    const float reach = wave_max(col < hn ? tied_reach(qq, a.D, a.scale, slope) : 0.f);
+    const int back = (int)fminf(reach, (float)ctx);
+    const int pb = __builtin_amdgcn_readfirstlane((ctx - back > 0 ? ctx - back : 0) / PAGE);
+    per = (npages - pb + a.splits - 1) / a.splits;
+    p0 = pb + split * per;
+    p1 = p0 + per < npages ? p0 + per : npages;
+  }
 
   float m = -INFINITY, l = 0.f;
   f32x4 O[2 * NRB];
@@ -190,7 +216,6 @@ __global__ __launch_bounds__(NW * WAVE, 2) void latent_attn_kernel(LatentAttn a)
     return *reinterpret_cast<const f32x4*>(a.key_scale + ((size_t)(page >= 0 && page < a.n_pages ? page : 0) * a.G + kvh) * PAGE + 4 * g);
   };
   f32x4 ksc = f32x4{0.f, 0.f, 0.f, 0.f};
-  const float slope = TIED ? a.slopes[h0 + (col < hn ? col : 0)] : 0.f;
   eltx8 kf[NRB], rf[2];
   bool ok = false, ok_next = false;
   const elt* kp = a.cache;
@@ -472,7 +497,7 @@ struct LatentPrefill {
   float scale;
   int H, pages, KN, KR, VB;
   const float* slopes;      // tied: [H]
-  int gs;                   // tied: heads per key/value head
+  int gs, D;                // tied: heads per key/value head, columns of a head
 };
 
 // Four waves own up to 128 consecutive queries of one head of one sequence, a wave 32 of them as two 16-query tiles.  Keys are
@@ -536,8 +561,31 @@ __global__ __launch_bounds__(LP_WAVES* WAVE, 2) void latent_prefill_kernel(Laten
                                        (__attribute__((address_space(3))) void*)(dst + i * 512), 16, 0, 0);
     }
   };
-  issue(0);
-  for (int b = 0; b < nblk; ++b) {
+  int b0 = 0;
+  if constexpr (TIED) {                                              // the first block within reach of any of the queries
+    __shared__ float qmax[LP_WAVES];
+    float qq = 0.f;
+#pragma unroll
+    for (int u = 0; u < LP_QT; ++u) {
+      float s = 0.f;
+#pragma unroll
+      for (int kb = 0; kb < KB_; ++kb)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) s = fmaf((float)qf[u][kb][e], (float)qf[u][kb][e], s);
+      s += __shfl_xor(s, 16, WAVE);
+      s += __shfl_xor(s, 32, WAVE);
+      qq = fmaxf(qq, s);
+    }
+    qq = wave_max(qq);
+    if (lane == 0) qmax[wave] = qq;
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < LP_WAVES; ++i) qq = fmaxf(qq, qmax[i]);
+    const int back = (int)fminf(tied_reach(qq, a.D, a.scale, a.slopes[h]), (float)(tile.w + 1));
+    b0 = __builtin_amdgcn_readfirstlane((tile.w - back > 0 ? tile.w - back : 0) / 64);
+  }
+  issue(b0);
+  for (int b = b0; b < nblk; ++b) {
     asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");      // this wave's pieces of block b have landed, its reads of b - 1 are done
     bare_barrier();
     if (b + 1 < nblk) issue(b + 1);                                  // into the buffer of block b - 1
@@ -1282,7 +1330,7 @@ extern "C" int mlora_tied_attn(void* out, int out_layout, const void* q, const v
   LatentAttn a = {};
   a.out = (elt*)out; a.q = (const elt*)q; a.cache = (const elt*)cache; a.block_table = block_table; a.max_blocks = max_blocks;
   a.n_pages = n_pages; a.n_seq = n_seq; a.tok_seq = tok_seq; a.tok_pos = tok_pos; a.scale = scale; a.T = T; a.H = H;
-  a.RB = a.NB = ceil_div(D, 32); a.splits = splits; a.key_scale = key_scale; a.slopes = slopes; a.G = G; a.gs = H / G; a.gt = ceil_div(H / G, 16);
+  a.RB = a.NB = ceil_div(D, 32); a.splits = splits; a.key_scale = key_scale; a.slopes = slopes; a.G = G; a.gs = H / G; a.gt = ceil_div(H / G, 16); a.D = D;
   a.frag_tt = out_layout == MLORA_FRAG ? mlora_frag_tiles(T) : 0; a.chunks = 1;
   hipStream_t s = (hipStream_t)stream;
 #ifdef MLORA_ELT_F32
@@ -1328,7 +1376,7 @@ extern "C" int mlora_tied_prefill(void* out, int out_layout, int ld_out, const v
   MLORA_CHECK(scratch_elems >= mlora_tied_prefill_scratch_elems(pages, G, D), MLORA_ERR_WORKSPACE, "tied_prefill: scratch too small");
   hipStream_t s = (hipStream_t)stream;
   LatentPrefill a = {};
-  a.KN = ceil_div(D, 32); a.KR = 0; a.VB = 2 * a.KN; a.H = H; a.pages = pages; a.gs = H / G;
+  a.KN = ceil_div(D, 32); a.KR = 0; a.VB = 2 * a.KN; a.H = H; a.pages = pages; a.gs = H / G; a.D = D;
   elt* k = (elt*)scratch;
   elt* v = k + (size_t)G * pages * a.KN * 512;
   hipLaunchKernelGGL(tied_expand_kernel, dim3(pages / 2, G), dim3(256), 0, s, k, v, (const elt*)cache, key_scale, phys, pages, n_pages, G, a.KN);

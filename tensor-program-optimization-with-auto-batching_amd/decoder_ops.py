@@ -167,6 +167,26 @@ def linear_sum(x, W, split=True):
     return y, ops.KSplitParts(part, ks, N) if ks > 1 else None
 
 
+def linear_groups(x, W, group_rows, ext):
+    """W's row groups of group_rows applied to activations of their own, the blocks of the FragActivation x one after the other: ->
+    (all groups' results [T, rows], those of the last `ext` rows [T, ext] fp32, a group of their own).  T <= 64."""
+    T, K = x.shape
+    n = W.shape[0] - ext
+    y = torch.empty((T, n), dtype=W.dtype, device=x.device)
+    y2 = torch.empty((T, ext), dtype=torch.float32, device=x.device)
+    stride = x.data.numel() // (n // group_rows + 1)
+    check(lib_of(W.dtype).mlora_gemv_frag_groups(_dev(y), _dev(y2), x.data.data_ptr(), stride, group_rows, W.data.data_ptr(), T, K, n, ext, _stream()),
+          W.dtype)
+    return y, y2
+
+
+def _cols(t, dtype):
+    """(pointer, row stride) of a column range of a row-major tensor."""
+    if not t.is_cuda or t.dtype != dtype or t.stride(1) != 1:
+        raise ValueError("column ranges of GPU tensors of one type")
+    return t.data_ptr(), t.stride(0) if t.shape[0] > 1 else max(t.shape[1], t.stride(0))
+
+
 def token_gate(x, W, table, col0, dim, ids):
     """gelu_tanh(W x) * table[ids, col0 : col0 + dim] (x: an activation) as the activation of the following linear, its width
     W's padded row count."""
@@ -243,13 +263,14 @@ def gate_up_silu(x, W, W_il, out):
 
 
 def time_mix(r, k, v, g, z, R, w2, w0, u, norm, eps, state, segs, tok_seq, tok_pos, out):
-    """The recurrence of time mixing (csrc/time_mix.hip) over a pass: r, k, v, g [T, ld], z [T, >= R] fp32, state [n, H, D, D] fp32
-    (updated), segs [n][4] int32 or None (a decode step) -> out, an activation [T, H * D rounded up]."""
-    T, ld = r.shape
+    """The recurrence of time mixing (csrc/time_mix.hip) over a pass: r, k, v, g [T, >= H * D] of one row stride, z [T, >= R] fp32, state
+    [n, H, D, D] fp32 (updated), segs [n][4] int32 or None (a decode step) -> out, an activation [T, H * D rounded up]."""
+    T = r.shape[0]
+    (r_p, ld), (k_p, _), (v_p, _), (g_p, _) = (_cols(t, r.dtype) for t in (r, k, v, g))
     n_seq, H, D, _ = state.shape
     frag = isinstance(out, FragActivation)
     check(lib_of(r.dtype).mlora_time_mix(out.data.data_ptr() if frag else _dev(out, r.dtype), FRAG if frag else ROWMAJOR, out.shape[1],
-                                         _dev(r), _dev(k, r.dtype), _dev(v, r.dtype), _dev(g, r.dtype), ld, _dev(z, torch.float32), z.shape[1], R,
+                                         r_p, k_p, v_p, g_p, ld, _dev(z, torch.float32), z.shape[1], R,
                                          _dev(w2, r.dtype), w2.shape[1], _dev(w0, torch.float32), _dev(u, torch.float32), _dev(norm, r.dtype), eps,
                                          _dev(state, torch.float32), n_seq, _ptr(segs), T if segs is None else segs.shape[0],
                                          _dev(tok_seq, torch.int32), _dev(tok_pos, torch.int32), T, H, D, _stream()), r.dtype)

@@ -306,6 +306,14 @@ class PackedWeight:
     def dtype(self):
         return self.data.dtype
 
+    def rows(self, n0: int, n: int) -> "PackedWeight":
+        """Rows n0 .. n0 + n - 1 (n0 a multiple of 16) as a weight of their own: a view."""
+        if n0 % 16 or n0 + n > self.N:
+            raise ValueError("PackedWeight.rows: whole tiles of 16 rows")
+        w = PackedWeight.__new__(PackedWeight)
+        w.N, w.K, w.data = n, self.K, self.data[n0 * self.K: (n0 + -(-n // 16) * 16) * self.K]
+        return w
+
     def unpack(self) -> torch.Tensor:
         """Back to row-major [N, K] (index arithmetic on the device tensor)."""
         nt = (self.N + 15) // 16

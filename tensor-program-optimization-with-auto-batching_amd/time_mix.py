@@ -36,9 +36,14 @@ class TimeMix:
         self.out_cols = pad64(cols)
         t = lambda n: w[n].to(device, dtype)
         self.mu = torch.stack([padded(t("mu." + s), Hp) for s in MIXES]).contiguous()
-        self.proj = {s: D.weight(padded(t(s), self.out_cols, Hp)) for s in "rkvg"}
         self.rank = w["w1"].shape[0]
-        self.w1 = D.weight(padded(t("w1"), pad32(self.rank), Hp))
+        rows = [padded(t(s), self.out_cols, Hp) for s in "rkvg"] + [padded(t("w1"), pad32(self.rank), Hp)]
+        if dtype == torch.float32:
+            self.all, (*proj, self.w1) = None, [D.weight(m) for m in rows]
+        else:                                                                    # one matrix for decode steps, and its parts
+            self.all = D.weight(torch.cat(rows))
+            *proj, self.w1 = (self.all.rows(i * self.out_cols, m.shape[0]) for i, m in enumerate(rows))
+        self.proj = dict(zip("rkvg", proj))
         self.w2 = padded(t("w2"), cols, pad32(self.rank)).contiguous()
         self.w0 = w["w0"].to(device, torch.float32).contiguous()
         self.u = w["u"].to(device, torch.float32).reshape(-1).contiguous()
@@ -47,22 +52,30 @@ class TimeMix:
         self.prompt_form = dtype != torch.float32 and D.time_mix_prompt_served(spec.dim)
 
     def mixes(self, T, width_p, device):
-        """Room for the five mixes of a pass: (what a stream step fills as out or out_row, the five activations)."""
+        """Room for the five mixes of a pass: (what a stream step fills as out or out_row, the five activations - which lie in it one
+        after the other)."""
         if self.dtype == torch.float32:
             rows = torch.empty((len(MIXES), T, width_p), dtype=self.dtype, device=device)
             return {"out_row": rows}, list(rows)
         n = ops.lib_of(self.dtype).mlora_frag_activation_elems(T, width_p)
         data = torch.empty(len(MIXES) * n, dtype=self.dtype, device=device)
         acts = [ops.FragActivation(T, width_p, device, data[i * n:(i + 1) * n]) for i in range(len(MIXES))]
+        acts[0].room = data                                                      # all five, for the product that takes them together
         return {"out": ops.FragActivation(T, width_p, device, data)}, acts
 
     def run(self, mixes, state, segs, tok_seq, tok_pos, plan=None):
         """mixes: the five activations -> the gated outputs of the heads, an activation of out_cols columns; updates state.
         segs: the sequences of the pass (None: a decode step); plan: a TimeMixPlan of the pass for the prompt form."""
-        r, k, v, g = (ops.linear(m, self.proj[s]) for m, s in zip(mixes, "rkvg"))
-        out = D.activation(r.shape[0], self.out_cols, self.dtype, r.device)
+        T, dev, n = mixes[0].shape[0], mixes[0].device, self.out_cols
+        out = D.activation(T, n, self.dtype, dev)
         rest = (self.w2, self.w0, self.u, self.norm, self.eps, state)
-        if plan is not None:
-            return D.time_mix_prompt(plan, r, k, v, g, mixes[4], self.w1, *rest, out)
-        z = ops.linear(mixes[4], self.w1, out_dtype=torch.float32)
+        if plan is None and self.all is not None and T <= 64 and self.w1.N <= n:
+            x = mixes[0]
+            y, z = D.linear_groups(ops.FragActivation(T, x.K, dev, x.room), self.all, n, self.w1.N)
+            r, k, v, g = (y[:, i * n:(i + 1) * n] for i in range(4))
+        else:
+            r, k, v, g = (ops.linear(m, self.proj[s]) for m, s in zip(mixes, "rkvg"))
+            if plan is not None:
+                return D.time_mix_prompt(plan, r, k, v, g, mixes[4], self.w1, *rest, out)
+            z = ops.linear(mixes[4], self.w1, out_dtype=torch.float32)
         return D.time_mix(r, k, v, g, z, self.rank, *rest, segs, tok_seq, tok_pos, out)

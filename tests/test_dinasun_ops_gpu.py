@@ -503,3 +503,19 @@ def test_gate_up_silu(D, ops, T, K, ff):
     torch.cuda.synchronize()
     z = f64(x) @ f64(gu).T
     assert err(out.unpack(), R.silu(z[:, :ff]) * z[:, ff:]) < 1.2e-2
+
+
+@pytest.mark.parametrize("T,K,rows,ext", [(1, 64, 64, 32), (16, 96, 128, 64), (30, 1056, 64, 32), (64, 128, 2048, 64), (32, 64, 4096, 32), (5, 4096, 1024, 160)])
+def test_linear_groups(D, ops, T, K, rows, ext):
+    """Four row groups and a narrow last one, each on activations of its own, in one launch."""
+    rng = np.random.default_rng(T)
+    dt = torch.bfloat16
+    xs, W = [rnd(rng, T, K, dt=dt) for _ in range(5)], rnd(rng, 4 * rows + ext, K, std=K ** -0.5, dt=dt)
+    data = torch.cat([ops.FragActivation.pack(x).data for x in xs])
+    Wp = ops.PackedWeight(W)
+    y, y2 = D.linear_groups(ops.FragActivation(T, K, DEV, data), Wp, rows, ext)
+    torch.cuda.synchronize()
+    for i in range(4):
+        assert err(y[:, i * rows:(i + 1) * rows], f64(xs[i]) @ f64(W[i * rows:(i + 1) * rows]).T) < 4e-3
+        assert torch.equal(Wp.rows(i * rows, rows).unpack(), W[i * rows:(i + 1) * rows])
+    assert err(y2, f64(xs[4]) @ f64(W[4 * rows:]).T) < 2e-6
