@@ -70,7 +70,9 @@ int mlora_stream_step(const mlora_stream_step_args* args, void* stream);
 int mlora_linear_ksplit_store(float* y, float* part, int ks, const void* xf, const void* Wp, int T, int K, int N, void* stream);
 
 /* y [T, N_main] = xf_g . Wp^T (bfloat16 library, T <= 64), row group g = row / group_rows (a multiple of 64) of the packed weight reading
- * the activation xf + g * x_stride; the N_ext rows behind N_main are a last group, whose result goes to y2 [T, N_ext] fp32. */
+ * the activation xf + g * x_stride; the N_ext rows behind N_main are a last group, whose result goes to y2
+ * [mlora_gemv_groups_parts(K), T, N_ext] fp32 as partial sums over ranges of K. */
+int mlora_gemv_groups_parts(int K);
 int mlora_gemv_frag_groups(void* y, float* y2, const void* xf, long x_stride, int group_rows, const void* Wp, int T, int K, int N_main, int N_ext,
                            void* stream);
 
@@ -79,11 +81,12 @@ int mlora_embed_scaled(float* x, void* out_frag, void* out_row, int ld_row, cons
                        void* stream);
 
 /* Time mixing (equations at the top of time_mix.hip): a recurrence per head over a matrix state, its decay, the norm of the
- * heads' outputs and their gate.  r, k, v, g [T, ld]; z [T, ld_z] fp32, R columns (before the tanh); w2 [H * D, ld_w2], zero behind R; w0, u fp32 and norm,
+ * heads' outputs and their gate.  r, k, v, g [T, ld]; z [n_z, T, ld_z] fp32, R columns: partial sums of the
+ * decay's low-rank projection (before the tanh); w2 [H * D, ld_w2], zero behind R; w0, u fp32 and norm,
  * each [H * D]; state [n_seq, H, D, D] fp32, updated.  segs [n_segs][4] int32 = {slot, first token, tokens, position of the first
  * token}; NULL: every token is a segment of its own (n_segs = T; a decode step).  y [T, ld_y], ld_y = H * D rounded up, zero behind H * D. */
-int mlora_time_mix(void* y, int y_layout, int ld_y, const void* r, const void* k, const void* v, const void* g, int ld, const float* z, int ld_z,
-                   int R, const void* w2, int ld_w2, const float* w0, const float* u, const void* norm, float eps, float* state, int n_seq,
+int mlora_time_mix(void* y, int y_layout, int ld_y, const void* r, const void* k, const void* v, const void* g, int ld, const float* z, int n_z,
+                   int ld_z, int R, const void* w2, int ld_w2, const float* w0, const float* u, const void* norm, float eps, float* state, int n_seq,
                    const int32_t* segs, int n_segs, const int32_t* tok_seq, const int32_t* tok_pos, int T, int H, int D, void* stream);
 
 /* The same for prompts (bfloat16 library), in chunks on the matrix cores.  zp [T, 3, ld_zp]: tanh of the decay's low-rank projection as

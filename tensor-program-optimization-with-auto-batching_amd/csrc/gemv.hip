@@ -122,13 +122,15 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE) void lora_expand_shares_kernel(Lo
 // With SHRINK the first `shrink_blocks` workgroups of the launch do LoRA shrink units (one per wave) on the same
 // x instead of a GEMV tile: the adapter work rides in the GEMV launch and finishes long before it does.
 // An accumulating launch without shrink units may instead carry `ride_blocks` delta riders (lora_delta_ride).
-// GX (fragment order): the rows are groups of gx_rows (a multiple of 16 NT) that read activations of their own, gx_stride elements apart.
+// GX (fragment order): the rows are groups of gx_rows (a multiple of 16 NT) that read activations of their own, gx_stride elements apart;
+// those behind n_main are cut into gx_kq ranges of K, each a workgroup that leaves a block of y2 (so that no unit gets a whole
+// workgroup more than the others).
 template <int NT, int TT, int OUT, bool PACKED, bool XFRAG, bool SHRINK, int PIPE = 4, bool GX = false>   // PIPE: k-steps in flight per wave
 __global__ __launch_bounds__(GEMV_WAVES* WAVE, (NT * TT > 8 ? 2 : 4)) void gemv_kernel(void* __restrict__ yv, const elt* __restrict__ x, int ldx,
                                                                 const elt* __restrict__ W, int T, int K, int N,
                                                                 LoraShrinkBatch sb, int shrink_blocks, int n_main,
                                                                 float* __restrict__ y2, int ksplit, float* __restrict__ part,
-                                                                LoraDeltaRide dr, int ride_blocks, GluArgs ga, int gx_rows = 0, long gx_stride = 0) {
+                                                                LoraDeltaRide dr, int ride_blocks, GluArgs ga, int gx_rows = 0, long gx_stride = 0, int gx_kq = 1) {
   constexpr int TILES = NT * TT;
   constexpr int HT = TILES > 8 ? TILES / 2 : TILES;   // accumulator tiles summed per pass through LDS (64 KiB holds 8)
   constexpr bool RIDE = OUT == OUT_ACC_F32 && PACKED && XFRAG && !SHRINK;   // the launches that may carry delta riders
@@ -161,6 +163,14 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE, (NT * TT > 8 ? 2 : 4)) void gemv_
     const int q = udiv_le4(bid, ksplit);
     slice = bid - q * ksplit;
     bid = q;
+  }
+  int gx_q = 0;                                    // GX: the range of K of a workgroup of the last group
+  if constexpr (GX) {
+    const int main_wgs = n_main / (16 * NT);
+    if (bid >= main_wgs) {                         // uniform
+      gx_q = (bid - main_wgs) % gx_kq;
+      bid = main_wgs + (bid - main_wgs) / gx_kq;
+    }
   }
   const int r16 = lane & 15;
   const int kg = lane >> 4;
@@ -205,8 +215,15 @@ __global__ __launch_bounds__(GEMV_WAVES* WAVE, (NT * TT > 8 ? 2 : 4)) void gemv_
 
   // wave w takes k-steps w, w + 8, w + 16, ...; stage s of this wave is k-step w + 8 s.
   // PIPE stages are always in flight: each buffer is refilled right after it is consumed.
-  const int kb0 = ksplit > 1 ? udiv_le4(slice * KB, ksplit) : 0;
-  const int kb1 = ksplit > 1 ? udiv_le4((slice + 1) * KB, ksplit) : KB;
+  int kb0 = ksplit > 1 ? udiv_le4(slice * KB, ksplit) : 0;
+  int kb1 = ksplit > 1 ? udiv_le4((slice + 1) * KB, ksplit) : KB;
+  if constexpr (GX) {
+    if (n0 >= n_main) {
+      kb0 = gx_q * KB / gx_kq;
+      kb1 = (gx_q + 1) * KB / gx_kq;
+      y2 += (size_t)gx_q * T * (N - n_main);
+    }
+  }
   const int S = (kb1 - kb0 - wave + GEMV_WAVES - 1) / GEMV_WAVES;
   eltx8 a[PIPE][NT], b[PIPE][TT];
   auto load_stage = [&](int u, int s) {
@@ -723,10 +740,18 @@ extern "C" int mlora_gemv_frag_acc_ksplit(float* y, float* y2, float* part, int 
                                           ks, part);
 }
 
+// ranges of K of the last group's rows: whole rounds of a workgroup's waves
+extern "C" int mlora_gemv_groups_parts(int K) {
+  const int by_k = K / KSTEP / GEMV_WAVES;
+  return by_k < 1 ? 1 : by_k < 8 ? by_k : 8;
+}
+
 template <int NT, int TT, int PIPE>
 static void launch_gemv_groups(void* y, float* y2, const elt* x, long stride, int rows, const elt* W, int T, int K, int N, int n_main, hipStream_t s) {
-  hipLaunchKernelGGL((gemv_kernel<NT, TT, OUT_F16, true, true, false, PIPE, true>), dim3(ceil_div(N, 16 * NT)), dim3(GEMV_WAVES * WAVE), 0, s, y, x, K, W, T,
-                     K, N, LoraShrinkBatch(), 0, n_main, y2, 1, (float*)nullptr, LoraDeltaRide(), 0, GluArgs(), rows, stride);
+  const int kq = mlora_gemv_groups_parts(K);
+  hipLaunchKernelGGL((gemv_kernel<NT, TT, OUT_F16, true, true, false, PIPE, true>), dim3(n_main / (16 * NT) + ceil_div(N - n_main, 16 * NT) * kq),
+                     dim3(GEMV_WAVES * WAVE), 0, s, y, x, K, W, T, K, N, LoraShrinkBatch(), 0, n_main, y2, 1, (float*)nullptr, LoraDeltaRide(), 0,
+                     GluArgs(), rows, stride, kq);
 }
 
 extern "C" int mlora_gemv_frag_groups(void* y, float* y2, const void* xf, long x_stride, int group_rows, const void* Wp, int T, int K, int N_main, int N_ext,

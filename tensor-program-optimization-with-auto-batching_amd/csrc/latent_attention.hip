@@ -515,7 +515,8 @@ __global__ __launch_bounds__(LP_WAVES* WAVE, 2) void latent_prefill_kernel(Laten
   const int qi = lane & 15, g = lane >> 4;
   const int KN = TIED && EXACT ? KB_ : a.KN, KR = TIED ? 0 : a.KR, KB = EXACT ? KB_ : KN + KR, VB = EXACT ? VB_ : a.VB;
   const int PIECES = 4 * KB + 2 * VB;                                // 1 KiB pieces of a key block
-  const int h = blockIdx.x;
+  // tied: the long ranges are those of the heads with small slopes, which the tiles take to another XCD each time
+  const int h = TIED ? (blockIdx.x + blockIdx.y) % gridDim.x : blockIdx.x;
   const int4 tile = a.tiles[blockIdx.y];
   const int wq = wave * LP_QT * 16;                                  // this wave's first query of the tile
   eltx8 qf[LP_QT][KB_];

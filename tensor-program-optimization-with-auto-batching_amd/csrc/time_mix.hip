@@ -22,8 +22,8 @@ struct TimeMix {
   const elt* v;
   const elt* g;
   int ld;
-  const float* z;           // [T, ld_z], R columns count
-  int ld_z, R;
+  const float* z;           // [n_z, T, ld_z] partial sums, R columns count
+  int n_z, ld_z, R;
   const elt* w2;            // [H * D, ld_w2], zero behind the R columns
   int ld_w2;
   const float* w0;          // [H * D]
@@ -36,6 +36,13 @@ struct TimeMix {
   const int32_t* tok_seq;
   const int32_t* tok_pos;
 };
+
+__device__ __forceinline__ float rank_tanh(const TimeMix& a, int t, int j) {
+  if (j >= a.R) return 0.f;
+  float z = 0.f;
+  for (int q = 0; q < a.n_z; ++q) z += a.z[((size_t)q * a.T + t) * a.ld_z + j];
+  return tanhf(z);
+}
 
 __device__ __forceinline__ int4 segment(const TimeMix& a, int i) {
   if (a.segs) return a.segs[i];
@@ -71,7 +78,7 @@ __global__ __launch_bounds__(C* KG) void time_mix_scan_kernel(TimeMix a) {
     __syncthreads();
     for (int i = threadIdx.x; i < n * a.ld_w2; i += NT) {
       const int t = i / a.ld_w2, j = i - t * a.ld_w2;
-      zs[t][j] = j < a.R ? tanhf(a.z[(size_t)(tb + t) * a.ld_z + j]) : 0.f;
+      zs[t][j] = rank_tanh(a, tb + t, j);
     }
     for (int i = threadIdx.x; i < n * DM; i += NT) {
       const int t = i / DM, d = i - t * DM;
@@ -179,7 +186,7 @@ __global__ __launch_bounds__(TS_THREADS) void time_mix_step_kernel(TimeMix a) {
 #pragma unroll
   for (int e = 0; e < 4; ++e)
     if (c + e < D) v4[e] = (float)a.v[o0 + c + e];
-  for (int j = threadIdx.x; j < a.ld_w2; j += TS_THREADS) zs[j] = j < a.R ? tanhf(a.z[(size_t)t * a.ld_z + j]) : 0.f;
+  for (int j = threadIdx.x; j < a.ld_w2; j += TS_THREADS) zs[j] = rank_tanh(a, t, j);
   if (threadIdx.x < C) {
     const int d = threadIdx.x;
     rk[d] = d < D ? (float)a.r[o0 + d] : 0.f;
@@ -287,7 +294,8 @@ typedef uint32_t u32x2 __attribute__((ext_vector_type(2)));
 typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
 __device__ __forceinline__ eltx8 operand(uint32_t a, uint32_t b, uint32_t c, uint32_t d) { return __builtin_bit_cast(eltx8, (u32x4{a, b, c, d})); }
 __device__ __forceinline__ eltx8 both(const HiLo& v) { return operand(v.h[0], v.h[1], v.l[0], v.l[1]); }
-__device__ __forceinline__ eltx8 twice(const uint32_t (&v)[2]) { return operand(v[0], v[1], v[0], v[1]); }
+// (a, b) and its halves swapped: two products with a pair of pairs make all four of their parts
+__device__ __forceinline__ eltx8 swapped(const HiLo& v) { return operand(v.l[0], v.l[1], v.h[0], v.h[1]); }
 __device__ __forceinline__ f32x4 floats(u32x2 v) {
   return f32x4{__uint_as_float(v[0] << 16), __uint_as_float(v[0] & 0xffff0000u), __uint_as_float(v[1] << 16), __uint_as_float(v[1] & 0xffff0000u)};
 }
@@ -308,8 +316,9 @@ __global__ __launch_bounds__(NT * WAVE, 2) void time_mix_chunk_kernel(TimeMix a,
   extern __shared__ __align__(16) char smem[];
   f32x4* part_o = reinterpret_cast<f32x4*>(smem);                    // [NT (keys)][NT (values)][64]
   f32x4* part_a = part_o + (OUT ? NT * NT * 64 : 0);                 // [NT][64]
-  u32x2* vs = reinterpret_cast<u32x2*>(part_a + (OUT ? NT * 64 : 0));   // [NT][64]
-  float* ssq = reinterpret_cast<float*>(vs + NT * 64);               // [NT][16]
+  elt* vs = reinterpret_cast<elt*>(part_a + (OUT ? NT * 64 : 0));    // [NT][64][8] values as operands
+  elt* zs = vs + NT * 512;                                           // [2][3 TC_RK][64][8] the decays' operands of this chunk and the next
+  float* ssq = reinterpret_cast<float*>(zs + 2 * 3 * TC_RK * 512);   // [NT][16]
   const TimeMixRange rg = ranges[blockIdx.y];
   if (rg.slot < 0 || rg.slot >= a.n_seq || rg.tokens <= 0 || (!OUT && rg.add < 0)) return;   // uniform
   const int h = blockIdx.x, D = FULL ? 16 * NT : a.D, hd = h * D;
@@ -364,22 +373,29 @@ __global__ __launch_bounds__(NT * WAVE, 2) void time_mix_chunk_kernel(TimeMix a,
   const int steps = (rg.tokens + 15) / 16, tl = rg.tokens - 1;
   // a chunk's inputs, requested one chunk ahead (tokens behind the range repeat its last one; their keys and queries are cleared)
   u32x2 r_n = u32x2{0, 0}, k_n, v_n, g_n = r_n;
-  eltx8 z_n[3][TC_RK];
+  const int nk = rb < TC_RK ? rb : TC_RK;
   auto row_of = [&](int c) { return (uint32_t)(rg.first + (c * 16 + q16 < tl ? c * 16 + q16 : tl)); };
   auto request = [&](int c) {
     const uint32_t t = row_of(c), row = t * (uint32_t)a.ld, zr = t * (uint32_t)(3 * 32 * rb) + g * 8;
+    for (int f = w; f < 3 * nk; f += NT) {                           // uniform: fragment p nk + i, shared by the waves
+      const int p = f / nk, i = f - p * nk;
+      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(zp + (zr + (uint32_t)((p * rb + i) * 32))),
+                                       (__attribute__((address_space(3))) void*)(zs + ((c & 1) * 3 * TC_RK + f) * 512), 16, 0, 0);
+    }
     k_n = load4(a.k, row);
     v_n = load4(a.v, row);
     if (OUT) {
       r_n = load4(a.r, row);
       g_n = load4(a.g, row);
     }
-#pragma unroll
-    for (int p = 0; p < 3; ++p)
-#pragma unroll
-      for (int i = 0; i < TC_RK; ++i) z_n[p][i] = ld8(zp + (zr + (uint32_t)((p * rb + (i < rb ? i : 0)) * 32)));
+  };
+  // a chunk's requests have landed (the wave's, then everybody's)
+  auto landed = [&]() {
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    lds_barrier();
   };
   request(0);
+  landed();
   for (int c = 0; c < steps; ++c) {
     const bool live = c * 16 + q16 <= tl;
     const f32x4 g4 = floats(g_n);
@@ -391,15 +407,15 @@ __global__ __launch_bounds__(NT * WAVE, 2) void time_mix_chunk_kernel(TimeMix a,
     }
     // values as operands: value 16 w + q16 of tokens 4 g .. + 3
     const f32x4 vt = mfma_16x16x32(operand(v_n[0], v_n[1], 0u, 0u), idh, f32x4{0.f, 0.f, 0.f, 0.f});
-    const uint32_t v4[2] = {__builtin_bit_cast(uint32_t, __builtin_convertvector((f32x2{vt[0], vt[1]}), eltx2)),
-                            __builtin_bit_cast(uint32_t, __builtin_convertvector((f32x2{vt[2], vt[3]}), eltx2))};
+    const u32x2 v2 = __builtin_bit_cast(u32x2, __builtin_convertvector(vt, eltx4));
+    const eltx8 vv = operand(v2[0], v2[1], v2[0], v2[1]);
     // logarithm (base 2) of the decays: lane (token q16; keys d0 ..)
     f32x4 lw = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int i = 0; i < TC_RK; ++i)
-      if (i < rb) {                                                  // uniform
+      if (i < nk) {                                                  // uniform
 #pragma unroll
-        for (int p = 0; p < 3; ++p) lw = mfma_16x16x32(w2r[i], z_n[p][i], lw);
+        for (int p = 0; p < 3; ++p) lw = mfma_16x16x32(w2r[i], ld8(zs + ((c & 1) * 3 * TC_RK + p * nk + i) * 512 + lane * 8), lw);
       }
     for (int i = TC_RK; i < rb; ++i) {
       const eltx8 wi = ld8(w2p + i * 32);
@@ -422,7 +438,7 @@ __global__ __launch_bounds__(NT * WAVE, 2) void time_mix_chunk_kernel(TimeMix a,
     }
     const f32x4 dec = exp2_4(Lt);
     const HiLo kd(k4 * exp2_4(Lt - Li));                             // keys as the state takes them
-    vs[w * 64 + lane] = u32x2{v4[0], v4[1]};
+    st8(vs + (w * 64 + lane) * 8, vv);
     if constexpr (OUT) {
       // this wave's keys' part of A: A^T[s = 4 g + r][t = q16]
       const f32x4 ru = r4 * u4;
@@ -439,14 +455,14 @@ __global__ __launch_bounds__(NT * WAVE, 2) void time_mix_chunk_kernel(TimeMix a,
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
           x[e] = up ? r4[e] : k4[e];
-          if (hb > 1) x[e] *= __builtin_amdgcn_exp2f(up ? Lx[e] - m[e] : m[e] - Li[e]);
+          if (hb > 1) x[e] *= __builtin_amdgcn_exp2f(-fabsf((up ? Lx[e] : Li[e]) - m[e]));   // Lx <= m <= L on the two sides
         }
         const HiLo p(x);
         f32x4 G;
         if (hb > 1) {
           const eltx8 b = both(p);
-          G = mfma_16x16x32(b, twice(p.h), f32x4{0.f, 0.f, 0.f, 0.f});
-          G = mfma_16x16x32(b, twice(p.l), G);
+          G = mfma_16x16x32(b, b, f32x4{0.f, 0.f, 0.f, 0.f});
+          G = mfma_16x16x32(b, swapped(p), G);
         } else {                                                     // r and k themselves: elements
           G = mfma_16x16x32(operand(p.h[0], p.h[1], 0u, 0u), operand(p.h[0], p.h[1], 0u, 0u), f32x4{0.f, 0.f, 0.f, 0.f});
         }
@@ -471,12 +487,12 @@ __global__ __launch_bounds__(NT * WAVE, 2) void time_mix_chunk_kernel(TimeMix a,
       part_a[w * 64 + lane] = A;
       // ... and of what comes out of the state: o^T[value 16 n + 4 g + r][t = q16]
       const HiLo R(r4 * exp2_4(Lx));
-      const eltx8 rh = twice(R.h), rl = twice(R.l);
+      const eltx8 ra = both(R), rs = swapped(R);
 #pragma unroll
       for (int n = 0; n < NT; ++n) {
         const eltx8 s8 = both(HiLo(S[n]));
-        const f32x4 o = mfma_16x16x32(s8, rh, f32x4{0.f, 0.f, 0.f, 0.f});
-        part_o[(w * NT + n) * 64 + lane] = mfma_16x16x32(s8, rl, o);
+        const f32x4 o = mfma_16x16x32(s8, ra, f32x4{0.f, 0.f, 0.f, 0.f});
+        part_o[(w * NT + n) * 64 + lane] = mfma_16x16x32(s8, rs, o);
       }
     }
     lds_barrier();
@@ -487,10 +503,7 @@ __global__ __launch_bounds__(NT * WAVE, 2) void time_mix_chunk_kernel(TimeMix a,
       const u32x2 uh = __builtin_bit_cast(u32x2, __builtin_convertvector(th, eltx4)), ul = __builtin_bit_cast(u32x2, __builtin_convertvector(tlo, eltx4));
       const eltx8 kt = operand(uh[0], uh[1], ul[0], ul[1]);
 #pragma unroll
-      for (int n = 0; n < NT; ++n) {
-        const u32x2 v = vs[n * 64 + lane];
-        S[n] = mfma_16x16x32(kt, operand(v[0], v[1], v[0], v[1]), S[n] * dec);
-      }
+      for (int n = 0; n < NT; ++n) S[n] = mfma_16x16x32(kt, ld8(vs + (n * 64 + lane) * 8), S[n] * dec);
       if (!OUT) keep *= dec;
     }
     if constexpr (OUT) {
@@ -500,12 +513,12 @@ __global__ __launch_bounds__(NT * WAVE, 2) void time_mix_chunk_kernel(TimeMix a,
         A += part_a[i * 64 + lane];
         o += part_o[(i * NT + w) * 64 + lane];
       }
-      o = mfma_16x16x32(twice(v4), both(HiLo(A)), o);                // o^T[value d0 + r][t = q16]
+      o = mfma_16x16x32(vv, both(HiLo(A)), o);                // o^T[value d0 + r][t = q16]
       float ss = fmaf(o[0], o[0], o[1] * o[1]) + fmaf(o[2], o[2], o[3] * o[3]);
       ss += __shfl_xor(ss, 16, WAVE);
       ss += __shfl_xor(ss, 32, WAVE);
       if (g == 0) ssq[w * 16 + q16] = ss;
-      lds_barrier();
+      landed();
       float tot = ssq[q16];
 #pragma unroll
       for (int i = 1; i < NT; ++i) tot += ssq[i * 16 + q16];
@@ -525,7 +538,7 @@ __global__ __launch_bounds__(NT * WAVE, 2) void time_mix_chunk_kernel(TimeMix a,
         }
       }
     } else {
-      lds_barrier();
+      landed();
     }
   }
   float* so = OUT ? a.state + ((size_t)rg.slot * a.H + h) * D * D : scratch + ((size_t)rg.add * a.H + h) * D * D;
@@ -582,18 +595,18 @@ __global__ __launch_bounds__(64) void time_mix_pad_kernel(elt* __restrict__ y, i
 }  // namespace
 
 extern "C" int mlora_time_mix(void* y, int y_layout, int ld_y, const void* r, const void* k, const void* v, const void* g, int ld, const float* z,
-                              int ld_z, int R, const void* w2, int ld_w2, const float* w0, const float* u, const void* norm, float eps, float* state,
+                              int n_z, int ld_z, int R, const void* w2, int ld_w2, const float* w0, const float* u, const void* norm, float eps, float* state,
                               int n_seq, const int32_t* segs, int n_segs, const int32_t* tok_seq, const int32_t* tok_pos, int T, int H, int D,
                               void* stream) {
   MLORA_CHECK(y && r && k && v && g && z && w2 && w0 && u && norm && state && (segs || (tok_seq && tok_pos)), MLORA_ERR_INVALID, "time_mix: null pointer");
-  MLORA_CHECK(T >= 0 && H > 0 && D > 0 && D <= 256 && R > 0 && R <= TM_MAX_R && ld >= H * D && ld_z >= R && ld_w2 >= R && ld_w2 % 8 == 0 && ld_w2 <= TM_MAX_R && ld_y >= H * D &&
+  MLORA_CHECK(T >= 0 && H > 0 && D > 0 && D <= 256 && n_z >= 1 && R > 0 && R <= TM_MAX_R && ld >= H * D && ld_z >= R && ld_w2 >= R && ld_w2 % 8 == 0 && ld_w2 <= TM_MAX_R && ld_y >= H * D &&
                   ld_y < H * D + 64 && n_seq > 0 && n_segs >= 0 && n_segs <= 65535 && (segs || n_segs == T),
               MLORA_ERR_UNSUPPORTED, "time_mix: need heads of at most 256 channels and a decay rank of at most %d (T=%d H=%d D=%d R=%d)", TM_MAX_R, T, H, D, R);
   MLORA_CHECK(y_layout == MLORA_ROWMAJOR || (ld_y % 32 == 0 && sizeof(elt) == 2), MLORA_ERR_UNSUPPORTED, "time_mix: fragment order needs whole blocks of 32");
   if (T == 0 || n_segs == 0) return MLORA_OK;
   TimeMix a;
   a.y = (elt*)y; a.frag_tt = y_layout == MLORA_FRAG ? mlora_frag_tiles(T) : 0; a.ld_y = ld_y;
-  a.r = (const elt*)r; a.k = (const elt*)k; a.v = (const elt*)v; a.g = (const elt*)g; a.ld = ld; a.z = z; a.ld_z = ld_z; a.R = R;
+  a.r = (const elt*)r; a.k = (const elt*)k; a.v = (const elt*)v; a.g = (const elt*)g; a.ld = ld; a.z = z; a.n_z = n_z; a.ld_z = ld_z; a.R = R;
   a.w2 = (const elt*)w2; a.ld_w2 = ld_w2; a.w0 = w0; a.u = u; a.norm = (const elt*)norm; a.eps = eps; a.state = state; a.n_seq = n_seq;
   a.H = H; a.D = D; a.T = T; a.segs = (const int4*)segs; a.tok_seq = tok_seq; a.tok_pos = tok_pos;
   hipStream_t s = (hipStream_t)stream;
@@ -612,7 +625,7 @@ extern "C" int mlora_time_mix(void* y, int y_layout, int ld_y, const void* r, co
 #ifndef MLORA_ELT_F32
 template <int NT, bool FULL, bool OUT>
 static int launch_time_mix_chunk(const TimeMix& a, const void* zp, int rb, const int32_t* ranges, int n_ranges, float* scratch, float* decay, hipStream_t s) {
-  constexpr size_t lds = (OUT ? (size_t)(NT * NT + NT) * 1024 : 0) + (size_t)NT * 512 + NT * 64;
+  constexpr size_t lds = (OUT ? (size_t)(NT * NT + NT) * 1024 : 0) + (size_t)(NT + 2 * 3 * TC_RK) * 1024 + NT * 64;
   static const hipError_t configured =               // the attribute is per kernel, set once per process, by one thread
       hipFuncSetAttribute((const void*)time_mix_chunk_kernel<NT, FULL, OUT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
   if (configured != hipSuccess) return mlora_set_error(MLORA_ERR_LAUNCH, "time_mix_prompt: cannot reserve %zu bytes of LDS", lds);

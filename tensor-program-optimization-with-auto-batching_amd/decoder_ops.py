@@ -169,11 +169,11 @@ def linear_sum(x, W, split=True):
 
 def linear_groups(x, W, group_rows, ext):
     """W's row groups of group_rows applied to activations of their own, the blocks of the FragActivation x one after the other: ->
-    (all groups' results [T, rows], those of the last `ext` rows [T, ext] fp32, a group of their own).  T <= 64."""
+    (all groups' results [T, rows], those of the last `ext` rows, a group of their own, as partial sums [n, T, ext] fp32).  T <= 64."""
     T, K = x.shape
     n = W.shape[0] - ext
     y = torch.empty((T, n), dtype=W.dtype, device=x.device)
-    y2 = torch.empty((T, ext), dtype=torch.float32, device=x.device)
+    y2 = torch.empty((lib_of(W.dtype).mlora_gemv_groups_parts(K), T, ext), dtype=torch.float32, device=x.device)
     stride = x.data.numel() // (n // group_rows + 1)
     check(lib_of(W.dtype).mlora_gemv_frag_groups(_dev(y), _dev(y2), x.data.data_ptr(), stride, group_rows, W.data.data_ptr(), T, K, n, ext, _stream()),
           W.dtype)
@@ -263,14 +263,14 @@ def gate_up_silu(x, W, W_il, out):
 
 
 def time_mix(r, k, v, g, z, R, w2, w0, u, norm, eps, state, segs, tok_seq, tok_pos, out):
-    """The recurrence of time mixing (csrc/time_mix.hip) over a pass: r, k, v, g [T, >= H * D] of one row stride, z [T, >= R] fp32, state
+    """The recurrence of time mixing (csrc/time_mix.hip) over a pass: r, k, v, g [T, >= H * D] of one row stride, z [n, T, >= R] fp32 (partial sums), state
     [n, H, D, D] fp32 (updated), segs [n][4] int32 or None (a decode step) -> out, an activation [T, H * D rounded up]."""
     T = r.shape[0]
     (r_p, ld), (k_p, _), (v_p, _), (g_p, _) = (_cols(t, r.dtype) for t in (r, k, v, g))
     n_seq, H, D, _ = state.shape
     frag = isinstance(out, FragActivation)
     check(lib_of(r.dtype).mlora_time_mix(out.data.data_ptr() if frag else _dev(out, r.dtype), FRAG if frag else ROWMAJOR, out.shape[1],
-                                         r_p, k_p, v_p, g_p, ld, _dev(z, torch.float32), z.shape[1], R,
+                                         r_p, k_p, v_p, g_p, ld, _dev(z, torch.float32), z.shape[0], z.shape[2], R,
                                          _dev(w2, r.dtype), w2.shape[1], _dev(w0, torch.float32), _dev(u, torch.float32), _dev(norm, r.dtype), eps,
                                          _dev(state, torch.float32), n_seq, _ptr(segs), T if segs is None else segs.shape[0],
                                          _dev(tok_seq, torch.int32), _dev(tok_pos, torch.int32), T, H, D, _stream()), r.dtype)

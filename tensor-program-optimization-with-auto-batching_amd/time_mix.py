@@ -77,5 +77,5 @@ class TimeMix:
             r, k, v, g = (ops.linear(m, self.proj[s]) for m, s in zip(mixes, "rkvg"))
             if plan is not None:
                 return D.time_mix_prompt(plan, r, k, v, g, mixes[4], self.w1, *rest, out)
-            z = ops.linear(mixes[4], self.w1, out_dtype=torch.float32)
+            z = ops.linear(mixes[4], self.w1, out_dtype=torch.float32)[None]
         return D.time_mix(r, k, v, g, z, self.rank, *rest, segs, tok_seq, tok_pos, out)

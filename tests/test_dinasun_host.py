@@ -86,7 +86,7 @@ def test_argument_validation():
     assert step(b, Hp=40) == -2 and step(b, x=None) == -1 and step(b, n_part=1) == -1 and step(b, rows=16) == -1 and step(b, ld_row=32) == -1
     assert step(f, out_frag=16) == -2 and step(b, mu=16) == -1
     assert step(b, mu=16, shift=16, tok_seq=16, tok_pos=16, n_seq=1, y=16, x_out=16) == -1          # would update in place what neighbours read
-    mix = lambda lib=b, lay=0, ld_y=64, D=32, R=8, segs=None, n=4: lib.mlora_time_mix(16, lay, ld_y, 16, 16, 16, 16, 64, 16, 32, R, 16, 64, 16, 16, 16, 1e-5, 16,
+    mix = lambda lib=b, lay=0, ld_y=64, D=32, R=8, segs=None, n=4: lib.mlora_time_mix(16, lay, ld_y, 16, 16, 16, 16, 64, 16, 1, 32, R, 16, 64, 16, 16, 16, 1e-5, 16,
                                                                                     2, segs, n, 16, 16, 4, 2, D, None)
     assert mix(D=33) == -2 and mix(R=300) == -2 and mix(f, lay=1) == -2 and mix(n=3) == -2 and mix(ld_y=128) == -2
     att = lambda lib, G=2, D=40, splits=1, ws=None, n=0: lib.mlora_tied_attn(16, 0, 16, 16, 16, 16, 4, 16, 16, 16, 0.1, 2, 6, G, D, 8, 2, splits, ws, n, None)
