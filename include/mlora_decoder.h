@@ -75,6 +75,9 @@ int mlora_linear_ksplit_store(float* y, float* part, int ks, const void* xf, con
 int mlora_gemv_groups_parts(int K);
 int mlora_gemv_frag_groups(void* y, float* y2, const void* xf, long x_stride, int group_rows, const void* Wp, int T, int K, int N_main, int N_ext,
                            void* stream);
+/* The same for more than 64 tokens, without the last group: mlora_narrow_linear, y [T, N] fp32 = xf . Wp^T for few rows N, takes that. */
+int mlora_gemm_frag_groups(void* y, const void* xf, long x_stride, int group_rows, const void* Wp, int T, int K, int N, void* stream);
+int mlora_narrow_linear(float* out, const void* xf, const void* Wp, int T, int K, int N, void* stream);
 
 /* x [T, H] fp32 = table[ids[t]] * scale (zero for an id outside 0..V-1), and the same in elements (out_frag and / or out_row). */
 int mlora_embed_scaled(float* x, void* out_frag, void* out_row, int ld_row, const void* table, const int32_t* ids, float scale, int T, int H, int V,

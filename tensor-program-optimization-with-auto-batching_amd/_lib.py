@@ -134,6 +134,8 @@ DECODER_SIGNATURES = {
     "mlora_stream_step": (_i, [C.POINTER(StreamStep), _p]),
     "mlora_embed_scaled": (_i, [_p, _p, _p, _i, _p, _p, _f, _i, _i, _i, _p]),
     "mlora_linear_ksplit_store": (_i, [_p, _p, _i, _p, _p, _i, _i, _i, _p]),
+    "mlora_gemm_frag_groups": (_i, [_p, _p, _l, _i, _p, _i, _i, _i, _p]),
+    "mlora_narrow_linear": (_i, [_p, _p, _p, _i, _i, _i, _p]),
     "mlora_gemv_groups_parts": (_i, [_i]),
     "mlora_gemv_frag_groups": (_i, [_p, _p, _p, _l, _i, _p, _i, _i, _i, _i, _p]),
     "mlora_time_mix": (_i, [_p, _i, _i, _p, _p, _p, _p, _i, _p, _i, _i, _i, _p, _i, _p, _p, _p, _f, _p, _i, _p, _i, _p, _p, _i, _i, _i, _p]),
@@ -171,7 +173,8 @@ DECODER_SIGNATURES = {
 # ... and those that the fp32 library does not have
 MATRIX_CORE_ONLY = ("mlora_token_gate", "mlora_latent_attn_out", "mlora_latent_prefill", "mlora_latent_prefill_tile_tokens", "mlora_latent_prefill_served",
                     "mlora_latent_prefill_scratch_elems", "mlora_tied_prefill", "mlora_tied_prefill_served", "mlora_tied_prefill_scratch_elems",
-                    "mlora_linear_ksplit_store", "mlora_gemv_frag_groups", "mlora_gemv_groups_parts", "mlora_tanh_parts", "mlora_time_mix_prompt", "mlora_time_mix_prompt_served")
+                    "mlora_linear_ksplit_store", "mlora_gemv_frag_groups", "mlora_gemv_groups_parts", "mlora_gemm_frag_groups",
+                    "mlora_narrow_linear", "mlora_tanh_parts", "mlora_time_mix_prompt", "mlora_time_mix_prompt_served")
 
 _libs = {}
 

@@ -734,10 +734,11 @@ int launch_gemm_pp(void* y, const elt* x, int ldx, int x_tt, const elt* Wp, int 
 // ---------------------------------------------------------------------------------------------
 constexpr int MID_KS = 2;                      // 32-k steps per stage
 
-template <int OUT, int FT, int FN>
+// GX: the rows are groups of gx_rows (a multiple of 16 FN) that read activations of their own, gx_stride elements apart.
+template <int OUT, int FT, int FN, bool GX = false>
 __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_mid_kernel(void* __restrict__ yv, float* __restrict__ part, int ld_part,
                                                                     const elt* __restrict__ xf, int x_tt, const elt* __restrict__ Wp,
-                                                                    int T, int K, int N) {
+                                                                    int T, int K, int N, int gx_rows = 0, long gx_stride = 0) {
   constexpr int MID_STAGES = FT == 16 ? 3 : 4;
   constexpr int SF = FN + FT;                  // fragments of one 32-k step: weights, then tokens
   constexpr int LF = MID_KS * SF;              // fragments per stage
@@ -756,6 +757,7 @@ __global__ __launch_bounds__(PP_WAVES* WAVE, 2) void gemm_mid_kernel(void* __res
   const int KB = K / 32;
   const int tiles = (N + 15) / 16;
   const int n0 = blockIdx.x * FN * 16, t0 = blockIdx.z * FT * 16;
+  if constexpr (GX) xf += (n0 / gx_rows) * gx_stride;
   const int per = (KB + gridDim.y - 1) / gridDim.y;
   const int kb0 = blockIdx.y * per;
   const int kb1 = kb0 + per < KB ? kb0 + per : KB;
@@ -968,17 +970,17 @@ MidShape gemm_mid_shape(int T, int K, int N, int ksplit_max) {
   return m;
 }
 
-template <int OUT, int FT, int FN>
+template <int OUT, int FT, int FN, bool GX = false>
 int launch_gemm_mid_shape(void* y, float* part, int ld_part, int ksplit, const elt* xf, int x_tt, const elt* Wp, int T, int K, int N,
-                          hipStream_t s) {
+                          hipStream_t s, int gx_rows = 0, long gx_stride = 0) {
   constexpr size_t lds = (size_t)(FT == 16 ? 3 : 4) * MID_KS * (FN + FT) * 512 * sizeof(elt);
   static_assert(lds >= (size_t)PP_WAVES * PP_OUT_ELEMS * sizeof(elt), "the output staging fits the ring");
   static const hipError_t configured =               // the attribute is per kernel, set once per process, by one thread
-      hipFuncSetAttribute((const void*)gemm_mid_kernel<OUT, FT, FN>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+      hipFuncSetAttribute((const void*)gemm_mid_kernel<OUT, FT, FN, GX>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
   if (configured != hipSuccess)
     return mlora_set_error(MLORA_ERR_LAUNCH, "linear_frag: cannot reserve %zu bytes of LDS: %s", lds, hipGetErrorString(configured));
   const dim3 grid(ceil_div(N, FN * 16), ksplit, ceil_div(T, FT * 16));
-  hipLaunchKernelGGL((gemm_mid_kernel<OUT, FT, FN>), grid, dim3(PP_WAVES * WAVE), lds, s, y, part, ld_part, xf, x_tt, Wp, T, K, N);
+  hipLaunchKernelGGL((gemm_mid_kernel<OUT, FT, FN, GX>), grid, dim3(PP_WAVES * WAVE), lds, s, y, part, ld_part, xf, x_tt, Wp, T, K, N, gx_rows, gx_stride);
   return MLORA_OK;
 }
 
@@ -1209,6 +1211,23 @@ int mlora_gemm_grouped(void* y, const void* xf, int x_tt, const void* Wp, const 
 #endif
 
 #ifdef MLORA_ELT_BF16
+extern "C" int mlora_gemm_frag_groups(void* y, const void* xf, long x_stride, int group_rows, const void* Wp, int T, int K, int N, void* stream) {
+  if (int e = mlora_check_linear("gemm_frag_groups", y, MLORA_F16, MLORA_STORE, xf, K, Wp, T, K, N)) return e;
+  MLORA_CHECK(T > 64 && T <= 65535 && group_rows > 0 && group_rows % 64 == 0 && N % group_rows == 0 && x_stride % 8 == 0 && ((uintptr_t)xf & 15) == 0,
+              MLORA_ERR_UNSUPPORTED, "gemm_frag_groups: more than 64 tokens and groups of whole 64 rows (T=%d rows=%d N=%d)", T, group_rows, N);
+  hipStream_t s = (hipStream_t)stream;
+  const elt* x = (const elt*)xf;
+  const elt* W = (const elt*)Wp;
+  const int tt = mlora_frag_tiles(T);
+  int e;
+  if (group_rows % 128 == 0 && (long)(N / 64) * ceil_div(T, 128) > 256)        // 128 rows a workgroup where that leaves one for every unit
+    e = T <= 128 ? launch_gemm_mid_shape<OUT_F16, 8, 8, true>(y, nullptr, 0, 1, x, tt, W, T, K, N, s, group_rows, x_stride)
+                 : launch_gemm_mid_shape<OUT_F16, 16, 8, true>(y, nullptr, 0, 1, x, tt, W, T, K, N, s, group_rows, x_stride);
+  else
+    e = launch_gemm_mid_shape<OUT_F16, 8, 4, true>(y, nullptr, 0, 1, x, tt, W, T, K, N, s, group_rows, x_stride);
+  return e ? e : mlora_launch_status("gemm_frag_groups");
+}
+
 int mlora_gemv_ksplit_store(float* y, float* part, int ks, const void* xf, const void* Wp, int T, int K, int N, void* stream);
 
 // y [T, N] fp32 = xf . Wp^T over ks K slices (mlora_gemv_ksplit): slice 0 into y, slices 1.. into part[ks - 1][T][N]

@@ -127,6 +127,12 @@ struct TokenGate {
     *reinterpret_cast<eltx4*>(out + frag_offset(t, n, frag_tt)) = o;
   }
 };
+//   s itself, out [T][N] fp32
+struct PlainRows {
+  float* out;
+  int N;
+  __device__ __forceinline__ void operator()(int t, int n, f32x4 s, int) const { *reinterpret_cast<f32x4*>(out + (size_t)t * N + n) = s; }
+};
 //   tanh(s) in full precision as the sum of three elements, out [T][3][N]
 struct TanhParts {
   elt* out;
@@ -524,6 +530,15 @@ extern "C" int mlora_token_gate(void* out_frag, const void* xf, const void* Wp, 
   if (T == 0) return MLORA_OK;
   launch_narrow(TokenGate{(elt*)out_frag, (const elt*)table, ld_table, col0, dim, ids, V}, xf, Wp, T, K, N, (hipStream_t)stream);
   return mlora_launch_status("token_gate");
+}
+
+extern "C" int mlora_narrow_linear(float* out, const void* xf, const void* Wp, int T, int K, int N, void* stream) {
+  MLORA_CHECK(out && xf && Wp, MLORA_ERR_INVALID, "narrow_linear: null pointer");
+  MLORA_CHECK(T >= 0 && K > 0 && K % 32 == 0 && N > 0 && N % 32 == 0 && ceil_div(T, 16) <= 65535, MLORA_ERR_UNSUPPORTED,
+              "narrow_linear: need K %% 32 == 0, N %% 32 == 0 (T=%d K=%d N=%d)", T, K, N);
+  if (T == 0) return MLORA_OK;
+  launch_narrow(PlainRows{out, N}, xf, Wp, T, K, N, (hipStream_t)stream);
+  return mlora_launch_status("narrow_linear");
 }
 
 extern "C" int mlora_tanh_parts(void* out, const void* xf, const void* Wp, int T, int K, int N, void* stream) {

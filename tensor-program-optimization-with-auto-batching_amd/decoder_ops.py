@@ -169,14 +169,18 @@ def linear_sum(x, W, split=True):
 
 def linear_groups(x, W, group_rows, ext):
     """W's row groups of group_rows applied to activations of their own, the blocks of the FragActivation x one after the other: ->
-    (all groups' results [T, rows], those of the last `ext` rows, a group of their own, as partial sums [n, T, ext] fp32).  T <= 64."""
+    (all groups' results [T, rows], those of the last `ext` rows, a group of their own, as partial sums [n, T, ext] fp32)."""
     T, K = x.shape
-    n = W.shape[0] - ext
+    n, L = W.shape[0] - ext, lib_of(W.dtype)
     y = torch.empty((T, n), dtype=W.dtype, device=x.device)
-    y2 = torch.empty((lib_of(W.dtype).mlora_gemv_groups_parts(K), T, ext), dtype=torch.float32, device=x.device)
     stride = x.data.numel() // (n // group_rows + 1)
-    check(lib_of(W.dtype).mlora_gemv_frag_groups(_dev(y), _dev(y2), x.data.data_ptr(), stride, group_rows, W.data.data_ptr(), T, K, n, ext, _stream()),
-          W.dtype)
+    if T > 64:
+        y2 = torch.empty((1, T, ext), dtype=torch.float32, device=x.device)
+        check(L.mlora_gemm_frag_groups(_dev(y), x.data.data_ptr(), stride, group_rows, W.data.data_ptr(), T, K, n, _stream()), W.dtype)
+        check(L.mlora_narrow_linear(_dev(y2), x.data[x.data.numel() - stride:].data_ptr(), W.rows(n, ext).data.data_ptr(), T, K, ext, _stream()), W.dtype)
+        return y, y2
+    y2 = torch.empty((L.mlora_gemv_groups_parts(K), T, ext), dtype=torch.float32, device=x.device)
+    check(L.mlora_gemv_frag_groups(_dev(y), _dev(y2), x.data.data_ptr(), stride, group_rows, W.data.data_ptr(), T, K, n, ext, _stream()), W.dtype)
     return y, y2
 
 

@@ -69,7 +69,7 @@ class TimeMix:
         T, dev, n = mixes[0].shape[0], mixes[0].device, self.out_cols
         out = D.activation(T, n, self.dtype, dev)
         rest = (self.w2, self.w0, self.u, self.norm, self.eps, state)
-        if plan is None and self.all is not None and T <= 64 and self.w1.N <= n:
+        if plan is None and self.all is not None and T <= 256 and self.w1.N <= n:
             x = mixes[0]
             y, z = D.linear_groups(ops.FragActivation(T, x.K, dev, x.room), self.all, n, self.w1.N)
             r, k, v, g = (y[:, i * n:(i + 1) * n] for i in range(4))
