@@ -258,8 +258,9 @@ __global__ __launch_bounds__(TS_THREADS) void time_mix_step_kernel(TimeMix a) {
 // token m of the lower half of their block of 2 h, exp(Lx_t - L_m) exp(L_m - L_s).  At every level h = 8, 4, 2, 1 a token is in one
 // half, so one vector x per token and level holds r's factor or k's, and the level's part of A is a part of x x^T.  Decays of any
 // strength are served; nothing overflows.
-// fp32 operands of the matrix cores are hi + lo pairs, in the two halves of the 32 k-slots: slot (g, e) is index 4 g + e for
-// e < 4 as hi (or of the one factor) and again for e >= 4 as lo.  That is also how a lane holds a result (rows 4 g + r), so a
+// fp32 operands of the matrix cores are hi + lo pairs (what enters the state has a third part, and values are elements, so that the
+// state is summed in fp32), in the two halves of the 32 k-slots: slot (g, e) is index 4 g + e for e < 4 as hi (or of the one factor)
+// and again for e >= 4 as lo.  That is also how a lane holds a result (rows 4 g + r), so a
 // state tile is an operand as it stands, and a product with the identity turns a factor over.
 //
 // A workgroup takes one head and up to a range of `tokens` of a sequence; wave w holds keys 16 w .. + 15 of the state (all values) and
@@ -437,7 +438,10 @@ __global__ __launch_bounds__(NT * WAVE, 2) void time_mix_chunk_kernel(TimeMix a,
       Lt[e] = row_lane<15>(x);
     }
     const f32x4 dec = exp2_4(Lt);
-    const HiLo kd(k4 * exp2_4(Lt - Li));                             // keys as the state takes them
+    // keys as the state takes them: three parts, all of fp32
+    const f32x4 kf = k4 * exp2_4(Lt - Li);
+    const HiLo kd(kf);
+    const u32x2 ke = __builtin_bit_cast(u32x2, __builtin_convertvector(kf - floats(u32x2{kd.h[0], kd.h[1]}) - floats(u32x2{kd.l[0], kd.l[1]}), eltx4));
     st8(vs + (w * 64 + lane) * 8, vv);
     if constexpr (OUT) {
       // this wave's keys' part of A: A^T[s = 4 g + r][t = q16]
@@ -501,9 +505,14 @@ __global__ __launch_bounds__(NT * WAVE, 2) void time_mix_chunk_kernel(TimeMix a,
       const eltx8 kb = both(kd);
       const f32x4 th = mfma_16x16x32(kb, idh, f32x4{0.f, 0.f, 0.f, 0.f}), tlo = mfma_16x16x32(kb, idl, f32x4{0.f, 0.f, 0.f, 0.f});   // [s = 4 g + r][key 16 w + q16]
       const u32x2 uh = __builtin_bit_cast(u32x2, __builtin_convertvector(th, eltx4)), ul = __builtin_bit_cast(u32x2, __builtin_convertvector(tlo, eltx4));
-      const eltx8 kt = operand(uh[0], uh[1], ul[0], ul[1]);
+      const f32x4 te = mfma_16x16x32(operand(ke[0], ke[1], 0u, 0u), idh, f32x4{0.f, 0.f, 0.f, 0.f});
+      const u32x2 ue = __builtin_bit_cast(u32x2, __builtin_convertvector(te, eltx4));
+      const eltx8 kt = operand(uh[0], uh[1], ul[0], ul[1]), kr = operand(ue[0], ue[1], 0u, 0u);
 #pragma unroll
-      for (int n = 0; n < NT; ++n) S[n] = mfma_16x16x32(kt, ld8(vs + (n * 64 + lane) * 8), S[n] * dec);
+      for (int n = 0; n < NT; ++n) {
+        const eltx8 v = ld8(vs + (n * 64 + lane) * 8);
+        S[n] = mfma_16x16x32(kr, v, mfma_16x16x32(kt, v, S[n] * dec));
+      }
       if (!OUT) keep *= dec;
     }
     if constexpr (OUT) {
