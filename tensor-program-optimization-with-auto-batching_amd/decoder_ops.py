@@ -117,9 +117,8 @@ class ResidualStream:
             return
         T, Hp = self.shape
         a = StreamStep(T=T, Hp=Hp, x=self.x.data_ptr(), mult=self.mult, row_weight=1.0)
-        keep = None
         if self.pending is not None:
-            y, parts, rows, a.row_weight, post, new = keep = self.pending
+            y, parts, rows, a.row_weight, post, new = self.pending
             if y is not None:
                 a.y = _dev(y, torch.float32)
             if parts is not None:
@@ -150,7 +149,6 @@ class ResidualStream:
             a.mu, a.shift, a.n_seq = _dev(mu, self.dtype), _dev(shift, torch.float32), shift.shape[0]
             a.tok_seq, a.tok_pos, a.tok_last = _dev(seq, torch.int32), _dev(pos, torch.int32), _ptr(last)
         check(lib_of(self.dtype).mlora_stream_step(ctypes.byref(a), _stream()), self.dtype)
-        del keep
 
 
 def linear_sum(x, W, split=True):

@@ -179,8 +179,8 @@ class DinasunForCausalLM(CausalLM):
                     stream.step(out=entry.columns(0, Hp))
                 stream.replace(*D.linear_sum(entry, self.loop_in, split))
             if isinstance(mixer, TimeMix):
-                room, mixes = mixer.mixes(T, Hp, stream.device)
-                stream.step(L["norm1"], mu=mixer.mu, shift=kv.shift(run), tokens=kv.token_meta(), **room)
+                mixes = mixer.mixes(T, Hp, stream.device)
+                stream.step(L["norm1"], mu=mixer.mu, shift=kv.shift(run), tokens=kv.token_meta(), **mixes.room())
                 y = kv.time_mix(run, mixes, mixer)
             else:
                 y = kv.tied_attention(run, ops.linear(self._normed(stream, L["norm1"])[0], mixer.proj, out_dtype=torch.float32), mixer)

@@ -219,18 +219,11 @@ class PagedStateCache(PageTable):
     kernels start a sequence's state from zero at its position 0."""
 
     def __init__(self, runs, width_p, n_pages, max_seqs, max_blocks, max_pos, dtype, device="cuda:0", free_pages=None, page_size=PAGE):
-        """runs: per layer run the mixer's spec (TiedSpec or TimeMixSpec); width_p: columns of the residual stream."""
+        """runs: per layer run the mixer's spec, whose cache_entry says what is kept; width_p: columns of the residual stream."""
         super().__init__(n_pages, max_seqs, max_blocks, max_pos, device, free_pages, page_size)
         self.dtype = dtype
-        self.entries = []
-        zeros = lambda *shape, dt=torch.float32: torch.zeros(shape, dtype=dt, device=self.device)
-        for s in runs:
-            if hasattr(s, "kv_heads"):
-                # pages [n_pages, G, dim / 32, 4, 16, 8] of values, and one key scale per token and head
-                self.entries.append((zeros(n_pages, s.kv_heads, -(-s.dim // 32), 4, PAGE, 8, dt=dtype), zeros(n_pages, s.kv_heads, PAGE)))
-            else:
-                # matrix states, and the previous token's normed row
-                self.entries.append((zeros(max_seqs, s.heads, s.dim, s.dim), zeros(max_seqs, width_p)))
+        self.entries = [tuple(torch.zeros(shape, dtype=dtype if elements else torch.float32, device=self.device)
+                              for shape, elements in s.cache_entry(n_pages, max_seqs, PAGE, width_p)) for s in runs]
         self._meta = None
 
     def values(self, run, sid):

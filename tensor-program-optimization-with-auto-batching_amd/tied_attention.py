@@ -32,6 +32,10 @@ class TiedSpec:
             raise ValueError(f"tied attention needs values as wide as its keys and whole groups of heads: {c}")
         return s
 
+    def cache_entry(self, n_pages, slots, page, width_p):
+        """Shapes of what a layer run keeps (and whether in elements rather than fp32): pages of values, and key scales."""
+        return ((n_pages, self.kv_heads, -(-self.dim // 32), 4, page, 8), True), ((n_pages, self.kv_heads, page), False)
+
 
 def distance_slopes(heads: int) -> torch.Tensor:
     """2^(-8 (h + 1) / heads)."""

@@ -24,6 +24,26 @@ class TimeMixSpec:
     def from_config(cls, c: dict) -> "TimeMixSpec":
         return cls(int(c["heads"]), int(c["dim"]))
 
+    def cache_entry(self, n_pages, slots, page, width_p):
+        """Shapes of what a layer run keeps (and whether in elements rather than fp32): matrix states, and previous tokens' rows."""
+        return ((slots, self.heads, self.dim, self.dim), False), ((slots, width_p), False)
+
+
+@dataclasses.dataclass
+class Mixes:
+    """The five mixes of a pass: activations that lie one after the other in one buffer."""
+    parts: list
+    data: torch.Tensor
+
+    def room(self) -> dict:
+        """What a stream step fills."""
+        return {"out_row": self.data} if self.data.dtype == torch.float32 else {"out": self.all()}
+
+    def all(self):
+        """All of them as one activation (bfloat16)."""
+        x = self.parts[0]
+        return ops.FragActivation(x.T, x.K, x.device, self.data)
+
 
 class TimeMix:
     """Weights of one layer in kernel order."""
@@ -51,31 +71,28 @@ class TimeMix:
         self.o = D.weight(padded(t("o"), Hp, self.out_cols))
         self.prompt_form = dtype != torch.float32 and D.time_mix_prompt_served(spec.dim)
 
-    def mixes(self, T, width_p, device):
-        """Room for the five mixes of a pass: (what a stream step fills as out or out_row, the five activations - which lie in it one
-        after the other)."""
+    def mixes(self, T, width_p, device) -> Mixes:
+        """Room for the five mixes of a pass."""
         if self.dtype == torch.float32:
             rows = torch.empty((len(MIXES), T, width_p), dtype=self.dtype, device=device)
-            return {"out_row": rows}, list(rows)
+            return Mixes(list(rows), rows)
         n = ops.lib_of(self.dtype).mlora_frag_activation_elems(T, width_p)
         data = torch.empty(len(MIXES) * n, dtype=self.dtype, device=device)
-        acts = [ops.FragActivation(T, width_p, device, data[i * n:(i + 1) * n]) for i in range(len(MIXES))]
-        acts[0].room = data                                                      # all five, for the product that takes them together
-        return {"out": ops.FragActivation(T, width_p, device, data)}, acts
+        return Mixes([ops.FragActivation(T, width_p, device, data[i * n:(i + 1) * n]) for i in range(len(MIXES))], data)
 
-    def run(self, mixes, state, segs, tok_seq, tok_pos, plan=None):
-        """mixes: the five activations -> the gated outputs of the heads, an activation of out_cols columns; updates state.
+    def run(self, mixes: Mixes, state, segs, tok_seq, tok_pos, plan=None):
+        """-> the gated outputs of the heads, an activation of out_cols columns; updates state.
         segs: the sequences of the pass (None: a decode step); plan: a TimeMixPlan of the pass for the prompt form."""
-        T, dev, n = mixes[0].shape[0], mixes[0].device, self.out_cols
+        parts = mixes.parts
+        T, dev, n = parts[0].shape[0], parts[0].device, self.out_cols
         out = D.activation(T, n, self.dtype, dev)
         rest = (self.w2, self.w0, self.u, self.norm, self.eps, state)
         if plan is None and self.all is not None and T <= 256 and self.w1.N <= n:
-            x = mixes[0]
-            y, z = D.linear_groups(ops.FragActivation(T, x.K, dev, x.room), self.all, n, self.w1.N)
+            y, z = D.linear_groups(mixes.all(), self.all, n, self.w1.N)
             r, k, v, g = (y[:, i * n:(i + 1) * n] for i in range(4))
         else:
-            r, k, v, g = (ops.linear(m, self.proj[s]) for m, s in zip(mixes, "rkvg"))
+            r, k, v, g = (ops.linear(m, self.proj[s]) for m, s in zip(parts, "rkvg"))
             if plan is not None:
-                return D.time_mix_prompt(plan, r, k, v, g, mixes[4], self.w1, *rest, out)
-            z = ops.linear(mixes[4], self.w1, out_dtype=torch.float32)[None]
+                return D.time_mix_prompt(plan, r, k, v, g, parts[4], self.w1, *rest, out)
+            z = ops.linear(parts[4], self.w1, out_dtype=torch.float32)[None]
         return D.time_mix(r, k, v, g, z, self.rank, *rest, segs, tok_seq, tok_pos, out)
